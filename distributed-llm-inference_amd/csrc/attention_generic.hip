@@ -18,6 +18,7 @@
 //   r1, r2        per query head, r1[h] * log(1 + r2[h] * (p - j)) is taken off the scaled score;
 //   sink != 0     the softmax's denominator has one more term, exp(0): a key of score 0 without a
 //                 value, so a row's weights may add up to less than one;
+//   sinks         the same with a score of its own per query head, exp(sinks[h]) in the denominator;
 //   value_dim     the size of a value where it differs from a key's;
 //   gate          float32 [tokens][gate_stride]: the result is multiplied by sigmoid(gate) element
 //                 by element (same layout as the output);
@@ -25,6 +26,7 @@
 //   v_heads       the value pages hold v_heads heads, a divisor of kv_heads, and kv head g reads the values of
 //                 head g % v_heads (several score maps over one set of values);
 //   out32         float32 [tokens][out_stride]: the result goes there unrounded instead of to `out`.
+//   v_pages == nullptr: the values are the keys, their first value_dim components (keys of up to 1,024 then).
 // tile_entry == nullptr: every entry is a single row (steps of single tokens, whose launches read
 // nothing that the host made from the step's lengths); a kernel of its own takes these, below.
 //
@@ -42,9 +44,17 @@ struct ScoreChanges {
   int keep_first;
   int v_heads;
   float* out32;
+  const float* sinks;
 };
 
-template <typename T, int RM, int RN, int DC>
+// What a row starts from: the sink's score and its weight, if there is one.
+__device__ __forceinline__ float sink_score(const ScoreChanges& sc, int head) {
+  return sc.sinks != nullptr ? sc.sinks[head] : sc.sink ? 0.f : -INFINITY;
+}
+__device__ __forceinline__ bool has_sink(const ScoreChanges& sc) { return sc.sinks != nullptr || sc.sink; }
+
+// KV: the values are the keys' first components.
+template <typename T, int RM, int RN, int DC, bool KV>
 __global__ __launch_bounds__(256) void attention_generic_kernel(
     const T* __restrict__ q, int64_t q_stride, const T* __restrict__ k_pages,
     const T* __restrict__ v_pages, T* __restrict__ out, int64_t out_stride,
@@ -55,7 +65,7 @@ __global__ __launch_bounds__(256) void attention_generic_kernel(
   constexpr int BM = 16 * RM, BN = 16 * RN, DMAX = 16 * DC;
   __shared__ float qs[BM][DMAX + 1];
   __shared__ float ks[BN][DMAX + 1];
-  __shared__ float vs[BN][DMAX + 1];
+  __shared__ float vs_[KV ? 1 : BN][KV ? 1 : DMAX + 1];
   __shared__ float ps[BM][BN + 1];
 
   const int tid = threadIdx.x, tx = tid % 16, ty = tid / 16;
@@ -81,8 +91,8 @@ __global__ __launch_bounds__(256) void attention_generic_kernel(
   float m_run[RM], l_run[RM], acc[RM][DC];
 #pragma unroll
   for (int i = 0; i < RM; ++i) {
-    m_run[i] = sc.sink ? 0.f : -INFINITY;  // the sink: a key of score 0 that brings no value
-    l_run[i] = sc.sink ? 1.f : 0.f;
+    m_run[i] = sink_score(sc, head);  // the sink: a key that brings no value
+    l_run[i] = has_sink(sc) ? 1.f : 0.f;
 #pragma unroll
     for (int c = 0; c < DC; ++c) acc[i][c] = 0.f;
   }
@@ -109,6 +119,7 @@ __global__ __launch_bounds__(256) void attention_generic_kernel(
       }
       ks[r][c] = kv;
     }
+    if constexpr (!KV)
     for (int idx = tid; idx < BN * value_dim; idx += 256) {
       const int c = idx / BN, r = idx - c * BN;  // key index fastest: contiguous in a V page
       const int j = j0 + r;
@@ -117,7 +128,7 @@ __global__ __launch_bounds__(256) void attention_generic_kernel(
         const int64_t page = max(table[j / page_size], 0);   // (a page that a window has passed: any page, its keys are not seen)
         vv = to_f32(v_pages[((page * sc.v_heads + vh) * value_dim + c) * page_size + j % page_size]);
       }
-      vs[r][c] = vv;
+      vs_[r][c] = vv;
     }
     __syncthreads();
 
@@ -184,7 +195,9 @@ __global__ __launch_bounds__(256) void attention_generic_kernel(
 #pragma unroll
       for (int c = 0; c < DC; ++c) {
         if (c * 16 < value_dim) {
-          const float vv = vs[jj][tx + 16 * c];
+          float vv;
+          if constexpr (KV) vv = ks[jj][tx + 16 * c];
+          else vv = vs_[jj][tx + 16 * c];
 #pragma unroll
           for (int i = 0; i < RM; ++i) acc[i][c] = fmaf(pv[i], vv, acc[i][c]);
         }
@@ -211,13 +224,13 @@ __global__ __launch_bounds__(256) void attention_generic_kernel(
   }
 }
 
-template <typename T, int RM, int RN, int DC>
+template <typename T, int RM, int RN, int DC, bool KV>
 static int launch_generic(const void* q, int64_t q_stride, const void* k_pages, const void* v_pages,
                           void* out, int64_t out_stride, const int* q_start, const int* kv_len,
                           const int* block_tables, int table_stride, const int* tile_entry,
                           const int* tile_q0, int tiles, int q_heads, int kv_heads, int head_dim,
                           int page_size, float scale, int window, ScoreChanges sc, hipStream_t stream) {
-  attention_generic_kernel<T, RM, RN, DC><<<dim3(tiles, q_heads), 256, 0, stream>>>(
+  attention_generic_kernel<T, RM, RN, DC, KV><<<dim3(tiles, q_heads), 256, 0, stream>>>(
       (const T*)q, q_stride, (const T*)k_pages, (const T*)v_pages, (T*)out, out_stride, q_start,
       kv_len, block_tables, table_stride, tile_entry, tile_q0, q_heads, kv_heads, head_dim,
       page_size, scale, window, sc);
@@ -237,7 +250,7 @@ template <typename T> struct Pack16;   // what 16 bytes hold
 template <> struct Pack16<bf16_t> { static constexpr int N = 8; typedef __bf16 type __attribute__((ext_vector_type(8))); };
 template <> struct Pack16<float> { static constexpr int N = 4; typedef float type __attribute__((ext_vector_type(4))); };
 
-template <typename T, int GQ, int VC>
+template <typename T, int GQ, int VC, bool KV>
 __global__ __launch_bounds__(512) void attention_scored_decode_kernel(
     const T* __restrict__ q, int64_t q_stride, const T* __restrict__ k_pages, const T* __restrict__ v_pages,
     T* __restrict__ out, int64_t out_stride, const int* __restrict__ kv_len, const int* __restrict__ block_tables,
@@ -270,8 +283,9 @@ __global__ __launch_bounds__(512) void attention_scored_decode_kernel(
   for (int h = 0; h < GQ; ++h) {
     r1[h] = sc.r1 != nullptr && h < nh ? sc.r1[h0 + h] : 0.f;
     r2[h] = sc.r1 != nullptr && h < nh ? sc.r2[h0 + h] : 0.f;
-    m_run[h] = sc.sink && wave == 0 && split == 0 ? 0.f : -INFINITY;           // the sink is counted once, by wave 0
-    l_run[h] = sc.sink && wave == 0 && split == 0 && lane == 0 ? 1.f : 0.f;    // (sums are kept lane by lane until the end)
+    const bool first = wave == 0 && split == 0;                                // the sink is counted once, by wave 0
+    m_run[h] = first && h < nh ? sink_score(sc, h0 + h) : -INFINITY;
+    l_run[h] = first && lane == 0 && h < nh && has_sink(sc) ? 1.f : 0.f;    // (sums are kept lane by lane until the end)
 #pragma unroll
     for (int c = 0; c < VC; ++c) acc[h][c] = 0.f;
   }
@@ -339,6 +353,29 @@ __global__ __launch_bounds__(512) void attention_scored_decode_kernel(
     // lanes are value columns now
     const int last = min(63, pos - j0);
     const int first = keep > 0 ? 0 : max(0, j_begin - j0);   // (keys that are not seen weigh nothing)
+    if constexpr (KV) {
+      // a value is the front of its key's row: the 64 lanes read neighbouring components of one key after
+      // the other, eight keys asked for at a time (keys that are not seen weigh nothing)
+      const int64_t my_row = ((int64_t)my_page * kv_heads + kvh) * page_size + j % page_size;
+#pragma unroll
+      for (int c = 0; c < VC; ++c) {
+        const int col = min(lane + 64 * c, value_dim - 1);
+        for (int jj = 0; jj < 64; jj += 8) {
+          float vf[8];
+#pragma unroll
+          for (int e = 0; e < 8; ++e) {
+            const int64_t row = (int64_t)__shfl((int)my_row, jj + e, DLI_WAVE);
+            vf[e] = to_f32(k_pages[row * head_dim + col]);
+          }
+#pragma unroll
+          for (int e = 0; e < 8; ++e)
+#pragma unroll
+            for (int h = 0; h < GQ; ++h) acc[h][c] = fmaf(ps[(wave * GQ + h) * 64 + jj + e], vf[e], acc[h][c]);
+        }
+      }
+      __builtin_amdgcn_wave_barrier();
+      continue;
+    }
     if (v_packs) {
       // every pack of the block's 64 keys is asked for before the first is used; keys that are not
       // seen have weight zero and lie in pages that exist (or in the table's last entry's page)
@@ -467,7 +504,7 @@ __global__ void attention_scored_merge_kernel(const float* __restrict__ parts, i
   }
 }
 
-template <typename T, int GQ>
+template <typename T, int GQ, bool KV>
 static int launch_scored_decode(const void* q, int64_t q_stride, const void* k_pages, const void* v_pages, void* out,
                                 int64_t out_stride, const int* kv_len, const int* block_tables, int table_stride,
                                 int entries, int q_heads, int kv_heads, int head_dim, int page_size, float scale,
@@ -484,13 +521,15 @@ static int launch_scored_decode(const void* q, int64_t q_stride, const void* k_p
     size_t bytes = 0;                                                                                       \
     for (;; waves /= 2) {                                                                                   \
       bytes = sizeof(float) * ((size_t)GQ * head_dim + waves * GQ * 64 + 2 * waves * GQ + waves * GQ * VC * 64); \
-      if (bytes <= 65536 || waves == 4) break;                                                              \
+      if (bytes <= 65536 || waves == (KV ? 1 : 4)) break;                                                   \
     }                                                                                                       \
-    attention_scored_decode_kernel<T, GQ, VC><<<grid, 64 * waves, bytes, stream>>>(                         \
+    attention_scored_decode_kernel<T, GQ, VC, KV><<<grid, 64 * waves, bytes, stream>>>(                         \
         (const T*)q, q_stride, (const T*)k_pages, (const T*)v_pages, (T*)out, out_stride, kv_len,           \
         block_tables, table_stride, q_heads, kv_heads, head_dim, page_size, scale, window, sc, parts, splits); \
   }
-  if (vc <= 1) DECODE_LAUNCH(1) else if (vc == 2) DECODE_LAUNCH(2) else DECODE_LAUNCH(4)
+  if (vc <= 1) DECODE_LAUNCH(1) else if (vc == 2) DECODE_LAUNCH(2) else if (vc <= 4) DECODE_LAUNCH(4)
+  else if constexpr (KV && GQ <= 4) { if (vc <= 8) DECODE_LAUNCH(8) else DECODE_LAUNCH(16) }
+  else return DLI_ERR_ARGUMENT;
 #undef DECODE_LAUNCH
   if (splits > 1) {
     const int status = dli_launch_status();
@@ -505,7 +544,7 @@ static int launch_scored_decode(const void* q, int64_t q_stride, const void* k_p
 // Queries per tile for a head_dim (the larger of the key's and the value's size): the host builds
 // its tile list with this.
 extern "C" int dli_attention_generic_tile_rows(int head_dim) {
-  if (head_dim <= 0 || head_dim > 256) return DLI_ERR_ARGUMENT;
+  if (head_dim <= 0 || head_dim > 1024) return DLI_ERR_ARGUMENT;
   return head_dim <= 128 ? 32 : 16;
 }
 
@@ -518,45 +557,59 @@ static int attention_scored(const void* q, int64_t q_stride, const void* k_pages
                             int tiles, int q_heads, int kv_heads, int head_dim, int value_dim,
                             int page_size, float scale, int window, int chunk, int sink,
                             const float* r1, const float* r2, const float* gate,
-                            int64_t gate_stride, int keep_first, int v_heads, float* out32, float* parts, int splits,
-                            int is_bf16, hipStream_t stream) {
+                            int64_t gate_stride, int keep_first, int v_heads, float* out32, const float* sinks, float* parts,
+                            int splits, int is_bf16, hipStream_t stream) {
   if (tiles <= 0) return DLI_OK;
   if (v_heads <= 0) v_heads = kv_heads;
   if (keep_first < 0 || kv_heads <= 0 || kv_heads % v_heads != 0) return DLI_ERR_ARGUMENT;
   const int dmax = head_dim > value_dim ? head_dim : value_dim;
-  if (head_dim <= 0 || value_dim <= 0 || dmax > 256 || q_heads <= 0 || kv_heads <= 0 ||
+  const bool kv = v_pages == nullptr;   // the values are the keys' first components
+  if (kv && (value_dim > head_dim || v_heads != kv_heads)) return DLI_ERR_ARGUMENT;
+  if (head_dim <= 0 || value_dim <= 0 || dmax > (kv ? 1024 : 256) || q_heads <= 0 || kv_heads <= 0 ||
       q_heads % kv_heads != 0 || q_heads > 65535 || page_size <= 0 || table_stride <= 0 ||
       window < 0 || chunk < 0 || (r1 == nullptr) != (r2 == nullptr) ||
       (tile_entry == nullptr) != (tile_q0 == nullptr))
     return DLI_ERR_ARGUMENT;
-  const ScoreChanges sc = {chunk, sink, r1, r2, value_dim, gate, gate_stride, keep_first, v_heads, out32};
+  const ScoreChanges sc = {chunk, sink, r1, r2, value_dim, gate, gate_stride, keep_first, v_heads, out32, sinks};
   if (tile_entry == nullptr) {
     // every entry is one row: the kernel whose lanes own keys, then value columns
     const int group = q_heads / kv_heads;
 #define DECODE_ARGS                                                                                      \
   q, q_stride, k_pages, v_pages, out, out_stride, kv_len, block_tables, table_stride, tiles, q_heads,   \
       kv_heads, head_dim, page_size, scale, window, sc, parts, splits, stream
+#define DECODE_CASE(T, KV)                                                                               \
+  if (group == 1) return launch_scored_decode<T, 1, KV>(DECODE_ARGS);                                    \
+  if (group <= 4 || value_dim > 256) return launch_scored_decode<T, 4, KV>(DECODE_ARGS);                 \
+  return launch_scored_decode<T, 8, KV>(DECODE_ARGS);
     if (is_bf16) {
-      if (group == 1) return launch_scored_decode<bf16_t, 1>(DECODE_ARGS);
-      if (group <= 4) return launch_scored_decode<bf16_t, 4>(DECODE_ARGS);
-      return launch_scored_decode<bf16_t, 8>(DECODE_ARGS);
+      if (kv) { DECODE_CASE(bf16_t, true) }
+      DECODE_CASE(bf16_t, false)
     }
-    if (group == 1) return launch_scored_decode<float, 1>(DECODE_ARGS);
-    if (group <= 4) return launch_scored_decode<float, 4>(DECODE_ARGS);
-    return launch_scored_decode<float, 8>(DECODE_ARGS);
+    if (kv) { DECODE_CASE(float, true) }
+    DECODE_CASE(float, false)
+#undef DECODE_CASE
 #undef DECODE_ARGS
   }
 #define GENERIC_ARGS                                                                              \
   q, q_stride, k_pages, v_pages, out, out_stride, q_start, kv_len, block_tables, table_stride,   \
       tile_entry, tile_q0, tiles, q_heads, kv_heads, head_dim, page_size, scale, window, sc, stream
+#define GENERIC_CASE(T, KV)                                                          \
+  if (dmax <= 64) return launch_generic<T, 2, 2, 4, KV>(GENERIC_ARGS);               \
+  if (dmax <= 128) return launch_generic<T, 2, 2, 8, KV>(GENERIC_ARGS);              \
+  if (dmax <= 256) return launch_generic<T, 1, 1, 16, KV>(GENERIC_ARGS);
+#define GENERIC_WIDE(T)                                                              \
+  if (dmax <= 576) return launch_generic<T, 1, 1, 36, true>(GENERIC_ARGS);           \
+  return launch_generic<T, 1, 1, 64, true>(GENERIC_ARGS);
   if (is_bf16) {
-    if (dmax <= 64) return launch_generic<bf16_t, 2, 2, 4>(GENERIC_ARGS);
-    if (dmax <= 128) return launch_generic<bf16_t, 2, 2, 8>(GENERIC_ARGS);
-    return launch_generic<bf16_t, 1, 1, 16>(GENERIC_ARGS);
+    if (kv) { GENERIC_CASE(bf16_t, true) GENERIC_WIDE(bf16_t) }
+    GENERIC_CASE(bf16_t, false)
+  } else {
+    if (kv) { GENERIC_CASE(float, true) GENERIC_WIDE(float) }
+    GENERIC_CASE(float, false)
   }
-  if (dmax <= 64) return launch_generic<float, 2, 2, 4>(GENERIC_ARGS);
-  if (dmax <= 128) return launch_generic<float, 2, 2, 8>(GENERIC_ARGS);
-  return launch_generic<float, 1, 1, 16>(GENERIC_ARGS);
+  return DLI_ERR_ARGUMENT;
+#undef GENERIC_CASE
+#undef GENERIC_WIDE
 #undef GENERIC_ARGS
 }
 
@@ -567,11 +620,11 @@ extern "C" int dli_attention_scored(const void* q, int64_t q_stride, const void*
                                     int tiles, int q_heads, int kv_heads, int head_dim, int value_dim,
                                     int page_size, float scale, int window, int chunk, int sink,
                                     const float* r1, const float* r2, const float* gate,
-                                    int64_t gate_stride, int keep_first, int v_heads, float* out32, int is_bf16,
-                                    hipStream_t stream) {
+                                    int64_t gate_stride, int keep_first, int v_heads, float* out32,
+                                    const float* sinks, int is_bf16, hipStream_t stream) {
   return attention_scored(q, q_stride, k_pages, v_pages, out, out_stride, q_start, kv_len, block_tables, table_stride,
                           tile_entry, tile_q0, tiles, q_heads, kv_heads, head_dim, value_dim, page_size, scale, window,
-                          chunk, sink, r1, r2, gate, gate_stride, keep_first, v_heads, out32, nullptr, 1, is_bf16, stream);
+                          chunk, sink, r1, r2, gate, gate_stride, keep_first, v_heads, out32, sinks, nullptr, 1, is_bf16, stream);
 }
 
 // How many workgroups share the keys of an (entry, group of query heads) in a step of single tokens: as
@@ -593,12 +646,12 @@ extern "C" int dli_attention_scored_single(const void* q, int64_t q_stride, cons
                                            int table_stride, int entries, int q_heads, int kv_heads, int head_dim,
                                            int value_dim, int page_size, float scale, int window, int chunk, int sink,
                                            const float* r1, const float* r2, const float* gate, int64_t gate_stride,
-                                           int keep_first, int v_heads, float* out32, float* parts, int splits,
-                                           int is_bf16, hipStream_t stream) {
+                                           int keep_first, int v_heads, float* out32, const float* sinks, float* parts,
+                                           int splits, int is_bf16, hipStream_t stream) {
   if (splits < 1 || splits > 64 || (splits > 1 && parts == nullptr)) return DLI_ERR_ARGUMENT;
   return attention_scored(q, q_stride, k_pages, v_pages, out, out_stride, nullptr, kv_len, block_tables, table_stride,
                           nullptr, nullptr, entries, q_heads, kv_heads, head_dim, value_dim, page_size, scale, window,
-                          chunk, sink, r1, r2, gate, gate_stride, keep_first, v_heads, out32, parts, splits, is_bf16, stream);
+                          chunk, sink, r1, r2, gate, gate_stride, keep_first, v_heads, out32, sinks, parts, splits, is_bf16, stream);
 }
 
 extern "C" int dli_attention_generic(const void* q, int64_t q_stride, const void* k_pages,
@@ -607,9 +660,9 @@ extern "C" int dli_attention_generic(const void* q, int64_t q_stride, const void
                                      int table_stride, const int* tile_entry, const int* tile_q0,
                                      int tiles, int q_heads, int kv_heads, int head_dim, int page_size,
                                      float scale, int window, int is_bf16, hipStream_t stream) {
-  if (head_dim % 16 != 0 || tile_entry == nullptr) return tiles <= 0 ? DLI_OK : DLI_ERR_ARGUMENT;
+  if (head_dim % 16 != 0 || tile_entry == nullptr || v_pages == nullptr) return tiles <= 0 ? DLI_OK : DLI_ERR_ARGUMENT;
   return attention_scored(q, q_stride, k_pages, v_pages, out, out_stride, q_start, kv_len,
                           block_tables, table_stride, tile_entry, tile_q0, tiles, q_heads,
                           kv_heads, head_dim, head_dim, page_size, scale, window, 0, 0, nullptr,
-                          nullptr, nullptr, 0, 0, kv_heads, nullptr, nullptr, 1, is_bf16, stream);
+                          nullptr, nullptr, 0, 0, kv_heads, nullptr, nullptr, nullptr, 1, is_bf16, stream);
 }

@@ -34,6 +34,7 @@ struct ScoredArgs {
   const float* gate; int64_t gate_stride;
   int keep_first, v_heads;
   float* out32;
+  const float* sinks;
 };
 
 template <int DT, int VT>   // head_dim = 16 DT, value_dim = 16 VT
@@ -74,8 +75,10 @@ __global__ __launch_bounds__(256) void attention_scored_mfma_kernel(ScoredArgs a
   float4s acc[VT];
 #pragma unroll
   for (int t = 0; t < VT; ++t) acc[t] = float4s{0.f, 0.f, 0.f, 0.f};
-  float m_run = a.sink ? 0.f : -INFINITY;              // the sink: a key of score 0 without a value,
-  float l_run = a.sink && grp == 0 ? 1.f : 0.f;        // counted once a query (sums are per lane until the end)
+  // the sink: a key of score 0 (or of the head's own score) without a value, counted once a query (sums are
+  // per lane until the end)
+  float m_run = a.sinks != nullptr ? a.sinks[head] * LOG2E : a.sink ? 0.f : -INFINITY;
+  float l_run = (a.sinks != nullptr || a.sink) && grp == 0 ? 1.f : 0.f;
 
   for (int j0 = keep > j_lo ? j_lo : j_begin; j0 <= p_hi; j0 += 64) {
     if (j0 >= keep && j0 < j_begin) j0 = j_begin;               // between the kept keys and the window: nothing
@@ -192,7 +195,7 @@ extern "C" int dli_attention_scored_mfma(const void* q, int64_t q_stride, const 
                                          const int* tile_q0, int tiles, int q_heads, int kv_heads, int head_dim,
                                          int value_dim, int page_size, float scale, int window, int chunk, int sink,
                                          const float* r1, const float* r2, const float* gate, int64_t gate_stride,
-                                         int keep_first, int v_heads, float* out32, hipStream_t stream) {
+                                         int keep_first, int v_heads, float* out32, const float* sinks, hipStream_t stream) {
   if (tiles <= 0) return DLI_OK;
   if (v_heads <= 0) v_heads = kv_heads;
   if (keep_first < 0 || kv_heads <= 0 || kv_heads % v_heads != 0) return DLI_ERR_ARGUMENT;
@@ -207,7 +210,7 @@ extern "C" int dli_attention_scored_mfma(const void* q, int64_t q_stride, const 
   a.block_tables = block_tables; a.table_stride = table_stride; a.tile_entry = tile_entry; a.tile_q0 = tile_q0;
   a.q_heads = q_heads; a.kv_heads = kv_heads; a.page_size = page_size; a.scale = scale; a.window = window;
   a.chunk = chunk; a.sink = sink; a.r1 = r1; a.r2 = r2; a.gate = gate; a.gate_stride = gate_stride;
-  a.keep_first = keep_first; a.v_heads = v_heads; a.out32 = out32;
+  a.keep_first = keep_first; a.v_heads = v_heads; a.out32 = out32; a.sinks = sinks;
   switch (head_dim / 16) {
     case 1: return launch_scored_mfma<1>(a, tiles, value_dim, stream);
     case 2: return launch_scored_mfma<2>(a, tiles, value_dim, stream);

@@ -27,6 +27,19 @@ template <typename T> __device__ __forceinline__ float round_to(float x) { retur
 // use it wait for memory.
 template <typename T> __device__ __forceinline__ float silu(float g) { return g / (1.f + expf(-g)); }
 
+// The gated activation of a feed-forward's two halves: g sigmoid(alpha g) (u + shift) with g = min(gate, limit),
+// u = clamp(up, -limit, limit). An infinite limit, alpha 1 and shift 0: silu(gate) * up.
+__device__ __forceinline__ float clamped_glu(float gate, float up, float limit, float alpha, float up_shift) {
+  const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+  return g / (1.f + expf(-alpha * g)) * (u + up_shift);
+}
+
+// The activation inside a few-row product: `clamped` 0 is cast(silu(gate)) * up, else the form above.
+struct GluForm { int clamped; float limit, alpha, up_shift; };
+__device__ __forceinline__ bf16_t glu_bf16(float gate, float up, const GluForm& f) {
+  if (f.clamped) return (bf16_t)clamped_glu(gate, up, f.limit, f.alpha, f.up_shift);
+  return (bf16_t)((float)(bf16_t)silu<bf16_t>(gate) * up);
+}
 
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll

@@ -110,7 +110,7 @@ __global__ __launch_bounds__(64) void conv_prepare_kernel(PrepArgs p) {
 #define GD_MAX_TAPS 16
 __global__ void conv_keep_kernel(const float* __restrict__ proj, int64_t stride, float* kept_base, int64_t state_stride,
                                  const int* __restrict__ q_start, const int* __restrict__ positions,
-                                 const int* __restrict__ state_slots, int channels, int taps) {
+                                 const int* __restrict__ state_slots, int channels, int taps, const float* __restrict__ in_bias) {
   const int e = blockIdx.x;
   const int first = q_start[e], end = q_start[e + 1];
   if (end <= first) return;
@@ -122,7 +122,7 @@ __global__ void conv_keep_kernel(const float* __restrict__ proj, int64_t stride,
   for (int i = 0; i < taps - 1; ++i) {            // new kept row i holds the input `taps-1-i` places before `end`
     const int src = end - (taps - 1 - i);
     float x;
-    if (src >= first) x = proj[(int64_t)src * stride + c];
+    if (src >= first) x = proj[(int64_t)src * stride + c] + (in_bias != nullptr ? in_bias[c] : 0.f);
     else if (pos0 - (first - src) < 0) x = 0.f;
     else x = kept[(int64_t)(taps - 1 - (first - src)) * channels + c];
     fresh[i] = x;
@@ -136,7 +136,8 @@ __global__ void causal_conv_kernel(const float* __restrict__ x, int64_t stride, 
                                    const float* __restrict__ bias, const float* kept_base, int64_t state_stride,
                                    const int* __restrict__ q_start, int entries, const int* __restrict__ positions,
                                    const int* __restrict__ state_slots, float* __restrict__ out, int64_t out_stride,
-                                   T* __restrict__ rounded, int64_t rounded_stride, int channels, int taps, int act) {
+                                   T* __restrict__ rounded, int64_t rounded_stride, int channels, int taps, int act,
+                                   const float* __restrict__ in_bias) {
   const int row = blockIdx.x;
   const int c = blockIdx.y * blockDim.x + threadIdx.x;
   if (c >= channels) return;
@@ -144,11 +145,12 @@ __global__ void causal_conv_kernel(const float* __restrict__ x, int64_t stride, 
   const int first = q_start[e], pos = positions[row];
   const float* kept = kept_base + (int64_t)state_slots[e] * state_stride;
   float acc = bias != nullptr ? bias[c] : 0.f;
+  const float ib = in_bias != nullptr ? in_bias[c] : 0.f;        // (part of every input that exists, not of the zeros before)
   for (int j = taps - 1; j >= 0; --j) {                          // oldest input first
     float in = 0.f;
     if (pos - j >= 0) {
       const int src = row - j;
-      in = src >= first ? x[(int64_t)src * stride + c] : kept[(int64_t)(taps - 1 - (first - src)) * channels + c];
+      in = src >= first ? x[(int64_t)src * stride + c] + ib : kept[(int64_t)(taps - 1 - (first - src)) * channels + c];
     }
     acc = fmaf(conv_w[(int64_t)c * taps + (taps - 1 - j)], in, acc);
   }
@@ -328,13 +330,13 @@ int dli_conv_prepare(const float* proj, int64_t stride, int b_off, int a_off, co
   if (taps > 1) {
     const dim3 grid(entries, (unsigned)((channels + 255) / 256));
     conv_keep_kernel<<<grid, 256, 0, stream>>>(proj, stride, state + kept_offset, state_stride, q_start, positions,
-                                               state_slots, (int)channels, taps);
+                                               state_slots, (int)channels, taps, nullptr);
   }
   return dli_launch_status();
 }
 
 // act: 0 none, 1 silu. rounded (may be nullptr): the result once more, bf16 if rounded_is_bf16 else float.
-int dli_causal_conv(const float* x, int64_t stride, const float* conv_w, const float* bias, float* state,
+int dli_causal_conv(const float* x, int64_t stride, const float* conv_w, const float* bias, const float* in_bias, float* state,
                     int64_t state_stride, int64_t kept_offset, const int* q_start, const int* positions,
                     const int* state_slots, float* out, int64_t out_stride, void* rounded, int64_t rounded_stride,
                     int rounded_is_bf16, int entries, int rows, int channels, int taps, int act, hipStream_t stream) {
@@ -348,16 +350,16 @@ int dli_causal_conv(const float* x, int64_t stride, const float* conv_w, const f
   if (rounded_is_bf16)
     causal_conv_kernel<bf16_t><<<grid, 256, 0, stream>>>(x, stride, conv_w, bias, state + kept_offset, state_stride, q_start,
                                                          entries, positions, state_slots, out, out_stride, (bf16_t*)rounded,
-                                                         rounded_stride, channels, taps, act);
+                                                         rounded_stride, channels, taps, act, in_bias);
   else
     causal_conv_kernel<float><<<grid, 256, 0, stream>>>(x, stride, conv_w, bias, state + kept_offset, state_stride, q_start,
                                                         entries, positions, state_slots, out, out_stride, (float*)rounded,
-                                                        rounded_stride, channels, taps, act);
+                                                        rounded_stride, channels, taps, act, in_bias);
   if (dli_launch_status() != DLI_OK) return DLI_ERR_LAUNCH;
   if (taps > 1) {
     const dim3 keep(entries, (channels + 255) / 256);
     conv_keep_kernel<<<keep, 256, 0, stream>>>(x, stride, state + kept_offset, state_stride, q_start, positions,
-                                               state_slots, channels, taps);
+                                               state_slots, channels, taps, in_bias);
   }
   return dli_launch_status();
 }

@@ -49,11 +49,6 @@ __global__ void poly_norm_kernel_f32in(const float* __restrict__ z, int64_t z_st
   }
 }
 
-__device__ __forceinline__ float clamped_glu(float gate, float up, float limit, float alpha, float up_shift) {
-  const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
-  return g / (1.f + expf(-alpha * g)) * (u + up_shift);
-}
-
 template <typename T>
 __global__ void clamped_glu_kernel(const T* __restrict__ gate_up, int64_t stride, T* __restrict__ out, int ff, float limit,
                                    float alpha, float up_shift) {

@@ -28,7 +28,7 @@
 //                 (RMSNorm: src/dli/model/llama.py:40-44)
 //   EPI_STORE     y (+ bias) stored as bf16
 //   EPI_SWIGLU    half of the quads are gate rows n, half up rows n + up_offset:
-//                 stores cast(silu(gate)) * up (src/dli/model/llama.py:190)
+//                 stores cast(silu(gate)) * up (src/dli/model/llama.py:190), or the clamped form (GluForm)
 //   EPI_RESIDUAL  stream[m][n] = cast(stream[m][n] + cast(y + bias)) in place, and this tile's part
 //                 of sum_n stream[m][n]^2 for the norm that follows
 //   EPI_F32       y stored as float32 (logits)
@@ -56,7 +56,7 @@ __global__ __launch_bounds__(KS * 64) void skinny4_kernel(
     const float* __restrict__ norm_w, float eps, const bf16_t* __restrict__ w,
     const bf16_t* __restrict__ bias, void* __restrict__ out, int64_t ldo,
     bf16_t* __restrict__ stream, int64_t lds_, float* __restrict__ ssq_out, int M, int N, int K,
-    int up_offset) {
+    int up_offset, GluForm glu) {
   constexpr int PAIRS = FQ * MG;                        // (quad, row group) accumulators per lane
   constexpr int OQ = EPI == EPI_SWIGLU ? FQ / 2 : FQ;   // quads of output features per tile
   __shared__ float4v red[KS][PAIRS][16];
@@ -376,8 +376,7 @@ __global__ __launch_bounds__(KS * 64) void skinny4_kernel(
           res.e[i] = (bf16_t)y[0][i];
         } else if (EPI == EPI_SWIGLU) {
           const float gt = (float)(bf16_t)y[0][i], up = (float)(bf16_t)y[1][i];
-          const float sg = (float)(bf16_t)silu<bf16_t>(gt);
-          res.e[i] = (bf16_t)(sg * up);
+          res.e[i] = glu_bf16(gt, up, glu);
         } else {  // EPI_RESIDUAL: the sum in 32-bit, rounded to the stream's type
           res.e[i] = (bf16_t)((float)old.e[i] + (float)(bf16_t)y[0][i]);
           if (nb + i < N) sq += (float)res.e[i] * (float)res.e[i];
@@ -408,9 +407,9 @@ __global__ __launch_bounds__(KS * 64) void skinny4_kernel(
 #define S4_PARAMS                                                                                 \
   const void *x, int64_t ldx, const float *ssq_in, int ssq_parts, const float *norm_w, float eps,   \
       const void *w, const void *bias, void *out, int64_t ldo, void *stream_buf, int64_t lds_,      \
-      float *ssq_out, int M, int N, int K, int up_offset, hipStream_t stream
+      float *ssq_out, int M, int N, int K, int up_offset, GluForm glu, hipStream_t stream
 #define S4_ARGS \
-  x, ldx, ssq_in, ssq_parts, norm_w, eps, w, bias, out, ldo, stream_buf, lds_, ssq_out, M, N, K, up_offset, stream
+  x, ldx, ssq_in, ssq_parts, norm_w, eps, w, bias, out, ldo, stream_buf, lds_, ssq_out, M, N, K, up_offset, glu, stream
 
 template <int KS, int FQ, int MG, int EPI, bool NORM>
 static void launch4(S4_PARAMS) {
@@ -430,7 +429,7 @@ static void launch4(S4_PARAMS) {
 #define S4_LAUNCH(XL_, DEPTH_)                                                                              \
   skinny4_kernel<KS, FQ, MG, EPI, NORM, XL_, DEPTH_><<<tiles, KS * 64, XL_ ? (size_t)x_lds : 0, stream>>>( \
       (const bf16_t*)x, ldx, ssq_in, ssq_parts, norm_w, eps, (const bf16_t*)w, (const bf16_t*)bias, out,    \
-      ldo, (bf16_t*)stream_buf, lds_, ssq_out, M, N, K, up_offset)
+      ldo, (bf16_t*)stream_buf, lds_, ssq_out, M, N, K, up_offset, glu)
   if (staged && by_four) S4_LAUNCH(true, 4);
   else if (staged) S4_LAUNCH(true, 2);
   else if (by_four) S4_LAUNCH(false, 4);
@@ -471,8 +470,9 @@ extern "C" int dli_skinny4_gemm(const void* x, int64_t ldx, const float* ssq_in,
                                 const float* norm_w, float eps, const void* w, const void* bias,
                                 void* out, int64_t ldo, void* stream_buf, int64_t lds_,
                                 float* ssq_out, int M, int N, int K, int up_offset, int epilogue,
-                                int shape, hipStream_t stream) {
+                                int shape, int clamped, float limit, float alpha, float up_shift, hipStream_t stream) {
   if (M <= 0 || N <= 0) return DLI_OK;
+  const GluForm glu{clamped, limit, alpha, up_shift};
   if (M > 16 || K <= 0 || K % 8 != 0 || ldx % 8 != 0 || ldx < K || (int64_t)M * ldx * 2 >= (int64_t)1 << 31 ||
       shape < 0 || shape > 2 || epilogue < 0 || epilogue > 3 ||
       (norm_w != nullptr && (ssq_in == nullptr || ssq_parts <= 0)) ||

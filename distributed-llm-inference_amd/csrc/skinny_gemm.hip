@@ -22,7 +22,7 @@
 //            (RMSNorm: src/dli/model/llama.py:40-44); otherwise xhat = x.
 //   EPI_STORE     y (+ bias) stored as bf16
 //   EPI_SWIGLU    two products per workgroup, rows n (gate) and n + up_offset (up) of w:
-//                 stores cast(silu(gate)) * up (src/dli/model/llama.py:190)
+//                 stores cast(silu(gate)) * up (src/dli/model/llama.py:190), or the clamped form (GluForm)
 //   EPI_RESIDUAL  stream[m][n] = cast(stream[m][n] + cast(y + bias)) in place (the residual sum, in
 //                 32-bit), and this tile's part of sum_n stream[m][n]^2 for the norm that follows
 //   EPI_F32       y stored as float32 (logits)
@@ -122,7 +122,7 @@ __global__ __launch_bounds__(KS * NS * 64) void skinny_gemm_kernel(
     const float* __restrict__ norm_w, float eps, const bf16_t* __restrict__ w,
     const bf16_t* __restrict__ bias, void* __restrict__ out, int64_t ldo,
     bf16_t* __restrict__ stream, int64_t lds_, float* __restrict__ ssq_out, int M, int N, int K,
-    int up_offset, QkvRope qr, MergedIn mi) {
+    int up_offset, QkvRope qr, MergedIn mi, GluForm glu) {
   static_assert(EPI != EPI_QKV || (TILED && MT == 1), "the q/k/v epilogue reads tiled weights, at most 16 rows");
   static_assert(!MERGED || (TILED && MT == 1 && NS == 1 && !NORM), "merged activations: tiled weights, one row tile");
   // MERGED: each wave's run of k for up to MERGE_ROWS rows
@@ -467,8 +467,7 @@ __global__ __launch_bounds__(KS * NS * 64) void skinny_gemm_kernel(
             reinterpret_cast<float*>(out)[(int64_t)m * ldo + n] = y[0][i];
           } else if (EPI == EPI_SWIGLU) {
             const float g = (float)(bf16_t)y[0][i], u = (float)(bf16_t)y[NA - 1][i];
-            const float sg = (float)(bf16_t)silu<bf16_t>(g);
-            reinterpret_cast<bf16_t*>(out)[(int64_t)m * ldo + n] = (bf16_t)(sg * u);
+            reinterpret_cast<bf16_t*>(out)[(int64_t)m * ldo + n] = glu_bf16(g, u, glu);
           } else {  // EPI_RESIDUAL
             bf16_t* sp = stream + (int64_t)m * lds_ + n;
             const bf16_t summed = (bf16_t)((float)old_s[EPI == EPI_RESIDUAL ? j : 0][EPI == EPI_RESIDUAL ? t : 0][i] + (float)(bf16_t)y[0][i]);
@@ -506,9 +505,9 @@ __global__ void embedding_ssq_kernel(const bf16_t* __restrict__ table, const int
 #define SK_PARAMS                                                                                 \
   const void *x, int64_t ldx, const float *ssq_in, int ssq_parts, const float *norm_w, float eps,   \
       const void *w, const void *bias, void *out, int64_t ldo, void *stream_buf, int64_t lds_,      \
-      float *ssq_out, int M, int N, int K, int up_offset, QkvRope qr, hipStream_t stream
+      float *ssq_out, int M, int N, int K, int up_offset, QkvRope qr, GluForm glu, hipStream_t stream
 #define SK_ARGS \
-  x, ldx, ssq_in, ssq_parts, norm_w, eps, w, bias, out, ldo, stream_buf, lds_, ssq_out, M, N, K, up_offset, qr, stream
+  x, ldx, ssq_in, ssq_parts, norm_w, eps, w, bias, out, ldo, stream_buf, lds_, ssq_out, M, N, K, up_offset, qr, glu, stream
 
 template <int KS, int NS, int NT, int MT, int EPI, bool NORM, bool TILED>
 static void launch_skinny(SK_PARAMS) {
@@ -516,7 +515,7 @@ static void launch_skinny(SK_PARAMS) {
   const int groups = (tiles + NS * NT - 1) / (NS * NT);
   skinny_gemm_kernel<KS, NS, NT, MT, EPI, NORM, TILED><<<groups, KS * NS * 64, 0, stream>>>(
       (const bf16_t*)x, ldx, ssq_in, ssq_parts, norm_w, eps, (const bf16_t*)w, (const bf16_t*)bias,
-      out, ldo, (bf16_t*)stream_buf, lds_, ssq_out, M, N, K, up_offset, qr, MergedIn{});
+      out, ldo, (bf16_t*)stream_buf, lds_, ssq_out, M, N, K, up_offset, qr, MergedIn{}, glu);
 }
 
 // shapes of the workgroup: 0: 4 k-waves x 1 tile (few tiles, short k); 1: 8 k-waves x 1 tile (few
@@ -552,8 +551,10 @@ extern "C" int dli_skinny_gemm(const void* x, int64_t ldx, const float* ssq_in, 
                                const float* norm_w, float eps, const void* w, const void* bias,
                                void* out, int64_t ldo, void* stream_buf, int64_t lds_,
                                float* ssq_out, int M, int N, int K, int up_offset, int epilogue,
-                               int shape, int tiled, hipStream_t stream) {
+                               int shape, int tiled, int clamped, float limit, float alpha, float up_shift,
+                               hipStream_t stream) {
   const QkvRope qr{};
+  const GluForm glu{clamped, limit, alpha, up_shift};
   if (M <= 0 || N <= 0) return DLI_OK;
   if (tiled && (M > 16 || K % 128 != 0 || N % 16 != 0 || up_offset % 16 != 0)) return DLI_ERR_ARGUMENT;
   if (M > 64 || K <= 0 || K % 32 != 0 || ldx % 8 != 0 || shape < 0 || shape > 4 || epilogue < 0 ||
@@ -598,6 +599,7 @@ extern "C" int dli_skinny_gemm_qkv_rope(const void* x, int64_t ldx, const float*
   float* ssq_out = nullptr;
   const int64_t lds_ = 0;
   const void* w = w_tiled;
+  const GluForm glu{};
   if (norm_w != nullptr) dispatch_shape<1, EPI_QKV, true, true>(shape, SK_ARGS);
   else dispatch_shape<1, EPI_QKV, false, true>(shape, SK_ARGS);
   return dli_launch_status();
@@ -623,7 +625,7 @@ extern "C" int dli_skinny_gemm_merged(const float* part_o, const float* part_ml,
 #define MERGED_LAUNCH(KS)                                                                          \
   skinny_gemm_kernel<KS, 1, 1, 1, EPI_RESIDUAL, false, true, true><<<groups, KS * 64, 0, stream>>>( \
       nullptr, 0, nullptr, 0, nullptr, 0.f, (const bf16_t*)w_tiled, (const bf16_t*)bias, nullptr, 0, \
-      (bf16_t*)stream_buf, lds_, ssq_out, M, N, K, 0, QkvRope{}, mi)
+      (bf16_t*)stream_buf, lds_, ssq_out, M, N, K, 0, QkvRope{}, mi, GluForm{})
   if (shape == 0) MERGED_LAUNCH(4);
   else MERGED_LAUNCH(8);
 #undef MERGED_LAUNCH

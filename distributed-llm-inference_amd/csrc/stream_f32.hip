@@ -3,10 +3,12 @@
 // write (float on the 32-bit path, bf16 when serving). Statistics, sums, angles and activations
 // are 32-bit.
 //
-//   embed_sinusoid     x = table[id] + pe(position), pe[2i] = sin(p f_i), pe[2i+1] = cos(p f_i)
+//   embed_sinusoid     x = scale table[id] + pe(position), pe[2i] = sin(p f_i), pe[2i+1] = cos(p f_i)
 //   cast_from_f32      the stream rounded to T, as the operand of a product
 //   norm_into_stream   x += w * y / sqrt(mean(y^2) + eps)   (a norm on a sublayer's output); like the embedding
 //                      it can leave the new stream once more in bf16, for the product that reads it next
+//   norm_stream_norm   the same sum, and of the new stream its norm by another weight, out(T) (norms before and after
+//                      every sublayer: one sublayer's second norm, the residual sum and the next one's first norm)
 //   rms_norm_from_f32  out(T) = w * x / sqrt(mean(x^2) + eps)
 //   post_norm_stream   x <- w * s / sqrt(mean(s^2) + eps) with s = alpha x + r y, r = sigmoid(g + b) element by element
 //                      or 1 (a norm after the residual sum, the summand under a gate of its own)
@@ -29,16 +31,17 @@
 //   rms_norm_pair      two norms of the same row (two weights) from one pass over its statistics
 //   add_pair_into_stream  x += a + b
 #include "common.h"
+#include "rotary.h"
 
 template <typename T>
 __global__ void embed_sinusoid_kernel(const T* __restrict__ table, const int* __restrict__ ids,
                                       const int* __restrict__ positions, const float* __restrict__ inv_freq,
-                                      float* __restrict__ out, bf16_t* __restrict__ rounded, int width) {
+                                      float* __restrict__ out, bf16_t* __restrict__ rounded, int width, float scale) {
   const int64_t row = blockIdx.x;
   const T* src = table + (int64_t)ids[row] * width;
   const float p = (float)positions[row];
   for (int i = threadIdx.x; i < width; i += blockDim.x) {
-    float sum = to_f32(src[i]);
+    float sum = to_f32(src[i]) * scale;
     if (inv_freq != nullptr) {   // (nullptr: the token's row alone)
       const float angle = p * inv_freq[i >> 1];
       sum += (i & 1) ? cosf(angle) : sinf(angle);
@@ -73,6 +76,94 @@ __global__ void norm_into_stream_kernel(const T* __restrict__ y, int64_t y_strid
     xr[i] = sum;
     if (rounded != nullptr) rounded[row * width + i] = from_f32<R>(sum);
   }
+}
+
+// x += w1 * y / sqrt(mean(y^2) + eps1), then out = w2 * x / sqrt(mean(x^2) + eps2). A workgroup a row, which stays in
+// registers in between: a thread holds PER runs of four neighbours (width a multiple of four, at most PER * 4 * threads).
+template <typename T, int PER>
+__global__ void norm_stream_norm_kernel(const float* __restrict__ y, int64_t y_stride, const float* __restrict__ w1,
+                                        float eps1, float* __restrict__ x, const float* __restrict__ w2, float eps2,
+                                        T* __restrict__ out, int width) {
+  typedef float f4 __attribute__((ext_vector_type(4)));
+  typedef T t4 __attribute__((ext_vector_type(4)));
+  __shared__ float scratch[16];
+  const int64_t row = blockIdx.x;
+  f4 yv[PER], xv[PER];
+  float ss = 0.f;
+#pragma unroll
+  for (int p = 0; p < PER; ++p) {
+    const int i = 4 * (threadIdx.x + p * blockDim.x);
+    yv[p] = xv[p] = f4{0.f, 0.f, 0.f, 0.f};
+    if (i < width) {
+      yv[p] = *reinterpret_cast<const f4*>(y + row * y_stride + i);
+      xv[p] = *reinterpret_cast<const f4*>(x + row * width + i);
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss += yv[p][e] * yv[p][e];
+  }
+  const float r1 = 1.f / sqrtf(block_sum(ss, scratch) / (float)width + eps1);
+  ss = 0.f;
+#pragma unroll
+  for (int p = 0; p < PER; ++p) {
+    const int i = 4 * (threadIdx.x + p * blockDim.x);
+    if (i < width) {
+      const f4 w = *reinterpret_cast<const f4*>(w1 + i);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        xv[p][e] += w[e] * (yv[p][e] * r1);
+        ss += xv[p][e] * xv[p][e];
+      }
+      *reinterpret_cast<f4*>(x + row * width + i) = xv[p];
+    }
+  }
+  const float r2 = 1.f / sqrtf(block_sum(ss, scratch) / (float)width + eps2);
+#pragma unroll
+  for (int p = 0; p < PER; ++p) {
+    const int i = 4 * (threadIdx.x + p * blockDim.x);
+    if (i < width) {
+      const f4 w = *reinterpret_cast<const f4*>(w2 + i);
+      t4 o;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) o[e] = from_f32<T>(w[e] * (xv[p][e] * r2));
+      *reinterpret_cast<t4*>(out + row * width + i) = o;
+    }
+  }
+}
+
+// The same for any width: each thread reads back only what it wrote itself.
+template <typename T>
+__global__ void norm_stream_norm_any_kernel(const float* __restrict__ y, int64_t y_stride, const float* __restrict__ w1,
+                                            float eps1, float* __restrict__ x, const float* __restrict__ w2, float eps2,
+                                            T* __restrict__ out, int width) {
+  __shared__ float scratch[16];
+  const int64_t row = blockIdx.x;
+  const float* yr = y + row * y_stride;
+  float* xr = x + row * width;
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < width; i += blockDim.x) ss += yr[i] * yr[i];
+  const float r1 = 1.f / sqrtf(block_sum(ss, scratch) / (float)width + eps1);
+  ss = 0.f;
+  for (int i = threadIdx.x; i < width; i += blockDim.x) {
+    const float s = xr[i] + w1[i] * (yr[i] * r1);
+    xr[i] = s;
+    ss += s * s;
+  }
+  const float r2 = 1.f / sqrtf(block_sum(ss, scratch) / (float)width + eps2);
+  for (int i = threadIdx.x; i < width; i += blockDim.x) out[row * width + i] = from_f32<T>(w2[i] * (xr[i] * r2));
+}
+
+template <typename T>
+static void launch_norm_stream_norm(const float* y, int64_t y_stride, const float* w1, float eps1, float* x, const float* w2,
+                                    float eps2, T* out, int rows, int width, hipStream_t stream) {
+  const bool runs = width % 4 == 0 && y_stride % 4 == 0 && width <= 16384 &&
+                    (((uintptr_t)y | (uintptr_t)w1 | (uintptr_t)x | (uintptr_t)w2) % 16) == 0 && (uintptr_t)out % 16 == 0;
+#define NSN_ARGS y, y_stride, w1, eps1, x, w2, eps2, out, width
+  if (!runs) norm_stream_norm_any_kernel<T><<<rows, width >= 2048 ? 512 : 256, 0, stream>>>(NSN_ARGS);
+  else if (width <= 1024) norm_stream_norm_kernel<T, 1><<<rows, 256, 0, stream>>>(NSN_ARGS);
+  else if (width <= 2048) norm_stream_norm_kernel<T, 1><<<rows, 512, 0, stream>>>(NSN_ARGS);
+  else if (width <= 4096) norm_stream_norm_kernel<T, 2><<<rows, 512, 0, stream>>>(NSN_ARGS);
+  else norm_stream_norm_kernel<T, 8><<<rows, 512, 0, stream>>>(NSN_ARGS);
+#undef NSN_ARGS
 }
 
 template <typename T>
@@ -241,34 +332,26 @@ __global__ void qk_unit_cache_kernel(const float* __restrict__ proj, int64_t str
   }
 }
 
-// cos and sin of position * freq with the product's rounding error taken back: the product's low
-// half (one fused multiply-add) turns the functions by their own derivatives.
-__device__ __forceinline__ void rotary_cos_sin(float position, float freq, float* c, float* s) {
-  const float hi = position * freq;
-  const float lo = fmaf(position, freq, -hi);
-  float sh, ch;
-  sincosf(hi, &sh, &ch);
-  *c = fmaf(-lo, sh, ch);
-  *s = fmaf(lo, ch, sh);
-}
-
 // proj [tokens][stride] float32 holds q (q_heads x dim), k (kv_heads x dim) and v (kv_heads x vdim) at
 // the given column offsets. The first rot_dims components of every q and k head are rotated by
 // position * inv_freq[i]: pair i is (2i, 2i+1) where `interleaved`, else (i, i + rot_dims/2); the
 // other components pass. q goes out in T; the rotated k and v go to the token's cache slot
 // (negative: not cached). A thread an element: it reads its partner from proj. `bias` (may be nullptr)
 // holds a value for every column of proj and is added before anything else. The pages may hold fewer
-// value heads than key heads (v_heads), and none at all where the mixer reads another's (kv_heads 0).
+// value heads than key heads (v_heads; 0: the values are the keys), and none at all where the mixer reads
+// another's (kv_heads 0). q_coef != 0: q is also multiplied by 1 + q_coef ln(floor((p + 1) / q_every) + 1).
 template <typename T>
 __global__ void rotary_cache_kernel(const float* __restrict__ proj, int64_t stride, int q_off, int k_off, int v_off,
                                     const float* __restrict__ bias,
                                     const int* __restrict__ positions, const float* __restrict__ inv_freq, int rot_dims,
                                     int interleaved, T* __restrict__ q_out, const int* __restrict__ slots,
                                     T* __restrict__ k_pages, T* __restrict__ v_pages, int q_heads, int kv_heads, int v_heads,
-                                    int dim, int vdim, int page_size) {
+                                    int dim, int vdim, int page_size, float q_coef, double q_every) {
   const int64_t row = blockIdx.x;
   const float* pr = proj + row * stride;
   const float p = (float)positions[row];
+  const float q_temp =
+      q_coef != 0.f ? 1.f + q_coef * logf((float)(floor((double)(positions[row] + 1) / q_every) + 1.0)) : 1.f;
   const int slot = slots != nullptr ? slots[row] : -1;
   const int64_t page = slot >= 0 ? slot / page_size : 0;
   const int off = slot >= 0 ? slot % page_size : 0;
@@ -290,7 +373,7 @@ __global__ void rotary_cache_kernel(const float* __restrict__ proj, int64_t stri
       const float other = src[partner] + (bs != nullptr ? bs[partner] : 0.f);
       y = first ? y * cs - other * sn : y * cs + other * sn;
     }
-    if (is_q) q_out[(row * q_heads + h) * dim + c] = from_f32<T>(y);
+    if (is_q) q_out[(row * q_heads + h) * dim + c] = from_f32<T>(y * q_temp);
     else if (slot >= 0) k_pages[((page * kv_heads + (h - q_heads)) * page_size + off) * dim + c] = from_f32<T>(y);
   }
   if (slot >= 0)
@@ -437,16 +520,16 @@ __global__ void add_pair_into_stream_kernel(float* __restrict__ x, const float* 
 extern "C" {
 
 int dli_embed_sinusoid(const void* table, const int* ids, const int* positions, const float* inv_freq, float* out,
-                       void* rounded_bf16, int rows, int width, int is_bf16, hipStream_t stream) {
+                       void* rounded_bf16, int rows, int width, float scale, int is_bf16, hipStream_t stream) {
   if (rows <= 0) return DLI_OK;
   if (width <= 0) return DLI_ERR_ARGUMENT;
   const int threads = width >= 1024 ? 256 : 128;
   if (is_bf16)
     embed_sinusoid_kernel<bf16_t><<<rows, threads, 0, stream>>>((const bf16_t*)table, ids, positions, inv_freq, out,
-                                                                (bf16_t*)rounded_bf16, width);
+                                                                (bf16_t*)rounded_bf16, width, scale);
   else
     embed_sinusoid_kernel<float><<<rows, threads, 0, stream>>>((const float*)table, ids, positions, inv_freq, out,
-                                                               (bf16_t*)rounded_bf16, width);
+                                                               (bf16_t*)rounded_bf16, width, scale);
   return dli_launch_status();
 }
 
@@ -470,6 +553,15 @@ int dli_norm_into_stream(const void* y, int64_t y_stride, const float* weight, f
   else
     norm_into_stream_kernel<float, bf16_t><<<rows, threads, 0, stream>>>((const float*)y, y_stride, weight, x,
                                                                          (bf16_t*)rounded_bf16, width, eps);
+  return dli_launch_status();
+}
+
+int dli_norm_stream_norm(const float* y, int64_t y_stride, const float* w1, float eps1, float* x, const float* w2, float eps2,
+                         void* out, int rows, int width, int is_bf16, hipStream_t stream) {
+  if (rows <= 0) return DLI_OK;
+  if (width <= 0 || y_stride < width) return DLI_ERR_ARGUMENT;
+  if (is_bf16) launch_norm_stream_norm<bf16_t>(y, y_stride, w1, eps1, x, w2, eps2, (bf16_t*)out, rows, width, stream);
+  else launch_norm_stream_norm<float>(y, y_stride, w1, eps1, x, w2, eps2, (float*)out, rows, width, stream);
   return dli_launch_status();
 }
 
@@ -558,20 +650,22 @@ int dli_qk_unit_cache(const float* proj, int64_t stride, int q_off, int k_off, i
 int dli_rotary_cache(const float* proj, int64_t stride, int q_off, int k_off, int v_off, const float* bias,
                      const int* positions, const float* inv_freq, int rot_dims, int interleaved, void* q_out,
                      const int* slots, void* k_pages, void* v_pages, int rows, int q_heads, int kv_heads, int v_heads,
-                     int dim, int vdim, int page_size, int is_bf16, hipStream_t stream) {
+                     int dim, int vdim, int page_size, float q_coef, double q_every, int is_bf16, hipStream_t stream) {
   if (rows <= 0) return DLI_OK;
-  if (q_heads <= 0 || kv_heads < 0 || v_heads < 0 || dim <= 0 || vdim <= 0 || page_size <= 0 || rot_dims < 0 ||
+  if (q_heads <= 0 || kv_heads < 0 || v_heads < 0 || dim <= 0 || vdim <= 0 || page_size <= 0 || rot_dims < 0 || !(q_every > 0.0) ||
       rot_dims > dim || rot_dims % 2 || (rot_dims > 0 && inv_freq == nullptr) ||
       (kv_heads > 0 && (k_pages == nullptr || slots == nullptr)) || (v_heads > 0 && (v_pages == nullptr || slots == nullptr)))
     return DLI_ERR_ARGUMENT;
   if (is_bf16)
     rotary_cache_kernel<bf16_t><<<rows, 256, 0, stream>>>(proj, stride, q_off, k_off, v_off, bias, positions, inv_freq,
                                                           rot_dims, interleaved, (bf16_t*)q_out, slots, (bf16_t*)k_pages,
-                                                          (bf16_t*)v_pages, q_heads, kv_heads, v_heads, dim, vdim, page_size);
+                                                          (bf16_t*)v_pages, q_heads, kv_heads, v_heads, dim, vdim, page_size, q_coef,
+                                                          q_every);
   else
     rotary_cache_kernel<float><<<rows, 256, 0, stream>>>(proj, stride, q_off, k_off, v_off, bias, positions, inv_freq,
                                                          rot_dims, interleaved, (float*)q_out, slots, (float*)k_pages,
-                                                         (float*)v_pages, q_heads, kv_heads, v_heads, dim, vdim, page_size);
+                                                         (float*)v_pages, q_heads, kv_heads, v_heads, dim, vdim, page_size, q_coef,
+                                                          q_every);
   return dli_launch_status();
 }
 

@@ -36,7 +36,8 @@ _SIGNATURES = {
     "dli_copy_pages": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_i64, _c_i64, _c_int, _c_ptr],
     "dli_fill": [_c_ptr, _c_float, _c_i64, _c_int, _c_ptr],
     "dli_skinny4_gemm": [_c_ptr, _c_i64, _c_ptr, _c_int, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr,
-                         _c_i64, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
+                         _c_i64, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
+                         _c_float, _c_float, _c_ptr],
     "dli_skinny4_tile_features": [_c_int, _c_int],
     "dli_rope_kv_write": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int,
                           _c_int, _c_int, _c_int, _c_int, _c_ptr],
@@ -52,7 +53,8 @@ _SIGNATURES = {
                            _c_int, _c_int, _c_ptr],
     "dli_skinny_gemm_max_rows": [],
     "dli_skinny_gemm": [_c_ptr, _c_i64, _c_ptr, _c_int, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr,
-                        _c_i64, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
+                        _c_i64, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
+                        _c_float, _c_float, _c_float, _c_ptr],
     "dli_skinny_gemm_qkv_rope": [_c_ptr, _c_i64, _c_ptr, _c_int, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_i64,
                                  _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
                                  _c_int, _c_ptr],
@@ -99,35 +101,40 @@ _SIGNATURES = {
                               _c_int, _c_int, _c_ptr],
     "dli_attention_scored": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr,
                              _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _c_ptr,
-                             _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_ptr, _c_int, _c_ptr],
+                             _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr],
     "dli_attention_scored_splits": [_c_int, _c_int, _c_int],
     "dli_attention_scored_single": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int,
                                     _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_i64,
-                                    _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr],
+                                    _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr],
     "dli_attention_scored_mfma_supports": [_c_int, _c_int, _c_int],
     "dli_attention_scored_mfma": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr,
                                   _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _c_ptr,
-                                  _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_ptr, _c_ptr],
-    "dli_embed_sinusoid": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr],
+                                  _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr],
+    "dli_embed_sinusoid": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_float, _c_int, _c_ptr],
+    "dli_norm_stream_norm": [_c_ptr, _c_i64, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_int, _c_int, _c_int, _c_ptr],
     "dli_cast_from_f32": [_c_ptr, _c_ptr, _c_i64, _c_int, _c_ptr],
     "dli_norm_into_stream": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_float, _c_int, _c_ptr],
     "dli_rms_norm_from_f32": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_float, _c_int, _c_ptr],
     "dli_softcap": [_c_ptr, _c_i64, _c_float, _c_ptr],
     "dli_post_norm_stream": [_c_ptr, _c_i64, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_float,
                              _c_float, _c_int, _c_ptr],
-    "dli_causal_conv": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_i64,
+    "dli_causal_conv": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_i64,
                         _c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "dli_selective_scan_max_states": [],
     "dli_selective_scan": [_c_ptr, _c_i64, _c_ptr, _c_i64, _c_ptr, _c_i64, _c_int, _c_int, _c_ptr, _c_i64, _c_ptr, _c_ptr,
                            _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_int,
                            _c_ptr],
+    "dli_gated_unit_tile_rows": [],
+    "dli_gated_unit": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_i64, _c_ptr,
+                       _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_int,
+                       _c_int, _c_int, _c_ptr],
     "dli_bounded_gates": [_c_ptr, _c_i64, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr],
     "dli_gated_linear_scan": [_c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
                               _c_i64, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "dli_latent_norm_cache": [_c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_ptr,
-                              _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr],
-    "dli_head_products": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_int, _c_int,
-                          _c_ptr],
+                              _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr],
+    "dli_head_products": [_c_ptr, _c_i64, _c_int, _c_ptr, _c_ptr, _c_i64, _c_int, _c_ptr, _c_i64, _c_int, _c_int, _c_int,
+                          _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr],
     "dli_token_shift": [_c_ptr, _c_ptr, _c_int, _c_ptr, _c_i64, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int,
                         _c_int, _c_ptr],
     "dli_lowrank_out": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_i64,
@@ -139,7 +146,7 @@ _SIGNATURES = {
                            _c_i64, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr,
                            _c_i64, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "dli_rotary_cache": [_c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr,
-                         _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
+                         _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, ctypes.c_double, _c_int, _c_ptr],
     "dli_diff_head_norm": [_c_ptr, _c_i64, _c_float, _c_float, _c_float, _c_ptr, _c_i64, _c_ptr, _c_i64, _c_int, _c_int,
                            _c_int, _c_int, _c_ptr],
     "dli_branch_weighted_sum": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_ptr],
@@ -524,13 +531,15 @@ def skinny_gemm(x: torch.Tensor, w: torch.Tensor, *, epilogue: int, out: Optiona
                 bias: Optional[torch.Tensor] = None, norm_w: Optional[torch.Tensor] = None, eps: float = 0.0,
                 ssq_in: Optional[torch.Tensor] = None, stream: Optional[torch.Tensor] = None,
                 ssq_out: Optional[torch.Tensor] = None, shape: Optional[int] = None,
-                blocks4: Optional[int] = None, w_tiled: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+                blocks4: Optional[int] = None, w_tiled: Optional[torch.Tensor] = None,
+                clamped: Optional[tuple] = None) -> Optional[torch.Tensor]:
     """``y = xhat @ w.T`` for at most 64 rows of bfloat16 ``x``, with fused surroundings.
 
     ``norm_w``/``eps``/``ssq_in [parts, rows]``: xhat is the RMSNorm of x, the row sums of squares
     being given in parts. Epilogues: ``SKINNY_STORE`` (``out`` bfloat16 ``[rows, n]``),
     ``SKINNY_SWIGLU`` (``w`` is ``[2n, k]``: gate rows then up rows; ``out [rows, n]`` gets
-    ``silu(gate) * up``), ``SKINNY_RESIDUAL`` (``stream [rows, n]`` becomes ``stream + y`` in place;
+    ``silu(gate) * up``, or with ``clamped = (limit, alpha, up_shift)`` what :func:`clamped_glu` computes),
+    ``SKINNY_RESIDUAL`` (``stream [rows, n]`` becomes ``stream + y`` in place;
     the parts of its row sums of squares are returned as ``[parts, rows]``, in ``ssq_out`` if that
     is given with the shape :func:`skinny_gemm_plan` names), ``SKINNY_F32`` (``out`` float32).
     ``shape`` forces the 16x16-tile kernel with that workgroup shape, ``blocks4`` the 4x4-block
@@ -543,6 +552,8 @@ def skinny_gemm(x: torch.Tensor, w: torch.Tensor, *, epilogue: int, out: Optiona
     _require(w.shape[1] == k, "x and w differ in inner size")
     _require(skinny_gemm_supports(m, k, x.dtype), f"the decode product takes 1..64 rows and k % 32 == 0, not {m} x {k}")
     _require(x.stride(0) % 8 == 0 and x.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0, "operands must be 16-byte aligned")
+    _require(clamped is None or epilogue == SKINNY_SWIGLU, "a clamped activation belongs to the gated epilogue")
+    glu = (0, 0.0, 0.0, 0.0) if clamped is None else (1, *(float(c) for c in clamped))
     n = w.shape[0] // 2 if epilogue == SKINNY_SWIGLU else w.shape[0]
     up_offset = n if epilogue == SKINNY_SWIGLU else 0
     if epilogue == SKINNY_SWIGLU:
@@ -595,11 +606,11 @@ def skinny_gemm(x: torch.Tensor, w: torch.Tensor, *, epilogue: int, out: Optiona
         _check(library().dli_skinny_gemm(
             _ptr(x), x.stride(0), _ptr(ssq_in), parts, _ptr(norm_w), float(eps), _ptr(w_tiled if tiled else w),
             _ptr(bias), _ptr(out), ldo, _ptr(stream), lds, _ptr(ssq_out), m, n, k, up_offset, epilogue, a,
-            int(tiled), _stream()), "skinny_gemm")
+            int(tiled), *glu, _stream()), "skinny_gemm")
     else:
         _check(library().dli_skinny4_gemm(
             _ptr(x), x.stride(0), _ptr(ssq_in), parts, _ptr(norm_w), float(eps), _ptr(w), _ptr(bias), _ptr(out), ldo,
-            _ptr(stream), lds, _ptr(ssq_out), m, n, k, up_offset, epilogue, a, _stream()), "skinny4_gemm")
+            _ptr(stream), lds, _ptr(ssq_out), m, n, k, up_offset, epilogue, a, *glu, _stream()), "skinny4_gemm")
     return ssq_out if epilogue == SKINNY_RESIDUAL else None
 
 
@@ -1399,8 +1410,8 @@ def _rounded_copy(rounded: Optional[torch.Tensor], like: torch.Tensor) -> None:
 
 
 def embed_sinusoid(table: torch.Tensor, ids: torch.Tensor, positions: torch.Tensor, inv_freq: Optional[torch.Tensor],
-                   out: torch.Tensor, rounded: Optional[torch.Tensor] = None) -> None:
-    """``out[t] = table[ids[t]] + pe(positions[t])`` in float32, ``pe[2i] = sin(p f_i)``,
+                   out: torch.Tensor, rounded: Optional[torch.Tensor] = None, scale: float = 1.0) -> None:
+    """``out[t] = scale table[ids[t]] + pe(positions[t])`` in float32, ``pe[2i] = sin(p f_i)``,
     ``pe[2i+1] = cos(p f_i)`` with ``f = inv_freq [ceil(width/2)]`` (``None``: the token's row alone, widened
     to float32). ``rounded``: the same rows once more in bfloat16."""
     _rounded_copy(rounded, out)
@@ -1414,7 +1425,7 @@ def embed_sinusoid(table: torch.Tensor, ids: torch.Tensor, positions: torch.Tens
         _dense(inv_freq, "inv_freq", torch.float32, 1)
         _require(inv_freq.shape[0] * 2 >= width, "inv_freq must hold a frequency for every pair of columns")
     _check(library().dli_embed_sinusoid(_ptr(table), _ptr(ids), _ptr(positions), _ptr(inv_freq), _ptr(out), _ptr(rounded), n, width,
-                                        _is_bf16(table.dtype), _stream()), "embed_sinusoid")
+                                        float(scale), _is_bf16(table.dtype), _stream()), "embed_sinusoid")
 
 
 def cast_from_f32(x: torch.Tensor, out: torch.Tensor) -> None:
@@ -1464,6 +1475,21 @@ def post_norm_stream(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, alp
     _check(library().dli_post_norm_stream(_ptr(y), y.stride(0), _ptr(gate), g_stride, _ptr(gate_bias), _ptr(weight), _ptr(x),
                                           _ptr(rounded), x.shape[0], x.shape[1], float(alpha), float(eps),
                                           _is_bf16(y.dtype), _stream()), "post_norm_stream")
+
+
+def norm_stream_norm(y: torch.Tensor, w1: torch.Tensor, eps1: float, x: torch.Tensor, w2: torch.Tensor, eps2: float,
+                     out: torch.Tensor) -> None:
+    """``x += w1 * y / sqrt(mean(y^2) + eps1)``, then ``out = w2 * x / sqrt(mean(x^2) + eps2)`` row by row: ``x`` and ``y``
+    float32 ``[n, width]`` (``y`` with contiguous rows), ``out`` float32 or bfloat16, rounded once."""
+    _f32_rows(y, "y")
+    _dense(x, "x", torch.float32, 2)
+    _dense(out, "out", ndim=2)
+    for name, w in (("w1", w1), ("w2", w2)):
+        _dense(w, name, torch.float32, 1)
+        _require(w.shape[0] == x.shape[1], f"{name} must hold a value per column")
+    _require(y.shape == x.shape and out.shape == x.shape, "y, x and out disagree on the sizes")
+    _check(library().dli_norm_stream_norm(_ptr(y), y.stride(0), _ptr(w1), float(eps1), _ptr(x), _ptr(w2), float(eps2), _ptr(out),
+                                          x.shape[0], x.shape[1], _is_bf16(out.dtype), _stream()), "norm_stream_norm")
 
 
 def rms_norm_from_f32(x: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Tensor) -> None:
@@ -1575,20 +1601,22 @@ def qk_unit_cache(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, q_out:
         _is_bf16(dtype), _stream()), "qk_unit_cache")
 
 
-def attention_scored(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, out: torch.Tensor,
+def attention_scored(q: torch.Tensor, k_pages: torch.Tensor, v_pages: Optional[torch.Tensor], out: torch.Tensor,
                      q_start: torch.Tensor, kv_len: torch.Tensor, block_tables: torch.Tensor,
                      tile_entry: Optional[torch.Tensor], tile_q0: Optional[torch.Tensor], q_heads: int, scale: float,
                      *, window: int = 0, chunk: int = 0, sink: bool = False, r1: Optional[torch.Tensor] = None,
-                     r2: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None, keep_first: int = 0) -> None:
+                     r2: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None, keep_first: int = 0,
+                     sinks: Optional[torch.Tensor] = None) -> None:
     """Paged causal attention on the vector units (32-bit arithmetic) with changes to the scores
     as parameters: ``window`` and ``chunk`` restrict the keys a query sees (under a window the first
     ``keep_first`` positions stay visible from any distance), ``r1, r2`` (float32
     ``[q_heads]``) take ``r1 log(1 + r2 (p - j))`` off the scaled score, ``sink`` adds ``exp(0)`` to the
-    softmax's denominator, ``gate`` (float32 ``[tokens, q_heads*value_dim]``, rows contiguous)
+    softmax's denominator (``sinks``, float32 ``[q_heads]``: ``exp(sinks[h])``), ``gate`` (float32 ``[tokens, q_heads*value_dim]``, rows contiguous)
     multiplies the result by its sigmoid. Values may differ from keys in size (``v_pages``), and the
     value pages may hold fewer heads than the key pages, a divisor of their number: kv head ``g`` then
     reads the values of head ``g % value_heads`` (several score maps over one set of values). ``out`` is
     of the pages' type, or float32 (the result unrounded).
+    ``v_pages`` ``None``: the values are the keys' first ``out.shape[1] / q_heads`` components.
     Without tile lists every entry is one row (a step of single tokens)."""
     _dense(k_pages, "k_pages", ndim=4)
     dtype = k_pages.dtype
@@ -1596,15 +1624,19 @@ def attention_scored(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tens
     out32 = out.dtype == torch.float32 and dtype != torch.float32
     _rows(out, "out", torch.float32 if out32 else dtype)
     pages, kv_heads, page_size, head_dim = k_pages.shape
-    _dense(v_pages, "v_pages", dtype, 4)
-    v_heads, value_dim = v_pages.shape[1], v_pages.shape[2]
-    _require(v_pages.shape == (pages, v_heads, value_dim, page_size) and v_heads > 0 and kv_heads % v_heads == 0,
+    if v_pages is None:
+        v_heads, value_dim = kv_heads, out.shape[1] // q_heads
+        _require(0 < value_dim <= head_dim <= 1024, "values that are keys are at most as long as them, keys at most 1024")
+    else:
+        _dense(v_pages, "v_pages", dtype, 4)
+        v_heads, value_dim = v_pages.shape[1], v_pages.shape[2]
+    _require(v_pages is None or v_pages.shape == (pages, v_heads, value_dim, page_size) and v_heads > 0 and kv_heads % v_heads == 0,
              "v_pages must be [pages, value heads, value_dim, page_size], the value heads a divisor of the kv heads")
     _require(keep_first >= 0, "keep_first must not be negative")
     _require(q.shape[1] == q_heads * head_dim and out.shape == (q.shape[0], q_heads * value_dim),
              "q must be [tokens, q_heads*head_dim] and out [tokens, q_heads*value_dim]")
     _require(q_heads % kv_heads == 0, "query heads are not a multiple of kv heads")
-    _require(max(head_dim, value_dim) <= 256, "heads of at most 256")
+    _require(v_pages is None or max(head_dim, value_dim) <= 256, "heads of at most 256")
     _dense(q_start, "q_start", torch.int32, 1)
     _dense(kv_len, "kv_len", torch.int32, 1)
     _dense(block_tables, "block_tables", torch.int32, 2)
@@ -1620,7 +1652,7 @@ def attention_scored(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tens
         _require(tile_entry.shape == tile_q0.shape, "tile lists differ in length")
         tiles = tile_entry.shape[0]
     _require((r1 is None) == (r2 is None), "r1 and r2 come together")
-    for name, t in (("r1", r1), ("r2", r2)):
+    for name, t in (("r1", r1), ("r2", r2), ("sinks", sinks)):
         if t is not None:
             _dense(t, name, torch.float32, 1)
             _require(t.shape[0] == q_heads, f"{name} must hold one value per query head")
@@ -1639,14 +1671,14 @@ def attention_scored(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tens
                 _ptr(q), q.stride(0), _ptr(k_pages), _ptr(v_pages), _ptr(out), out.stride(0), _ptr(kv_len),
                 _ptr(block_tables), block_tables.stride(0), entries, q_heads, kv_heads, head_dim, value_dim, page_size,
                 float(scale), int(window), int(chunk), int(bool(sink)), _ptr(r1), _ptr(r2), _ptr(gate), gate_stride,
-                int(keep_first), v_heads, _ptr(out if out32 else None), _ptr(parts), splits, _is_bf16(dtype), _stream()),
+                int(keep_first), v_heads, _ptr(out if out32 else None), _ptr(sinks), _ptr(parts), splits, _is_bf16(dtype), _stream()),
                 "attention_scored_single")
             return
     _check(library().dli_attention_scored(
         _ptr(q), q.stride(0), _ptr(k_pages), _ptr(v_pages), _ptr(out), out.stride(0), _ptr(q_start), _ptr(kv_len),
         _ptr(block_tables), block_tables.stride(0), _ptr(tile_entry), _ptr(tile_q0), tiles, q_heads, kv_heads,
         head_dim, value_dim, page_size, float(scale), int(window), int(chunk), int(bool(sink)), _ptr(r1), _ptr(r2),
-        _ptr(gate), gate_stride, int(keep_first), v_heads, _ptr(out if out32 else None), _is_bf16(dtype), _stream()),
+        _ptr(gate), gate_stride, int(keep_first), v_heads, _ptr(out if out32 else None), _ptr(sinks), _is_bf16(dtype), _stream()),
         "attention_scored")
 
 
@@ -1662,7 +1694,8 @@ def attention_scored_mfma(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch
                           q_start: torch.Tensor, kv_len: torch.Tensor, block_tables: torch.Tensor,
                           tile_entry: torch.Tensor, tile_q0: torch.Tensor, q_heads: int, scale: float, *,
                           window: int = 0, chunk: int = 0, sink: bool = False, r1: Optional[torch.Tensor] = None,
-                          r2: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None, keep_first: int = 0) -> None:
+                          r2: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None, keep_first: int = 0,
+                          sinks: Optional[torch.Tensor] = None) -> None:
     """:func:`attention_scored` for the portions of a bfloat16 step on the matrix cores: the same
     operands and parameters, tiles of ``SCORED_MFMA_TILE_ROWS`` queries, sizes that
     :func:`attention_scored_mfma_supports` takes."""
@@ -1691,7 +1724,7 @@ def attention_scored_mfma(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch
              "q_start/kv_len/block_tables disagree on the number of requests")
     _require(tile_entry.shape == tile_q0.shape, "tile lists differ in length")
     _require((r1 is None) == (r2 is None), "r1 and r2 come together")
-    for name, t in (("r1", r1), ("r2", r2)):
+    for name, t in (("r1", r1), ("r2", r2), ("sinks", sinks)):
         if t is not None:
             _dense(t, name, torch.float32, 1)
             _require(t.shape[0] == q_heads, f"{name} must hold one value per query head")
@@ -1704,7 +1737,7 @@ def attention_scored_mfma(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch
         _ptr(q), q.stride(0), _ptr(k_pages), _ptr(v_pages), _ptr(out), out.stride(0), _ptr(q_start), _ptr(kv_len),
         _ptr(block_tables), block_tables.stride(0), _ptr(tile_entry), _ptr(tile_q0), tile_entry.shape[0], q_heads,
         kv_heads, head_dim, value_dim, page_size, float(scale), int(window), int(chunk), int(bool(sink)), _ptr(r1),
-        _ptr(r2), _ptr(gate), gate_stride, int(keep_first), v_heads, _ptr(out if out32 else None), _stream()),
+        _ptr(r2), _ptr(gate), gate_stride, int(keep_first), v_heads, _ptr(out if out32 else None), _ptr(sinks), _stream()),
         "attention_scored_mfma")
 
 
@@ -1761,13 +1794,15 @@ def recurrent_scan(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, w: torch.T
 def rotary_cache(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, positions: torch.Tensor,
                  inv_freq: Optional[torch.Tensor], rot_dims: int, interleaved: bool, q_out: torch.Tensor,
                  slots: Optional[torch.Tensor], k_pages: Optional[torch.Tensor], v_pages: Optional[torch.Tensor], q_heads: int,
-                 bias: Optional[torch.Tensor] = None) -> None:
+                 bias: Optional[torch.Tensor] = None, query_temperature: Optional[tuple] = None) -> None:
     """From the float32 projections ``proj [n, >= ...]`` (q at ``q_off``, k at ``k_off``, v at ``v_off``):
     the first ``rot_dims`` components of every q and k head rotated by ``position * inv_freq[i]`` (pair
     ``i`` is ``(2i, 2i+1)`` where ``interleaved``, else ``(i, i + rot_dims/2)``; 32-bit angles),
     ``q_out [n, q_heads*dim]``; rotated k and v written at each token's cache slot. ``bias`` (float32, a
     value for every column of ``proj``) is added first. The value pages may hold fewer heads than the key
-    pages; without pages (``None``: the mixer reads another's) only q is made."""
+    pages, or be left out (``v_pages`` ``None``: the values are the keys); without key pages (``None``: the mixer reads
+    another's) only q is made. ``query_temperature = (coef, every)``: q is also multiplied by
+    ``1 + coef ln(floor((position + 1) / every) + 1)``."""
     _f32_rows(proj, "proj")
     n = proj.shape[0]
     dtype = q_out.dtype
@@ -1780,9 +1815,10 @@ def rotary_cache(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, positio
         _dense(k_pages, "k_pages", dtype, 4)
         pages, kv_heads, page_size, kdim = k_pages.shape
         _require(kdim == dim, "keys and queries differ in size")
-        _dense(v_pages, "v_pages", dtype, 4)
-        v_heads, vdim = v_pages.shape[1], v_pages.shape[2]
-        _require(v_pages.shape == (pages, v_heads, vdim, page_size), "v_pages must be [pages, value heads, vdim, page_size]")
+        if v_pages is not None:
+            _dense(v_pages, "v_pages", dtype, 4)
+            v_heads, vdim = v_pages.shape[1], v_pages.shape[2]
+            _require(v_pages.shape == (pages, v_heads, vdim, page_size), "v_pages must be [pages, value heads, vdim, page_size]")
         _dense(slots, "slots", torch.int32, 1)
         _require(slots.shape[0] == n, "slots differ from proj in rows")
     else:
@@ -1799,10 +1835,12 @@ def rotary_cache(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, positio
     if rot_dims:
         _dense(inv_freq, "inv_freq", torch.float32, 1)
         _require(inv_freq.shape[0] * 2 == rot_dims, "inv_freq must hold rot_dims/2 frequencies")
+    coef, every = (0.0, 1.0) if query_temperature is None else (float(c) for c in query_temperature)
+    _require(every > 0, "a temperature needs a positive period")
     _check(library().dli_rotary_cache(
         _ptr(proj), proj.stride(0), q_off, k_off, v_off, _ptr(bias), _ptr(positions), _ptr(inv_freq if rot_dims else None),
         int(rot_dims), int(bool(interleaved)), _ptr(q_out), _ptr(slots if k_pages is not None else None), _ptr(k_pages),
-        _ptr(v_pages), n, q_heads, kv_heads, v_heads, dim, vdim, page_size, _is_bf16(dtype), _stream()), "rotary_cache")
+        _ptr(v_pages), n, q_heads, kv_heads, v_heads, dim, vdim, page_size, coef, every, _is_bf16(dtype), _stream()), "rotary_cache")
 
 
 def group_norm(x: torch.Tensor, weight: torch.Tensor, groups: int, eps: float, out: torch.Tensor,
@@ -2064,14 +2102,16 @@ def _state_rows(state: torch.Tensor, floats: int) -> None:
 
 def causal_conv(x: torch.Tensor, conv_w: torch.Tensor, bias: Optional[torch.Tensor], state: torch.Tensor, kept_offset: int,
                 q_start: torch.Tensor, positions: torch.Tensor, state_slots: torch.Tensor, out: torch.Tensor,
-                rounded: Optional[torch.Tensor] = None, act: str = "silu") -> None:
+                rounded: Optional[torch.Tensor] = None, act: str = "silu",
+                in_bias: Optional[torch.Tensor] = None) -> None:
     """A short causal convolution over time per channel: ``out[t, c] = act(bias[c] + sum_j conv_w[c, taps-1-j] x[t-j, c])``
     with zeros before position 0. ``x`` float32 ``[n, >= channels]`` (rows contiguous; the channels from
     column 0), ``conv_w`` float32 ``[channels, taps]`` (the last column is the current token's). The inputs
     before an entry's first row come from ``state[slot, kept_offset:]`` (``[taps-1, channels]``, the newest
     last), which then receives the entry's last ``taps - 1`` inputs. ``out`` float32 ``[n, channels]``;
     ``rounded``: the result once more (float32 or bfloat16), for the product that reads it next.
-    ``act``: ``"silu"`` or ``"none"``."""
+    ``act``: ``"silu"`` or ``"none"``. ``in_bias`` (float32 ``[channels]``): added to every input that exists (the kept inputs
+    carry it, the zeros before position 0 do not)."""
     _f32_rows(x, "x")
     _dense(conv_w, "conv_w", torch.float32, 2)
     channels, taps = conv_w.shape
@@ -2081,6 +2121,9 @@ def causal_conv(x: torch.Tensor, conv_w: torch.Tensor, bias: Optional[torch.Tens
     if bias is not None:
         _dense(bias, "bias", torch.float32, 1)
         _require(bias.shape[0] == channels, "bias must hold a value per channel")
+    if in_bias is not None:
+        _dense(in_bias, "in_bias", torch.float32, 1)
+        _require(in_bias.shape[0] == channels, "in_bias must hold a value per channel")
     _f32_rows(out, "out")
     _require(out.shape == (n, channels), "out must be [n, channels]")
     r_stride, r_bf16 = 0, 0
@@ -2092,7 +2135,7 @@ def causal_conv(x: torch.Tensor, conv_w: torch.Tensor, bias: Optional[torch.Tens
     _state_rows(state, kept_offset + (taps - 1) * channels)
     entries = _step_arrays(q_start, positions, state_slots, n)
     _check(library().dli_causal_conv(
-        _ptr(x), x.stride(0), _ptr(conv_w), _ptr(bias), _ptr(state), state.stride(0), int(kept_offset), _ptr(q_start),
+        _ptr(x), x.stride(0), _ptr(conv_w), _ptr(bias), _ptr(in_bias), _ptr(state), state.stride(0), int(kept_offset), _ptr(q_start),
         _ptr(positions), _ptr(state_slots), _ptr(out), out.stride(0), _ptr(rounded), r_stride, r_bf16, entries, n,
         channels, taps, int(act == "silu"), _stream()), "causal_conv")
 
@@ -2179,51 +2222,77 @@ def gated_linear_scan(proj: torch.Tensor, q_off: int, f_off: int, v_off: int, st
 # ----------------------------------------------------------------------------- attention through a latent
 
 def latent_norm_cache(proj: torch.Tensor, q_off: int, q_rank: int, c_off: int, rank: int, q_weight: torch.Tensor,
-                      c_weight: torch.Tensor, eps: float, q_out: torch.Tensor, slots: torch.Tensor, k_pages: torch.Tensor,
-                      v_pages: torch.Tensor) -> None:
+                      c_weight: Optional[torch.Tensor], eps: float, q_out: torch.Tensor, slots: Optional[torch.Tensor],
+                      k_pages: Optional[torch.Tensor], v_pages: Optional[torch.Tensor] = None, *, rot: int = 0,
+                      inv_freq: Optional[torch.Tensor] = None, positions: Optional[torch.Tensor] = None) -> None:
     """From float32 ``proj [n, >=]``: the ``q_rank`` columns from ``q_off`` and the ``rank`` columns from ``c_off``
     each divided by their root mean square (eps inside the root) and multiplied by their weight; the first
     goes to ``q_out [n, q_rank]``, the second into the token's cache slot (negative: not cached) as a key,
-    ``k_pages [pages, 1, page_size, rank]``, and as a value, ``v_pages [pages, 1, rank, page_size]``."""
+    ``k_pages [pages, 1, page_size, rank + rot]``, and as a value, ``v_pages [pages, 1, rank, page_size]`` (``None``: the
+    values are the keys). ``rot`` > 0: the ``rot`` columns behind the latent are rotated by ``position * inv_freq[i]``
+    (component ``i`` with ``i + rot/2``, 32-bit angles) and cached behind it. ``rank`` 0 (no pages): the query's latent alone."""
     _f32_rows(proj, "proj")
     n = proj.shape[0]
     _dense(q_weight, "q_weight", torch.float32, 1)
-    _dense(c_weight, "c_weight", torch.float32, 1)
-    _require(q_weight.shape[0] == q_rank and c_weight.shape[0] == rank, "the weights must fit the latents")
-    _require(0 <= q_off and q_off + q_rank <= proj.shape[1] and 0 <= c_off and c_off + rank <= proj.shape[1],
+    _require(q_weight.shape[0] == q_rank, "the weights must fit the latents")
+    _require(0 <= q_off and q_off + q_rank <= proj.shape[1] and 0 <= c_off and c_off + rank + rot <= proj.shape[1],
              "the latents lie outside proj")
     _dense(q_out, "q_out", ndim=2)
     _require(q_out.shape == (n, q_rank), "q_out must be [n, q_rank]")
-    _dense(k_pages, "k_pages", q_out.dtype, 4)
-    _dense(v_pages, "v_pages", q_out.dtype, 4)
-    pages, _, page_size, _ = k_pages.shape
-    _require(k_pages.shape == (pages, 1, page_size, rank) and v_pages.shape == (pages, 1, rank, page_size),
-             "the pages must hold one latent a token: k [pages, 1, page_size, rank], v [pages, 1, rank, page_size]")
-    _dense(slots, "slots", torch.int32, 1)
-    _require(slots.shape[0] == n, "a cache slot per row")
+    page_size = 1
+    if rank == 0:
+        _require(rot == 0 and k_pages is None and v_pages is None, "without a latent nothing is cached")
+    else:
+        _dense(c_weight, "c_weight", torch.float32, 1)
+        _require(c_weight.shape[0] == rank, "the weights must fit the latents")
+        _dense(k_pages, "k_pages", q_out.dtype, 4)
+        pages, _, page_size, _ = k_pages.shape
+        _require(k_pages.shape == (pages, 1, page_size, rank + rot), "the key pages must hold one latent a token: [pages, 1, page_size, rank + rot]")
+        if v_pages is not None:
+            _dense(v_pages, "v_pages", q_out.dtype, 4)
+            _require(rot == 0 and v_pages.shape == (pages, 1, rank, page_size), "value pages must be [pages, 1, rank, page_size]")
+        _dense(slots, "slots", torch.int32, 1)
+        _require(slots.shape[0] == n, "a cache slot per row")
+    _rotation(rot, inv_freq, positions, n)
     _check(library().dli_latent_norm_cache(
         _ptr(proj), proj.stride(0), int(q_off), int(q_rank), int(c_off), int(rank), _ptr(q_weight), _ptr(c_weight),
-        float(eps), _ptr(q_out), _ptr(slots), _ptr(k_pages), _ptr(v_pages), n, page_size, _is_bf16(q_out.dtype),
-        _stream()), "latent_norm_cache")
+        float(eps), _ptr(q_out), _ptr(slots), _ptr(k_pages), _ptr(v_pages), n, page_size, int(rot), _ptr(inv_freq),
+        _ptr(positions), _is_bf16(q_out.dtype), _stream()), "latent_norm_cache")
 
 
-def head_products(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, gate: Optional[torch.Tensor] = None) -> None:
-    """``out[t, h] = w[h] x[t, h]`` for every head (32-bit sums, ascending k): ``x [n, heads*k]``,
-    ``w [heads, m, k]``, ``out [n, heads*m]``, all of one type (float32 or bfloat16, rows contiguous);
-    ``gate`` (float32 ``[n, heads*m]``): the result is multiplied by its sigmoid."""
+def _rotation(rot: int, inv_freq: Optional[torch.Tensor], positions: Optional[torch.Tensor], n: int) -> None:
+    _require(rot >= 0 and rot % 2 == 0, "an even number of components turns")
+    if rot:
+        _dense(inv_freq, "inv_freq", torch.float32, 1)
+        _dense(positions, "positions", torch.int32, 1)
+        _require(inv_freq.shape[0] * 2 == rot and positions.shape[0] == n, "inv_freq must hold rot/2 frequencies, positions one per row")
+
+
+def head_products(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, gate: Optional[torch.Tensor] = None, *,
+                  rot: int = 0, inv_freq: Optional[torch.Tensor] = None, positions: Optional[torch.Tensor] = None) -> None:
+    """``out[t, h] = w[h] x[t, h]`` for every head (32-bit sums, ascending k): ``x [n, heads*xs]``,
+    ``w [heads, m, k]``, ``out [n, heads*os]``, all of one type (float32 or bfloat16, rows contiguous), where a head's
+    ``xs >= k + rot`` components hold its operand first and ``os >= m + rot`` receive its result first;
+    ``gate`` (float32, ``[n, heads*m]`` or one number a head, ``[n, heads]``): the result is multiplied by its sigmoid.
+    ``rot`` > 0: the ``rot`` components behind a head's operand are rotated (component ``i`` with ``i + rot/2`` by
+    ``position * inv_freq[i]``) to the place behind its result."""
     _dense(w, "w", ndim=3)
     heads, m, k = w.shape
     _rows(x, "x", w.dtype)
     _rows(out, "out", w.dtype)
     n = x.shape[0]
-    _require(x.shape == (n, heads * k) and out.shape == (n, heads * m), "x must be [n, heads*k] and out [n, heads*m]")
-    g_stride = 0
+    _require(x.shape[1] % heads == 0 and out.shape[0] == n and out.shape[1] % heads == 0, "x must be [n, heads*xs] and out [n, heads*os]")
+    x_head, out_head = x.shape[1] // heads, out.shape[1] // heads
+    _require(x_head >= k + rot and out_head >= m + rot, "a head's operand or result does not fit its row")
+    _rotation(rot, inv_freq, positions, n)
+    g_stride, per_head = 0, 0
     if gate is not None:
         _f32_rows(gate, "gate")
-        _require(gate.shape == out.shape, "gate differs from out in shape")
-        g_stride = gate.stride(0)
-    _check(library().dli_head_products(_ptr(x), x.stride(0), _ptr(w), _ptr(out), out.stride(0), _ptr(gate), g_stride, n,
-                                       heads, m, k, _is_bf16(w.dtype), _stream()), "head_products")
+        _require(gate.shape in ((n, heads * m), (n, heads)), "gate must hold a value per output or per head")
+        g_stride, per_head = gate.stride(0), int(gate.shape[1] == heads)
+    _check(library().dli_head_products(_ptr(x), x.stride(0), x_head, _ptr(w), _ptr(out), out.stride(0), out_head, _ptr(gate),
+                                       g_stride, per_head, n, heads, m, k, int(rot), _ptr(inv_freq), _ptr(positions),
+                                       _is_bf16(w.dtype), _stream()), "head_products")
 
 
 # ----------------------------------------------------------------------------- recurrences under scalar gates, differential maps
@@ -2370,3 +2439,53 @@ def silu_columns(x: torch.Tensor) -> None:
     """``x <- silu(x)`` in place: float32 ``[n, width]`` with contiguous rows (columns of a wider matrix will do)."""
     _f32_rows(x, "x")
     _check(library().dli_silu_columns(_ptr(x), x.stride(0), x.shape[0], x.shape[1], _stream()), "silu_columns")
+
+
+# ----------------------------------------------------------------------------- the gated unit recurrence
+
+def gated_unit_tile_rows() -> int:
+    return int(library().dli_gated_unit_tile_rows())
+
+
+def gated_unit(u: torch.Tensor, w_r: torch.Tensor, w_i: torch.Tensor, r_bias: torch.Tensor, i_bias: torch.Tensor,
+               decay: torch.Tensor, y: torch.Tensor, y_bias: Optional[torch.Tensor], state: torch.Tensor, q_start: torch.Tensor,
+               positions: torch.Tensor, state_slots: torch.Tensor, tiles: Optional[tuple], out: torch.Tensor) -> None:
+    """Per request and channel, over the step's rows in order: with block-diagonal gates ``r = sigmoid(w_r u + r_bias)``,
+    ``i = sigmoid(w_i u + i_bias)`` and ``a = exp(-r decay)``, ``S <- a S + sqrt(1 - a^2) i u``, ``out = S gelu(y + y_bias)``
+    (tanh form). ``u`` and ``y`` float32 ``[n, channels]`` (rows contiguous), ``w_r, w_i [blocks, s, s]`` of ``out``'s type (a row an
+    output), biases and ``decay`` (not negative) float32 ``[channels]``. ``S`` float32 ``[channels]`` at the start of
+    ``state[slot]`` (zeros at position 0). ``tiles``: the step's tiles of :func:`gated_unit_tile_rows` rows, every entry's
+    (``StepContext.q_tiles``); ``None``: every entry is one row."""
+    _f32_rows(u, "u")
+    _f32_rows(y, "y")
+    n, channels = u.shape
+    _dense(w_r, "w_r", out.dtype, 3)
+    _dense(w_i, "w_i", out.dtype, 3)
+    blocks, s = w_r.shape[0], w_r.shape[1]
+    _require(w_r.shape == (blocks, s, s) and w_i.shape == w_r.shape and blocks * s == channels,
+             "the gates' maps must be [blocks, s, s], blocks * s the channels")
+    for name, t in (("r_bias", r_bias), ("i_bias", i_bias), ("decay", decay), ("y_bias", y_bias)):
+        if t is not None:
+            _dense(t, name, torch.float32, 1)
+            _require(t.shape[0] == channels, f"{name} must hold a value per channel")
+    _rows(out, "out", out.dtype)
+    _require(y.shape == (n, channels) and out.shape == (n, channels), "y and out must be [n, channels]")
+    _state_rows(state, channels)
+    entries = _step_arrays(q_start, positions, state_slots, n)
+    s_local = p_local = ends = tile_entry = tile_q0 = None
+    count = 0
+    if tiles is None:
+        _require(entries == n, "without tile lists every entry must be one row")
+    else:
+        tile_entry, tile_q0 = tiles
+        _dense(tile_entry, "tile_entry", torch.int32, 1)
+        _dense(tile_q0, "tile_q0", torch.int32, 1)
+        _require(tile_entry.shape == tile_q0.shape, "tile lists differ in length")
+        count = tile_entry.shape[0]
+        s_local, p_local = (torch.empty(n, channels, device=u.device, dtype=torch.float32) for _ in range(2))
+        ends = torch.empty(max(count, 1), 2, channels, device=u.device, dtype=torch.float32)
+    _check(library().dli_gated_unit(
+        _ptr(u), u.stride(0), _ptr(w_r), _ptr(w_i), _ptr(r_bias), _ptr(i_bias), _ptr(decay), _ptr(y), y.stride(0), _ptr(y_bias),
+        _ptr(state), state.stride(0), _ptr(q_start), _ptr(positions), _ptr(state_slots), _ptr(tile_entry), _ptr(tile_q0), count,
+        _ptr(s_local), _ptr(p_local), _ptr(ends), _ptr(out), out.stride(0), entries, n, channels, blocks, _is_bf16(out.dtype),
+        _stream()), "gated_unit")

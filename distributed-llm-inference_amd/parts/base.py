@@ -287,6 +287,9 @@ class Block(Part):
     roles of the layer's :class:`LayerSpec` to built parts."""
 
     roles: tuple[str, ...] = ()
+    # Whether ``forward`` takes a keyword ``following``: the norm that the stream meets after this block
+    # (the next block's ``first_norm``, the final norm, or None), for a block whose last kernel can apply it.
+    takes_following: bool = False
 
     def forward(self, x: torch.Tensor, delta: Optional[torch.Tensor], ctx: Any, cache: Any,
                 parts: Mapping[str, Part]) -> tuple[torch.Tensor, Optional[torch.Tensor]]:

@@ -11,7 +11,7 @@ from typing import Any, Mapping, Optional
 import torch
 
 from .base import Block, DecodeStream, Part, Runtime
-from .linear import as_operand
+from .linear import NormedStream, as_operand
 from .registry import register_part
 
 
@@ -211,6 +211,55 @@ class ParallelNormsBlock(Block):
         y = _as_f32(parts["mixer"].forward(h1, ctx, cache))
         f = _as_f32(parts["feed_forward"].forward(h2, ctx))
         ops.add_pair_into_stream(x, y, f)
+        return x, None
+
+
+@register_part("block", "sandwich_norms")
+class SandwichNormsBlock(Block):
+    """A norm before and a norm after every sublayer, around a 32-bit residual stream:
+    ``x <- x + out_norm1(mixer(norm1(x)))``, then ``x <- x + out_norm2(feed_forward(norm2(x)))`` (a constant on the summands
+    goes into the out-norms' weights). The feed-forward and its norms may be absent. ``x`` is float32 in both
+    runtimes. A sublayer's out-norm, the residual sum and the norm that the stream meets next are one kernel."""
+
+    roles = ("mixer_norm", "mixer", "mixer_out_norm")   # and "feed_forward_norm", "feed_forward", "feed_forward_out_norm"
+    takes_following = True
+
+    def __init__(self, runtime: Runtime) -> None:
+        super().__init__(runtime)
+
+    def graph_capturable(self, page_size: int) -> bool:
+        return True  # kernels on device arrays only
+
+    def first_norm(self, parts: Mapping[str, Part]) -> Optional[Part]:
+        return parts["mixer_norm"]
+
+    def _add(self, x: torch.Tensor, y: torch.Tensor, out_norm: Part, following: Optional[Part], ctx: Any) -> None:
+        """``x += out_norm(y)``; the rows normalised by ``following`` are left on the context where one kernel makes both."""
+        if following is not None and hasattr(out_norm, "add_normed_then") and hasattr(following, "fused_params"):
+            NormedStream.offer(ctx, x, following, out_norm.add_normed_then(x, _as_f32(y), following))
+        else:
+            out_norm.add_normed(x, y, ctx)
+            NormedStream.offer(ctx, x, None, None)
+
+    def _normed(self, x: torch.Tensor, norm: Part, ctx: Any) -> torch.Tensor:
+        ready = NormedStream.take(ctx, x, norm)
+        return ready if ready is not None else norm.forward(x)
+
+    def forward(self, x: torch.Tensor, delta: Optional[torch.Tensor], ctx: Any, cache: Any, parts: Mapping[str, Part],
+                following: Optional[Part] = None) -> tuple[torch.Tensor, Optional[torch.Tensor]]:
+        if x.dtype != torch.float32:
+            raise RuntimeError("the sandwich_norms block keeps a float32 residual stream")
+        if delta is not None:
+            from ..kernels import ops
+
+            ops.add(x, delta, x)
+            NormedStream.offer(ctx, x, None, None)
+        h = self._normed(x, parts["mixer_norm"], ctx)
+        y = parts["mixer"].forward(h, ctx, cache)
+        self._add(x, y, parts["mixer_out_norm"], parts.get("feed_forward_norm", following), ctx)
+        if "feed_forward" in parts:
+            h = self._normed(x, parts["feed_forward_norm"], ctx)
+            self._add(x, parts["feed_forward"].forward(h, ctx), parts["feed_forward_out_norm"], following, ctx)
         return x, None
 
 

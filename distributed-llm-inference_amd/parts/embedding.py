@@ -16,17 +16,22 @@ from .spec import PartSpec, WeightSpec
 @register_part("embedding", "token_embedding")
 class TokenEmbedding(Embedding):
     def __init__(self, runtime: Runtime, *, vocab_size: int, hidden_size: int, weight_name: str = "weight",
-                 float32_rows: bool = False, norm: Optional[PartSpec] = None) -> None:
+                 float32_rows: bool = False, norm: Optional[PartSpec] = None,
+                 scale: float = 1.0) -> None:
         """``float32_rows``: the rows go out widened to float32 whatever the runtime's type, for a
         model that keeps its residual stream in 32-bit (the table keeps the runtime's type). ``norm``: a norm
-        (a part with ``forward_f32``) that the float32 rows pass before they become the stream."""
+        (a part with ``forward_f32``) that the float32 rows pass before they become the stream. ``scale``: the float32
+        rows are multiplied by it (a tied head reads the table without it)."""
         super().__init__(runtime)
         self.vocab_size, self.hidden_size = vocab_size, hidden_size
         self.weight_name, self.float32_rows = weight_name, bool(float32_rows)
         self.weight: torch.Tensor | None = None
         if norm is not None and not self.float32_rows:
             raise ValueError("a norm on the embedded rows belongs to a float32 stream")
+        if scale != 1.0 and not self.float32_rows:
+            raise ValueError("a scale on the embedded rows belongs to a float32 stream")
         self.norm = build_part("norm", norm, runtime) if norm is not None else None
+        self.scale = float(scale)
 
     def sub_parts(self) -> dict:
         return {"norm": self.norm} if self.norm is not None else {}
@@ -55,7 +60,7 @@ class TokenEmbedding(Embedding):
         if not self.float32_rows:
             return self.forward(ctx.token_ids)
         out = torch.empty(ctx.token_ids.shape[0], self.hidden_size, device=self.rt.device, dtype=torch.float32)
-        ops.embed_sinusoid(self.table(), ctx.token_ids, ctx.positions, None, out)
+        ops.embed_sinusoid(self.table(), ctx.token_ids, ctx.positions, None, out, scale=self.scale)
         return out if self.norm is None else self.norm.forward_f32(out)
 
     def streams(self, ctx) -> bool:

@@ -1,5 +1,6 @@
 """Gated feed-forward: ``down(act(gate(x)) * up(x))`` with ``act = silu`` (SwiGLU; reference:
-src/dli/model/llama.py:180-191). Gate and up matrices are stacked at load, so one product gives
+src/dli/model/llama.py:180-191), or ``down(g sigmoid(alpha g) (u + up_shift))`` with clamped halves
+``g = min(gate(x), limit)``, ``u = clamp(up(x), -limit, limit)`` (``activation="clamped"``). Gate and up matrices are stacked at load, so one product gives
 both halves; the activation kernel reads them side by side."""
 
 from __future__ import annotations
@@ -10,7 +11,7 @@ import torch
 
 from ..kernels import ops
 from .base import DecodeStream, FeedForward, Norm, Runtime
-from .linear import decode_copy, finish_residual, linear
+from .linear import decode_copy, finish_residual, linear, linear_f32
 from .registry import register_part
 from .spec import WeightSpec
 
@@ -21,7 +22,10 @@ class GatedMLP(FeedForward):
 
     def __init__(self, runtime: Runtime, *, hidden_size: int, intermediate_size: int,
                  activation: str = "silu", bias: bool = False, names: Optional[Mapping[str, str]] = None,
-                 few_rows_fused: bool = False) -> None:
+                 few_rows_fused: bool = False, limit: float = float("inf"), alpha: float = 1.0, up_shift: float = 0.0,
+                 float32_out: bool = False) -> None:
+        """``limit``, ``alpha``, ``up_shift``: of the clamped activation. ``float32_out``: the result is the second product's
+        32-bit sums (for a norm or a residual stream that is 32-bit)."""
         super().__init__(runtime)
         # forward() itself takes the few-row kernels (SwiGLU inside the first product) for up to 16
         # rows: for blocks that have no fused decode path of their own
@@ -30,8 +34,12 @@ class GatedMLP(FeedForward):
         self.names = {**self.NAMES, **dict(names or {})}
         if bias and names:
             raise ValueError("gated_mlp: other tensor names are taken for the matrices only")
-        if activation != "silu":
-            raise ValueError(f"gated_mlp has no kernel for activation {activation!r} (only 'silu')")
+        if activation not in ("silu", "clamped"):
+            raise ValueError(f"gated_mlp has no kernel for activation {activation!r} (only 'silu' and 'clamped')")
+        if bias and (activation != "silu" or float32_out):
+            raise ValueError("gated_mlp: biases go with the plain activation and a result of the runtime's type")
+        self.clamped = (float(limit), float(alpha), float(up_shift)) if activation == "clamped" else None
+        self.float32_out = bool(float32_out)
         self.hidden_size, self.intermediate_size, self.bias = hidden_size, intermediate_size, bias
         self.w_gate_up = self.b_gate_up = self.w_down = self.b_down = None
         self.w_gate_up_tiled = self.w_down_tiled = None
@@ -63,7 +71,7 @@ class GatedMLP(FeedForward):
         from .native import _bf16_matrix, _bf16_vector
 
         h, i = self.hidden_size, self.intermediate_size
-        if type(self) is not GatedMLP:
+        if type(self) is not GatedMLP or self.clamped is not None or self.float32_out:
             return None  # a subclass computes something else: it must describe itself
         if not (self.rt.is_bf16 and _bf16_matrix(self.w_gate_up, 2 * i, h) and _bf16_matrix(self.w_down, h, i)
                 and _bf16_vector(self.b_gate_up, 2 * i) and _bf16_vector(self.b_down, h)):
@@ -71,30 +79,39 @@ class GatedMLP(FeedForward):
         return {"kind": "gated_silu", "w_gate_up": self.w_gate_up, "b_gate_up": self.b_gate_up, "w_down": self.w_down, "b_down": self.b_down,
                 "hidden": h, "intermediate": i}
 
+    def _takes_few_rows(self, x: torch.Tensor) -> bool:
+        n = x.shape[0]
+        return (self.rt.is_bf16 and 0 < n <= self.FEW_ROWS and x.dtype == torch.bfloat16 and x.stride(0) % 8 == 0
+                and x.data_ptr() % 16 == 0 and ops.skinny_gemm_supports(n, self.hidden_size, x.dtype)
+                and ops.skinny_gemm_supports(n, self.intermediate_size, x.dtype))
+
     def forward(self, x: torch.Tensor, ctx: Any) -> torch.Tensor:
         n = x.shape[0]
-        if (self.few_rows_fused and self.rt.is_bf16 and 0 < n <= self.FEW_ROWS and x.dtype == torch.bfloat16 and x.stride(0) % 8 == 0
-                and x.data_ptr() % 16 == 0 and ops.skinny_gemm_supports(n, self.hidden_size, x.dtype)
-                and ops.skinny_gemm_supports(n, self.intermediate_size, x.dtype)):
+        act = self.rt.empty(n, self.intermediate_size)
+        if (self.few_rows_fused or self.float32_out) and self._takes_few_rows(x):
             # a few rows outside the fused decode path (a block that keeps its stream in 32-bit, say):
-            # the few-row products, SwiGLU inside the first
-            act = self.rt.empty(n, self.intermediate_size)
+            # the few-row products, the activation inside the first
             ops.skinny_gemm(x, self.w_gate_up, w_tiled=self.w_gate_up_tiled, epilogue=ops.SKINNY_SWIGLU, out=act,
-                            bias=self.b_gate_up)
-            out = self.rt.empty(n, self.hidden_size)
-            ops.skinny_gemm(act, self.w_down, w_tiled=self.w_down_tiled, epilogue=ops.SKINNY_STORE, out=out,
-                            bias=self.b_down)
+                            bias=self.b_gate_up, clamped=self.clamped)
+            out = torch.empty(n, self.hidden_size, device=self.rt.device,
+                              dtype=torch.float32 if self.float32_out else self.rt.dtype)
+            ops.skinny_gemm(act, self.w_down, w_tiled=self.w_down_tiled, bias=self.b_down, out=out,
+                            epilogue=ops.SKINNY_F32 if self.float32_out else ops.SKINNY_STORE)
             return out
         gate_up = linear(self.rt, x, self.w_gate_up, self.b_gate_up)
-        act = self.rt.empty(x.shape[0], self.intermediate_size)
-        ops.silu_mul(gate_up, act)
+        if self.clamped is not None:
+            ops.clamped_glu(gate_up, act, *self.clamped)
+        else:
+            ops.silu_mul(gate_up, act)
+        if self.float32_out:
+            return linear_f32(self.rt, act, self.w_down)
         return linear(self.rt, act, self.w_down, self.b_down)
 
     FEW_ROWS = 16  # the few-row product kernels; 17 to 64 rows take the one that shares activations
 
     def streams(self, ctx: Any) -> bool:
         n = ctx.num_tokens
-        if not (self.rt.is_bf16 and self.hidden_size % 8 == 0):
+        if self.clamped is not None or self.float32_out or not (self.rt.is_bf16 and self.hidden_size % 8 == 0):
             return False
         if n > self.FEW_ROWS:
             return (self.w_gate_up_tiled is not None and self.w_down_tiled is not None
@@ -156,8 +173,6 @@ class PolyNormMLP(FeedForward):
         self.coef = tensors[self.names["act"]].contiguous()
 
     def forward(self, x: torch.Tensor, ctx: Any) -> torch.Tensor:
-        from .linear import linear_f32
-
         z = linear_f32(self.rt, x, self.w_up)
         act = self.rt.empty(x.shape[0], self.intermediate_size)
         ops.poly_norm(z, self.coef, self.norm_eps, act)

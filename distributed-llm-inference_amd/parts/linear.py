@@ -15,7 +15,7 @@ from typing import Optional
 import torch
 
 from ..kernels import ops
-from .base import DecodeStream, Norm, Runtime
+from .base import DecodeStream, Norm, Runtime, norm_key
 
 
 def linear(rt: Runtime, x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor] = None,
@@ -98,6 +98,30 @@ class RoundedStream:
     def take(ctx, x: torch.Tensor) -> Optional[torch.Tensor]:
         hit = getattr(ctx, "_memo", {}).get(RoundedStream.KEY) if ctx is not None else None
         return hit[2] if hit is not None and hit[:2] == (x.data_ptr(), tuple(x.shape)) else None
+
+
+class NormedStream:
+    """The rows of a 32-bit residual stream already normalised by a named norm, where the kernel that last wrote
+    the stream was told which norm follows: kept on the step's context for whoever applies that norm next, and
+    dropped by whoever changes the stream."""
+
+    KEY = "normed stream"
+
+    @staticmethod
+    def offer(ctx, x: torch.Tensor, norm: Optional[Norm], rows: Optional[torch.Tensor]) -> None:
+        if ctx is not None and hasattr(ctx, "_memo"):
+            if rows is None:
+                ctx._memo.pop(NormedStream.KEY, None)
+            else:
+                ctx._memo[NormedStream.KEY] = (x.data_ptr(), tuple(x.shape), norm_key(norm), rows)
+
+    @staticmethod
+    def take(ctx, x: torch.Tensor, norm: Norm) -> Optional[torch.Tensor]:
+        hit = getattr(ctx, "_memo", {}).get(NormedStream.KEY) if ctx is not None else None
+        key = norm_key(norm)
+        if hit is None or key is None or hit[:3] != (x.data_ptr(), tuple(x.shape), key):
+            return None
+        return ctx._memo.pop(NormedStream.KEY)[3]   # (applied once: the stream changes after it)
 
 
 def as_operand(rt: Runtime, x: torch.Tensor, ctx=None) -> torch.Tensor:

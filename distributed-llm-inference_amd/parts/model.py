@@ -16,12 +16,13 @@ import torch
 
 from ..kernels import ops
 from .base import Part, Runtime
+from .linear import NormedStream
 from .registry import build_part
 from .spec import ModelSpec, WeightSpec
 
 # importing the modules registers the built-in parts
 from . import (  # noqa: F401,E402
-    attention, block, embedding, experts, feed_forward, head, latent_attention, norm, parallel, position, recurrent,
+    attention, block, embedding, experts, feed_forward, gated_unit, head, latent_attention, norm, parallel, position, recurrent,
     scored_attention, selective_scan, token_shift,
 )
 
@@ -203,12 +204,22 @@ class Model:
             delta = native.run(x, ctx)      # every layer's launches from one call; None: nothing ran
             self.native_runs += delta is not None
         if delta is None:
-            for entry, cache in zip(self.spec.schedule, caches):
-                layer = self.layers[entry.layer]
-                x, delta = layer.block.forward(x, delta, ctx, cache, layer.parts)
+            order = [self.layers[entry.layer] for entry in self.spec.schedule]
+            for i, (layer, cache) in enumerate(zip(order, caches)):
+                if layer.block.takes_following:
+                    # (the final norm reads the wanted rows: it follows where those are all rows, in order)
+                    after = (order[i + 1].block.first_norm(order[i + 1].parts) if i + 1 < len(order)
+                             else self.final_norm if getattr(ctx, "all_rows_wanted", False) else None)
+                    x, delta = layer.block.forward(x, delta, ctx, cache, layer.parts, following=after)
+                else:
+                    x, delta = layer.block.forward(x, delta, ctx, cache, layer.parts)
         k = ctx.logit_rows.shape[0]
         if k == 0:
             return torch.empty(0, self.spec.vocab_size, device=self.rt.device, dtype=torch.float32)
+        if delta is None and getattr(ctx, "all_rows_wanted", False):
+            ready = NormedStream.take(ctx, x, self.final_norm)
+            if ready is not None:
+                return self.head.forward(ready)
         xs = torch.empty(k, x.shape[1], device=x.device, dtype=x.dtype)
         ops.gather_rows(x, ctx.logit_rows, xs)
         ds = None

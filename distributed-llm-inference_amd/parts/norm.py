@@ -16,11 +16,13 @@ from .spec import WeightSpec
 @register_part("norm", "rms_norm")
 class RMSNorm(Norm):
     def __init__(self, runtime: Runtime, *, width: int, eps: float, weight_name: str = "weight",
-                 unit_offset: bool = False) -> None:
+                 unit_offset: bool = False, weight_scale: float = 1.0) -> None:
         """``unit_offset``: the checkpoint stores the weight around zero and the norm multiplies by one plus it
-        (the sum is made once, at load, in 32-bit; every kernel then sees an ordinary weight)."""
+        (the sum is made once, at load, in 32-bit; every kernel then sees an ordinary weight). ``weight_scale``: a constant that
+        the norm's result is multiplied by, in the weight likewise."""
         super().__init__(runtime)
         self.width, self.eps, self.weight_name, self.unit_offset = width, float(eps), weight_name, bool(unit_offset)
+        self.weight_scale = float(weight_scale)
         self.weight: torch.Tensor | None = None
 
     def graph_capturable(self, page_size: int) -> bool:
@@ -31,7 +33,8 @@ class RMSNorm(Norm):
 
     def load_weights(self, tensors: Mapping[str, torch.Tensor]) -> None:
         w = tensors[self.weight_name]
-        self.weight = (w + 1.0).contiguous() if self.unit_offset else w
+        w = (w + 1.0).contiguous() if self.unit_offset else w
+        self.weight = w if self.weight_scale == 1.0 else (w * self.weight_scale).contiguous()
 
     def forward_f32(self, x: torch.Tensor) -> torch.Tensor:
         """The norm of a float32 ``x`` as float32 whatever the runtime's type (a norm inside a 32-bit stream)."""
@@ -61,6 +64,14 @@ class RMSNorm(Norm):
         rounded = self.rt.empty(*x.shape) if self.rt.is_bf16 and ctx is not None else None
         ops.norm_into_stream(y, self.weight, self.eps, x, rounded=rounded)
         RoundedStream.offer(ctx, x, rounded)
+
+    def add_normed_then(self, x: torch.Tensor, y: torch.Tensor, following: "RMSNorm") -> torch.Tensor:
+        """``x += norm(y)`` as :meth:`add_normed`, and in the same kernel the norm that the new stream meets next:
+        the rows normalised by ``following``, in the runtime's type. ``y`` float32."""
+        w2, eps2 = following.fused_params()
+        out = self.rt.empty(*x.shape)
+        ops.norm_stream_norm(y, self.weight, self.eps, x, w2, eps2, out)
+        return out
 
     def post_norm(self, x: torch.Tensor, y: torch.Tensor, alpha: float, ctx=None, gate: Optional[torch.Tensor] = None,
                   gate_bias: Optional[torch.Tensor] = None) -> None:

@@ -1,9 +1,10 @@
 """Grouped-query attention over the paged cache whose scores are changed by parameters: unit-RMS
 queries and keys or a rotary position encoding, a per-head logarithmic distance penalty, a chunked
-mask, a window that keeps the first positions, a softmax with a sink, value mixing across layers, a sigmoid
-output gate, biases on the projections, several score maps a head over the same values whose results are
-subtracted (differential attention), and keys and values read from another layer's cache. Each is a
-parameter, so another design may take any subset.
+mask, a window that keeps the first positions, a softmax with a sink (of score 0 or of a learnt score per head),
+a temperature on the queries that grows with the position, value mixing across layers, a sigmoid output gate,
+biases on the projections, several score maps a head over the same values whose results are subtracted
+(differential attention), values that are the keys, and keys and values read from another layer's cache. Each
+is a parameter, so another design may take any subset.
 
 Order of work for the rows ``h`` of a step (``x`` may be a 32-bit residual stream; the products read
 it in the runtime's type):
@@ -31,6 +32,10 @@ the head's result is ``d / sqrt(mean(d^2) + norm_eps) * (1 - diff)`` with ``d = 
 ``sigmoid(W_g h)_head`` where ``head_gate`` (one number a head). ``own_kv=False``: the layer has no key and value
 projections and reads the cache of the schedule entry it is given (keys as that layer rotated them).
 
+``head_sink``: a learnt number ``sink`` per head instead of the 1 above, ``exp(sink_h)``. ``keys_as_values``: there is no value
+projection; the values are the keys as cached, and the pages hold keys alone. ``query_temperature = (coef, every)``: q is
+multiplied by ``1 + coef ln(floor((p + 1) / every) + 1)`` at position ``p``, before it is rounded.
+
 Scores, weights, norms and the mixing are 32-bit; keys and values are cached in the runtime's type.
 """
 
@@ -55,14 +60,15 @@ def paged_scored_attention(rt: Runtime, ctx: Any, cache: Any, q: torch.Tensor, o
     values there: steps of single tokens go to the kernel that reads the context's device arrays alone,
     the portions of other steps to the matrix cores where they take the sizes (single tokens, which come
     first, to their kernel), else to the vector-unit tile kernel. ``changes``: ``window``, ``chunk``, ``sink``,
-    ``r1``, ``r2`` as :func:`dli_amd.kernels.ops.attention_scored` takes them."""
+    ``r1``, ``r2``, ``sinks`` as :func:`dli_amd.kernels.ops.attention_scored` takes them. A cache without value pages: the
+    values are the keys' first ``value_dim`` components."""
     grp = ctx.groups[cache.group]
     nd = ctx.num_decode
     if nd == ctx.num_entries:
         # every entry is one row: nothing is derived from the step's lengths on the host
         ops.attention_scored(q, cache.k_pages, cache.v_pages, out, ctx.q_start, ctx.kv_len, grp.block_tables,
                              None, None, num_heads, scale, gate=gate, **changes)
-    elif ops.attention_scored_mfma_supports(head_dim, value_dim, ctx.page_size, rt.dtype):
+    elif cache.v_pages is not None and ops.attention_scored_mfma_supports(head_dim, value_dim, ctx.page_size, rt.dtype):
         if nd:
             ops.attention_scored(q[:nd], cache.k_pages, cache.v_pages, out[:nd], ctx.q_start[:nd + 1], ctx.kv_len[:nd],
                                  grp.block_tables[:nd], None, None, num_heads, scale,
@@ -86,7 +92,8 @@ class ScoredAttention(Mixer):
                  sink: bool = False, output_gate: bool = False, value_mix: str = "none",
                  value_mix_key: str = "first_values", names: Optional[Mapping[str, str]] = None,
                  position: Optional[PartSpec] = None, bias: bool = False, keep_first: int = 0, maps: int = 1,
-                 diff: float = 0.0, head_gate: bool = False, own_kv: bool = True, cache_window: Optional[int] = None) -> None:
+                 diff: float = 0.0, head_gate: bool = False, own_kv: bool = True, cache_window: Optional[int] = None,
+                 keys_as_values: bool = False, head_sink: bool = False, query_temperature: Optional[tuple] = None) -> None:
         """``cache_window``: how many of the latest keys the pages must keep where that is not this layer's own
         window (0: all): other layers that read this layer's cache may look further back than it does."""
         super().__init__(runtime)
@@ -110,8 +117,17 @@ class ScoredAttention(Mixer):
         if num_heads < 1 or num_kv_heads < 1 or num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} query heads do not group onto {num_kv_heads} kv heads")
         value_dim = head_dim if value_dim is None else value_dim
-        if not 0 < head_dim <= 256 or not 0 < value_dim <= 256:
-            raise ops.KernelArgumentError(f"attention takes heads of 1 to 256, not {head_dim} / {value_dim}")
+        self.keys_as_values, self.head_sink = bool(keys_as_values), bool(head_sink)
+        self.query_temperature = tuple(float(c) for c in query_temperature) if query_temperature is not None else None
+        if (keys_as_values or head_sink or query_temperature is not None) and (qk_unit or maps == 2 or value_mix != "none"):
+            raise ValueError("scored_attention: values that are keys, a sink per head and a query temperature go with one map of rotary or plain keys")
+        if keys_as_values and value_dim != head_dim:
+            raise ValueError("scored_attention: values that are keys have their size")
+        if head_sink and sink:
+            raise ValueError("scored_attention: one sink")
+        most = 1024 if keys_as_values else 256
+        if not 0 < head_dim <= most or not 0 < value_dim <= most:
+            raise ops.KernelArgumentError(f"attention takes heads of 1 to {most}, not {head_dim} / {value_dim}")
         if value_mix not in self.VALUE_MIX:
             raise ValueError(f"value_mix must be one of {self.VALUE_MIX}")
         if chunk < 0 or window < 0:
@@ -128,9 +144,9 @@ class ScoredAttention(Mixer):
             raise ValueError("scored_attention: unit keys and a position encoding together have no kernel")
         if not self.qk_unit and value_mix != "none":
             raise ValueError("scored_attention: value mixing belongs to the kernel that makes unit keys")
-        self.names = {"q": "q", "k": "k", "v": "v", "g": "g", "o": "o", "mix": "vmix", "r1": "r1", "r2": "r2",
+        self.names = {"q": "q", "k": "k", "v": "v", "g": "g", "o": "o", "mix": "vmix", "r1": "r1", "r2": "r2", "sink": "sink",
                       "lq1": "lq1", "lk1": "lk1", "lq2": "lq2", "lk2": "lk2", **dict(names or {})}
-        self.w_in = self.w_o = self.mix = self.r1 = self.r2 = None
+        self.w_in = self.w_o = self.mix = self.r1 = self.r2 = self.sinks = None
 
     # -- sizes of the stacked projection's parts
     @property
@@ -143,7 +159,7 @@ class ScoredAttention(Mixer):
 
     @property
     def _v(self) -> int:
-        return self.num_kv_heads * self.value_dim if self.own_kv else 0
+        return self.num_kv_heads * self.value_dim if self.own_kv and not self.keys_as_values else 0
 
     @property
     def _o(self) -> int:
@@ -153,7 +169,9 @@ class ScoredAttention(Mixer):
         n, h = self.names, self.hidden_size
         specs = {n["q"]: WeightSpec((self._q, h)), n["o"]: WeightSpec((h, self._o))}
         if self.own_kv:
-            specs.update({n["k"]: WeightSpec((self._k, h)), n["v"]: WeightSpec((self._v, h))})
+            specs.update({n[s]: WeightSpec((size, h)) for s, size in (("k", self._k), ("v", self._v)) if size})
+        if self.head_sink:
+            specs[n["sink"]] = WeightSpec((self.num_heads,), role="float32", init="zeros")
         if self.bias:
             specs.update({n[s] + ".b": WeightSpec((size,), role="float32", init="zeros")
                           for s, size in (("q", self._q), ("k", self._k), ("v", self._v)) if size})
@@ -180,7 +198,7 @@ class ScoredAttention(Mixer):
                 return t
             return t.reshape(heads, self.maps, self.head_dim, *t.shape[1:]).transpose(0, 1).reshape(t.shape)
 
-        kinds = [("q", self.num_heads)] + ([("k", self.num_kv_heads), ("v", 0)] if self.own_kv else [])
+        kinds = [("q", self.num_heads)] + ([("k", self.num_kv_heads)] if self.own_kv else []) + ([("v", 0)] if self._v else [])
         stacked = [by_map(tensors[n[s]], heads) if heads else tensors[n[s]] for s, heads in kinds]
         if self.output_gate or self.head_gate:
             stacked.append(tensors[n["g"]])
@@ -192,6 +210,8 @@ class ScoredAttention(Mixer):
             lq1, lk1, lq2, lk2 = (tensors[n[s]].float() for s in ("lq1", "lk1", "lq2", "lk2"))
             self.lam = float(torch.exp((lq1 * lk1).sum()) - torch.exp((lq2 * lk2).sum())) + self.diff
         self.w_o = tensors[n["o"]]
+        if self.head_sink:
+            self.sinks = tensors[n["sink"]].contiguous()
         if self.distance_penalty:
             self.r1, self.r2 = tensors[n["r1"]].contiguous(), tensors[n["r2"]].contiguous()
         if self.value_mix == "mix":
@@ -213,6 +233,8 @@ class ScoredAttention(Mixer):
             return None   # the schedule hands this layer another entry's cache
         # (a window that keeps its first positions gives no page back while the request runs)
         kept = self.cache_window if self.cache_window is not None else (0 if self.keep_first else self.window)
+        if self.keys_as_values:
+            return PagedKVSpec(self.num_kv_heads, self.head_dim, kept, 0)
         return PagedKVSpec(self.num_kv_heads * self.maps, self.head_dim, kept,
                            None if self.value_dim == self.head_dim else self.value_dim,
                            self.num_kv_heads if self.maps > 1 else None)
@@ -253,7 +275,8 @@ class ScoredAttention(Mixer):
             ops.rotary_cache(proj, 0, self._q, self._q + self._k, ctx.positions, None if table is None else table.inv_freq,
                              0 if table is None else table.dim, table is not None and table.pairing == "interleaved",
                              q, grp.slots if self.own_kv else None, cache.k_pages if self.own_kv else None,
-                             cache.v_pages if self.own_kv else None, self.num_heads * self.maps, bias=self.b_in)
+                             cache.v_pages if self.own_kv else None, self.num_heads * self.maps, bias=self.b_in,
+                             query_temperature=self.query_temperature)
         g0 = self._q + self._k + self._v
         if self.maps == 2:
             # each map is a head of its own to the attention kernels; their results stay 32-bit until they are combined
@@ -269,5 +292,5 @@ class ScoredAttention(Mixer):
         gate = proj[:, g0:g0 + self._o] if self.output_gate else None
         paged_scored_attention(self.rt, ctx, cache, q, out, self.num_heads, self.head_dim, self.value_dim, self.scale,
                                gate=gate, window=self.window, chunk=self.chunk, sink=self.sink, r1=self.r1, r2=self.r2,
-                               keep_first=self.keep_first)
+                               keep_first=self.keep_first, sinks=self.sinks)
         return linear_f32(self.rt, out, self.w_o)
