@@ -318,13 +318,33 @@ def betepel_shape(width, heads, kv_heads, ff, layers, vocab, chunk):
     return {"architecture": "Betepel", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "logit_scale": 0.5, "layers": out}
 
 
+def pibuvik_shape(width, heads, kv_heads, ff, layers, vocab, chunk):
+    """A Pibuvik of sizes that resemble a real model's layers, in the order gated unit recurrence (as many channels as
+    the width, parts of 128, four taps), attention whose values are its keys (heads of 64), attention through a
+    latent of 256 values with a rotated part of 32 (heads of 64, queries through a latent of three quarters of the
+    width, a window of the chunk's size), attention on that layer's latents; the Llama layer's feed-forward."""
+    latent = {"heads": heads, "dim": 64, "rot_dim": 32, "vdim": 64, "kv_rank": 256, "q_rank": 3 * width // 4,
+              "mask": {"size": chunk}, "rot": {"base": 5e5, "dims": 32}, "scale": 96 ** -0.5}
+    mixers = {"rglru": {"width": width, "blocks": width // 128, "conv": 4},
+              "attention": {"heads": heads, "kv_heads": kv_heads, "dim": 64, "vdim": 64, "scale": 0.125,
+                            "q_temp": {"coef": 0.3, "every": 2048}},
+              "latent_attention": latent}
+    order = ["rglru", "attention", "latent_attention", "latent_attention"]
+    out = []
+    for i in range(layers):
+        mixer = dict(latent, kv_from=i - 1) if i % 4 == 3 else mixers[order[i % 4]]
+        out.append({"type": order[i % 4], "mixer": mixer, "mlp": {"kind": "dense", "ff": ff, "limit": 7.0}})
+    return {"architecture": "Pibuvik", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": 3.0},
+            "residual_mult": 0.3, "logit_scale": 0.5, "layers": out}
+
+
 DESIGN_SIZES = {  # width, heads (of 64), kv heads, feed-forward, layers, vocabulary, attention chunk
     "1024": (1024, 16, 4, 4096, 8, 32000, 1024),
     "2048": (2048, 32, 8, 8192, 8, 32000, 2048),
 }
 
 
-BESIDE = {"miberax": "makodra and ", "zarinex": "miberax and ", "betepel": "miberax and "}
+BESIDE = {"miberax": "makodra and ", "zarinex": "miberax and ", "betepel": "miberax and ", "pibuvik": "zarinex and "}
 
 
 def design_compare(args):
@@ -338,8 +358,10 @@ def design_compare(args):
     for name in args.design_sizes.split(","):
         width, heads, kv_heads, ff, layers, vocab, chunk = DESIGN_SIZES[name]
         shapes = {
+            **({"pibuvik": pibuvik_shape(width, heads, kv_heads, ff, layers, vocab, chunk)} if args.design == "pibuvik" else {}),
             **({"betepel": betepel_shape(width, heads, kv_heads, ff, layers, vocab, chunk)} if args.design == "betepel" else {}),
-            **({"zarinex": zarinex_shape(width, heads, kv_heads, ff, layers, vocab, chunk)} if args.design == "zarinex" else {}),
+            **({"zarinex": zarinex_shape(width, heads, kv_heads, ff, layers, vocab, chunk)}
+               if args.design in ("zarinex", "pibuvik") else {}),
             **({"miberax": miberax_shape(width, heads, kv_heads, ff, layers, vocab, chunk)}
                if args.design in ("miberax", "zarinex", "betepel") else {}),
             **({"makodra": makodra_shape(width, heads, kv_heads, ff, layers, vocab, chunk)}
@@ -458,13 +480,13 @@ def main() -> int:
                     help="prompt length of --only-prefill (the line of the default run always has 2,048)")
     ap.add_argument("--portion", type=int, default=None,
                     help="with --only-prefill: the prompt runs in steps of at most this many tokens")
-    ap.add_argument("--design", default=None, choices=["makodra", "miberax", "zarinex", "betepel"],
+    ap.add_argument("--design", default=None, choices=["makodra", "miberax", "zarinex", "betepel", "pibuvik"],
                     help="instead of the default run: prefill (2,048 and 8,192 tokens) and decode (batch 1, 8, 64 at "
                          "--context) of this design beside the Llama decoder at equal sizes, random weights")
     ap.add_argument("--design-sizes", default="1024,2048", help="widths of --design, of " + ", ".join(DESIGN_SIZES))
     ap.add_argument("--design-phases", default="prefill2048,prefill8192,decode_b1,decode_b8,decode_b64",
                     help="with --design: which of these measurements to make")
-    ap.add_argument("--design-only", default=None, choices=["makodra", "miberax", "zarinex", "betepel", "llama"],
+    ap.add_argument("--design-only", default=None, choices=["makodra", "miberax", "zarinex", "betepel", "pibuvik", "llama"],
                     help="with --design: measure this one of the pair alone (for profiling)")
     args = ap.parse_args()
     if args.gpus != 1:

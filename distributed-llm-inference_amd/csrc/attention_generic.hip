@@ -654,6 +654,16 @@ extern "C" int dli_attention_scored_single(const void* q, int64_t q_stride, cons
                           chunk, sink, r1, r2, gate, gate_stride, keep_first, v_heads, out32, sinks, parts, splits, is_bf16, stream);
 }
 
+// The merge alone, for another kernel that leaves its shares in this layout.
+extern "C" int dli_attention_scored_merge_bf16(const float* parts, int splits, int entries, int q_heads, int value_dim,
+                                               void* out, int64_t out_stride, hipStream_t stream) {
+  if (entries <= 0) return DLI_OK;
+  if (parts == nullptr || splits < 1 || q_heads <= 0 || q_heads > 65535 || value_dim <= 0) return DLI_ERR_ARGUMENT;
+  attention_scored_merge_kernel<bf16_t><<<dim3(entries, q_heads), value_dim <= 64 ? 64 : value_dim <= 128 ? 128 : 256, 0, stream>>>(
+      parts, splits, q_heads, value_dim, nullptr, 0, (bf16_t*)out, out_stride, nullptr);
+  return dli_launch_status();
+}
+
 extern "C" int dli_attention_generic(const void* q, int64_t q_stride, const void* k_pages,
                                      const void* v_pages, void* out, int64_t out_stride,
                                      const int* q_start, const int* kv_len, const int* block_tables,

@@ -110,6 +110,11 @@ _SIGNATURES = {
     "dli_attention_scored_mfma": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr,
                                   _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _c_ptr,
                                   _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr],
+    "dli_attention_keyvalue_supports": [_c_int, _c_int],
+    "dli_attention_keyvalue_tile_tokens": [_c_int, _c_int],
+    "dli_attention_keyvalue_splits": [_c_int, _c_int, _c_int],
+    "dli_attention_keyvalue": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int,
+                               _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr],
     "dli_embed_sinusoid": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_float, _c_int, _c_ptr],
     "dli_norm_stream_norm": [_c_ptr, _c_i64, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_int, _c_int, _c_int, _c_ptr],
     "dli_cast_from_f32": [_c_ptr, _c_ptr, _c_i64, _c_int, _c_ptr],
@@ -1739,6 +1744,61 @@ def attention_scored_mfma(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch
         kv_heads, head_dim, value_dim, page_size, float(scale), int(window), int(chunk), int(bool(sink)), _ptr(r1),
         _ptr(r2), _ptr(gate), gate_stride, int(keep_first), v_heads, _ptr(out if out32 else None), _ptr(sinks), _stream()),
         "attention_scored_mfma")
+
+
+def attention_keyvalue_supports(head_dim: int, value_dim: int, dtype: torch.dtype) -> bool:
+    return dtype == torch.bfloat16 and bool(library().dli_attention_keyvalue_supports(int(head_dim), int(value_dim)))
+
+
+def attention_keyvalue_tile_tokens(q_heads: int, kv_heads: int) -> int:
+    return int(library().dli_attention_keyvalue_tile_tokens(int(q_heads), int(kv_heads)))
+
+
+def attention_keyvalue(q: torch.Tensor, k_pages: torch.Tensor, out: torch.Tensor, q_start: torch.Tensor, kv_len: torch.Tensor,
+                       block_tables: torch.Tensor, tile_entry: Optional[torch.Tensor], tile_q0: Optional[torch.Tensor],
+                       q_heads: int, scale: float, *, window: int = 0, sinks: Optional[torch.Tensor] = None,
+                       splits: Optional[int] = None) -> None:
+    """Paged causal attention whose values are the first ``out.shape[1] / q_heads`` components of its keys, bfloat16 on
+    the matrix cores (sizes that :func:`attention_keyvalue_supports` takes): tiles of
+    :func:`attention_keyvalue_tile_tokens` tokens, or without tile lists every entry one row (an entry's keys then
+    cut over several workgroups, as many as ``splits`` says or the heads and the number of entries decide).
+    ``window``: only the last so many keys are seen; ``sinks`` (float32 ``[q_heads]``): ``exp(sinks[h])`` in the denominator."""
+    _dense(k_pages, "k_pages", torch.bfloat16, 4)
+    _rows(q, "q", torch.bfloat16)
+    _rows(out, "out", torch.bfloat16)
+    _, kv_heads, page_size, head_dim = k_pages.shape
+    _require(q_heads % kv_heads == 0 and q.shape[1] == q_heads * head_dim and out.shape[0] == q.shape[0]
+             and out.shape[1] % q_heads == 0, "q must be [tokens, q_heads*head_dim], out [tokens, q_heads*value_dim]")
+    value_dim = out.shape[1] // q_heads
+    _require(attention_keyvalue_supports(head_dim, value_dim, k_pages.dtype), "the matrix-core kernel does not take these sizes")
+    _require(q.stride(0) % 8 == 0 and out.stride(0) % 4 == 0 and q.data_ptr() % 16 == 0 and k_pages.data_ptr() % 16 == 0
+             and out.data_ptr() % 8 == 0, "q and the pages must be aligned for eight values at once, out for four")
+    for name, t in (("q_start", q_start), ("kv_len", kv_len)):
+        _dense(t, name, torch.int32, 1)
+    _dense(block_tables, "block_tables", torch.int32, 2)
+    entries = kv_len.shape[0]
+    _require(q_start.shape[0] == entries + 1 and block_tables.shape[0] >= entries,
+             "q_start/kv_len/block_tables disagree on the number of requests")
+    parts = None
+    if tile_entry is None:
+        _require(tile_q0 is None and q.shape[0] == entries, "without tile lists every entry must be one row")
+        tiles = entries
+        if splits is None:
+            splits = int(library().dli_attention_keyvalue_splits(q_heads, kv_heads, max(entries, 1)))
+        if splits > 1:
+            parts = torch.empty(entries * q_heads * splits * (value_dim + 2), device=q.device, dtype=torch.float32)
+    else:
+        _dense(tile_entry, "tile_entry", torch.int32, 1)
+        _dense(tile_q0, "tile_q0", torch.int32, 1)
+        _require(tile_entry.shape == tile_q0.shape and splits in (None, 1), "tile lists differ in length, or tiles with splits")
+        tiles, splits = tile_entry.shape[0], 1
+    if sinks is not None:
+        _dense(sinks, "sinks", torch.float32, 1)
+        _require(sinks.shape[0] == q_heads, "sinks must hold one value per query head")
+    _check(library().dli_attention_keyvalue(
+        _ptr(q), q.stride(0), _ptr(k_pages), _ptr(out), out.stride(0), _ptr(q_start), _ptr(kv_len), _ptr(block_tables),
+        block_tables.stride(0), _ptr(tile_entry), _ptr(tile_q0), tiles, q_heads, kv_heads, head_dim, value_dim, page_size,
+        float(scale), int(window), _ptr(sinks), _ptr(parts), splits, _stream()), "attention_keyvalue")
 
 
 RULE_DELTA, RULE_BONUS = 0, 1

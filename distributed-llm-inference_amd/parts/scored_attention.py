@@ -64,6 +64,17 @@ def paged_scored_attention(rt: Runtime, ctx: Any, cache: Any, q: torch.Tensor, o
     values are the keys' first ``value_dim`` components."""
     grp = ctx.groups[cache.group]
     nd = ctx.num_decode
+    if cache.v_pages is None and gate is None and _keyvalue_takes(rt, head_dim, value_dim, out, changes):
+        # values that are keys, bfloat16: the matrix cores, single tokens (which come first) apart from portions
+        own = {n: changes[n] for n in ("window", "sinks") if n in changes}
+        if nd:
+            ops.attention_keyvalue(q[:nd], cache.k_pages, out[:nd], ctx.q_start[:nd + 1], ctx.kv_len[:nd],
+                                   grp.block_tables[:nd], None, None, num_heads, scale, **own)
+        if nd < ctx.num_entries:
+            tiles = ctx.q_tiles(ops.attention_keyvalue_tile_tokens(num_heads, cache.k_pages.shape[1]), first_entry=nd)
+            ops.attention_keyvalue(q, cache.k_pages, out, ctx.q_start, ctx.kv_len, grp.block_tables, tiles[0], tiles[1],
+                                   num_heads, scale, **own)
+        return
     if nd == ctx.num_entries:
         # every entry is one row: nothing is derived from the step's lengths on the host
         ops.attention_scored(q, cache.k_pages, cache.v_pages, out, ctx.q_start, ctx.kv_len, grp.block_tables,
@@ -80,6 +91,14 @@ def paged_scored_attention(rt: Runtime, ctx: Any, cache: Any, q: torch.Tensor, o
         tiles = ctx.q_tiles(ops.attention_generic_tile_rows(max(head_dim, value_dim)))
         ops.attention_scored(q, cache.k_pages, cache.v_pages, out, ctx.q_start, ctx.kv_len, grp.block_tables,
                              tiles[0], tiles[1], num_heads, scale, gate=gate, **changes)
+
+
+def _keyvalue_takes(rt: Runtime, head_dim: int, value_dim: int, out: torch.Tensor, changes: Mapping[str, Any]) -> bool:
+    """Whether the matrix-core kernel for values that are keys computes this attention: its sizes, and no change to
+    the scores but a window and a sink per head."""
+    others = any(bool(v) if not isinstance(v, torch.Tensor) else True
+                 for n, v in changes.items() if n not in ("window", "sinks") and v is not None)
+    return not others and out.dtype == rt.dtype and ops.attention_keyvalue_supports(head_dim, value_dim, rt.dtype)
 
 
 @register_part("mixer", "scored_attention")
