@@ -73,7 +73,7 @@ def test_config_is_read_and_becomes_parts():
     specs = model.cache_specs()
     assert len(specs) == 5
     assert specs[0] == specs[4] == CompositeCacheSpec((shift, ("inner", StateSpec((40 * 5 + 3 * 40,), torch.float32))))
-    assert specs[1] == specs[3] == CompositeCacheSpec((shift, ("inner", PagedKVSpec(1, 20, 0))))
+    assert specs[1] == specs[3] == CompositeCacheSpec((shift, ("inner", PagedKVSpec(1, 20, 0, 0))))
     assert specs[2] == CompositeCacheSpec((shift, ("inner", StateSpec((2 * 6 * 8,), torch.float32))))
     assert model.head.tied and model.embedding.float32_rows
 
