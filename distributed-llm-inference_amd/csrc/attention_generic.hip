@@ -476,27 +476,39 @@ __global__ __launch_bounds__(512) void attention_scored_decode_kernel(
   }
 }
 
-// The shares of the workgroups that split an entry's keys meet: parts [entries][q_heads][splits][value_dim + 2].
-// One workgroup an (entry, head), a thread a value column; sums in the order of the splits.
+// The shares of the workgroups that split an entry's keys meet: parts [entries][q_heads][splits][value_dim + 2],
+// at most 64 splits. One workgroup an (entry, head), a thread a value column; the shares' factors are made once, by the
+// first wave, a lane a share; sums in the order of the splits.
 template <typename T>
 __global__ void attention_scored_merge_kernel(const float* __restrict__ parts, int splits, int q_heads, int value_dim,
                                               const float* __restrict__ gate, int64_t gate_stride, T* __restrict__ out,
                                               int64_t out_stride, float* __restrict__ out32) {
+  __shared__ float factor[64];
   const int entry = blockIdx.x, head = blockIdx.y;
-  const float* base = parts + ((int64_t)entry * q_heads + head) * splits * (value_dim + 2);
-  float m = -INFINITY;
-  for (int s = 0; s < splits; ++s) m = fmaxf(m, base[s * (value_dim + 2) + value_dim]);
+  const int64_t width = value_dim + 2;
+  const float* base = parts + ((int64_t)entry * q_heads + head) * splits * width;
+  if (threadIdx.x < 64) {
+    const int s = threadIdx.x;
+    const float ms = s < splits ? base[s * width + value_dim] : -INFINITY;
+    const float ls = s < splits ? base[s * width + value_dim + 1] : 0.f;
+    const float m = wave_max(ms);
+    const float f = ms > -INFINITY ? expf(ms - m) : 0.f;
+    const float l = wave_sum(ls * f);
+    factor[s] = l > 0.f ? f / l : 0.f;
+  }
+  __syncthreads();
   for (int col = threadIdx.x; col < value_dim; col += blockDim.x) {
-    float l = 0.f, o = 0.f;
-    for (int s = 0; s < splits; ++s) {
-      const float ms = base[s * (value_dim + 2) + value_dim];
-      if (ms > -INFINITY) {
-        const float f = expf(ms - m);
-        l += base[s * (value_dim + 2) + value_dim + 1] * f;
-        o += base[s * (value_dim + 2) + col] * f;
-      }
+    float o = 0.f;
+    int s = 0;
+    for (; s + 4 <= splits; s += 4) {
+      float p[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) p[e] = base[(s + e) * width + col];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) o = fmaf(p[e], factor[s + e], o);
     }
-    float y = l > 0.f ? o / l : 0.f;
+    for (; s < splits; ++s) o = fmaf(base[s * width + col], factor[s], o);
+    float y = o;
     const int64_t at = (int64_t)head * value_dim + col;
     if (gate != nullptr) y *= 1.f / (1.f + expf(-gate[(int64_t)entry * gate_stride + at]));
     if (out32 != nullptr) out32[(int64_t)entry * out_stride + at] = y;
@@ -658,7 +670,7 @@ extern "C" int dli_attention_scored_single(const void* q, int64_t q_stride, cons
 extern "C" int dli_attention_scored_merge_bf16(const float* parts, int splits, int entries, int q_heads, int value_dim,
                                                void* out, int64_t out_stride, hipStream_t stream) {
   if (entries <= 0) return DLI_OK;
-  if (parts == nullptr || splits < 1 || q_heads <= 0 || q_heads > 65535 || value_dim <= 0) return DLI_ERR_ARGUMENT;
+  if (parts == nullptr || splits < 1 || splits > 64 || q_heads <= 0 || q_heads > 65535 || value_dim <= 0) return DLI_ERR_ARGUMENT;
   attention_scored_merge_kernel<bf16_t><<<dim3(entries, q_heads), value_dim <= 64 ? 64 : value_dim <= 128 ? 128 : 256, 0, stream>>>(
       parts, splits, q_heads, value_dim, nullptr, 0, (bf16_t*)out, out_stride, nullptr);
   return dli_launch_status();

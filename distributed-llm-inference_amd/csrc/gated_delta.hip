@@ -159,6 +159,92 @@ __global__ void causal_conv_kernel(const float* __restrict__ x, int64_t stride, 
   if (rounded != nullptr) rounded[(int64_t)row * rounded_stride + c] = from_f32<T>(acc);
 }
 
+// Every entry one row (a step of single tokens): the thread that reads a channel's kept inputs also moves them on.
+template <typename T>
+__global__ void causal_conv_single_kernel(const float* __restrict__ x, int64_t stride, const float* __restrict__ conv_w,
+                                          const float* __restrict__ bias, float* kept_base, int64_t state_stride,
+                                          const int* __restrict__ positions, const int* __restrict__ state_slots,
+                                          float* __restrict__ out, int64_t out_stride, T* __restrict__ rounded,
+                                          int64_t rounded_stride, int channels, int taps, int act,
+                                          const float* __restrict__ in_bias) {
+  const int row = blockIdx.x, c = blockIdx.y * blockDim.x + threadIdx.x;
+  if (c >= channels) return;
+  float* kept = kept_base + (int64_t)state_slots[row] * state_stride + c;
+  const int pos = positions[row];
+  const float now = x[(int64_t)row * stride + c] + (in_bias != nullptr ? in_bias[c] : 0.f);
+  float acc = bias != nullptr ? bias[c] : 0.f, old[GD_MAX_TAPS];
+  for (int i = 0; i < taps - 1; ++i)                             // kept row i: the input taps - 1 - i places back
+    old[i] = pos - (taps - 1 - i) >= 0 ? kept[(int64_t)i * channels] : 0.f;
+  for (int i = 0; i < taps - 1; ++i) acc = fmaf(conv_w[(int64_t)c * taps + i], old[i], acc);   // oldest input first
+  acc = fmaf(conv_w[(int64_t)c * taps + taps - 1], now, acc);
+  for (int i = 0; i + 1 < taps - 1; ++i) kept[(int64_t)i * channels] = old[i + 1];
+  if (taps > 1) kept[(int64_t)(taps - 2) * channels] = now;
+  if (act == 1) acc = acc / (1.f + expf(-acc));
+  out[(int64_t)row * out_stride + c] = acc;
+  if (rounded != nullptr) rounded[(int64_t)row * rounded_stride + c] = from_f32<T>(acc);
+}
+
+// The same as causal_conv, a thread RUN neighbouring rows of a channel: an input is read once for all rows it reaches where the run
+// lies in one entry with its inputs among the step's rows; other runs take the rows one by one. TAPS at least `taps`.
+template <typename T, int TAPS, int RUN>
+__global__ __launch_bounds__(256) void causal_conv_run_kernel(const float* __restrict__ x, int64_t stride,
+                                                              const float* __restrict__ conv_w, const float* __restrict__ bias,
+                                                              const float* kept_base, int64_t state_stride,
+                                                              const int* __restrict__ q_start, int entries,
+                                                              const int* __restrict__ positions,
+                                                              const int* __restrict__ state_slots, float* __restrict__ out,
+                                                              int64_t out_stride, T* __restrict__ rounded, int64_t rounded_stride,
+                                                              int rows, int channels, int taps, int act,
+                                                              const float* __restrict__ in_bias) {
+  const int row0 = blockIdx.x * RUN, c = blockIdx.y * 256 + threadIdx.x;
+  if (c >= channels) return;
+  const float ib = in_bias != nullptr ? in_bias[c] : 0.f, b = bias != nullptr ? bias[c] : 0.f;
+  float w[TAPS];                                                // w[j]: the input j places back
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j) w[j] = j < taps ? conv_w[(int64_t)c * taps + (taps - 1 - j)] : 0.f;
+  const int e0 = gd_entry_of_row(q_start, entries, row0);
+  const bool inside = row0 - (TAPS - 1) >= q_start[e0] && row0 + RUN <= q_start[e0 + 1];
+  float y[RUN];
+  if (inside) {                                                 // (the same for the whole workgroup)
+    float in[RUN + TAPS - 1];
+#pragma unroll
+    for (int k = 0; k < RUN + TAPS - 1; ++k) in[k] = x[(int64_t)(row0 - (TAPS - 1) + k) * stride + c] + ib;
+#pragma unroll
+    for (int r = 0; r < RUN; ++r) {
+      y[r] = b;
+#pragma unroll
+      for (int j = TAPS - 1; j >= 0; --j) y[r] = fmaf(w[j], in[r + TAPS - 1 - j], y[r]);   // oldest input first
+    }
+  } else {
+    for (int r = 0; r < RUN; ++r) {
+      const int row = row0 + r;
+      float acc = b;
+      if (row < rows) {
+        const int e = gd_entry_of_row(q_start, entries, row);
+        const int first = q_start[e], pos = positions[row];
+        const float* kept = kept_base + (int64_t)state_slots[e] * state_stride;
+#pragma unroll
+        for (int j = TAPS - 1; j >= 0; --j)
+          if (j < taps && pos - j >= 0) {
+            const int src = row - j;
+            acc = fmaf(w[j], src >= first ? x[(int64_t)src * stride + c] + ib : kept[(int64_t)(taps - 1 - (first - src)) * channels + c], acc);
+          }
+      }
+#pragma unroll
+      for (int q = 0; q < RUN; ++q) y[q] = q == r ? acc : y[q];
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < RUN; ++r) {
+    const int row = row0 + r;
+    if (row >= rows) break;
+    float v = y[r];
+    if (act == 1) v = v / (1.f + expf(-v));
+    out[(int64_t)row * out_stride + c] = v;
+    if (rounded != nullptr) rounded[(int64_t)row * rounded_stride + c] = from_f32<T>(v);
+  }
+}
+
 struct GdArgs {
   const float* prep; int64_t stride;   // [rows][stride]: q | k | v | beta | g as conv_prepare leaves them
   float* state; int64_t state_stride;
@@ -347,6 +433,25 @@ int dli_causal_conv(const float* x, int64_t stride, const float* conv_w, const f
     return DLI_ERR_ARGUMENT;
   const dim3 grid(rows, (channels + 255) / 256);
   if (grid.y > 65535) return DLI_ERR_ARGUMENT;
+  if (rows == entries) {
+#define CONV_SINGLE(T)                                                                                                 \
+  causal_conv_single_kernel<T><<<grid, 256, 0, stream>>>(x, stride, conv_w, bias, state + kept_offset, state_stride,   \
+                                                         positions, state_slots, out, out_stride, (T*)rounded,         \
+                                                         rounded_stride, channels, taps, act, in_bias)
+    if (rounded_is_bf16) CONV_SINGLE(bf16_t);
+    else CONV_SINGLE(float);
+#undef CONV_SINGLE
+    return dli_launch_status();
+  }
+#define CONV_RUN(T, TAPS)                                                                                              \
+  causal_conv_run_kernel<T, TAPS, 8><<<dim3((rows + 7) / 8, grid.y), 256, 0, stream>>>(                                \
+      x, stride, conv_w, bias, state + kept_offset, state_stride, q_start, entries, positions, state_slots, out,      \
+      out_stride, (T*)rounded, rounded_stride, rows, channels, taps, act, in_bias)
+  if (taps <= 4 && rows >= 8 * entries && rows >= 256) {       // portions: runs of rows
+    if (rounded_is_bf16) CONV_RUN(bf16_t, 4);
+    else CONV_RUN(float, 4);
+  } else
+#undef CONV_RUN
   if (rounded_is_bf16)
     causal_conv_kernel<bf16_t><<<grid, 256, 0, stream>>>(x, stride, conv_w, bias, state + kept_offset, state_stride, q_start,
                                                          entries, positions, state_slots, out, out_stride, (bf16_t*)rounded,

@@ -38,28 +38,44 @@ struct GuArgs {
   int rows, entries, C, s, blocks;
 };
 
-__device__ __forceinline__ float gu_sigmoid(float x) { return 1.f / (1.f + expf(-x)); }
+// (the hardware's exp2, reciprocal and square root are good to an ulp or so; the step is held by their number)
+__device__ __forceinline__ float gu_sigmoid(float x) { return __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
 __device__ __forceinline__ float gu_gelu(float z) {
-  return z / (1.f + expf(-1.5957691216057308f * (z + 0.044715f * z * z * z)));   // 2 sqrt(2 / pi)
+  return z * gu_sigmoid(1.5957691216057308f * (z + 0.044715f * z * z * z));      // 2 sqrt(2 / pi)
 }
-// a and the recurrence's input from the gates' pre-activations
+// a and the recurrence's input from the gates' pre-activations. 1 - a^2 = 1 - exp(-t), t = 2 r decay: near t = 0 by its
+// Taylor series (the next term is below 2e-8 of the sum at t = 1/4), where a^2 would lose what is left of it.
 __device__ __forceinline__ void gu_gates(float r_pre, float i_pre, float u, float decay, float* a, float* in) {
-  const float x = gu_sigmoid(r_pre) * decay;
-  *a = expf(-x);
-  *in = sqrtf(-expm1f(-2.f * x)) * gu_sigmoid(i_pre) * u;
+  const float x = gu_sigmoid(r_pre) * decay, t = 2.f * x;
+  *a = __expf(-x);
+  const float series = t * (1.f - t * (1.f / 2) * (1.f - t * (1.f / 3) * (1.f - t * (1.f / 4) * (1.f - t * (1.f / 5) *
+                       (1.f - t * (1.f / 6) * (1.f - t * (1.f / 7)))))));
+  const float rest = t < 0.25f ? series : fmaf(-*a, *a, 1.f);
+  *in = __builtin_amdgcn_sqrtf(rest) * gu_sigmoid(i_pre) * u;
 }
 
-// One token of one entry at channel c.
+// What a single token's step at channel c reads besides the gates, asked for before they are made.
+struct GuSingle {
+  float u, y, old;
+  float* state;
+  bool fresh;
+};
+__device__ __forceinline__ GuSingle gu_single_read(const GuArgs& p, int row, int c) {
+  GuSingle x;
+  x.u = p.u[(int64_t)row * p.u_stride + c];
+  x.y = p.y[(int64_t)row * p.y_stride + c];
+  x.state = p.state + (int64_t)p.state_slots[row] * p.state_stride + c;
+  x.old = *x.state;
+  x.fresh = p.positions[row] == 0;
+  return x;
+}
 template <typename T>
-__device__ __forceinline__ void gu_single(const GuArgs& p, int row, int c, float r_pre, float i_pre) {
+__device__ __forceinline__ void gu_single_step(const GuArgs& p, const GuSingle& x, int row, int c, float r_pre, float i_pre) {
   float a, in;
-  gu_gates(r_pre + p.br[c], i_pre + p.bi[c], p.u[(int64_t)row * p.u_stride + c], p.decay[c], &a, &in);
-  float* st = p.state + (int64_t)p.state_slots[row] * p.state_stride + c;
-  const float old = *st;
-  const float S = fmaf(a, p.positions[row] == 0 ? 0.f : old, in);
-  *st = S;
-  ((T*)p.out)[(int64_t)row * p.out_stride + c] =
-      from_f32<T>(S * gu_gelu(p.y[(int64_t)row * p.y_stride + c] + (p.y_bias != nullptr ? p.y_bias[c] : 0.f)));
+  gu_gates(r_pre + p.br[c], i_pre + p.bi[c], x.u, p.decay[c], &a, &in);
+  const float S = fmaf(a, x.fresh ? 0.f : x.old, in);
+  *x.state = S;
+  ((T*)p.out)[(int64_t)row * p.out_stride + c] = from_f32<T>(S * gu_gelu(x.y + (p.y_bias != nullptr ? p.y_bias[c] : 0.f)));
 }
 
 // Eight floats as the sum of three bfloat16 vectors.
@@ -106,35 +122,66 @@ __global__ __launch_bounds__(64 * WAVES) void gated_unit_mfma_kernel(GuArgs p) {
   for (int t = 0; t < TB; ++t)
 #pragma unroll
     for (int n = 0; n < NC; ++n) ar[t][n] = ai[t][n] = gu_f4{0.f, 0.f, 0.f, 0.f};
-  for (int k0 = 0; k0 < s; k0 += 32) {
-    const int at = k0 + 8 * grp;
-    const bool in = at < s;                     // (s is a multiple of 8)
-    gu_bf8 br[NC], bi[NC];
+  GuSingle single[SINGLE ? 4 : 1][SINGLE ? NC : 1];
+  if constexpr (SINGLE) {
 #pragma unroll
-    for (int n = 0; n < NC; ++n) {
-      br[n] = *reinterpret_cast<const gu_bf8*>(wr[n] + (in ? at : 0));
-      bi[n] = *reinterpret_cast<const gu_bf8*>(wi[n] + (in ? at : 0));
-      if (!in) br[n] = bi[n] = gu_bf8{};
-    }
+    for (int n = 0; n < NC; ++n)
 #pragma unroll
-    for (int t = 0; t < TB; ++t) {
-      const float* ur = p.u + (int64_t)(row0 + min(16 * t + col, n_rows - 1)) * p.u_stride + (int64_t)block * s + (in ? at : 0);
-      float x[8];
+      for (int i = 0; i < 4; ++i)               // (rows and outputs past the last are the last again; nothing is stored for them)
+        single[i][n] = gu_single_read(p, row0 + min(4 * grp + i, n_rows - 1), block * s + min(n0 + 16 * n + col, s - 1));
+  }
+  // KU steps of 32 k are asked for at once, and the next KU before these are multiplied
+  constexpr int KU = SINGLE ? 4 : 1;
+  struct Operands { gu_bf8 r[KU][NC], i[KU][NC]; gu_f4 u[KU][TB][2]; };
+  const float* ur[TB];
 #pragma unroll
-      for (int e = 0; e < 8; e += 4) {
-        const gu_f4 v = *reinterpret_cast<const gu_f4*>(ur + e);
+  for (int t = 0; t < TB; ++t) ur[t] = p.u + (int64_t)(row0 + min(16 * t + col, n_rows - 1)) * p.u_stride + (int64_t)block * s;
+  auto fetch = [&](Operands& o, int k0) {
 #pragma unroll
-        for (int f = 0; f < 4; ++f) x[e + f] = in ? v[f] : 0.f;
+    for (int j = 0; j < KU; ++j) {
+      const int k = k0 + 32 * j + 8 * grp, at = k < s ? k : 0;   // (s is a multiple of 8; what lies past it counts as zero)
+#pragma unroll
+      for (int n = 0; n < NC; ++n) {
+        o.r[j][n] = *reinterpret_cast<const gu_bf8*>(wr[n] + at);
+        o.i[j][n] = *reinterpret_cast<const gu_bf8*>(wi[n] + at);
       }
-      gu_bf8 h[3];
-      gu_split(x, h);
 #pragma unroll
-      for (int j = 2; j >= 0; --j)              // the small parts first
+      for (int t = 0; t < TB; ++t)
 #pragma unroll
-        for (int n = 0; n < NC; ++n) {
-          ar[t][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(h[j], br[n], ar[t][n], 0, 0, 0);
-          ai[t][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(h[j], bi[n], ai[t][n], 0, 0, 0);
-        }
+        for (int e = 0; e < 2; ++e) o.u[j][t][e] = *reinterpret_cast<const gu_f4*>(ur[t] + at + 4 * e);
+    }
+  };
+  auto multiply = [&](const Operands& o, int k0) {
+#pragma unroll
+    for (int j = 0; j < KU; ++j) {
+      const bool in = k0 + 32 * j + 8 * grp < s;
+      if (KU > 1 && k0 + 32 * j >= s) break;
+#pragma unroll
+      for (int t = 0; t < TB; ++t) {
+        float x[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[e] = in ? o.u[j][t][e / 4][e % 4] : 0.f;
+        gu_bf8 h[3];
+        gu_split(x, h);
+#pragma unroll
+        for (int q = 2; q >= 0; --q)            // the small parts first
+#pragma unroll
+          for (int n = 0; n < NC; ++n) {
+            ar[t][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(h[q], o.r[j][n], ar[t][n], 0, 0, 0);
+            ai[t][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(h[q], o.i[j][n], ai[t][n], 0, 0, 0);
+          }
+      }
+    }
+  };
+  {
+    Operands o0, o1;
+    fetch(o0, 0);
+    for (int k0 = 0; k0 < s; k0 += 64 * KU) {
+      fetch(o1, k0 + 32 * KU);
+      multiply(o0, k0);
+      if (k0 + 32 * KU >= s) break;
+      fetch(o0, k0 + 64 * KU);
+      multiply(o1, k0 + 32 * KU);
     }
   }
   // ar[t][n][i]: token 16 t + 4 grp + i, output n0 + 16 n + col
@@ -146,7 +193,8 @@ __global__ __launch_bounds__(64 * WAVES) void gated_unit_mfma_kernel(GuArgs p) {
     if constexpr (SINGLE) {
 #pragma unroll
       for (int i = 0; i < 4; ++i)
-        if (live && 4 * grp + i < n_rows) gu_single<bf16_t>(p, row0 + 4 * grp + i, c, ar[0][n][i], ai[0][n][i]);
+        if (live && 4 * grp + i < n_rows) 
+          gu_single_step<bf16_t>(p, single[i][n], row0 + 4 * grp + i, c, ar[0][n][i], ai[0][n][i]);
     } else {
       const float cr = p.br[c], ci = p.bi[c], decay = p.decay[c];
       float P0 = 1.f, S0 = 0.f;                 // at the beginning of this part of 16 tokens
@@ -239,7 +287,7 @@ __global__ __launch_bounds__(256) void gated_unit_any_kernel(GuArgs p) {
     }
     const bool live = o < s && t0 + ty < n_rows;
     if constexpr (SINGLE) {
-      if (live) gu_single<T>(p, row0 + ty, c, ar, ai);
+      if (live) gu_single_step<T>(p, gu_single_read(p, row0 + ty, c), row0 + ty, c, ar, ai);
     } else {
       float a = 1.f, b = 0.f;
       if (live)
@@ -273,20 +321,32 @@ __global__ void gated_unit_carry_kernel(GuArgs p) {
   const float old = *st;
   float S = p.positions[row0] == 0 ? 0.f : old;
   float* e = p.ends + (int64_t)first * 2 * p.C + c;
-  for (int t0 = 0; t0 < tiles; t0 += 8) {
-    float P[8], E[8];
+  constexpr int N = 16;                         // tiles asked for at once, the next ones before these are walked
+  float P[2][N], E[2][N];
+  auto fetch = [&](int w, int t0) {
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {               // (tiles past the last repeat it)
+    for (int j = 0; j < N; ++j) {               // (tiles past the last repeat it)
       const int64_t at = (int64_t)min(t0 + j, tiles - 1) * 2 * p.C;
-      P[j] = e[at];
-      E[j] = e[at + p.C];
+      P[w][j] = e[at];
+      E[w][j] = e[at + p.C];
     }
+  };
+  auto walk = [&](int w, int t0) {
 #pragma unroll
-    for (int j = 0; j < 8; ++j)
+    for (int j = 0; j < N; ++j)
       if (t0 + j < tiles) {
         e[(int64_t)(t0 + j) * 2 * p.C] = S;
-        S = fmaf(P[j], S, E[j]);
+        S = fmaf(P[w][j], S, E[w][j]);
       }
+  };
+  fetch(0, 0);
+  for (int t0 = 0; t0 < tiles; t0 += 2 * N) {
+    // (what is fetched ahead lies past what is being written: a tile's P is read before its place is taken)
+    if (t0 + N < tiles) fetch(1, t0 + N);
+    walk(0, t0);
+    if (t0 + N >= tiles) break;
+    if (t0 + 2 * N < tiles) fetch(0, t0 + 2 * N);
+    walk(1, t0 + N);
   }
   *st = S;
 }

@@ -29,18 +29,29 @@ __global__ void latent_norm_cache_kernel(const float* __restrict__ proj, int64_t
                                          float eps, T* __restrict__ q_out, const int* __restrict__ slots,
                                          T* __restrict__ k_pages, T* __restrict__ v_pages, int page_size, int rot,
                                          const float* __restrict__ inv_freq, const int* __restrict__ positions) {
-  __shared__ float scratch[16];
+  __shared__ float scratch[2][16];
   const int64_t row = blockIdx.x;
   const float* pr = proj + row * stride;
-  float ss = 0.f;
-  for (int i = threadIdx.x; i < q_rank; i += blockDim.x) ss += pr[q_off + i] * pr[q_off + i];
-  const float rq = 1.f / sqrtf(block_sum(ss, scratch) / (float)q_rank + eps);
+  float sq = 0.f, sc = 0.f;
+  for (int i = threadIdx.x; i < q_rank; i += blockDim.x) sq += pr[q_off + i] * pr[q_off + i];
+  for (int i = threadIdx.x; i < rank; i += blockDim.x) sc += pr[c_off + i] * pr[c_off + i];
+  sq = wave_sum(sq);
+  sc = wave_sum(sc);
+  if (threadIdx.x % DLI_WAVE == 0) {
+    scratch[0][threadIdx.x / DLI_WAVE] = sq;
+    scratch[1][threadIdx.x / DLI_WAVE] = sc;
+  }
+  __syncthreads();
+  sq = sc = 0.f;
+  for (int w = 0; w < (int)blockDim.x / DLI_WAVE; ++w) {     // same order in every thread
+    sq += scratch[0][w];
+    sc += scratch[1][w];
+  }
+  const float rq = 1.f / sqrtf(sq / (float)q_rank + eps);
   for (int i = threadIdx.x; i < q_rank; i += blockDim.x)
     q_out[row * q_rank + i] = from_f32<T>(q_weight[i] * (pr[q_off + i] * rq));
   if (rank == 0) return;
-  ss = 0.f;
-  for (int i = threadIdx.x; i < rank; i += blockDim.x) ss += pr[c_off + i] * pr[c_off + i];
-  const float rc = 1.f / sqrtf(block_sum(ss, scratch) / (float)rank + eps);
+  const float rc = 1.f / sqrtf(sc / (float)rank + eps);
   const int slot = slots[row];
   if (slot < 0) return;                                // a padding row: nothing is cached
   const int64_t page = slot / page_size;
@@ -142,8 +153,9 @@ __global__ __launch_bounds__(256) void head_products_kernel(HeadProductArgs p) {
 }
 
 // On the matrix cores, in transposed form, out^T = M_h x^T (v_mfma_f32_16x16x32_bf16: lane l supplies row l%16 of
-// either operand and the k-indices 8 (l/16) .. + 7): a lane ends with four neighbouring outputs of one row. A wave
-// takes 16 MB outputs of 16 RB rows of one head, every operand straight from memory, 16 bytes a lane.
+// either operand and the k-indices 8 (l/16) .. + 7). A wave takes 16 MB outputs of 16 RB rows of one head, every operand
+// straight from memory, 16 bytes a lane. Which output is which row of a product is free: output
+// n0 + 4 MB (j/4) + 4 a + j%4 is row j of product a, so a lane ends with 4 MB neighbouring outputs of one row.
 template <int MB, int RB, int WAVES>
 __global__ __launch_bounds__(64 * WAVES) void head_products_mfma_kernel(HeadProductArgs p) {
   const int lane = threadIdx.x % 64, wave = threadIdx.x / 64, col = lane & 15, grp = lane >> 4;
@@ -158,7 +170,7 @@ __global__ __launch_bounds__(64 * WAVES) void head_products_mfma_kernel(HeadProd
   const bf16_t* wr[MB];
   const bf16_t* xr[RB];
 #pragma unroll
-  for (int b = 0; b < MB; ++b) wr[b] = wh + (int64_t)min(n0 + 16 * b + col, p.m - 1) * p.k;
+  for (int b = 0; b < MB; ++b) wr[b] = wh + (int64_t)min(n0 + 4 * MB * (col / 4) + 4 * b + col % 4, p.m - 1) * p.k;
 #pragma unroll
   for (int b = 0; b < RB; ++b)
     xr[b] = (const bf16_t*)p.x + (int64_t)min(r0 + 16 * b + col, p.rows - 1) * p.x_stride + (int64_t)head * p.x_head;
@@ -194,7 +206,7 @@ __global__ __launch_bounds__(64 * WAVES) void head_products_mfma_kernel(HeadProd
     const float g1 = p.gate_per_head ? hp_gate(p, r, head, 0) : 1.f;
 #pragma unroll
     for (int a = 0; a < MB; ++a) {
-      const int n = n0 + 16 * a + 4 * grp;
+      const int n = n0 + 4 * MB * grp + 4 * a;
       if (n >= p.m) continue;                       // (m is a multiple of four)
       hp_bf4 y;
 #pragma unroll
@@ -216,7 +228,7 @@ int dli_latent_norm_cache(const float* proj, int64_t stride, int q_off, int q_ra
       (rot > 0 && (rank == 0 || inv_freq == nullptr || positions == nullptr || v_pages != nullptr)))
     return DLI_ERR_ARGUMENT;
   const int widest = q_rank > rank ? q_rank : rank;
-  const int threads = widest >= 1024 ? 256 : widest >= 256 ? 128 : 64;
+  const int threads = widest >= 1024 ? 512 : widest >= 256 ? 256 : 64;
   if (is_bf16)
     latent_norm_cache_kernel<bf16_t><<<rows, threads, 0, stream>>>(
         proj, stride, q_off, q_rank, c_off, rank, q_weight, c_weight, eps, (bf16_t*)q_out, slots, (bf16_t*)k_pages,

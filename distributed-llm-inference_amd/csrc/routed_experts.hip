@@ -58,6 +58,25 @@ __global__ void clamped_glu_kernel(const T* __restrict__ gate_up, int64_t stride
     out[row * ff + i] = from_f32<T>(clamped_glu(to_f32(gate_up[row * stride + i]), to_f32(gate_up[row * stride + ff + i]), limit, alpha, up_shift));
 }
 
+// Eight neighbours a thread (rows and sizes of whole 16 bytes).
+__global__ __launch_bounds__(256) void clamped_glu_bf16x8_kernel(const bf16_t* __restrict__ gate_up, int64_t stride,
+                                                                 bf16_t* __restrict__ out, int ff, float limit, float alpha,
+                                                                 float up_shift) {
+  typedef __bf16 b8 __attribute__((ext_vector_type(8)));
+  const int64_t row = blockIdx.x;
+  const int i = 8 * (blockIdx.y * 256 + threadIdx.x);
+  if (i >= ff) return;
+  const b8 g = *reinterpret_cast<const b8*>(gate_up + row * stride + i);
+  const b8 u = *reinterpret_cast<const b8*>(gate_up + row * stride + ff + i);
+  b8 y;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const float a = fminf((float)g[e], limit), b = fminf(fmaxf((float)u[e], -limit), limit);
+    y[e] = (bf16_t)(a * __builtin_amdgcn_rcpf(1.f + __expf(-alpha * a)) * (b + up_shift));
+  }
+  *reinterpret_cast<b8*>(out + row * ff + i) = y;
+}
+
 // The better of two (value, index) pairs: the larger value, the lower index on a tie.
 __device__ __forceinline__ void wave_argmax(float& v, int& i) {
 #pragma unroll
@@ -486,7 +505,10 @@ int dli_clamped_glu(const void* gate_up, int64_t stride, void* out, int rows, in
   if (rows <= 0) return DLI_OK;
   if (ff <= 0 || stride < 2 * (int64_t)ff) return DLI_ERR_ARGUMENT;
   const dim3 grid(rows, (ff + 255) / 256);
-  if (is_bf16) clamped_glu_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)gate_up, stride, (bf16_t*)out, ff, limit, alpha, up_shift);
+  if (is_bf16 && ff % 8 == 0 && stride % 8 == 0 && ((uintptr_t)gate_up | (uintptr_t)out) % 16 == 0)
+    clamped_glu_bf16x8_kernel<<<dim3(rows, (ff / 8 + 255) / 256), 256, 0, stream>>>((const bf16_t*)gate_up, stride, (bf16_t*)out,
+                                                                                   ff, limit, alpha, up_shift);
+  else if (is_bf16) clamped_glu_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)gate_up, stride, (bf16_t*)out, ff, limit, alpha, up_shift);
   else clamped_glu_kernel<float><<<grid, 256, 0, stream>>>((const float*)gate_up, stride, (float*)out, ff, limit, alpha, up_shift);
   return dli_launch_status();
 }

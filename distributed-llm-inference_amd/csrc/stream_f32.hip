@@ -356,7 +356,9 @@ __global__ void rotary_cache_kernel(const float* __restrict__ proj, int64_t stri
   const int64_t page = slot >= 0 ? slot / page_size : 0;
   const int off = slot >= 0 ? slot % page_size : 0;
   const int half = rot_dims / 2;
-  for (int i = threadIdx.x; i < (q_heads + kv_heads) * dim; i += blockDim.x) {
+  // (a row of a step with few rows is shared by gridDim.y workgroups)
+  const int at0 = blockIdx.y * blockDim.x + threadIdx.x, stride0 = gridDim.y * blockDim.x;
+  for (int i = at0; i < (q_heads + kv_heads) * dim; i += stride0) {
     const int h = i / dim, c = i - h * dim;
     const bool is_q = h < q_heads;
     const int64_t at = is_q ? q_off + (int64_t)h * dim : k_off + (int64_t)(h - q_heads) * dim;
@@ -377,7 +379,7 @@ __global__ void rotary_cache_kernel(const float* __restrict__ proj, int64_t stri
     else if (slot >= 0) k_pages[((page * kv_heads + (h - q_heads)) * page_size + off) * dim + c] = from_f32<T>(y);
   }
   if (slot >= 0)
-    for (int i = threadIdx.x; i < v_heads * vdim; i += blockDim.x) {
+    for (int i = at0; i < v_heads * vdim; i += stride0) {
       const int g = i / vdim, c = i - g * vdim;
       v_pages[((page * v_heads + g) * vdim + c) * page_size + off] =
           from_f32<T>(pr[v_off + i] + (bias != nullptr ? bias[v_off + i] : 0.f));
@@ -656,13 +658,15 @@ int dli_rotary_cache(const float* proj, int64_t stride, int q_off, int k_off, in
       rot_dims > dim || rot_dims % 2 || (rot_dims > 0 && inv_freq == nullptr) ||
       (kv_heads > 0 && (k_pages == nullptr || slots == nullptr)) || (v_heads > 0 && (v_pages == nullptr || slots == nullptr)))
     return DLI_ERR_ARGUMENT;
+  const int64_t shares = ((int64_t)(q_heads + kv_heads) * dim + 511) / 512;
+  const dim3 grid(rows, rows >= 128 ? 1 : (unsigned)(shares < 16 ? shares : 16));
   if (is_bf16)
-    rotary_cache_kernel<bf16_t><<<rows, 256, 0, stream>>>(proj, stride, q_off, k_off, v_off, bias, positions, inv_freq,
+    rotary_cache_kernel<bf16_t><<<grid, 256, 0, stream>>>(proj, stride, q_off, k_off, v_off, bias, positions, inv_freq,
                                                           rot_dims, interleaved, (bf16_t*)q_out, slots, (bf16_t*)k_pages,
                                                           (bf16_t*)v_pages, q_heads, kv_heads, v_heads, dim, vdim, page_size, q_coef,
                                                           q_every);
   else
-    rotary_cache_kernel<float><<<rows, 256, 0, stream>>>(proj, stride, q_off, k_off, v_off, bias, positions, inv_freq,
+    rotary_cache_kernel<float><<<grid, 256, 0, stream>>>(proj, stride, q_off, k_off, v_off, bias, positions, inv_freq,
                                                          rot_dims, interleaved, (float*)q_out, slots, (float*)k_pages,
                                                          (float*)v_pages, q_heads, kv_heads, v_heads, dim, vdim, page_size, q_coef,
                                                           q_every);

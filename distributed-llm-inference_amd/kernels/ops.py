@@ -112,7 +112,7 @@ _SIGNATURES = {
                                   _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr],
     "dli_attention_keyvalue_supports": [_c_int, _c_int],
     "dli_attention_keyvalue_tile_tokens": [_c_int, _c_int],
-    "dli_attention_keyvalue_splits": [_c_int, _c_int, _c_int],
+    "dli_attention_keyvalue_splits": [_c_int, _c_int, _c_int, _c_int],
     "dli_attention_keyvalue": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int,
                                _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr],
     "dli_embed_sinusoid": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_float, _c_int, _c_ptr],
@@ -1784,7 +1784,7 @@ def attention_keyvalue(q: torch.Tensor, k_pages: torch.Tensor, out: torch.Tensor
         _require(tile_q0 is None and q.shape[0] == entries, "without tile lists every entry must be one row")
         tiles = entries
         if splits is None:
-            splits = int(library().dli_attention_keyvalue_splits(q_heads, kv_heads, max(entries, 1)))
+            splits = int(library().dli_attention_keyvalue_splits(q_heads, kv_heads, head_dim, max(entries, 1)))
         if splits > 1:
             parts = torch.empty(entries * q_heads * splits * (value_dim + 2), device=q.device, dtype=torch.float32)
     else:

@@ -27,7 +27,7 @@ import torch
 
 from ..kernels import ops
 from .base import Mixer, PagedKVSpec, Runtime
-from .linear import as_operand, linear, linear_f32, stack_rows
+from .linear import as_operand, linear_few, linear_f32, stack_rows
 from .registry import build_part, register_part
 from .scored_attention import paged_scored_attention
 from .spec import PartSpec, WeightSpec
@@ -120,7 +120,7 @@ class LatentAttention(Mixer):
                                   grp.slots, cache.k_pages, **turn)
         else:
             ops.latent_norm_cache(proj, 0, self.q_rank, self.q_rank, 0, self.q_norm, None, self.norm_eps, cq, None, None)
-        q = linear(self.rt, cq, self.w_uq)
+        q = linear_few(self.rt, cq, self.w_uq)
         q_latent = self.rt.empty(n, H * (r + e))
         ops.head_products(q, self.w_uk_t, q_latent, **turn)
         mixed = self.rt.empty(n, H * r)

@@ -39,6 +39,18 @@ def linear(rt: Runtime, x: torch.Tensor, weight: torch.Tensor, bias: Optional[to
     return out
 
 
+def linear_few(rt: Runtime, x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """:func:`linear` for a part outside the fused decode path: up to 16 rows on the few-row product, which streams
+    the weights faster than the library does."""
+    n, k = x.shape
+    if (rt.is_bf16 and 0 < n <= F32_FEW_ROWS and x.dtype == torch.bfloat16 and ops.skinny_gemm_supports(n, k, x.dtype)
+            and x.stride(0) % 8 == 0 and x.data_ptr() % 16 == 0 and weight.is_contiguous()):
+        out = rt.empty(n, weight.shape[0])
+        ops.skinny_gemm(x, weight, epilogue=ops.SKINNY_STORE, out=out)
+        return out
+    return linear(rt, x, weight)
+
+
 def decode_copy(rt: Runtime, weight: Optional[torch.Tensor], epilogue: int) -> Optional[torch.Tensor]:
     """The matrix once more in the tile order of the decode product (``ops.tile_weights``), or
     ``None`` where that would not be used: another type, sizes that do not tile, a product that
