@@ -324,7 +324,7 @@ def pibuvik_shape(width, heads, kv_heads, ff, layers, vocab, chunk):
     latent of 256 values with a rotated part of 32 (heads of 64, queries through a latent of three quarters of the
     width, a window of the chunk's size), attention on that layer's latents; the Llama layer's feed-forward."""
     latent = {"heads": heads, "dim": 64, "rot_dim": 32, "vdim": 64, "kv_rank": 256, "q_rank": 3 * width // 4,
-              "mask": {"size": chunk}, "rot": {"base": 5e5, "dims": 32}, "scale": 96 ** -0.5}
+              "mask": {"size": chunk}, "rot": {"base": 1e5, "dims": 32}, "scale": 96 ** -0.5}
     mixers = {"rglru": {"width": width, "blocks": width // 128, "conv": 4},
               "attention": {"heads": heads, "kv_heads": kv_heads, "dim": 64, "vdim": 64, "scale": 0.125,
                             "q_temp": {"coef": 0.3, "every": 2048}},
@@ -334,8 +334,8 @@ def pibuvik_shape(width, heads, kv_heads, ff, layers, vocab, chunk):
     for i in range(layers):
         mixer = dict(latent, kv_from=i - 1) if i % 4 == 3 else mixers[order[i % 4]]
         out.append({"type": order[i % 4], "mixer": mixer, "mlp": {"kind": "dense", "ff": ff, "limit": 7.0}})
-    return {"architecture": "Pibuvik", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": 3.0},
-            "residual_mult": 0.3, "logit_scale": 0.5, "layers": out}
+    return {"architecture": "Pibuvik", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": 2.0},
+            "residual_mult": 0.4, "logit_scale": 0.8, "layers": out}
 
 
 DESIGN_SIZES = {  # width, heads (of 64), kv heads, feed-forward, layers, vocabulary, attention chunk
