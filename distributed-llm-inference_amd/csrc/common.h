@@ -34,10 +34,20 @@ __device__ __forceinline__ float clamped_glu(float gate, float up, float limit, 
   return g / (1.f + expf(-alpha * g)) * (u + up_shift);
 }
 
-// The activation inside a few-row product: `clamped` 0 is cast(silu(gate)) * up, else the form above.
-struct GluForm { int clamped; float limit, alpha, up_shift; };
+// gelu(gate) * up in its tanh form, 0.5 z (1 + tanh t) = z sigmoid(2 t), t = sqrt(2 / pi) (z + 0.044715 z^3).
+__device__ __forceinline__ float gelu_glu(float z, float up) {
+  const float t2 = 1.5957691216057308f * (z + 0.044715f * z * z * z);
+  return z / (1.f + expf(-t2)) * up;
+}
+
+// The activation inside a few-row product: `form` 0 is cast(silu(gate)) * up, 1 the clamped form, 2 gelu(gate) * up.
+#define GLU_SILU 0
+#define GLU_CLAMPED 1
+#define GLU_GELU 2
+struct GluForm { int form; float limit, alpha, up_shift; };
 __device__ __forceinline__ bf16_t glu_bf16(float gate, float up, const GluForm& f) {
-  if (f.clamped) return (bf16_t)clamped_glu(gate, up, f.limit, f.alpha, f.up_shift);
+  if (f.form == GLU_CLAMPED) return (bf16_t)clamped_glu(gate, up, f.limit, f.alpha, f.up_shift);
+  if (f.form == GLU_GELU) return (bf16_t)gelu_glu(gate, up);
   return (bf16_t)((float)(bf16_t)silu<bf16_t>(gate) * up);
 }
 

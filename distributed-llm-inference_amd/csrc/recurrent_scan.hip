@@ -34,6 +34,7 @@
 #define RULE_DELTA 0
 #define RULE_BONUS 1
 #define GATE_NONE 2   // head_norm_gate alone: the per-head norm without a gate
+#define GATE_FIRST 3  // head_norm_gate alone: o times silu(g_pre), then the norm of that
 
 struct ScanArgs {
   const float* r; const float* k; const float* v;   // [rows][heads * D], each with its row stride
@@ -249,7 +250,11 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
     const float* oh = o + row * o_stride + (int64_t)h * dim;
     const float dn = den != nullptr ? 1.f / den[row * heads + h] : 1.f;
     float ss = 0.f;
-    for (int c = lane; c < dim; c += DLI_WAVE) ss += (oh[c] * dn) * (oh[c] * dn);
+    for (int c = lane; c < dim; c += DLI_WAVE) {
+      float v = oh[c] * dn;
+      if (RULE == GATE_FIRST) v *= silu<float>(g_pre[row * g_stride + (int64_t)h * dim + c]);
+      ss += v * v;
+    }
     const float r = dn / sqrtf(wave_sum(ss) / (float)dim + eps);
     for (int c = lane; c < dim; c += DLI_WAVE) {
       float gate = 1.f;                                   // RULE 2: no gate (g_pre is not read)
@@ -262,7 +267,7 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
   }
 }
 
-// The same for one head that spans a long row: a workgroup a row.
+// The same for heads that span a long row: a workgroup a (row, head).
 template <typename T, int RULE>
 __global__ __launch_bounds__(256) void row_norm_gate_kernel(const float* __restrict__ o, int64_t o_stride,
                                                             const float* __restrict__ g_pre, int64_t g_stride,
@@ -270,10 +275,18 @@ __global__ __launch_bounds__(256) void row_norm_gate_kernel(const float* __restr
                                                             int64_t out_stride, int dim, const float* __restrict__ den) {
   __shared__ float scratch[16];
   const int64_t row = blockIdx.x;
-  const float* oh = o + row * o_stride;
-  const float dn = den != nullptr ? 1.f / den[row] : 1.f;
+  const int64_t at = (int64_t)blockIdx.y * dim;            // (several long heads a row: a workgroup each)
+  const float* oh = o + row * o_stride + at;
+  const float dn = den != nullptr ? 1.f / den[row * gridDim.y + blockIdx.y] : 1.f;
+  g_pre += at;
+  norm_w += at;
+  out += at;
   float ss = 0.f;
-  for (int c = threadIdx.x; c < dim; c += blockDim.x) ss += (oh[c] * dn) * (oh[c] * dn);
+  for (int c = threadIdx.x; c < dim; c += blockDim.x) {
+    float v = oh[c] * dn;
+    if (RULE == GATE_FIRST) v *= silu<float>(g_pre[row * g_stride + c]);
+    ss += v * v;
+  }
   const float r = dn / sqrtf(block_sum(ss, scratch) / (float)dim + eps);
   for (int c = threadIdx.x; c < dim; c += blockDim.x) {
     float gate = 1.f;
@@ -353,22 +366,23 @@ extern "C" int dli_recurrent_scan(const float* r, int64_t r_stride, const float*
 extern "C" int dli_head_norm_gate(const float* o, int64_t o_stride, const float* g_pre, int64_t g_stride,
                                   const float* norm_w, float eps, void* out, int64_t out_stride, int rows, int heads,
                                   int dim, int gate, const float* den, int out_is_bf16, hipStream_t stream) {
-  // gate: 0 sigmoid(g_pre), 1 silu(g_pre), 2 none
+  // gate: 0 sigmoid(g_pre), 1 silu(g_pre), 2 none, 3 silu(g_pre) on o before the norm
   if (rows <= 0) return DLI_OK;
   const int64_t width = (int64_t)heads * dim;
-  if (heads <= 0 || dim <= 0 || o_stride < width || out_stride < width || gate < 0 || gate > 2 ||
+  if (heads <= 0 || dim <= 0 || o_stride < width || out_stride < width || gate < 0 || gate > 3 ||
       (gate != GATE_NONE && (g_pre == nullptr || g_stride < width)))
     return DLI_ERR_ARGUMENT;
   const dim3 grid(rows, (heads + 3) / 4);
   if (grid.y > 65535) return DLI_ERR_ARGUMENT;
 #define HNG(T, RULE)                                                                                                     \
   do {                                                                                                                   \
-    if (heads == 1 && dim > 256)                                                                                         \
-      row_norm_gate_kernel<T, RULE><<<rows, 256, 0, stream>>>(o, o_stride, g_pre, g_stride, norm_w, eps, (T*)out, out_stride, dim, den); \
+    if (dim > 256 && (heads == 1 || gate == GATE_FIRST))                                                                 \
+      row_norm_gate_kernel<T, RULE><<<dim3(rows, heads), 256, 0, stream>>>(o, o_stride, g_pre, g_stride, norm_w, eps, (T*)out, out_stride, dim, den); \
     else                                                                                                                 \
       head_norm_gate_kernel<T, RULE><<<grid, 256, 0, stream>>>(o, o_stride, g_pre, g_stride, norm_w, eps, (T*)out, out_stride, heads, dim, den); \
   } while (0)
-  if (out_is_bf16) { if (gate == GATE_NONE) HNG(bf16_t, GATE_NONE); else if (gate) HNG(bf16_t, RULE_BONUS); else HNG(bf16_t, RULE_DELTA); }
+  if (gate == GATE_FIRST) { if (out_is_bf16) HNG(bf16_t, GATE_FIRST); else HNG(float, GATE_FIRST); }
+  else if (out_is_bf16) { if (gate == GATE_NONE) HNG(bf16_t, GATE_NONE); else if (gate) HNG(bf16_t, RULE_BONUS); else HNG(bf16_t, RULE_DELTA); }
   else { if (gate == GATE_NONE) HNG(float, GATE_NONE); else if (gate) HNG(float, RULE_BONUS); else HNG(float, RULE_DELTA); }
 #undef HNG
   return dli_launch_status();

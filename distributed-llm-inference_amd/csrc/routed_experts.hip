@@ -6,13 +6,15 @@
 //                    over the row; z is the 32-bit result of the product before it
 //   clamped_glu      y = g sigmoid(alpha g) (u + shift), g = min(gate, limit), u = clamp(up, -limit, limit); an infinite
 //                    limit, alpha 1 and shift 0 give the plain silu(gate) * up
-//   router_choose    softmax over all router outputs; choice = score + correction; only the `keep` groups of
-//                    neighbours with the largest best choice stay; the `top` largest choices; weights = the chosen
-//                    scores (without correction) / (their sum + 1e-20) * scale
+//   gelu_glu         y = gelu(gate) * up, tanh form (the same kernels)
+//   router_choose    softmax over all router outputs, or the sigmoid of each; choice = score + correction; only the
+//                    `keep` groups of neighbours with the largest best choice stay; the `top` largest choices; weights =
+//                    the chosen scores (without correction) / (their sum + 1e-20) * scale, or scores * scale alone
 //   expert_sort      the (token, choice) slots of real experts in runs by expert, and the list of row tiles
 //   expert_up/down   the experts' products over those tiles (on the matrix cores for bfloat16 and sizes that are
 //                    multiples of 32, else on the vector units, any size), the clamped activation between
-//                    them; the down product leaves each slot's 32-bit result in the slot's own row
+//                    them; the down product leaves each slot's 32-bit result in the slot's own row. Where a slot's
+//                    weight belongs on the expert's input, the up kernels multiply their 32-bit sums by it
 //   expert_combine   out = sum_j w_j (expert j's result, or the input itself for an identity expert)
 //                    + sigmoid(shared gate) * shared expert's result
 //
@@ -50,18 +52,18 @@ __global__ void poly_norm_kernel_f32in(const float* __restrict__ z, int64_t z_st
 }
 
 template <typename T>
-__global__ void clamped_glu_kernel(const T* __restrict__ gate_up, int64_t stride, T* __restrict__ out, int ff, float limit,
-                                   float alpha, float up_shift) {
+__global__ void clamped_glu_kernel(const T* __restrict__ gate_up, int64_t stride, T* __restrict__ out, int ff, GluForm f) {
   const int64_t row = blockIdx.x;
   const int i = blockIdx.y * blockDim.x + threadIdx.x;
-  if (i < ff)
-    out[row * ff + i] = from_f32<T>(clamped_glu(to_f32(gate_up[row * stride + i]), to_f32(gate_up[row * stride + ff + i]), limit, alpha, up_shift));
+  if (i >= ff) return;
+  const float g = to_f32(gate_up[row * stride + i]), u = to_f32(gate_up[row * stride + ff + i]);
+  out[row * ff + i] = from_f32<T>(f.form == GLU_GELU ? gelu_glu(g, u) : clamped_glu(g, u, f.limit, f.alpha, f.up_shift));
 }
 
 // Eight neighbours a thread (rows and sizes of whole 16 bytes).
+template <bool GELU>
 __global__ __launch_bounds__(256) void clamped_glu_bf16x8_kernel(const bf16_t* __restrict__ gate_up, int64_t stride,
-                                                                 bf16_t* __restrict__ out, int ff, float limit, float alpha,
-                                                                 float up_shift) {
+                                                                 bf16_t* __restrict__ out, int ff, GluForm f) {
   typedef __bf16 b8 __attribute__((ext_vector_type(8)));
   const int64_t row = blockIdx.x;
   const int i = 8 * (blockIdx.y * 256 + threadIdx.x);
@@ -71,8 +73,13 @@ __global__ __launch_bounds__(256) void clamped_glu_bf16x8_kernel(const bf16_t* _
   b8 y;
 #pragma unroll
   for (int e = 0; e < 8; ++e) {
-    const float a = fminf((float)g[e], limit), b = fminf(fmaxf((float)u[e], -limit), limit);
-    y[e] = (bf16_t)(a * __builtin_amdgcn_rcpf(1.f + __expf(-alpha * a)) * (b + up_shift));
+    if (GELU) {
+      const float z = (float)g[e];
+      y[e] = (bf16_t)(z * __builtin_amdgcn_rcpf(1.f + __expf(-1.5957691216057308f * (z + 0.044715f * z * z * z))) * (float)u[e]);
+    } else {
+      const float a = fminf((float)g[e], f.limit), b = fminf(fmaxf((float)u[e], -f.limit), f.limit);
+      y[e] = (bf16_t)(a * __builtin_amdgcn_rcpf(1.f + __expf(-f.alpha * a)) * (b + f.up_shift));
+    }
   }
   *reinterpret_cast<b8*>(out + row * ff + i) = y;
 }
@@ -91,23 +98,27 @@ __device__ __forceinline__ void wave_argmax(float& v, int& i) {
 __global__ __launch_bounds__(64) void router_choose_kernel(const float* __restrict__ logits, int64_t stride,
                                                            const float* __restrict__ bias,
                                                            const float* __restrict__ correction, int total, int count,
-                                                           int keep, int top, float scale, int* __restrict__ ids,
-                                                           float* __restrict__ weights) {
+                                                           int keep, int top, float scale, int sigmoid, int normalize,
+                                                           int* __restrict__ ids, float* __restrict__ weights) {
   extern __shared__ float sh[];
   float *s = sh, *choice = sh + total, *gbest = sh + 2 * total;
   const int64_t row = blockIdx.x;
   const int lane = threadIdx.x;
   const float* z = logits + row * stride;
-  float m = -INFINITY;
-  for (int i = lane; i < total; i += DLI_WAVE) m = fmaxf(m, z[i] + (bias != nullptr ? bias[i] : 0.f));
-  m = wave_max(m);
-  float sum = 0.f;
-  for (int i = lane; i < total; i += DLI_WAVE) {
-    const float e = expf(z[i] + (bias != nullptr ? bias[i] : 0.f) - m);
-    s[i] = e;
-    sum += e;
+  float m = -INFINITY, sum = 0.f;
+  if (sigmoid) {
+    for (int i = lane; i < total; i += DLI_WAVE) s[i] = 1.f / (1.f + expf(-(z[i] + (bias != nullptr ? bias[i] : 0.f))));
+    sum = 1.f;
+  } else {
+    for (int i = lane; i < total; i += DLI_WAVE) m = fmaxf(m, z[i] + (bias != nullptr ? bias[i] : 0.f));
+    m = wave_max(m);
+    for (int i = lane; i < total; i += DLI_WAVE) {
+      const float e = expf(z[i] + (bias != nullptr ? bias[i] : 0.f) - m);
+      s[i] = e;
+      sum += e;
+    }
+    sum = wave_sum(sum);
   }
-  sum = wave_sum(sum);
   for (int i = lane; i < total; i += DLI_WAVE) {
     const float p = s[i] / sum;
     s[i] = p;
@@ -160,7 +171,7 @@ __global__ __launch_bounds__(64) void router_choose_kernel(const float* __restri
   }
   if (lane < top) {
     ids[row * top + lane] = my_id;
-    weights[row * top + lane] = mine / (chosen_sum + 1e-20f) * scale;
+    weights[row * top + lane] = (normalize ? mine / (chosen_sum + 1e-20f) : mine) * scale;
   }
 }
 
@@ -210,6 +221,7 @@ __global__ __launch_bounds__(1024) void expert_sort_kernel(const int* __restrict
 struct ExpertArgs {
   const int* tile_expert; const int* tile_row0; const int* tile_count; const int* offsets; const int* order;
   int top, width, ff;
+  const float* in_weight;   // [slots], what multiplies an expert's input (nullptr: nothing)
 };
 
 // y[sorted row][ff] = clamped_glu(h[token] . w_gate[e], h[token] . w_up[e]); w_gate, w_up [experts][ff][width].
@@ -259,10 +271,11 @@ __global__ __launch_bounds__(256) void expert_up_kernel(ExpertArgs p, const T* _
   for (int i = 0; i < 2; ++i) {
     const int r = r0 + ty * 2 + i;
     if (r >= rend) continue;
+    const float iw = p.in_weight != nullptr ? p.in_weight[p.order[r]] : 1.f;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int c = n0 + tx * 4 + j;
-      if (c < p.ff) y[(int64_t)r * p.ff + c] = from_f32<T>(clamped_glu(accg[i][j], accu[i][j], limit, alpha, up_shift));
+      if (c < p.ff) y[(int64_t)r * p.ff + c] = from_f32<T>(clamped_glu(iw * accg[i][j], iw * accu[i][j], limit, alpha, up_shift));
     }
   }
 }
@@ -389,12 +402,14 @@ __global__ __launch_bounds__(256) void expert_up_mfma_kernel(ExpertArgs p, const
   for (int mb = 0; mb < EXM_MB; ++mb) {
     const int r = r0 + mb * 16 + c;
     if (r >= rend) continue;
+    const float iw = p.in_weight != nullptr ? p.in_weight[p.order[r]] : 1.f;
 #pragma unroll
     for (int nb = 0; nb < 2; ++nb) {
       const int n0 = nw + nb * 16 + (lane / 16) * 4;
 #pragma unroll
       for (int i = 0; i < 4; ++i)
-        if (n0 + i < p.ff) y[(int64_t)r * p.ff + n0 + i] = (bf16_t)clamped_glu(accg[nb][mb][i], accu[nb][mb][i], limit, alpha, up_shift);
+        if (n0 + i < p.ff)
+          y[(int64_t)r * p.ff + n0 + i] = (bf16_t)clamped_glu(iw * accg[nb][mb][i], iw * accu[nb][mb][i], limit, alpha, up_shift);
     }
   }
 }
@@ -454,6 +469,7 @@ __global__ __launch_bounds__(256) void expert_down_mfma_kernel(ExpertArgs p, con
   }
 }
 
+// (weights nullptr: ones)
 // out[token] = sum_j weights[token][j] * (ids[token][j] < experts ? z[token * top + j] : h[token])
 //            + sigmoid(shared_gate[token]) * shared[token]       (the shared expert, if there is one)
 template <typename T>
@@ -469,7 +485,7 @@ __global__ void expert_combine_kernel(const int* __restrict__ ids, const float* 
   for (int j = 0; j < top; ++j) {
     const int e = ids[row * top + j];
     const float v = e < experts ? z[(row * top + j) * width + c] : to_f32(h[row * h_stride + c]);
-    sum = fmaf(weights[row * top + j], v, sum);
+    sum = fmaf(weights != nullptr ? weights[row * top + j] : 1.f, v, sum);
   }
   if (shared != nullptr) {
     const float g = shared_gate != nullptr ? 1.f / (1.f + expf(-shared_gate[row * gate_stride])) : 1.f;
@@ -500,27 +516,28 @@ int dli_poly_norm(const float* z, int64_t z_stride, const float* coef, void* out
   return dli_launch_status();
 }
 
-int dli_clamped_glu(const void* gate_up, int64_t stride, void* out, int rows, int ff, float limit, float alpha, float up_shift, int is_bf16,
-                    hipStream_t stream) {
+int dli_clamped_glu(const void* gate_up, int64_t stride, void* out, int rows, int ff, int form, float limit, float alpha, float up_shift,
+                    int is_bf16, hipStream_t stream) {
   if (rows <= 0) return DLI_OK;
-  if (ff <= 0 || stride < 2 * (int64_t)ff) return DLI_ERR_ARGUMENT;
-  const dim3 grid(rows, (ff + 255) / 256);
-  if (is_bf16 && ff % 8 == 0 && stride % 8 == 0 && ((uintptr_t)gate_up | (uintptr_t)out) % 16 == 0)
-    clamped_glu_bf16x8_kernel<<<dim3(rows, (ff / 8 + 255) / 256), 256, 0, stream>>>((const bf16_t*)gate_up, stride, (bf16_t*)out,
-                                                                                   ff, limit, alpha, up_shift);
-  else if (is_bf16) clamped_glu_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)gate_up, stride, (bf16_t*)out, ff, limit, alpha, up_shift);
-  else clamped_glu_kernel<float><<<grid, 256, 0, stream>>>((const float*)gate_up, stride, (float*)out, ff, limit, alpha, up_shift);
+  if (ff <= 0 || stride < 2 * (int64_t)ff || (form != GLU_CLAMPED && form != GLU_GELU)) return DLI_ERR_ARGUMENT;
+  const dim3 grid(rows, (ff + 255) / 256), grid8(rows, (ff / 8 + 255) / 256);
+  const GluForm f{form, limit, alpha, up_shift};
+  if (is_bf16 && ff % 8 == 0 && stride % 8 == 0 && ((uintptr_t)gate_up | (uintptr_t)out) % 16 == 0) {
+    if (form == GLU_GELU) clamped_glu_bf16x8_kernel<true><<<grid8, 256, 0, stream>>>((const bf16_t*)gate_up, stride, (bf16_t*)out, ff, f);
+    else clamped_glu_bf16x8_kernel<false><<<grid8, 256, 0, stream>>>((const bf16_t*)gate_up, stride, (bf16_t*)out, ff, f);
+  } else if (is_bf16) clamped_glu_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)gate_up, stride, (bf16_t*)out, ff, f);
+  else clamped_glu_kernel<float><<<grid, 256, 0, stream>>>((const float*)gate_up, stride, (float*)out, ff, f);
   return dli_launch_status();
 }
 
 int dli_router_choose(const float* logits, int64_t stride, const float* bias, const float* correction, int rows, int total, int count, int keep,
-                      int top, float scale, int* ids, float* weights, hipStream_t stream) {
+                      int top, float scale, int sigmoid, int normalize, int* ids, float* weights, hipStream_t stream) {
   if (rows <= 0) return DLI_OK;
   if (total <= 0 || total > 4096 || stride < total || top < 1 || top > 64 || top > total || count < 1 || total % count ||
       keep < 1 || keep > count || (int64_t)keep * (total / count) < top)
     return DLI_ERR_ARGUMENT;
   router_choose_kernel<<<rows, 64, (2 * total + count) * sizeof(float), stream>>>(logits, stride, bias, correction, total, count, keep,
-                                                                                  top, scale, ids, weights);
+                                                                                  top, scale, sigmoid, normalize, ids, weights);
   return dli_launch_status();
 }
 
@@ -530,11 +547,12 @@ int dli_expert_tile_rows(int width, int ff, int is_bf16) { return expert_mfma(wi
 
 // The experts' part of a mixture for `rows` tokens: sort, up product with activation, down product.
 // ids [rows][top]; scratch: offsets [experts + 1], order [rows * top], tile_expert and tile_row0 [max_tiles],
-// tile_count [1] (int32), y [rows * top][ff] (T), z [rows * top][width] (float32).
+// tile_count [1] (int32), y [rows * top][ff] (T), z [rows * top][width] (float32). in_weight [rows][top] (may be nullptr):
+// what each slot's expert input is multiplied by.
 int dli_expert_products(const int* ids, const void* h, int64_t h_stride, const void* w_gate, const void* w_up,
                         const void* w_down, int* offsets, int* order, int* tile_expert, int* tile_row0, int* tile_count,
-                        int max_tiles, void* y, float* z, int rows, int top, int experts, int width, int ff, float limit,
-                        float alpha, float up_shift, int is_bf16, hipStream_t stream) {
+                        int max_tiles, void* y, float* z, const float* in_weight, int rows, int top, int experts, int width,
+                        int ff, float limit, float alpha, float up_shift, int is_bf16, hipStream_t stream) {
   if (rows <= 0) return DLI_OK;
   const int64_t slots = (int64_t)rows * top;
   if (top < 1 || experts < 1 || experts > 4096 || width <= 0 || ff <= 0 || h_stride < width || slots > (1 << 30) ||
@@ -549,7 +567,7 @@ int dli_expert_products(const int* ids, const void* h, int64_t h_stride, const v
   if (dli_launch_status() != DLI_OK) return DLI_ERR_LAUNCH;
   ExpertArgs p;
   p.tile_expert = tile_expert; p.tile_row0 = tile_row0; p.tile_count = tile_count; p.offsets = offsets; p.order = order;
-  p.top = top; p.width = width; p.ff = ff;
+  p.top = top; p.width = width; p.ff = ff; p.in_weight = in_weight;
   const int bn = mfma ? EXM_BN : EX_BN;
   const dim3 up_grid(max_tiles, (ff + bn - 1) / bn), down_grid(max_tiles, (width + bn - 1) / bn);
   if (mfma) {

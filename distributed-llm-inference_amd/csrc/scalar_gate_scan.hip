@@ -3,15 +3,18 @@
 //
 //   S_t = a_t S_(t-1) + b_t k_t v_t^T,   o_t = S_t^T q_t      (o is made from the state that already holds the token)
 //
-// Two uses: a constant decay per head (a = decay[head], b = 1: linear attention with a decay), and a matrix
-// memory with exponential input and forget gates, whose factors come from log gates i_t, f_t under a running
-// reference point m (m_0 = 0):
+// Three uses: a constant decay per head (a = decay[head], b = 1: linear attention with a decay); a step size per token and
+// head (a state-space recurrence: dt = softplus(step + bias), log a = -exp(rate) dt, b = dt, and the result o + skip v; the
+// scan makes a and b itself); and a matrix memory with exponential input and forget gates, whose factors come from log
+// gates i_t, f_t under a running reference point m (m_0 = 0):
 //
 //   m_t = max(f_t + m_(t-1), i_t),  a_t = exp(f_t + m_(t-1) - m_t),  b_t = exp(i_t - m_t)
 //
 // and whose result is divided by max(|n_t . q_t|, exp(-m_t)) + 1e-6 with n_t = a_t n_(t-1) + b_t k_t. n is the
 // state's column for a value that is always one, so the scan carries V + 1 columns and leaves the
 // denominators in an array of their own (`den`), for the kernel that normalises the heads.
+//
+// Several heads may share one query and key: head h reads those of head h / (heads / qk_heads).
 //
 // S is float32 [heads][V (+ 1)][D] in the request's state slot (then m [heads] for the matrix memory) and
 // starts from zeros where the entry's first row has position 0; an entry's rows are walked in order from
@@ -45,7 +48,18 @@ struct SgArgs {
   float* o; int64_t o_stride;            // [rows][heads * V]
   int heads, vdim;
   float q_scale; int silu;
+  int qk_heads;                          // q and k hold that many heads
+  const float* step; int64_t step_stride;                        // [rows][heads] before the bias: with it a and b are
+  const float* step_bias; const float* step_rate;                // made here ([heads] each)
+  const float* skip;                     // [heads]: o + skip v (nullptr: o)
 };
+
+// How a and b come about.
+#define SG_DECAY 0   // decay[head] and one
+#define SG_EXP 1     // keep and write, with a normaliser (the column of n)
+#define SG_STEP 2    // from a step size
+
+__device__ __forceinline__ float sg_softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 
 __device__ __forceinline__ float sg_row_sum(float x) {
   x += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, x), 0xB1, 0xF, 0xF, false));
@@ -57,12 +71,13 @@ __device__ __forceinline__ float sg_row_sum(float x) {
 
 __device__ __forceinline__ float sg_act(float x, int silu) { return silu ? x / (1.f + expf(-x)) : x; }
 
-// NK keys a lane, D = 16 NK; TB tokens staged at once (1 in a step of single tokens). GATED: keep and write factors
-// per token (else the head's constant decay and one), and with them the column of n and the denominators; SILU:
+// NK keys a lane, D = 16 NK; TB tokens staged at once (1 in a step of single tokens). MODE SG_EXP: keep and write
+// factors per token, and with them the column of n and the denominators; SILU:
 // q, k and v pass through silu on their way into LDS. No load hangs on a condition (what is not wanted is read
 // from a clamped place and dropped), so that a batch's loads stay in flight while the chain of the one before runs.
-template <int NK, int TB, bool GATED, bool SILU>
+template <int NK, int TB, int MODE, bool SILU>
 __global__ __launch_bounds__(64) void scalar_gate_scan_kernel(SgArgs p) {
+  constexpr bool GATED = MODE == SG_EXP;
   constexpr int D = NK * 16, COLS = 4, PER = (TB * D + 63) / 64;
   __shared__ float sk[PER * 64], sq[PER * 64], sv[TB * COLS], sa[TB], sb[TB], sfl[TB];
   const int lane = threadIdx.x, vloc = lane / 16, part = lane % 16;
@@ -73,7 +88,7 @@ __global__ __launch_bounds__(64) void scalar_gate_scan_kernel(SgArgs p) {
   const bool live = my_col < VX, is_n = GATED && col == V;
   const int row0 = p.q_start[entry], n_rows = p.q_start[entry + 1] - row0;
   if (n_rows <= 0) return;
-  const int64_t qk_col = (int64_t)head * D, v_col = (int64_t)head * V;
+  const int64_t qk_col = (int64_t)(head / (p.heads / p.qk_heads)) * D, v_col = (int64_t)head * V;
   float* st = p.state + (int64_t)p.state_slots[entry] * p.state_stride + ((int64_t)head * VX + col) * D + part * NK;
   float s[NK];
   const bool fresh = p.positions[row0] == 0;
@@ -82,7 +97,9 @@ __global__ __launch_bounds__(64) void scalar_gate_scan_kernel(SgArgs p) {
     const float old = st[i];
     s[i] = fresh ? 0.f : old;
   }
-  const float decay = GATED ? 1.f : p.decay[head];
+  const float decay = MODE == SG_DECAY ? p.decay[head] : 1.f;
+  const float bias = MODE == SG_STEP ? p.step_bias[head] : 0.f, rate = MODE == SG_STEP ? -expf(p.step_rate[head]) : 0.f;
+  const float skip = MODE == SG_STEP && p.skip != nullptr ? p.skip[head] : 0.f;
   float pk[PER], pq[PER], pv = 0.f, pa = 1.f, pb = 1.f, pf = 0.f;
   auto fetch = [&](int t0) {
 #pragma unroll
@@ -103,6 +120,7 @@ __global__ __launch_bounds__(64) void scalar_gate_scan_kernel(SgArgs p) {
       pb = p.write[row * p.gate_stride + head];
       pf = p.floor[row * p.gate_stride + head];
     }
+    if (MODE == SG_STEP) pa = p.step[(int64_t)(row0 + min(t0 + min(lane, TB - 1), n_rows - 1)) * p.step_stride + head];
   };
   auto step = [&](int t, int64_t row) {
     const float* kt = sk + t * D + part * NK;
@@ -117,7 +135,7 @@ __global__ __launch_bounds__(64) void scalar_gate_scan_kernel(SgArgs p) {
     const float o = sg_row_sum(o0 + o1);
     if (part == 0 && live) {
       if (is_n) p.den[row * p.heads + head] = fmaxf(fabsf(o), sfl[t]) + 1e-6f;
-      else p.o[row * p.o_stride + v_col + col] = o;
+      else p.o[row * p.o_stride + v_col + col] = MODE == SG_STEP ? fmaf(skip, sv[t * COLS + vloc], o) : o;
     }
   };
   fetch(0);
@@ -132,7 +150,12 @@ __global__ __launch_bounds__(64) void scalar_gate_scan_kernel(SgArgs p) {
       sv[lane] = GATED && c >= V ? 1.f : sg_act(pv, SILU);   // the column of n reads a value of one
     }
     if (lane < TB) {
-      sa[lane] = GATED ? pa : decay;
+      if (MODE == SG_STEP) {
+        pb = sg_softplus(pa + bias);
+        sa[lane] = expf(rate * pb);
+      } else {
+        sa[lane] = GATED ? pa : decay;
+      }
       sb[lane] = pb;
       sfl[lane] = pf;
     }
@@ -162,7 +185,7 @@ __global__ void scalar_gate_any_kernel(SgArgs p, int D) {
   const int entry = blockIdx.x, head = blockIdx.y;
   const int row0 = p.q_start[entry], n_rows = p.q_start[entry + 1] - row0;
   if (n_rows <= 0) return;
-  const int64_t qk_col = (int64_t)head * D, v_col = (int64_t)head * V;
+  const int64_t qk_col = (int64_t)(head / (p.heads / p.qk_heads)) * D, v_col = (int64_t)head * V;
   float* st = p.state + (int64_t)p.state_slots[entry] * p.state_stride + ((int64_t)head * VX + (live ? c : 0)) * D;
   if (live && p.positions[row0] == 0)
     for (int i = 0; i < D; ++i) st[i] = 0.f;
@@ -175,9 +198,17 @@ __global__ void scalar_gate_any_kernel(SgArgs p, int D) {
     }
     __syncthreads();
     if (!live) continue;
-    const float a = p.keep != nullptr ? p.keep[row * p.gate_stride + head] : p.decay[head];
-    const float b = p.keep != nullptr ? p.write[row * p.gate_stride + head] : 1.f;
-    const float bv = b * (is_n ? 1.f : sg_act(p.v[row * p.v_stride + v_col + c], p.silu));
+    float a, b = 1.f;
+    if (p.step != nullptr) {
+      b = sg_softplus(p.step[row * p.step_stride + head] + p.step_bias[head]);
+      a = expf(-expf(p.step_rate[head]) * b);
+    } else if (p.keep != nullptr) {
+      a = p.keep[row * p.gate_stride + head];
+      b = p.write[row * p.gate_stride + head];
+    } else {
+      a = p.decay[head];
+    }
+    const float v = is_n ? 1.f : sg_act(p.v[row * p.v_stride + v_col + c], p.silu), bv = b * v;
     float o = 0.f;
     for (int i = 0; i < D; ++i) {
       const float s = fmaf(a, st[i], bv * sk[i]);
@@ -185,7 +216,7 @@ __global__ void scalar_gate_any_kernel(SgArgs p, int D) {
       o = fmaf(sq[i], s, o);
     }
     if (is_n) p.den[row * p.heads + head] = fmaxf(fabsf(o), p.floor[row * p.gate_stride + head]) + 1e-6f;
-    else p.o[row * p.o_stride + v_col + c] = o;
+    else p.o[row * p.o_stride + v_col + c] = p.skip != nullptr ? fmaf(p.skip[head], v, o) : o;
   }
 }
 
@@ -207,8 +238,9 @@ __global__ void scalar_gate_any_kernel(SgArgs p, int D) {
 // q = k = v = 0. The slice that holds column 0 also carries n and writes the denominators.
 typedef float sg_f4 __attribute__((ext_vector_type(4)));
 
-template <int D, bool GATED>
+template <int D, int MODE>
 __global__ __launch_bounds__(256) void scalar_gate_chunk_kernel(SgArgs p, const float* __restrict__ log_keep) {
+  constexpr bool GATED = MODE == SG_EXP;
   constexpr int C = 64, VS = 16, DS = D + 4, PS = C + 4, QK_PER = C * D / 256, V_PER = C * VS / 256;
   __shared__ __attribute__((aligned(16))) float sQ[C * DS], sK[C * DS], sP[C * PS], sVt[VS * PS], sSt[VS * DS], sW[C];
   __shared__ float sN[D], sB[C], sFl[C];
@@ -222,7 +254,7 @@ __global__ __launch_bounds__(256) void scalar_gate_chunk_kernel(SgArgs p, const 
   if (n_rows <= 0) return;
   const bool fresh = p.positions[row0] == 0, with_n = GATED && blockIdx.z == 0;
   float* st = p.state + (int64_t)p.state_slots[entry] * p.state_stride + (int64_t)head * VX * D;
-  const int64_t qk_col = (int64_t)head * D, v_col = (int64_t)head * V;
+  const int64_t qk_col = (int64_t)(head / (p.heads / p.qk_heads)) * D, v_col = (int64_t)head * V;
   for (int idx = tid; idx < D * VS; idx += 256) {
     const int j = idx / D, d = idx - j * D;                 // the state keeps a column's keys side by side
     const float old = v0 + j < V ? st[(int64_t)(v0 + j) * D + d] : 0.f;
@@ -232,7 +264,9 @@ __global__ __launch_bounds__(256) void scalar_gate_chunk_kernel(SgArgs p, const 
     const float old = with_n ? st[(int64_t)V * D + tid] : 0.f;
     sN[tid] = fresh ? 0.f : old;
   }
-  const float log_decay = GATED ? 0.f : fmaxf(logf(p.decay[head]), -1e30f);
+  const float log_decay = MODE == SG_DECAY ? fmaxf(logf(p.decay[head]), -1e30f) : 0.f;
+  const float bias = MODE == SG_STEP ? p.step_bias[head] : 0.f, rate = MODE == SG_STEP ? -expf(p.step_rate[head]) : 0.f;
+  const float skip = MODE == SG_STEP && p.skip != nullptr ? p.skip[head] : 0.f;
   float rq[QK_PER], rk[QK_PER], rv[V_PER], rla = 0.f, rb = 0.f, rfl = 0.f;
   auto fetch = [&](int t0) {                                // rows past the last: the last row again, dropped when staged
 #pragma unroll
@@ -254,6 +288,7 @@ __global__ __launch_bounds__(256) void scalar_gate_chunk_kernel(SgArgs p, const 
       rb = p.write[at];
       rfl = p.floor[at];
     }
+    if (MODE == SG_STEP) rla = p.step[(int64_t)(row0 + min(t0 + lane, n_rows - 1)) * p.step_stride + head];
   };
   fetch(0);
   for (int t0 = 0; t0 < n_rows; t0 += C) {
@@ -273,6 +308,10 @@ __global__ __launch_bounds__(256) void scalar_gate_chunk_kernel(SgArgs p, const 
     if (wave == 0) {
       double la = GATED ? rla : log_decay;
       float b = GATED ? rb : 1.f;
+      if (MODE == SG_STEP) {
+        b = sg_softplus(rla + bias);
+        la = rate * b;
+      }
       if (lane >= nb) { la = 0.0; b = 0.f; }
 #pragma unroll
       for (int d = 1; d < 64; d <<= 1) {
@@ -331,7 +370,8 @@ __global__ __launch_bounds__(256) void scalar_gate_chunk_kernel(SgArgs p, const 
       for (int r = 0; r < 4; ++r) {
         const int t = 16 * wave + 4 * lk + r;
         if (t < nb && v0 + li < V)
-          p.o[(int64_t)(row0 + t0 + t) * p.o_stride + v_col + v0 + li] = fmaf(expf((float)sA[t]), far[r], acc[r]);
+          p.o[(int64_t)(row0 + t0 + t) * p.o_stride + v_col + v0 + li] =
+              fmaf(expf((float)sA[t]), far[r], MODE == SG_STEP ? fmaf(skip, sVt[li * PS + t], acc[r]) : acc[r]);
       }
       if (with_n) {                                         // row t = 16 wave + li, a quarter of its sums a lane
         const int t = 16 * wave + li;
@@ -470,25 +510,31 @@ int dli_exp_gates(const float* pre, int64_t stride, int i_off, int f_off, const 
 }
 
 // keep, write: [rows][heads] or both nullptr (then decay [heads] and a write factor of one); floor and den
-// [rows][heads] come together, and with them the state has a column more a head.
+// [rows][heads] come together, and with them the state has a column more a head. step [rows][heads] instead: factors from
+// softplus(step + step_bias) and -exp(step_rate), the result plus skip (may be nullptr) times v.
 int dli_scalar_gate_scan(const float* q, int64_t q_stride, const float* k, int64_t k_stride, const float* v, int64_t v_stride,
                          const float* keep, const float* write, const float* log_keep, int64_t gate_stride, const float* decay,
                          const float* floor, float* den, float* state, int64_t state_stride, const int* q_start, const int* positions,
                          const int* state_slots, float* o, int64_t o_stride, int entries, int rows, int heads, int dim,
-                         int vdim, float q_scale, int silu, int chunked, hipStream_t stream) {
+                         int vdim, float q_scale, int silu, int chunked, int qk_heads, const float* step, int64_t step_stride,
+                         const float* step_bias, const float* step_rate, const float* skip, hipStream_t stream) {
   if (rows <= 0 || entries <= 0) return DLI_OK;
+  if (qk_heads <= 0 || heads % qk_heads || (step != nullptr && (step_stride < heads || step_bias == nullptr || step_rate == nullptr ||
+      keep != nullptr || silu)) || (skip != nullptr && step == nullptr))
+    return DLI_ERR_ARGUMENT;
   const int vx = vdim + (floor != nullptr ? 1 : 0);
   if (rows < entries || heads <= 0 || heads > 65535 || dim <= 0 || dim > 4096 || vdim <= 0 ||
-      state_stride < (int64_t)heads * vx * dim || o_stride < (int64_t)heads * vdim || q_stride < (int64_t)heads * dim ||
-      k_stride < (int64_t)heads * dim || v_stride < (int64_t)heads * vdim || (keep == nullptr) != (write == nullptr) ||
-      (keep == nullptr && decay == nullptr) || (keep != nullptr && gate_stride < heads) || (floor == nullptr) != (den == nullptr) ||
+      state_stride < (int64_t)heads * vx * dim || o_stride < (int64_t)heads * vdim || q_stride < (int64_t)qk_heads * dim ||
+      k_stride < (int64_t)qk_heads * dim || v_stride < (int64_t)heads * vdim || (keep == nullptr) != (write == nullptr) ||
+      (keep == nullptr && decay == nullptr && step == nullptr) || (keep != nullptr && gate_stride < heads) || (floor == nullptr) != (den == nullptr) ||
       (floor != nullptr && keep == nullptr))
     return DLI_ERR_ARGUMENT;
   SgArgs p;
   p.q = q; p.q_stride = q_stride; p.k = k; p.k_stride = k_stride; p.v = v; p.v_stride = v_stride; p.keep = keep;
   p.write = write; p.gate_stride = gate_stride; p.decay = decay; p.floor = floor; p.den = den; p.state = state;
   p.state_stride = state_stride; p.q_start = q_start; p.positions = positions; p.state_slots = state_slots; p.o = o;
-  p.o_stride = o_stride; p.heads = heads; p.vdim = vdim; p.q_scale = q_scale; p.silu = silu;
+  p.o_stride = o_stride; p.heads = heads; p.vdim = vdim; p.q_scale = q_scale; p.silu = silu; p.qk_heads = qk_heads;
+  p.step = step; p.step_stride = step_stride; p.step_bias = step_bias; p.step_rate = step_rate; p.skip = skip;
   const bool single = rows == entries;
   const dim3 grid(entries, heads, (vx + 3) / 4);
   if (grid.z > 65535) return DLI_ERR_ARGUMENT;
@@ -500,8 +546,9 @@ int dli_scalar_gate_scan(const float* q, int64_t q_stride, const float* k, int64
     if (cgrid.z > 65535) return DLI_ERR_ARGUMENT;
 #define SG_CHUNK(DIM)                                                                                   \
   case DIM:                                                                                             \
-    if (gated) scalar_gate_chunk_kernel<DIM, true><<<cgrid, 256, 0, stream>>>(p, log_keep);             \
-    else scalar_gate_chunk_kernel<DIM, false><<<cgrid, 256, 0, stream>>>(p, log_keep);                  \
+    if (gated) scalar_gate_chunk_kernel<DIM, SG_EXP><<<cgrid, 256, 0, stream>>>(p, log_keep);           \
+    else if (step != nullptr) scalar_gate_chunk_kernel<DIM, SG_STEP><<<cgrid, 256, 0, stream>>>(p, log_keep); \
+    else scalar_gate_chunk_kernel<DIM, SG_DECAY><<<cgrid, 256, 0, stream>>>(p, log_keep);               \
     break;
     switch (dim) { SG_CHUNK(16) SG_CHUNK(32) SG_CHUNK(48) SG_CHUNK(64) }
 #undef SG_CHUNK
@@ -509,9 +556,10 @@ int dli_scalar_gate_scan(const float* q, int64_t q_stride, const float* k, int64
   }
 #define SG_LAUNCH(NK, TBV)                                                                                  \
   {                                                                                                         \
-    if (gated) scalar_gate_scan_kernel<NK, TBV, true, false><<<grid, 64, 0, stream>>>(p);                  \
-    else if (silu) scalar_gate_scan_kernel<NK, TBV, false, true><<<grid, 64, 0, stream>>>(p);              \
-    else scalar_gate_scan_kernel<NK, TBV, false, false><<<grid, 64, 0, stream>>>(p);                       \
+    if (gated) scalar_gate_scan_kernel<NK, TBV, SG_EXP, false><<<grid, 64, 0, stream>>>(p);                \
+    else if (step != nullptr) scalar_gate_scan_kernel<NK, TBV, SG_STEP, false><<<grid, 64, 0, stream>>>(p); \
+    else if (silu) scalar_gate_scan_kernel<NK, TBV, SG_DECAY, true><<<grid, 64, 0, stream>>>(p);           \
+    else scalar_gate_scan_kernel<NK, TBV, SG_DECAY, false><<<grid, 64, 0, stream>>>(p);                    \
   }
 #define SG_CASE(NK, TBM)                                                                     \
   case NK * 16:                                                                              \

@@ -28,7 +28,7 @@
 //                 (RMSNorm: src/dli/model/llama.py:40-44)
 //   EPI_STORE     y (+ bias) stored as bf16
 //   EPI_SWIGLU    half of the quads are gate rows n, half up rows n + up_offset:
-//                 stores cast(silu(gate)) * up (src/dli/model/llama.py:190), or the clamped form (GluForm)
+//                 stores cast(silu(gate)) * up (src/dli/model/llama.py:190), or another form (GluForm)
 //   EPI_RESIDUAL  stream[m][n] = cast(stream[m][n] + cast(y + bias)) in place, and this tile's part
 //                 of sum_n stream[m][n]^2 for the norm that follows
 //   EPI_F32       y stored as float32 (logits)
@@ -470,9 +470,9 @@ extern "C" int dli_skinny4_gemm(const void* x, int64_t ldx, const float* ssq_in,
                                 const float* norm_w, float eps, const void* w, const void* bias,
                                 void* out, int64_t ldo, void* stream_buf, int64_t lds_,
                                 float* ssq_out, int M, int N, int K, int up_offset, int epilogue,
-                                int shape, int clamped, float limit, float alpha, float up_shift, hipStream_t stream) {
+                                int shape, int glu_form, float limit, float alpha, float up_shift, hipStream_t stream) {
   if (M <= 0 || N <= 0) return DLI_OK;
-  const GluForm glu{clamped, limit, alpha, up_shift};
+  const GluForm glu{glu_form, limit, alpha, up_shift};
   if (M > 16 || K <= 0 || K % 8 != 0 || ldx % 8 != 0 || ldx < K || (int64_t)M * ldx * 2 >= (int64_t)1 << 31 ||
       shape < 0 || shape > 2 || epilogue < 0 || epilogue > 3 ||
       (norm_w != nullptr && (ssq_in == nullptr || ssq_parts <= 0)) ||

@@ -22,7 +22,7 @@
 //            (RMSNorm: src/dli/model/llama.py:40-44); otherwise xhat = x.
 //   EPI_STORE     y (+ bias) stored as bf16
 //   EPI_SWIGLU    two products per workgroup, rows n (gate) and n + up_offset (up) of w:
-//                 stores cast(silu(gate)) * up (src/dli/model/llama.py:190), or the clamped form (GluForm)
+//                 stores cast(silu(gate)) * up (src/dli/model/llama.py:190), or another form (GluForm)
 //   EPI_RESIDUAL  stream[m][n] = cast(stream[m][n] + cast(y + bias)) in place (the residual sum, in
 //                 32-bit), and this tile's part of sum_n stream[m][n]^2 for the norm that follows
 //   EPI_F32       y stored as float32 (logits)
@@ -551,10 +551,10 @@ extern "C" int dli_skinny_gemm(const void* x, int64_t ldx, const float* ssq_in, 
                                const float* norm_w, float eps, const void* w, const void* bias,
                                void* out, int64_t ldo, void* stream_buf, int64_t lds_,
                                float* ssq_out, int M, int N, int K, int up_offset, int epilogue,
-                               int shape, int tiled, int clamped, float limit, float alpha, float up_shift,
+                               int shape, int tiled, int glu_form, float limit, float alpha, float up_shift,
                                hipStream_t stream) {
   const QkvRope qr{};
-  const GluForm glu{clamped, limit, alpha, up_shift};
+  const GluForm glu{glu_form, limit, alpha, up_shift};
   if (M <= 0 || N <= 0) return DLI_OK;
   if (tiled && (M > 16 || K % 128 != 0 || N % 16 != 0 || up_offset % 16 != 0)) return DLI_ERR_ARGUMENT;
   if (M > 64 || K <= 0 || K % 32 != 0 || ldx % 8 != 0 || shape < 0 || shape > 4 || epilogue < 0 ||

@@ -30,6 +30,8 @@
 //   scale_f32          y *= c in place
 //   rms_norm_pair      two norms of the same row (two weights) from one pass over its statistics
 //   add_pair_into_stream  x += a + b
+//   tanh_norm_stream   x += s1 a + s2 b + c (each a vector over the row; any may be left out), and of the new stream
+//                      out(T) = tanh(alpha x) * w + o (a tanh in place of a norm: no statistics, so sum and norm are one pass)
 #include "common.h"
 #include "rotary.h"
 
@@ -340,13 +342,19 @@ __global__ void qk_unit_cache_kernel(const float* __restrict__ proj, int64_t str
 // holds a value for every column of proj and is added before anything else. The pages may hold fewer
 // value heads than key heads (v_heads; 0: the values are the keys), and none at all where the mixer reads
 // another's (kv_heads 0). q_coef != 0: q is also multiplied by 1 + q_coef ln(floor((p + 1) / q_every) + 1).
-template <typename T>
-__global__ void rotary_cache_kernel(const float* __restrict__ proj, int64_t stride, int q_off, int k_off, int v_off,
+// NORM: q, over all its heads at once, is divided by its root mean square and multiplied by q_norm (a value a
+// column), and k alike by k_norm, after the bias and before the rotation.
+// The cos and sin of a row's angles are made once, in LDS (rows of more pairs: element by element).
+#define ROTARY_LDS_PAIRS 512
+template <typename T, bool NORM>
+__global__ __launch_bounds__(256) void rotary_cache_kernel(const float* __restrict__ proj, int64_t stride, int q_off, int k_off, int v_off,
                                     const float* __restrict__ bias,
                                     const int* __restrict__ positions, const float* __restrict__ inv_freq, int rot_dims,
                                     int interleaved, T* __restrict__ q_out, const int* __restrict__ slots,
                                     T* __restrict__ k_pages, T* __restrict__ v_pages, int q_heads, int kv_heads, int v_heads,
-                                    int dim, int vdim, int page_size, float q_coef, double q_every) {
+                                    int dim, int vdim, int page_size, float q_coef, double q_every,
+                                    const float* __restrict__ q_norm, const float* __restrict__ k_norm, float eps) {
+  __shared__ float cs_[ROTARY_LDS_PAIRS], sn_[ROTARY_LDS_PAIRS], scratch[16];
   const int64_t row = blockIdx.x;
   const float* pr = proj + row * stride;
   const float p = (float)positions[row];
@@ -356,6 +364,23 @@ __global__ void rotary_cache_kernel(const float* __restrict__ proj, int64_t stri
   const int64_t page = slot >= 0 ? slot / page_size : 0;
   const int off = slot >= 0 ? slot % page_size : 0;
   const int half = rot_dims / 2;
+  const bool in_lds = half <= ROTARY_LDS_PAIRS;
+  if (in_lds)
+    for (int i = threadIdx.x; i < half; i += blockDim.x) rotary_cos_sin(p, inv_freq[i], &cs_[i], &sn_[i]);
+  float rq = 1.f, rk = 1.f;
+  if (NORM) {
+    auto rms = [&](int off, int size) {
+      float ss = 0.f;
+      for (int i = threadIdx.x; i < size; i += blockDim.x) {
+        const float v = pr[off + i] + (bias != nullptr ? bias[off + i] : 0.f);
+        ss += v * v;
+      }
+      return 1.f / sqrtf(block_sum(ss, scratch) / (float)size + eps);
+    };
+    rq = rms(q_off, q_heads * dim);
+    if (kv_heads > 0) rk = rms(k_off, kv_heads * dim);
+  }
+  __syncthreads();
   // (a row of a step with few rows is shared by gridDim.y workgroups)
   const int at0 = blockIdx.y * blockDim.x + threadIdx.x, stride0 = gridDim.y * blockDim.x;
   for (int i = at0; i < (q_heads + kv_heads) * dim; i += stride0) {
@@ -364,15 +389,20 @@ __global__ void rotary_cache_kernel(const float* __restrict__ proj, int64_t stri
     const int64_t at = is_q ? q_off + (int64_t)h * dim : k_off + (int64_t)(h - q_heads) * dim;
     const float* src = pr + at;
     const float* bs = bias != nullptr ? bias + at : nullptr;
+    const float r = is_q ? rq : rk;
+    const float* nw = NORM ? (is_q ? q_norm + (int64_t)h * dim : k_norm + (int64_t)(h - q_heads) * dim) : nullptr;
     float y = src[c] + (bs != nullptr ? bs[c] : 0.f);
+    if (NORM) y = y * r * nw[c];
     if (c < rot_dims) {
       int pair, partner;
       bool first;
       if (interleaved) { pair = c >> 1; partner = c ^ 1; first = (c & 1) == 0; }
       else { first = c < half; pair = first ? c : c - half; partner = first ? c + half : c - half; }
       float cs, sn;
-      rotary_cos_sin(p, inv_freq[pair], &cs, &sn);
-      const float other = src[partner] + (bs != nullptr ? bs[partner] : 0.f);
+      if (in_lds) { cs = cs_[pair]; sn = sn_[pair]; }
+      else rotary_cos_sin(p, inv_freq[pair], &cs, &sn);
+      float other = src[partner] + (bs != nullptr ? bs[partner] : 0.f);
+      if (NORM) other = other * r * nw[partner];
       y = first ? y * cs - other * sn : y * cs + other * sn;
     }
     if (is_q) q_out[(row * q_heads + h) * dim + c] = from_f32<T>(y * q_temp);
@@ -519,7 +549,70 @@ __global__ void add_pair_into_stream_kernel(float* __restrict__ x, const float* 
   if (i < n) x[i] += a[i] + b[i];
 }
 
+// x += s1 a + s2 b + c, out = tanh(alpha x) w + o. a, b: [rows][stride], b and c may be nullptr, and a too (nothing is added
+// then); out may be nullptr (the sum alone). A thread four neighbours, or one (VEC 1).
+struct TanhArgs {
+  float* x; const float* a; int64_t a_stride; const float* b; int64_t b_stride;
+  const float* s1; const float* s2; const float* c;
+  const float* w; const float* o; float alpha;
+  int width;
+};
+template <typename T, int VEC, bool SUM>
+__global__ __launch_bounds__(256) void tanh_norm_stream_kernel(TanhArgs p, T* __restrict__ out) {
+  typedef float fv __attribute__((ext_vector_type(VEC)));
+  typedef T tv __attribute__((ext_vector_type(VEC)));
+  const int64_t row = blockIdx.x;
+  const int i = VEC * (blockIdx.y * 256 + threadIdx.x);
+  if (i >= p.width) return;
+  auto load = [&](const float* at) { return *reinterpret_cast<const fv*>(at); };
+  fv x = load(p.x + row * p.width + i);
+  if (SUM) {
+    fv add = load(p.a + row * p.a_stride + i);
+    if (p.s1 != nullptr) add *= load(p.s1 + i);
+    if (p.b != nullptr) {
+      fv more = load(p.b + row * p.b_stride + i);
+      if (p.s2 != nullptr) more *= load(p.s2 + i);
+      add += more;
+    }
+    if (p.c != nullptr) add += load(p.c + i);
+    x += add;
+    *reinterpret_cast<fv*>(p.x + row * p.width + i) = x;
+  }
+  if (out == nullptr) return;
+  const fv w = load(p.w + i), o = load(p.o + i);
+  tv y;
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) y[e] = from_f32<T>(fmaf(tanhf(p.alpha * x[e]), w[e], o[e]));
+  *reinterpret_cast<tv*>(out + row * p.width + i) = y;
+}
+
 extern "C" {
+
+int dli_tanh_norm_stream(float* x, const float* a, int64_t a_stride, const float* b, int64_t b_stride, const float* s1,
+                         const float* s2, const float* c, const float* w, const float* o, float alpha, void* out, int rows,
+                         int width, int is_bf16, hipStream_t stream) {
+  if (rows <= 0) return DLI_OK;
+  if (width <= 0 || (a != nullptr && a_stride < width) || (b != nullptr && (a == nullptr || b_stride < width)) ||
+      (out != nullptr && (w == nullptr || o == nullptr)))
+    return DLI_ERR_ARGUMENT;
+  TanhArgs p;
+  p.x = x; p.a = a; p.a_stride = a_stride; p.b = b; p.b_stride = b_stride; p.s1 = s1; p.s2 = s2; p.c = c; p.w = w; p.o = o;
+  p.alpha = alpha; p.width = width;
+  const bool four = width % 4 == 0 && a_stride % 4 == 0 && b_stride % 4 == 0 &&
+                    (((uintptr_t)x | (uintptr_t)a | (uintptr_t)b | (uintptr_t)s1 | (uintptr_t)s2 | (uintptr_t)c | (uintptr_t)w |
+                      (uintptr_t)o | (uintptr_t)out) % 16) == 0;
+  const dim3 grid(rows, four ? (width / 4 + 255) / 256 : (width + 255) / 256);
+  if (grid.y > 65535) return DLI_ERR_ARGUMENT;
+#define TANH_STREAM(T, VEC)                                                                                       \
+  do {                                                                                                            \
+    if (a != nullptr) tanh_norm_stream_kernel<T, VEC, true><<<grid, 256, 0, stream>>>(p, (T*)out);                \
+    else if (out != nullptr) tanh_norm_stream_kernel<T, VEC, false><<<grid, 256, 0, stream>>>(p, (T*)out);        \
+  } while (0)
+  if (is_bf16) { if (four) TANH_STREAM(bf16_t, 4); else TANH_STREAM(bf16_t, 1); }
+  else { if (four) TANH_STREAM(float, 4); else TANH_STREAM(float, 1); }
+#undef TANH_STREAM
+  return dli_launch_status();
+}
 
 int dli_embed_sinusoid(const void* table, const int* ids, const int* positions, const float* inv_freq, float* out,
                        void* rounded_bf16, int rows, int width, float scale, int is_bf16, hipStream_t stream) {
@@ -652,24 +745,23 @@ int dli_qk_unit_cache(const float* proj, int64_t stride, int q_off, int k_off, i
 int dli_rotary_cache(const float* proj, int64_t stride, int q_off, int k_off, int v_off, const float* bias,
                      const int* positions, const float* inv_freq, int rot_dims, int interleaved, void* q_out,
                      const int* slots, void* k_pages, void* v_pages, int rows, int q_heads, int kv_heads, int v_heads,
-                     int dim, int vdim, int page_size, float q_coef, double q_every, int is_bf16, hipStream_t stream) {
+                     int dim, int vdim, int page_size, float q_coef, double q_every, const float* q_norm, const float* k_norm,
+                     float eps, int is_bf16, hipStream_t stream) {
   if (rows <= 0) return DLI_OK;
   if (q_heads <= 0 || kv_heads < 0 || v_heads < 0 || dim <= 0 || vdim <= 0 || page_size <= 0 || rot_dims < 0 || !(q_every > 0.0) ||
-      rot_dims > dim || rot_dims % 2 || (rot_dims > 0 && inv_freq == nullptr) ||
+      rot_dims > dim || rot_dims % 2 || (rot_dims > 0 && inv_freq == nullptr) || (q_norm != nullptr && kv_heads > 0 && k_norm == nullptr) ||
       (kv_heads > 0 && (k_pages == nullptr || slots == nullptr)) || (v_heads > 0 && (v_pages == nullptr || slots == nullptr)))
     return DLI_ERR_ARGUMENT;
   const int64_t shares = ((int64_t)(q_heads + kv_heads) * dim + 511) / 512;
   const dim3 grid(rows, rows >= 128 ? 1 : (unsigned)(shares < 16 ? shares : 16));
-  if (is_bf16)
-    rotary_cache_kernel<bf16_t><<<grid, 256, 0, stream>>>(proj, stride, q_off, k_off, v_off, bias, positions, inv_freq,
-                                                          rot_dims, interleaved, (bf16_t*)q_out, slots, (bf16_t*)k_pages,
-                                                          (bf16_t*)v_pages, q_heads, kv_heads, v_heads, dim, vdim, page_size, q_coef,
-                                                          q_every);
-  else
-    rotary_cache_kernel<float><<<grid, 256, 0, stream>>>(proj, stride, q_off, k_off, v_off, bias, positions, inv_freq,
-                                                         rot_dims, interleaved, (float*)q_out, slots, (float*)k_pages,
-                                                         (float*)v_pages, q_heads, kv_heads, v_heads, dim, vdim, page_size, q_coef,
-                                                          q_every);
+#define ROTARY_CACHE(T, NORM)                                                                                             \
+  rotary_cache_kernel<T, NORM><<<grid, 256, 0, stream>>>(proj, stride, q_off, k_off, v_off, bias, positions, inv_freq,    \
+                                                         rot_dims, interleaved, (T*)q_out, slots, (T*)k_pages, (T*)v_pages, \
+                                                         q_heads, kv_heads, v_heads, dim, vdim, page_size, q_coef, q_every, \
+                                                         q_norm, k_norm, eps)
+  if (is_bf16) { if (q_norm != nullptr) ROTARY_CACHE(bf16_t, true); else ROTARY_CACHE(bf16_t, false); }
+  else { if (q_norm != nullptr) ROTARY_CACHE(float, true); else ROTARY_CACHE(float, false); }
+#undef ROTARY_CACHE
   return dli_launch_status();
 }
 

@@ -151,20 +151,23 @@ _SIGNATURES = {
                            _c_i64, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr,
                            _c_i64, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "dli_rotary_cache": [_c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr,
-                         _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, ctypes.c_double, _c_int, _c_ptr],
+                         _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, ctypes.c_double, _c_ptr, _c_ptr,
+                         _c_float, _c_int, _c_ptr],
     "dli_diff_head_norm": [_c_ptr, _c_i64, _c_float, _c_float, _c_float, _c_ptr, _c_i64, _c_ptr, _c_i64, _c_int, _c_int,
                            _c_int, _c_int, _c_ptr],
     "dli_branch_weighted_sum": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_ptr],
     "dli_scale_f32": [_c_ptr, _c_i64, _c_float, _c_ptr],
     "dli_silu_columns": [_c_ptr, _c_i64, _c_int, _c_int, _c_ptr],
     "dli_rms_norm_pair": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_float, _c_int, _c_ptr],
+    "dli_tanh_norm_stream": [_c_ptr, _c_ptr, _c_i64, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_float, _c_ptr,
+                             _c_int, _c_int, _c_int, _c_ptr],
     "dli_add_pair_into_stream": [_c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr],
     "dli_table_choose": [_c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr],
     "dli_exp_gates": [_c_ptr, _c_i64, _c_int, _c_int, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_i64, _c_i64, _c_ptr, _c_ptr,
                       _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr],
     "dli_scalar_gate_scan": [_c_ptr, _c_i64, _c_ptr, _c_i64, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr,
                              _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_int,
-                             _c_int, _c_float, _c_int, _c_int, _c_ptr],
+                             _c_int, _c_float, _c_int, _c_int, _c_int, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr],
     "dli_group_norm": [_c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_int, _c_ptr],
     "dli_branch_norm_mean": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_float, _c_ptr],
     "dli_head_norm_gate": [_c_ptr, _c_i64, _c_ptr, _c_i64, _c_ptr, _c_float, _c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_int,
@@ -175,12 +178,12 @@ _SIGNATURES = {
     "dli_gated_delta_scan": [_c_ptr, _c_i64, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_int,
                              _c_int, _c_int, _c_int, _c_ptr],
     "dli_poly_norm": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_float, _c_int, _c_ptr],
-    "dli_clamped_glu": [_c_ptr, _c_i64, _c_ptr, _c_int, _c_int, _c_float, _c_float, _c_float, _c_int, _c_ptr],
-    "dli_router_choose": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_ptr, _c_ptr,
-                          _c_ptr],
+    "dli_clamped_glu": [_c_ptr, _c_i64, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_int, _c_ptr],
+    "dli_router_choose": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int,
+                          _c_ptr, _c_ptr, _c_ptr],
     "dli_expert_tile_rows": [_c_int, _c_int, _c_int],
     "dli_expert_products": [_c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int,
-                            _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_int,
+                            _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_int,
                             _c_ptr],
     "dli_expert_combine": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_i64, _c_ptr, _c_i64, _c_ptr, _c_int, _c_int,
                            _c_int, _c_int, _c_int, _c_ptr],
@@ -537,13 +540,14 @@ def skinny_gemm(x: torch.Tensor, w: torch.Tensor, *, epilogue: int, out: Optiona
                 ssq_in: Optional[torch.Tensor] = None, stream: Optional[torch.Tensor] = None,
                 ssq_out: Optional[torch.Tensor] = None, shape: Optional[int] = None,
                 blocks4: Optional[int] = None, w_tiled: Optional[torch.Tensor] = None,
-                clamped: Optional[tuple] = None) -> Optional[torch.Tensor]:
+                clamped: Optional[tuple] = None, gelu: bool = False) -> Optional[torch.Tensor]:
     """``y = xhat @ w.T`` for at most 64 rows of bfloat16 ``x``, with fused surroundings.
 
     ``norm_w``/``eps``/``ssq_in [parts, rows]``: xhat is the RMSNorm of x, the row sums of squares
     being given in parts. Epilogues: ``SKINNY_STORE`` (``out`` bfloat16 ``[rows, n]``),
     ``SKINNY_SWIGLU`` (``w`` is ``[2n, k]``: gate rows then up rows; ``out [rows, n]`` gets
-    ``silu(gate) * up``, or with ``clamped = (limit, alpha, up_shift)`` what :func:`clamped_glu` computes),
+    ``silu(gate) * up``, or with ``clamped = (limit, alpha, up_shift)`` what :func:`clamped_glu` computes, or with ``gelu``
+    what :func:`gelu_glu` computes),
     ``SKINNY_RESIDUAL`` (``stream [rows, n]`` becomes ``stream + y`` in place;
     the parts of its row sums of squares are returned as ``[parts, rows]``, in ``ssq_out`` if that
     is given with the shape :func:`skinny_gemm_plan` names), ``SKINNY_F32`` (``out`` float32).
@@ -557,8 +561,9 @@ def skinny_gemm(x: torch.Tensor, w: torch.Tensor, *, epilogue: int, out: Optiona
     _require(w.shape[1] == k, "x and w differ in inner size")
     _require(skinny_gemm_supports(m, k, x.dtype), f"the decode product takes 1..64 rows and k % 32 == 0, not {m} x {k}")
     _require(x.stride(0) % 8 == 0 and x.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0, "operands must be 16-byte aligned")
-    _require(clamped is None or epilogue == SKINNY_SWIGLU, "a clamped activation belongs to the gated epilogue")
-    glu = (0, 0.0, 0.0, 0.0) if clamped is None else (1, *(float(c) for c in clamped))
+    _require((clamped is None and not gelu) or (epilogue == SKINNY_SWIGLU and not (gelu and clamped is not None)),
+             "another activation belongs to the gated epilogue")
+    glu = (2, 0.0, 0.0, 0.0) if gelu else (0, 0.0, 0.0, 0.0) if clamped is None else (1, *(float(c) for c in clamped))
     n = w.shape[0] // 2 if epilogue == SKINNY_SWIGLU else w.shape[0]
     up_offset = n if epilogue == SKINNY_SWIGLU else 0
     if epilogue == SKINNY_SWIGLU:
@@ -1854,7 +1859,8 @@ def recurrent_scan(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, w: torch.T
 def rotary_cache(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, positions: torch.Tensor,
                  inv_freq: Optional[torch.Tensor], rot_dims: int, interleaved: bool, q_out: torch.Tensor,
                  slots: Optional[torch.Tensor], k_pages: Optional[torch.Tensor], v_pages: Optional[torch.Tensor], q_heads: int,
-                 bias: Optional[torch.Tensor] = None, query_temperature: Optional[tuple] = None) -> None:
+                 bias: Optional[torch.Tensor] = None, query_temperature: Optional[tuple] = None,
+                 row_norm: Optional[tuple] = None) -> None:
     """From the float32 projections ``proj [n, >= ...]`` (q at ``q_off``, k at ``k_off``, v at ``v_off``):
     the first ``rot_dims`` components of every q and k head rotated by ``position * inv_freq[i]`` (pair
     ``i`` is ``(2i, 2i+1)`` where ``interleaved``, else ``(i, i + rot_dims/2)``; 32-bit angles),
@@ -1862,7 +1868,9 @@ def rotary_cache(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, positio
     value for every column of ``proj``) is added first. The value pages may hold fewer heads than the key
     pages, or be left out (``v_pages`` ``None``: the values are the keys); without key pages (``None``: the mixer reads
     another's) only q is made. ``query_temperature = (coef, every)``: q is also multiplied by
-    ``1 + coef ln(floor((position + 1) / every) + 1)``."""
+    ``1 + coef ln(floor((position + 1) / every) + 1)``. ``row_norm = (q_weight, k_weight, eps)``: after the bias and before the
+    rotation q is divided by its root mean square over all its heads at once and multiplied by ``q_weight``
+    (float32 ``[q_heads*dim]``), k alike by ``k_weight`` (``None`` without key pages)."""
     _f32_rows(proj, "proj")
     n = proj.shape[0]
     dtype = q_out.dtype
@@ -1897,10 +1905,17 @@ def rotary_cache(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, positio
         _require(inv_freq.shape[0] * 2 == rot_dims, "inv_freq must hold rot_dims/2 frequencies")
     coef, every = (0.0, 1.0) if query_temperature is None else (float(c) for c in query_temperature)
     _require(every > 0, "a temperature needs a positive period")
+    q_norm, k_norm, norm_eps = (None, None, 0.0) if row_norm is None else row_norm
+    if row_norm is not None:
+        for name, w, size in (("q_weight", q_norm, q_heads * dim), ("k_weight", k_norm, kv_heads * dim)):
+            if size:
+                _dense(w, name, torch.float32, 1)
+                _require(w.shape[0] == size, f"{name} must hold a value for every column it multiplies")
     _check(library().dli_rotary_cache(
         _ptr(proj), proj.stride(0), q_off, k_off, v_off, _ptr(bias), _ptr(positions), _ptr(inv_freq if rot_dims else None),
         int(rot_dims), int(bool(interleaved)), _ptr(q_out), _ptr(slots if k_pages is not None else None), _ptr(k_pages),
-        _ptr(v_pages), n, q_heads, kv_heads, v_heads, dim, vdim, page_size, coef, every, _is_bf16(dtype), _stream()), "rotary_cache")
+        _ptr(v_pages), n, q_heads, kv_heads, v_heads, dim, vdim, page_size, coef, every, _ptr(q_norm), _ptr(k_norm),
+        float(norm_eps), _is_bf16(dtype), _stream()), "rotary_cache")
 
 
 def group_norm(x: torch.Tensor, weight: torch.Tensor, groups: int, eps: float, out: torch.Tensor,
@@ -2004,14 +2019,15 @@ def gated_delta_scan(prep: torch.Tensor, state: torch.Tensor, q_start: torch.Ten
         _ptr(o), o.stride(0), entries, n, heads, kv_heads, dim, vdim, _stream()), "gated_delta_scan")
 
 
-HEAD_GATES = {"sigmoid": 0, "silu": 1, "none": 2}
+HEAD_GATES = {"sigmoid": 0, "silu": 1, "none": 2, "silu_first": 3}
 
 
 def head_norm_gate(o: torch.Tensor, g_pre: Optional[torch.Tensor], norm_w: torch.Tensor, eps: float, out: torch.Tensor,
                    heads: int, dim: int, gate: str = "silu", den: Optional[torch.Tensor] = None) -> None:
     """``out = o / sqrt(mean_head(o^2) + eps) * norm_w * gate(g_pre)`` head by head: ``o`` and ``g_pre`` float32
-    ``[n, heads*dim]`` (rows contiguous), ``norm_w`` float32 ``[heads*dim]``, ``gate`` ``"silu"``, ``"sigmoid"`` or
-    ``"none"`` (the per-head norm alone; ``g_pre`` is then ``None``)."""
+    ``[n, heads*dim]`` (rows contiguous), ``norm_w`` float32 ``[heads*dim]``, ``gate`` ``"silu"``, ``"sigmoid"``,
+    ``"none"`` (the per-head norm alone; ``g_pre`` is then ``None``) or ``"silu_first"``: ``o`` is multiplied by
+    ``silu(g_pre)`` and the norm is of that product."""
     _f32_rows(o, "o")
     _rows(out, "out", out.dtype)
     _dense(norm_w, "norm_w", torch.float32, 1)
@@ -2052,17 +2068,29 @@ def clamped_glu(gate_up: torch.Tensor, out: torch.Tensor, limit: float, alpha: f
     _dense(out, "out", ndim=2)
     n, ff = out.shape
     _require(gate_up.shape[0] == n and gate_up.shape[1] >= 2 * ff, "gate_up must hold gate and up for every row")
-    _check(library().dli_clamped_glu(_ptr(gate_up), gate_up.stride(0), _ptr(out), n, ff, float(limit), float(alpha),
+    _check(library().dli_clamped_glu(_ptr(gate_up), gate_up.stride(0), _ptr(out), n, ff, 1, float(limit), float(alpha),
                                      float(up_shift), _is_bf16(out.dtype), _stream()), "clamped_glu")
 
 
+def gelu_glu(gate_up: torch.Tensor, out: torch.Tensor) -> None:
+    """``out = gelu(gate) * up``, gelu in its tanh form; operands as :func:`clamped_glu` takes them."""
+    _rows(gate_up, "gate_up", out.dtype)
+    _dense(out, "out", ndim=2)
+    n, ff = out.shape
+    _require(gate_up.shape[0] == n and gate_up.shape[1] >= 2 * ff, "gate_up must hold gate and up for every row")
+    _check(library().dli_clamped_glu(_ptr(gate_up), gate_up.stride(0), _ptr(out), n, ff, 2, 0.0, 0.0, 0.0, _is_bf16(out.dtype),
+                                     _stream()), "gelu_glu")
+
+
 def router_choose(logits: torch.Tensor, total: int, correction: Optional[torch.Tensor], groups: int, keep: int, top: int,
-                  scale: float, ids: torch.Tensor, weights: torch.Tensor, bias: Optional[torch.Tensor] = None) -> None:
+                  scale: float, ids: torch.Tensor, weights: torch.Tensor, bias: Optional[torch.Tensor] = None,
+                  sigmoid: bool = False, normalize: bool = True) -> None:
     """The router's choice per row of float32 ``logits [n, >= total]``: scores ``softmax`` over the first
     ``total`` columns (plus ``bias``, float32 ``[total]``, where the router has one); choice scores add ``correction``; with ``groups`` > 1 only the ``keep`` groups of
     neighbours with the largest best choice score can be chosen; ``ids [n, top]`` int32 are the largest
     choice scores (lowest index on a tie), ``weights [n, top]`` their scores (without correction) divided
-    by their sum + 1e-20, times ``scale``."""
+    by their sum + 1e-20, times ``scale``. ``sigmoid``: the scores are each output's sigmoid instead; ``normalize=False``: the
+    weights are the scores times ``scale``, not divided by their sum."""
     _f32_rows(logits, "logits")
     n = logits.shape[0]
     _require(logits.shape[1] >= total, "logits must hold every router output")
@@ -2078,16 +2106,19 @@ def router_choose(logits: torch.Tensor, total: int, correction: Optional[torch.T
     _require(1 <= top <= min(total, 64) and groups >= 1 and total % groups == 0 and 1 <= keep <= groups
              and keep * (total // groups) >= top, "the router's sizes do not fit each other")
     _check(library().dli_router_choose(_ptr(logits), logits.stride(0), _ptr(bias), _ptr(correction), n, int(total), int(groups),
-                                       int(keep), int(top), float(scale), _ptr(ids), _ptr(weights), _stream()),
+                                       int(keep), int(top), float(scale), int(bool(sigmoid)), int(bool(normalize)), _ptr(ids),
+                                       _ptr(weights), _stream()),
            "router_choose")
 
 
 def expert_products(ids: torch.Tensor, h: torch.Tensor, w_gate: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor,
-                    limit: float, alpha: float, up_shift: float = 1.0) -> torch.Tensor:
+                    limit: float, alpha: float, up_shift: float = 1.0,
+                    in_weights: Optional[torch.Tensor] = None) -> torch.Tensor:
     """The chosen experts' results for every (token, choice): ``z [n * top, width]`` float32, row
     ``t * top + j`` holding ``w_down[e] clamped_glu(w_gate[e] h_t, w_up[e] h_t)`` for ``e = ids[t, j]`` (rows of
     ids at or above the number of experts are left unwritten). ``w_gate, w_up [experts, ff, width]``,
-    ``w_down [experts, width, ff]`` of ``h``'s type. Nothing here waits for the device: the rows are
+    ``w_down [experts, width, ff]`` of ``h``'s type. ``in_weights`` (float32 ``[n, top]``): what each choice's input ``h_t`` is
+    multiplied by (the products being linear, their 32-bit sums are). Nothing here waits for the device: the rows are
     sorted by expert and cut into tiles on the device."""
     _dense(ids, "ids", torch.int32, 2)
     n, top = ids.shape
@@ -2097,6 +2128,9 @@ def expert_products(ids: torch.Tensor, h: torch.Tensor, w_gate: torch.Tensor, w_
     experts, ff, width = w_gate.shape
     _require(w_up.shape == w_gate.shape and w_down.shape == (experts, width, ff) and h.shape == (n, width),
              "h [n, width], w_gate/w_up [experts, ff, width], w_down [experts, width, ff] do not fit")
+    if in_weights is not None:
+        _dense(in_weights, "in_weights", torch.float32, 2)
+        _require(in_weights.shape == (n, top), "in_weights must be [n, top]")
     slots = n * top
     tile_rows = int(library().dli_expert_tile_rows(width, ff, _is_bf16(h.dtype)))
     max_tiles = max(1, min(slots, slots // tile_rows + experts))
@@ -2108,24 +2142,25 @@ def expert_products(ids: torch.Tensor, h: torch.Tensor, w_gate: torch.Tensor, w_
     z = torch.empty(slots, width, device=h.device, dtype=torch.float32)
     _check(library().dli_expert_products(
         _ptr(ids), _ptr(h), h.stride(0), _ptr(w_gate), _ptr(w_up), _ptr(w_down), _ptr(offsets), _ptr(order),
-        _ptr(tile_expert), _ptr(tile_row0), _ptr(tile_count), max_tiles, _ptr(y), _ptr(z), n, top, experts, width, ff,
+        _ptr(tile_expert), _ptr(tile_row0), _ptr(tile_count), max_tiles, _ptr(y), _ptr(z), _ptr(in_weights), n, top, experts, width, ff,
         float(limit), float(alpha), float(up_shift), _is_bf16(h.dtype), _stream()), "expert_products")
     return z
 
 
-def expert_combine(ids: torch.Tensor, weights: torch.Tensor, z: Optional[torch.Tensor], h: torch.Tensor, experts: int,
+def expert_combine(ids: torch.Tensor, weights: Optional[torch.Tensor], z: Optional[torch.Tensor], h: torch.Tensor, experts: int,
                    out: torch.Tensor, shared: Optional[torch.Tensor] = None,
                    shared_gate: Optional[torch.Tensor] = None) -> None:
     """``out[t] = sum_j weights[t, j] * (z[t * top + j] if ids[t, j] < experts else h[t])
-    + sigmoid(shared_gate[t]) * shared[t]``; ``out`` float32 ``[n, width]``, ``shared`` float32 ``[n, width]``
+    + sigmoid(shared_gate[t]) * shared[t]`` (``weights`` ``None``: ones); ``out`` float32 ``[n, width]``, ``shared`` float32 ``[n, width]``
     and ``shared_gate`` float32 ``[n, 1]`` (a column of a wider matrix will do), both optional."""
     _dense(ids, "ids", torch.int32, 2)
-    _dense(weights, "weights", torch.float32, 2)
     n, top = ids.shape
+    if weights is not None:
+        _dense(weights, "weights", torch.float32, 2)
     _rows(h, "h", h.dtype)
     _dense(out, "out", torch.float32, 2)
     width = out.shape[1]
-    _require(weights.shape == (n, top) and h.shape == (n, width) and out.shape[0] == n, "ids, weights, h and out disagree")
+    _require((weights is None or weights.shape == (n, top)) and h.shape == (n, width) and out.shape[0] == n, "ids, weights, h and out disagree")
     if z is not None:
         _dense(z, "z", torch.float32, 2)
         _require(z.shape == (n * top, width), "z must be [n * top, width]")
@@ -2389,7 +2424,9 @@ def scalar_gate_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: t
                      keep: Optional[torch.Tensor] = None, write: Optional[torch.Tensor] = None,
                      decay: Optional[torch.Tensor] = None, floor: Optional[torch.Tensor] = None,
                      den: Optional[torch.Tensor] = None, q_scale: float = 1.0, silu: bool = False,
-                     log_keep: Optional[torch.Tensor] = None, chunked: bool = True) -> None:
+                     log_keep: Optional[torch.Tensor] = None, chunked: bool = True, qk_heads: Optional[int] = None,
+                     step: Optional[torch.Tensor] = None, step_bias: Optional[torch.Tensor] = None,
+                     step_rate: Optional[torch.Tensor] = None, skip: Optional[torch.Tensor] = None) -> None:
     """Per request and head ``S <- a S + b k v^T``, ``o = S^T q`` over the step's rows in order, with
     ``a, b = keep, write`` (float32 ``[n, heads]``) or ``a = decay[head]``, ``b = 1``. ``q, k [n, heads*dim]`` and
     ``v [n, heads*vdim]`` are float32 with contiguous rows (columns of a wider matrix will do); with ``silu`` all
@@ -2398,13 +2435,29 @@ def scalar_gate_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: t
     ``max(|that column's result|, floor) + 1e-6``. ``S`` float32 ``[heads][vdim (+ 1)][dim]`` at the start of
     ``state[slot]`` (zeros at position 0); ``o [n, heads*vdim]`` float32. A step with portions whose heads hold 16 to 64
     keys in steps of 16 runs 64 tokens at a time on the matrix cores, in 32-bit (``chunked``; under gates it needs
-    ``log_keep``, the logarithm of ``keep``; not with ``silu``); any other walks the tokens one by one."""
-    for name, t, width in (("q", q, heads * dim), ("k", k, heads * dim), ("v", v, heads * vdim), ("o", o, heads * vdim)):
+    ``log_keep``, the logarithm of ``keep``; not with ``silu``); any other walks the tokens one by one.
+
+    ``qk_heads``: q and k hold that many heads, each shared by ``heads / qk_heads`` neighbours. ``step`` (float32 ``[n, heads]``,
+    columns of a wider matrix will do) instead of factors: ``b = softplus(step + step_bias)``, ``a = exp(-exp(step_rate) b)``
+    (float32 ``[heads]`` each), and ``o`` gets ``skip * v`` on top (float32 ``[heads]``; ``None``: nothing)."""
+    qk_heads = heads if qk_heads is None else int(qk_heads)
+    _require(qk_heads > 0 and heads % qk_heads == 0, "the heads do not group onto qk_heads")
+    for name, t, width in (("q", q, qk_heads * dim), ("k", k, qk_heads * dim), ("v", v, heads * vdim), ("o", o, heads * vdim)):
         _f32_rows(t, name)
         _require(t.shape[1] == width, f"{name} must hold {width} columns")
     n = q.shape[0]
     _require(k.shape[0] == n and v.shape[0] == n and o.shape[0] == n, "q, k, v and o differ in rows")
-    _require((keep is None) == (write is None) and (keep is not None or decay is not None), "keep and write, or decay")
+    _require((keep is None) == (write is None) and sum(t is not None for t in (keep, decay, step)) == 1,
+             "keep and write, or decay, or step")
+    _require((step is not None) == (step_bias is not None) == (step_rate is not None) and (skip is None or step is not None)
+             and not (step is not None and silu), "a step size comes with its bias and rate, skip with a step size, silu without")
+    if step is not None:
+        _f32_rows(step, "step")
+        _require(step.shape == (n, heads), "step must be [n, heads]")
+    for name, t in (("step_bias", step_bias), ("step_rate", step_rate), ("skip", skip)):
+        if t is not None:
+            _dense(t, name, torch.float32, 1)
+            _require(t.shape[0] == heads, f"{name} must hold a value per head")
     _require((floor is None) == (den is None) and (floor is None or keep is not None), "floor and den come with the gates")
     for name, t in (("keep", keep), ("write", write), ("floor", floor), ("den", den), ("log_keep", log_keep)):
         if t is not None:
@@ -2418,7 +2471,8 @@ def scalar_gate_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: t
     _check(library().dli_scalar_gate_scan(
         _ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(v), v.stride(0), _ptr(keep), _ptr(write), _ptr(log_keep), heads,
         _ptr(decay), _ptr(floor), _ptr(den), _ptr(state), state.stride(0), _ptr(q_start), _ptr(positions), _ptr(state_slots),
-        _ptr(o), o.stride(0), entries, n, heads, dim, vdim, float(q_scale), int(bool(silu)), int(bool(chunked)), _stream()),
+        _ptr(o), o.stride(0), entries, n, heads, dim, vdim, float(q_scale), int(bool(silu)), int(bool(chunked)),
+        qk_heads, _ptr(step), 0 if step is None else step.stride(0), _ptr(step_bias), _ptr(step_rate), _ptr(skip), _stream()),
         "scalar_gate_scan")
 
 
@@ -2493,6 +2547,38 @@ def add_pair_into_stream(x: torch.Tensor, a: torch.Tensor, b: torch.Tensor) -> N
         _dense(t, name, torch.float32, 2)
     _require(a.shape == x.shape and b.shape == x.shape, "a and b differ from x in shape")
     _check(library().dli_add_pair_into_stream(_ptr(x), _ptr(a), _ptr(b), x.numel(), _stream()), "add_pair_into_stream")
+
+
+def tanh_norm_stream(x: torch.Tensor, *, a: Optional[torch.Tensor] = None, b: Optional[torch.Tensor] = None,
+                     a_scale: Optional[torch.Tensor] = None, b_scale: Optional[torch.Tensor] = None,
+                     constant: Optional[torch.Tensor] = None, norm: Optional[tuple] = None,
+                     out: Optional[torch.Tensor] = None) -> None:
+    """``x += a_scale * a + b_scale * b + constant`` in place (float32 ``[n, width]``; the scales and the constant float32
+    ``[width]``; ``b``, a scale, the constant or all summands may be left out), and with ``norm = (alpha, weight, offset)``
+    ``out = tanh(alpha x) * weight + offset`` of the new ``x`` in the same pass (``out`` float32 or bfloat16)."""
+    _dense(x, "x", torch.float32, 2)
+    n, width = x.shape
+    _require(a is not None or (b is None and a_scale is None and constant is None), "summands begin with a")
+    _require(b is not None or b_scale is None, "b_scale comes with b")
+    for name, t in (("a", a), ("b", b)):
+        if t is not None:
+            _f32_rows(t, name)
+            _require(t.shape == x.shape, f"{name} differs from x in shape")
+    _require((norm is None) == (out is None), "norm and out come together")
+    alpha, w, o = norm if norm is not None else (0.0, None, None)
+    for name, t in (("a_scale", a_scale), ("b_scale", b_scale), ("constant", constant), ("weight", w), ("offset", o)):
+        if t is not None:
+            _dense(t, name, torch.float32, 1)
+            _require(t.shape[0] == width, f"{name} must hold a value per column")
+    bf16 = 0
+    if out is not None:
+        _require(w is not None and o is not None, "a tanh norm has a weight and an offset")
+        _dense(out, "out", ndim=2)
+        _require(out.shape == x.shape, "out differs from x in shape")
+        bf16 = _is_bf16(out.dtype)
+    _check(library().dli_tanh_norm_stream(
+        _ptr(x), _ptr(a), 0 if a is None else a.stride(0), _ptr(b), 0 if b is None else b.stride(0), _ptr(a_scale), _ptr(b_scale),
+        _ptr(constant), _ptr(w), _ptr(o), float(alpha), _ptr(out), n, width, bf16, _stream()), "tanh_norm_stream")
 
 
 def silu_columns(x: torch.Tensor) -> None:

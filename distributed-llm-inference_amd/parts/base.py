@@ -126,7 +126,10 @@ class DecodeStream:
 
 
 def norm_key(norm: Any) -> Optional[tuple]:
-    """What identifies a norm for :class:`DecodeStream`: its weight's address and its eps."""
+    """What identifies a norm for :class:`DecodeStream` and ``NormedStream``: its weight's address and its eps, or what the
+    norm itself answers (``stream_key()``)."""
+    if norm is not None and hasattr(norm, "stream_key"):
+        return norm.stream_key()
     if norm is None or not hasattr(norm, "fused_params"):
         return None
     w, eps = norm.fused_params()
@@ -151,6 +154,10 @@ class Part:
         or ``None`` (the default) for a part that this route does not cover; the step then runs
         part by part."""
         return None
+
+    # A bias that this part leaves out of its result because whoever adds the result into the stream adds it as well
+    # (set only where the part was built for such a block; None: the result is complete).
+    output_bias: Optional[torch.Tensor] = None
 
     def load_weights(self, tensors: Mapping[str, torch.Tensor]) -> None:
         """Receive the tensors of :meth:`weight_specs`, already on the device and typed by role."""
@@ -294,6 +301,10 @@ class Block(Part):
     def forward(self, x: torch.Tensor, delta: Optional[torch.Tensor], ctx: Any, cache: Any,
                 parts: Mapping[str, Part]) -> tuple[torch.Tensor, Optional[torch.Tensor]]:
         raise NotImplementedError
+
+    def bind_parts(self, parts: Mapping[str, Part]) -> None:
+        """Called once after the weights of all parts are loaded and finalized: what the arrangement derives from its
+        parts' tensors (default: nothing)."""
 
     def native_fields(self, parts: Mapping[str, Part]) -> Optional[dict]:  # type: ignore[override]
         """This arrangement with its parts' tensors and constants, for the loop in C that issues a

@@ -214,6 +214,72 @@ class ParallelNormsBlock(Block):
         return x, None
 
 
+@register_part("block", "parallel_scaled")
+class ParallelScaledBlock(Block):
+    """Mixer and feed-forward side by side behind one norm, each result multiplied by a vector of its own:
+    ``x <- x + (s1 * mixer(h) + s2 * feed_forward(h))``, ``h = norm(x)``, around a 32-bit residual stream. ``scales``: role ->
+    the name of its vector below this block's prefix (a role left out: ones). The feed-forward may be absent. ``x`` is
+    float32 in both runtimes. A part that leaves its output bias to the block (``output_bias``) has it added here, inside the
+    same 32-bit sum. Where the norm that the stream meets next works element by element (``tanh_params``), the
+    kernel that makes the sums applies it too."""
+
+    roles = ("norm", "mixer")   # and, unless the layer has no feed-forward, "feed_forward"
+    takes_following = True
+
+    def __init__(self, runtime: Runtime, *, hidden_size: int, scales: Optional[Mapping[str, str]] = None) -> None:
+        super().__init__(runtime)
+        self.hidden_size, self.scale_names = hidden_size, dict(scales or {})
+        if any(role not in ("mixer", "feed_forward") for role in self.scale_names):
+            raise ValueError("parallel_scaled multiplies the results of the mixer and the feed-forward")
+        self.scales: dict[str, torch.Tensor] = {}
+        self.constant: Optional[torch.Tensor] = None      # what the parts' output biases add up to
+
+    def graph_capturable(self, page_size: int) -> bool:
+        return True  # kernels on device arrays only
+
+    def weight_specs(self) -> dict:
+        from .spec import WeightSpec
+
+        return {name: WeightSpec((self.hidden_size,), role="float32", init="norm") for name in self.scale_names.values()}
+
+    def load_weights(self, tensors: Mapping[str, torch.Tensor]) -> None:
+        self.scales = {role: tensors[name].contiguous() for role, name in self.scale_names.items()}
+
+    def first_norm(self, parts: Mapping[str, Part]) -> Optional[Part]:
+        return parts["norm"]
+
+    def bind_parts(self, parts: Mapping[str, Part]) -> None:
+        """``constant = sum_role s_role * bias_role`` over the parts that leave their output bias to this block, in 32-bit."""
+        self.constant = None
+        for role in ("mixer", "feed_forward"):
+            b = parts[role].output_bias if role in parts else None
+            if b is not None:
+                term = b.float() * self.scales[role] if role in self.scales else b.float()
+                self.constant = term.contiguous() if self.constant is None else (self.constant + term).contiguous()
+
+    def forward(self, x: torch.Tensor, delta: Optional[torch.Tensor], ctx: Any, cache: Any, parts: Mapping[str, Part],
+                following: Optional[Part] = None) -> tuple[torch.Tensor, Optional[torch.Tensor]]:
+        from ..kernels import ops
+
+        if x.dtype != torch.float32:
+            raise RuntimeError("the parallel_scaled block keeps a float32 residual stream")
+        if delta is not None:
+            ops.add(x, delta, x)
+            NormedStream.offer(ctx, x, None, None)
+        h = NormedStream.take(ctx, x, parts["norm"])
+        if h is None:
+            h = parts["norm"].forward(x)
+        y = _as_f32(parts["mixer"].forward(h, ctx, cache))
+        f = _as_f32(parts["feed_forward"].forward(h, ctx)) if "feed_forward" in parts else None
+        fused = following is not None and hasattr(following, "tanh_params")
+        out = self.rt.empty(*x.shape) if fused else None
+        ops.tanh_norm_stream(x, a=y, b=f, a_scale=self.scales.get("mixer"),
+                             b_scale=self.scales.get("feed_forward") if f is not None else None, constant=self.constant,
+                             norm=following.tanh_params() if fused else None, out=out)
+        NormedStream.offer(ctx, x, following if fused else None, out)
+        return x, None
+
+
 @register_part("block", "sandwich_norms")
 class SandwichNormsBlock(Block):
     """A norm before and a norm after every sublayer, around a 32-bit residual stream:

@@ -1,12 +1,13 @@
 """A mixture of small feed-forward experts behind a router.
 
 Router: ``z = W_router h`` (``+ b_router`` with ``router_bias``) in 32-bit over ``experts + identity`` outputs, scores
-``s = softmax(z)``. The
+``s = softmax(z)`` (or ``scoring="sigmoid"``: each output's sigmoid). The
 choice scores add a per-output ``correction`` (the weights do not). The outputs form ``groups`` equal
 groups of neighbours; a group's score is its largest choice score, and only outputs of the best
 ``groups_kept`` groups can be chosen. The ``top`` largest choice scores are chosen; their weights are
 their scores ``s`` divided by their sum (+ 1e-20), times ``scale`` (with ``scale = 1`` and without correction and
-groups that is the softmax over the chosen logits alone). The last ``identity`` outputs are
+groups that is the softmax over the chosen logits alone); with ``normalize=False`` they are the scores times ``scale`` as they
+are. A weight multiplies its expert's result, or with ``weight_input`` the expert's input: ``expert(w h)``. The last ``identity`` outputs are
 identity experts: their result is the input itself; they have no tensors.
 
 Expert ``e`` (tensors ``e<e>.gate``, ``e<e>.up``, ``e<e>.down``, no biases): ``g = min(W_gate h, limit)``,
@@ -44,8 +45,13 @@ class RoutedExperts(FeedForward):
                  limit: float, alpha: float = 1.702, identity: int = 0, groups: int = 1, groups_kept: int = 1,
                  scale: float = 1.0, correction: bool = True, shared_size: int = 0, shared_limit: float = 0.0,
                  shared_gate: bool = True, up_shift: float = 1.0, router_bias: bool = False, routing: str = "router",
-                 vocab_size: int = 0) -> None:
+                 vocab_size: int = 0, scoring: str = "softmax", normalize: bool = True, weight_input: bool = False) -> None:
         super().__init__(runtime)
+        if scoring not in ("softmax", "sigmoid"):
+            raise ValueError(f"scoring must be 'softmax' or 'sigmoid', not {scoring!r}")
+        if weight_input and identity:
+            raise ValueError("weights on the inputs of experts that are the identity have no kernel")
+        self.scoring, self.normalize, self.weight_input = scoring, bool(normalize), bool(weight_input)
         if routing not in ("router", "table"):
             raise ValueError(f"routing must be 'router' or 'table', not {routing!r}")
         if routing == "table" and (identity or vocab_size < 1 or shared_gate and shared_size):
@@ -118,10 +124,11 @@ class RoutedExperts(FeedForward):
         else:
             logits = linear_f32(self.rt, x, self.w_router)
             ops.router_choose(logits, self.total, self.correction, self.groups, self.groups_kept, self.top, self.scale, ids,
-                              weights, bias=self.router_bias)
+                              weights, bias=self.router_bias, sigmoid=self.scoring == "sigmoid", normalize=self.normalize)
         z = None
         if self.experts:
-            z = ops.expert_products(ids, x, self.w_gate, self.w_up, self.w_down, self.limit, self.alpha, self.up_shift)
+            z = ops.expert_products(ids, x, self.w_gate, self.w_up, self.w_down, self.limit, self.alpha, self.up_shift,
+                                    in_weights=weights if self.weight_input else None)
         shared = gate = None
         if self.shared_size:
             gate_up = linear(self.rt, x, self.ws_gate_up)
@@ -131,5 +138,5 @@ class RoutedExperts(FeedForward):
             if self.shared_gate:
                 gate = logits[:, self.total:self.total + 1]
         out = torch.empty(n, self.hidden_size, device=dev, dtype=torch.float32)
-        ops.expert_combine(ids, weights, z, x, self.experts, out, shared=shared, shared_gate=gate)
+        ops.expert_combine(ids, None if self.weight_input else weights, z, x, self.experts, out, shared=shared, shared_gate=gate)
         return out

@@ -1,6 +1,7 @@
 """Gated feed-forward: ``down(act(gate(x)) * up(x))`` with ``act = silu`` (SwiGLU; reference:
 src/dli/model/llama.py:180-191), or ``down(g sigmoid(alpha g) (u + up_shift))`` with clamped halves
-``g = min(gate(x), limit)``, ``u = clamp(up(x), -limit, limit)`` (``activation="clamped"``). Gate and up matrices are stacked at load, so one product gives
+``g = min(gate(x), limit)``, ``u = clamp(up(x), -limit, limit)`` (``activation="clamped"``), or with the gate's gelu in its tanh form
+(``activation="gelu_tanh"``). Gate and up matrices are stacked at load, so one product gives
 both halves; the activation kernel reads them side by side."""
 
 from __future__ import annotations
@@ -19,25 +20,32 @@ from .spec import WeightSpec
 @register_part("feed_forward", "gated_mlp")
 class GatedMLP(FeedForward):
     NAMES = {"gate": "gate_proj.weight", "up": "up_proj.weight", "down": "down_proj.weight"}
+    BIAS_NAMES = {"gate": "gate_proj.bias", "up": "up_proj.bias", "down": "down_proj.bias"}
+    ACTIVATIONS = ("silu", "clamped", "gelu_tanh")
 
     def __init__(self, runtime: Runtime, *, hidden_size: int, intermediate_size: int,
                  activation: str = "silu", bias: bool = False, names: Optional[Mapping[str, str]] = None,
                  few_rows_fused: bool = False, limit: float = float("inf"), alpha: float = 1.0, up_shift: float = 0.0,
-                 float32_out: bool = False) -> None:
+                 float32_out: bool = False, bias_names: Optional[Mapping[str, str]] = None, defer_output_bias: bool = False) -> None:
         """``limit``, ``alpha``, ``up_shift``: of the clamped activation. ``float32_out``: the result is the second product's
-        32-bit sums (for a norm or a residual stream that is 32-bit)."""
+        32-bit sums (for a norm or a residual stream that is 32-bit). ``defer_output_bias``: the second product's bias is
+        left to the block (``output_bias``)."""
         super().__init__(runtime)
         # forward() itself takes the few-row kernels (SwiGLU inside the first product) for up to 16
         # rows: for blocks that have no fused decode path of their own
         self.few_rows_fused = bool(few_rows_fused)
         # checkpoint names of the three matrices below the part's prefix, where they are not the usual ones
         self.names = {**self.NAMES, **dict(names or {})}
-        if bias and names:
-            raise ValueError("gated_mlp: other tensor names are taken for the matrices only")
-        if activation not in ("silu", "clamped"):
-            raise ValueError(f"gated_mlp has no kernel for activation {activation!r} (only 'silu' and 'clamped')")
-        if bias and (activation != "silu" or float32_out):
-            raise ValueError("gated_mlp: biases go with the plain activation and a result of the runtime's type")
+        self.bias_names = {**self.BIAS_NAMES, **dict(bias_names or {})}
+        if bias and bool(names) != bool(bias_names):
+            raise ValueError("gated_mlp: other tensor names are taken for the matrices and the biases alike")
+        if activation not in self.ACTIVATIONS:
+            raise ValueError(f"gated_mlp has no kernel for activation {activation!r} (only {', '.join(self.ACTIVATIONS)})")
+        if bias and activation == "clamped":
+            raise ValueError("gated_mlp: the clamped activation takes no biases")
+        if defer_output_bias and not (bias and float32_out):
+            raise ValueError("gated_mlp: a bias that the block adds belongs to a 32-bit result with biases")
+        self.activation, self.defer_output_bias = activation, bool(defer_output_bias)
         self.clamped = (float(limit), float(alpha), float(up_shift)) if activation == "clamped" else None
         self.float32_out = bool(float32_out)
         self.hidden_size, self.intermediate_size, self.bias = hidden_size, intermediate_size, bias
@@ -52,16 +60,19 @@ class GatedMLP(FeedForward):
         specs = {self.names["gate"]: WeightSpec((i, h)), self.names["up"]: WeightSpec((i, h)),
                  self.names["down"]: WeightSpec((h, i))}
         if self.bias:
-            specs.update({"gate_proj.bias": WeightSpec((i,)), "up_proj.bias": WeightSpec((i,)),
-                          "down_proj.bias": WeightSpec((h,))})
+            n = self.bias_names
+            specs.update({n["gate"]: WeightSpec((i,)), n["up"]: WeightSpec((i,)), n["down"]: WeightSpec((h,))})
         return specs
 
     def load_weights(self, tensors: Mapping[str, torch.Tensor]) -> None:
         self.w_gate_up = torch.cat([tensors[self.names["gate"]], tensors[self.names["up"]]], 0).contiguous()
         self.w_down = tensors[self.names["down"]]
         if self.bias:
-            self.b_gate_up = torch.cat([tensors["gate_proj.bias"], tensors["up_proj.bias"]], 0).contiguous()
-            self.b_down = tensors["down_proj.bias"]
+            n = self.bias_names
+            self.b_gate_up = torch.cat([tensors[n["gate"]], tensors[n["up"]]], 0).contiguous()
+            self.b_down = tensors[n["down"]].contiguous()
+            if self.defer_output_bias:
+                self.output_bias, self.b_down = self.b_down, None
 
     def finalize(self) -> None:
         self.w_gate_up_tiled = decode_copy(self.rt, self.w_gate_up, ops.SKINNY_SWIGLU)
@@ -71,7 +82,7 @@ class GatedMLP(FeedForward):
         from .native import _bf16_matrix, _bf16_vector
 
         h, i = self.hidden_size, self.intermediate_size
-        if type(self) is not GatedMLP or self.clamped is not None or self.float32_out:
+        if type(self) is not GatedMLP or self.activation != "silu" or self.float32_out:
             return None  # a subclass computes something else: it must describe itself
         if not (self.rt.is_bf16 and _bf16_matrix(self.w_gate_up, 2 * i, h) and _bf16_matrix(self.w_down, h, i)
                 and _bf16_vector(self.b_gate_up, 2 * i) and _bf16_vector(self.b_down, h)):
@@ -92,7 +103,7 @@ class GatedMLP(FeedForward):
             # a few rows outside the fused decode path (a block that keeps its stream in 32-bit, say):
             # the few-row products, the activation inside the first
             ops.skinny_gemm(x, self.w_gate_up, w_tiled=self.w_gate_up_tiled, epilogue=ops.SKINNY_SWIGLU, out=act,
-                            bias=self.b_gate_up, clamped=self.clamped)
+                            bias=self.b_gate_up, clamped=self.clamped, gelu=self.activation == "gelu_tanh")
             out = torch.empty(n, self.hidden_size, device=self.rt.device,
                               dtype=torch.float32 if self.float32_out else self.rt.dtype)
             ops.skinny_gemm(act, self.w_down, w_tiled=self.w_down_tiled, bias=self.b_down, out=out,
@@ -101,17 +112,19 @@ class GatedMLP(FeedForward):
         gate_up = linear(self.rt, x, self.w_gate_up, self.b_gate_up)
         if self.clamped is not None:
             ops.clamped_glu(gate_up, act, *self.clamped)
+        elif self.activation == "gelu_tanh":
+            ops.gelu_glu(gate_up, act)
         else:
             ops.silu_mul(gate_up, act)
         if self.float32_out:
-            return linear_f32(self.rt, act, self.w_down)
+            return linear_f32(self.rt, act, self.w_down, bias=self.b_down)
         return linear(self.rt, act, self.w_down, self.b_down)
 
     FEW_ROWS = 16  # the few-row product kernels; 17 to 64 rows take the one that shares activations
 
     def streams(self, ctx: Any) -> bool:
         n = ctx.num_tokens
-        if self.clamped is not None or self.float32_out or not (self.rt.is_bf16 and self.hidden_size % 8 == 0):
+        if self.activation != "silu" or self.float32_out or not (self.rt.is_bf16 and self.hidden_size % 8 == 0):
             return False
         if n > self.FEW_ROWS:
             return (self.w_gate_up_tiled is not None and self.w_down_tiled is not None

@@ -155,10 +155,18 @@ def as_operand(rt: Runtime, x: torch.Tensor, ctx=None) -> torch.Tensor:
 F32_FEW_ROWS = 16  # up to here the few-row product streams the weights faster than the library does
 
 
-def linear_f32(rt: Runtime, x: torch.Tensor, weight: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """``x [n, k] @ weight[m, k].T -> float32 [n, m]``: the 32-bit sums of the product as they are,
+def linear_f32(rt: Runtime, x: torch.Tensor, weight: torch.Tensor, out: Optional[torch.Tensor] = None,
+               bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``x [n, k] @ weight[m, k].T (+ bias) -> float32 [n, m]``: the 32-bit sums of the product as they are,
     for what is computed in 32-bit after a projection (recurrences, norms, gates). ``out`` may be a
-    view of some columns of a wider float32 matrix."""
+    view of some columns of a wider float32 matrix. ``bias`` (any float type) is added in 32-bit, by a kernel of its own."""
+    if bias is not None:
+        y = linear_f32(rt, x, weight)
+        ops.add(y, None, y, bias=bias.float())
+        if out is None:
+            return y
+        out.copy_(y)
+        return out
     n, m = x.shape[0], weight.shape[0]
     if out is None:
         out = torch.empty(n, m, device=rt.device, dtype=torch.float32)

@@ -23,7 +23,7 @@ from .spec import ModelSpec, WeightSpec
 # importing the modules registers the built-in parts
 from . import (  # noqa: F401,E402
     attention, block, embedding, experts, feed_forward, gated_unit, head, latent_attention, norm, parallel, position, recurrent,
-    scored_attention, selective_scan, token_shift,
+    scored_attention, selective_scan, state_space, token_shift,
 )
 
 
@@ -103,6 +103,8 @@ class Model:
         self.head.tie(self.embedding.table())
         for part in self._all_parts():
             part.finalize()
+        for layer in self.layers:
+            layer.block.bind_parts(layer.parts)
         self.weights_version += 1
 
     # ------------------------------------------------------------------ cache needs

@@ -102,6 +102,48 @@ class RMSNorm(Norm):
         return out
 
 
+@register_part("norm", "tanh_norm")
+class TanhNorm(Norm):
+    """A tanh in place of a norm, on a 32-bit residual stream: ``tanh(alpha x) * w + b`` with one number ``alpha`` and two
+    vectors (tensors ``<weight_name>``, ``<weight_name>.alpha``, ``<weight_name>.b``). It has no statistics, so it is
+    element by element and may be made by whichever kernel writes the stream (``tanh_params``, ``ops.tanh_norm_stream``)."""
+
+    def __init__(self, runtime: Runtime, *, width: int, weight_name: str = "weight") -> None:
+        super().__init__(runtime)
+        self.width, self.weight_name = width, weight_name
+        self.alpha = 0.0
+        self.weight: torch.Tensor | None = None
+        self.offset: torch.Tensor | None = None
+
+    def graph_capturable(self, page_size: int) -> bool:
+        return True  # kernels on device arrays only
+
+    def weight_specs(self) -> dict[str, WeightSpec]:
+        n = self.weight_name
+        return {n: WeightSpec((self.width,), role="float32", init="norm"), n + ".b": WeightSpec((self.width,), role="float32", init="zeros"),
+                n + ".alpha": WeightSpec((), role="float32", init="ones")}
+
+    def load_weights(self, tensors: Mapping[str, torch.Tensor]) -> None:
+        n = self.weight_name
+        self.weight, self.offset = tensors[n].contiguous(), tensors[n + ".b"].contiguous()
+        self.alpha = float(tensors[n + ".alpha"])
+
+    def tanh_params(self) -> tuple[float, torch.Tensor, torch.Tensor]:
+        """``alpha``, weight and offset, for a kernel that writes the stream and applies this to it."""
+        return self.alpha, self.weight, self.offset
+
+    def stream_key(self) -> tuple:
+        """What identifies this norm where rows that it has normalised are handed on."""
+        return ("tanh", self.weight.data_ptr(), self.alpha)
+
+    def forward(self, x: torch.Tensor, delta: Optional[torch.Tensor] = None) -> torch.Tensor:
+        if x.dtype != torch.float32:
+            raise RuntimeError("tanh_norm reads a float32 residual stream")
+        out = self.rt.empty(*x.shape)
+        ops.tanh_norm_stream(x, a=delta, norm=self.tanh_params(), out=out)
+        return out
+
+
 @register_part("norm", "group_rms_norm")
 class GroupRMSNorm(Norm):
     """RMS norm in groups, on a 32-bit residual stream: a row is split into ``groups`` equal

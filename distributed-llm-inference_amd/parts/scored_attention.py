@@ -2,7 +2,7 @@
 queries and keys or a rotary position encoding, a per-head logarithmic distance penalty, a chunked
 mask, a window that keeps the first positions, a softmax with a sink (of score 0 or of a learnt score per head),
 a temperature on the queries that grows with the position, value mixing across layers, a sigmoid output gate,
-biases on the projections, several score maps a head over the same values whose results are subtracted
+biases on the projections, norms over the whole query and key projections, several score maps a head over the same values whose results are subtracted
 (differential attention), values that are the keys, and keys and values read from another layer's cache. Each
 is a parameter, so another design may take any subset.
 
@@ -35,6 +35,10 @@ projections and reads the cache of the schedule entry it is given (keys as that 
 ``head_sink``: a learnt number ``sink`` per head instead of the 1 above, ``exp(sink_h)``. ``keys_as_values``: there is no value
 projection; the values are the keys as cached, and the pages hold keys alone. ``query_temperature = (coef, every)``: q is
 multiplied by ``1 + coef ln(floor((p + 1) / every) + 1)`` at position ``p``, before it is rounded.
+
+``qk_row_norm``: q, over all its heads at once, is divided by its root mean square and multiplied by the weight ``q.norm``, k
+alike by ``k.norm``, after the biases and before the rotation. ``out_bias``: the output product has a bias; with
+``defer_output_bias`` it is left to the block (``output_bias``).
 
 Scores, weights, norms and the mixing are 32-bit; keys and values are cached in the runtime's type.
 """
@@ -112,7 +116,8 @@ class ScoredAttention(Mixer):
                  value_mix_key: str = "first_values", names: Optional[Mapping[str, str]] = None,
                  position: Optional[PartSpec] = None, bias: bool = False, keep_first: int = 0, maps: int = 1,
                  diff: float = 0.0, head_gate: bool = False, own_kv: bool = True, cache_window: Optional[int] = None,
-                 keys_as_values: bool = False, head_sink: bool = False, query_temperature: Optional[tuple] = None) -> None:
+                 keys_as_values: bool = False, head_sink: bool = False, query_temperature: Optional[tuple] = None,
+                 qk_row_norm: bool = False, out_bias: bool = False, defer_output_bias: bool = False) -> None:
         """``cache_window``: how many of the latest keys the pages must keep where that is not this layer's own
         window (0: all): other layers that read this layer's cache may look further back than it does."""
         super().__init__(runtime)
@@ -127,6 +132,13 @@ class ScoredAttention(Mixer):
             raise ValueError("scored_attention: the gate per head belongs to the kernel that combines two maps")
         if (bias or not own_kv) and qk_unit:
             raise ValueError("scored_attention: biases and borrowed keys go with rotary or plain keys")
+        if qk_row_norm and (qk_unit or maps == 2 or not own_kv):
+            raise ValueError("scored_attention: norms over the whole projections go with one map of own rotary or plain keys")
+        if defer_output_bias and not out_bias:
+            raise ValueError("scored_attention: there is no output bias to leave to the block")
+        self.qk_row_norm, self.out_bias, self.defer_output_bias = bool(qk_row_norm), bool(out_bias), bool(defer_output_bias)
+        self.row_norm: Optional[tuple] = None
+        self.b_o: Optional[torch.Tensor] = None
         if keep_first < 0 or (keep_first and not window):
             raise ValueError("scored_attention: kept first positions belong to a window")
         self.bias, self.keep_first, self.maps, self.diff = bool(bias), int(keep_first), int(maps), float(diff)
@@ -164,6 +176,7 @@ class ScoredAttention(Mixer):
         if not self.qk_unit and value_mix != "none":
             raise ValueError("scored_attention: value mixing belongs to the kernel that makes unit keys")
         self.names = {"q": "q", "k": "k", "v": "v", "g": "g", "o": "o", "mix": "vmix", "r1": "r1", "r2": "r2", "sink": "sink",
+                      "q_norm": "q.norm", "k_norm": "k.norm",
                       "lq1": "lq1", "lk1": "lk1", "lq2": "lq2", "lk2": "lk2", **dict(names or {})}
         self.w_in = self.w_o = self.mix = self.r1 = self.r2 = self.sinks = None
 
@@ -194,6 +207,11 @@ class ScoredAttention(Mixer):
         if self.bias:
             specs.update({n[s] + ".b": WeightSpec((size,), role="float32", init="zeros")
                           for s, size in (("q", self._q), ("k", self._k), ("v", self._v)) if size})
+        if self.qk_row_norm:
+            specs.update({n[s]: WeightSpec((size,), role="float32", init="norm")
+                          for s, size in (("q_norm", self._q), ("k_norm", self._k)) if size})
+        if self.out_bias:
+            specs[n["o"] + ".b"] = WeightSpec((h,), role="float32", init="zeros")
         if self.output_gate:
             specs[n["g"]] = WeightSpec((self._o, h))
         if self.head_gate:
@@ -229,6 +247,12 @@ class ScoredAttention(Mixer):
             lq1, lk1, lq2, lk2 = (tensors[n[s]].float() for s in ("lq1", "lk1", "lq2", "lk2"))
             self.lam = float(torch.exp((lq1 * lk1).sum()) - torch.exp((lq2 * lk2).sum())) + self.diff
         self.w_o = tensors[n["o"]]
+        if self.qk_row_norm:
+            self.row_norm = (tensors[n["q_norm"]].contiguous(), tensors[n["k_norm"]].contiguous(), self.norm_eps)
+        if self.out_bias:
+            self.b_o = tensors[n["o"] + ".b"].contiguous()
+            if self.defer_output_bias:
+                self.output_bias, self.b_o = self.b_o, None
         if self.head_sink:
             self.sinks = tensors[n["sink"]].contiguous()
         if self.distance_penalty:
@@ -295,7 +319,7 @@ class ScoredAttention(Mixer):
                              0 if table is None else table.dim, table is not None and table.pairing == "interleaved",
                              q, grp.slots if self.own_kv else None, cache.k_pages if self.own_kv else None,
                              cache.v_pages if self.own_kv else None, self.num_heads * self.maps, bias=self.b_in,
-                             query_temperature=self.query_temperature)
+                             query_temperature=self.query_temperature, row_norm=self.row_norm)
         g0 = self._q + self._k + self._v
         if self.maps == 2:
             # each map is a head of its own to the attention kernels; their results stay 32-bit until they are combined
@@ -306,10 +330,10 @@ class ScoredAttention(Mixer):
             out = self.rt.empty(n, self._o)
             ops.diff_head_norm(both, self.lam, 1.0 - self.diff, self.norm_eps,
                                proj[:, g0:g0 + self.num_heads] if self.head_gate else None, out, self.num_heads, self.value_dim)
-            return linear_f32(self.rt, out, self.w_o)
+            return linear_f32(self.rt, out, self.w_o, bias=self.b_o)
         out = self.rt.empty(n, self._o)
         gate = proj[:, g0:g0 + self._o] if self.output_gate else None
         paged_scored_attention(self.rt, ctx, cache, q, out, self.num_heads, self.head_dim, self.value_dim, self.scale,
                                gate=gate, window=self.window, chunk=self.chunk, sink=self.sink, r1=self.r1, r2=self.r2,
                                keep_first=self.keep_first, sinks=self.sinks)
-        return linear_f32(self.rt, out, self.w_o)
+        return linear_f32(self.rt, out, self.w_o, bias=self.b_o)
