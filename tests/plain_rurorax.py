@@ -171,8 +171,19 @@ def expert(h: torch.Tensor, gate: torch.Tensor, up: torch.Tensor, down: torch.Te
     return (silu(h @ gate.t()) * (h @ up.t())) @ down.t()
 
 
-def experts(h: torch.Tensor, p: Mapping[str, torch.Tensor], f: Mapping[str, Any]) -> torch.Tensor:
-    ids, s = choose(h @ p["router"].t(), f["router"]["top"])
+def call_margins(z: torch.Tensor, top: int) -> torch.Tensor:
+    """How far each row's last chosen logit lies above the first that is not chosen (all chosen: infinity)."""
+    if top >= z.shape[1]:
+        return torch.full((z.shape[0],), math.inf, dtype=F)
+    best = torch.sort(z, dim=1, descending=True).values
+    return best[:, top - 1] - best[:, top]
+
+
+def experts(h: torch.Tensor, p: Mapping[str, torch.Tensor], f: Mapping[str, Any], margins: Optional[list] = None) -> torch.Tensor:
+    z = h @ p["router"].t()
+    if margins is not None:
+        margins.append(call_margins(z, f["router"]["top"]))
+    ids, s = choose(z, f["router"]["top"])
     out = torch.zeros_like(h)
     for t in range(h.shape[0]):
         for e, w in zip(ids[t].tolist(), s[t]):
@@ -198,7 +209,7 @@ class PlainRurorax:
     def norm(self, name: str, x: torch.Tensor) -> torch.Tensor:
         return tanh_norm(x, self.t[name + ".alpha"], self.t[name], self.t[name + ".b"])
 
-    def layer(self, i: int, x: torch.Tensor, first: int, states: list) -> torch.Tensor:
+    def layer(self, i: int, x: torch.Tensor, first: int, states: list, margins: Optional[list] = None) -> torch.Tensor:
         entry, p = self.cfg["layers"][i], f"l{i}."
         h, mix = self.norm(p + "norm1", x), sub_tensors(self.t, p + "mix.")
         if entry["type"] == "mamba2":
@@ -211,16 +222,18 @@ class PlainRurorax:
         f = entry.get("mlp")
         if f is not None:
             own = sub_tensors(self.t, p + "mlp.")
-            out = out + self.t[p + "ls2"] * (dense(h, own) if f["kind"] == "dense" else experts(h, own, f))
+            out = out + self.t[p + "ls2"] * (dense(h, own) if f["kind"] == "dense" else experts(h, own, f, margins))
         return out
 
-    def forward(self, tokens, states: Optional[list] = None, start: int = 0, layers_out: Optional[list] = None) -> torch.Tensor:
+    def forward(self, tokens, states: Optional[list] = None, start: int = 0, layers_out: Optional[list] = None,
+                margins: Optional[list] = None) -> torch.Tensor:
         """Logits ``[tokens, vocab]`` of ``tokens`` at positions ``start, start+1, ...``; ``states`` (from
-        :meth:`new_state`) carries the sequence from call to call."""
+        :meth:`new_state`) carries the sequence from call to call. ``margins`` receives, per mixture of
+        experts, how close each token's choice was."""
         states = self.new_state() if states is None else states
         x = self.t["embed"][torch.as_tensor(tokens, dtype=torch.long)]
         for i in range(len(self.cfg["layers"])):
-            x = self.layer(i, x, start, states)
+            x = self.layer(i, x, start, states, margins)
             if layers_out is not None:
                 layers_out.append(x.clone())
         logits = self.norm("final.norm", x) @ self.t["embed"].t()
