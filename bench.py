@@ -338,13 +338,27 @@ def pibuvik_shape(width, heads, kv_heads, ff, layers, vocab, chunk):
             "residual_mult": 0.4, "logit_scale": 0.8, "layers": out}
 
 
+def rurorax_shape(width, heads, kv_heads, ff, layers, vocab, chunk):
+    """A Rurorax of sizes that resemble a real model's layers, state-space and attention layers in turn: the recurrence with
+    twice the width in heads of 64 with 128 states, as many groups as the attention has kv heads and four taps; the
+    attention with heads of 64 in chunks, half of each head rotated; the feed-forward in turn dense (the Llama layer's) and
+    a mixture of 32 experts of an eighth of its size, four of them chosen."""
+    mixers = {"mamba2": {"heads": 2 * width // 64, "vdim": 64, "state": 128, "groups": kv_heads, "norm_groups": kv_heads, "conv": 4},
+              "attention": {"heads": heads, "kv_heads": kv_heads, "dim": 64, "vdim": 64, "scale": 0.125, "mask": {"size": chunk},
+                            "rot": {"dims": 32, "base": 1e6, "scaling": {"factor": 2.0}}}}
+    mlps = [{"kind": "dense", "ff": ff}, {"kind": "moe", "expert": {"ff": ff // 8}, "router": {"experts": 32, "top": 4}}]
+    order = [("mamba2", 0), ("attention", 1), ("mamba2", 1), ("attention", 0)]
+    return {"architecture": "Rurorax", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "logit_softcap": 30.0,
+            "layers": [{"type": order[i % 4][0], "mixer": mixers[order[i % 4][0]], "mlp": mlps[order[i % 4][1]]} for i in range(layers)]}
+
+
 DESIGN_SIZES = {  # width, heads (of 64), kv heads, feed-forward, layers, vocabulary, attention chunk
     "1024": (1024, 16, 4, 4096, 8, 32000, 1024),
     "2048": (2048, 32, 8, 8192, 8, 32000, 2048),
 }
 
 
-BESIDE = {"miberax": "makodra and ", "zarinex": "miberax and ", "betepel": "miberax and ", "pibuvik": "zarinex and "}
+BESIDE = {"miberax": "makodra and ", "zarinex": "miberax and ", "betepel": "miberax and ", "pibuvik": "zarinex and ", "rurorax": "betepel and "}
 
 
 def design_compare(args):
@@ -358,8 +372,10 @@ def design_compare(args):
     for name in args.design_sizes.split(","):
         width, heads, kv_heads, ff, layers, vocab, chunk = DESIGN_SIZES[name]
         shapes = {
+            **({"rurorax": rurorax_shape(width, heads, kv_heads, ff, layers, vocab, chunk)} if args.design == "rurorax" else {}),
             **({"pibuvik": pibuvik_shape(width, heads, kv_heads, ff, layers, vocab, chunk)} if args.design == "pibuvik" else {}),
-            **({"betepel": betepel_shape(width, heads, kv_heads, ff, layers, vocab, chunk)} if args.design == "betepel" else {}),
+            **({"betepel": betepel_shape(width, heads, kv_heads, ff, layers, vocab, chunk)}
+               if args.design in ("betepel", "rurorax") else {}),
             **({"zarinex": zarinex_shape(width, heads, kv_heads, ff, layers, vocab, chunk)}
                if args.design in ("zarinex", "pibuvik") else {}),
             **({"miberax": miberax_shape(width, heads, kv_heads, ff, layers, vocab, chunk)}
@@ -480,13 +496,13 @@ def main() -> int:
                     help="prompt length of --only-prefill (the line of the default run always has 2,048)")
     ap.add_argument("--portion", type=int, default=None,
                     help="with --only-prefill: the prompt runs in steps of at most this many tokens")
-    ap.add_argument("--design", default=None, choices=["makodra", "miberax", "zarinex", "betepel", "pibuvik"],
+    ap.add_argument("--design", default=None, choices=["makodra", "miberax", "zarinex", "betepel", "pibuvik", "rurorax"],
                     help="instead of the default run: prefill (2,048 and 8,192 tokens) and decode (batch 1, 8, 64 at "
                          "--context) of this design beside the Llama decoder at equal sizes, random weights")
     ap.add_argument("--design-sizes", default="1024,2048", help="widths of --design, of " + ", ".join(DESIGN_SIZES))
     ap.add_argument("--design-phases", default="prefill2048,prefill8192,decode_b1,decode_b8,decode_b64",
                     help="with --design: which of these measurements to make")
-    ap.add_argument("--design-only", default=None, choices=["makodra", "miberax", "zarinex", "betepel", "pibuvik", "llama"],
+    ap.add_argument("--design-only", default=None, choices=["makodra", "miberax", "zarinex", "betepel", "pibuvik", "rurorax", "llama"],
                     help="with --design: measure this one of the pair alone (for profiling)")
     args = ap.parse_args()
     if args.gpus != 1:

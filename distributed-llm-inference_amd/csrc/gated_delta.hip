@@ -155,7 +155,7 @@ __global__ void causal_conv_kernel(const float* __restrict__ x, int64_t stride, 
     acc = fmaf(conv_w[(int64_t)c * taps + (taps - 1 - j)], in, acc);
   }
   if (act == 1) acc = acc / (1.f + expf(-acc));
-  out[(int64_t)row * out_stride + c] = acc;
+  if (out != nullptr) out[(int64_t)row * out_stride + c] = acc;
   if (rounded != nullptr) rounded[(int64_t)row * rounded_stride + c] = from_f32<T>(acc);
 }
 
@@ -180,7 +180,7 @@ __global__ void causal_conv_single_kernel(const float* __restrict__ x, int64_t s
   for (int i = 0; i + 1 < taps - 1; ++i) kept[(int64_t)i * channels] = old[i + 1];
   if (taps > 1) kept[(int64_t)(taps - 2) * channels] = now;
   if (act == 1) acc = acc / (1.f + expf(-acc));
-  out[(int64_t)row * out_stride + c] = acc;
+  if (out != nullptr) out[(int64_t)row * out_stride + c] = acc;
   if (rounded != nullptr) rounded[(int64_t)row * rounded_stride + c] = from_f32<T>(acc);
 }
 
@@ -240,7 +240,7 @@ __global__ __launch_bounds__(256) void causal_conv_run_kernel(const float* __res
     if (row >= rows) break;
     float v = y[r];
     if (act == 1) v = v / (1.f + expf(-v));
-    out[(int64_t)row * out_stride + c] = v;
+    if (out != nullptr) out[(int64_t)row * out_stride + c] = v;
     if (rounded != nullptr) rounded[(int64_t)row * rounded_stride + c] = from_f32<T>(v);
   }
 }
@@ -421,13 +421,14 @@ int dli_conv_prepare(const float* proj, int64_t stride, int b_off, int a_off, co
   return dli_launch_status();
 }
 
-// act: 0 none, 1 silu. rounded (may be nullptr): the result once more, bf16 if rounded_is_bf16 else float.
+// act: 0 none, 1 silu. rounded (may be nullptr): the result once more, bf16 if rounded_is_bf16 else float; out may be nullptr
+// where it is not.
 int dli_causal_conv(const float* x, int64_t stride, const float* conv_w, const float* bias, const float* in_bias, float* state,
                     int64_t state_stride, int64_t kept_offset, const int* q_start, const int* positions,
                     const int* state_slots, float* out, int64_t out_stride, void* rounded, int64_t rounded_stride,
                     int rounded_is_bf16, int entries, int rows, int channels, int taps, int act, hipStream_t stream) {
   if (rows <= 0 || entries <= 0) return DLI_OK;
-  if (channels <= 0 || taps < 1 || taps > GD_MAX_TAPS || stride < channels || out_stride < channels ||
+  if (channels <= 0 || taps < 1 || taps > GD_MAX_TAPS || stride < channels || (out != nullptr ? out_stride < channels : rounded == nullptr) ||
       (rounded != nullptr && rounded_stride < channels) || act < 0 || act > 1 ||
       state_stride < kept_offset + (int64_t)(taps - 1) * channels)
     return DLI_ERR_ARGUMENT;

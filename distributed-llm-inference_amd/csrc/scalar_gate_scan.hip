@@ -36,9 +36,9 @@
 #include "common.h"
 
 struct SgArgs {
-  const float* q; int64_t q_stride;      // [rows][>= heads * D], already at the first column
-  const float* k; int64_t k_stride;
-  const float* v; int64_t v_stride;      // [rows][>= heads * V]
+  const void* q; int64_t q_stride;       // [rows][>= heads * D], already at the first column; float, or bfloat16 where the
+  const void* k; int64_t k_stride;       // kernel is built for it
+  const void* v; int64_t v_stride;       // [rows][>= heads * V]
   const float* keep; const float* write; int64_t gate_stride;   // [rows][heads]; keep == nullptr: decay[head] and 1
   const float* decay;                    // [heads]
   const float* floor;                    // [rows][heads] exp(-m_t): with it the last column is n, and den is written
@@ -75,7 +75,7 @@ __device__ __forceinline__ float sg_act(float x, int silu) { return silu ? x / (
 // factors per token, and with them the column of n and the denominators; SILU:
 // q, k and v pass through silu on their way into LDS. No load hangs on a condition (what is not wanted is read
 // from a clamped place and dropped), so that a batch's loads stay in flight while the chain of the one before runs.
-template <int NK, int TB, int MODE, bool SILU>
+template <int NK, int TB, int MODE, bool SILU, typename T>
 __global__ __launch_bounds__(64) void scalar_gate_scan_kernel(SgArgs p) {
   constexpr bool GATED = MODE == SG_EXP;
   constexpr int D = NK * 16, COLS = 4, PER = (TB * D + 63) / 64;
@@ -106,13 +106,13 @@ __global__ __launch_bounds__(64) void scalar_gate_scan_kernel(SgArgs p) {
     for (int m = 0; m < PER; ++m) {
       const int e = min(lane + 64 * m, TB * D - 1), t = e / D, c = e - t * D;
       const int64_t row = row0 + min(t0 + t, n_rows - 1);
-      pk[m] = p.k[row * p.k_stride + qk_col + c];
-      pq[m] = p.q[row * p.q_stride + qk_col + c];
+      pk[m] = to_f32(((const T*)p.k)[row * p.k_stride + qk_col + c]);
+      pq[m] = to_f32(((const T*)p.q)[row * p.q_stride + qk_col + c]);
     }
     {
       const int64_t row = row0 + min(t0 + min(lane / COLS, TB - 1), n_rows - 1);
       const int c = (int)blockIdx.z * COLS + lane % COLS;
-      pv = p.v[row * p.v_stride + v_col + min(c, V - 1)];
+      pv = to_f32(((const T*)p.v)[row * p.v_stride + v_col + min(c, V - 1)]);
     }
     if (GATED) {
       const int64_t row = row0 + min(t0 + min(lane, TB - 1), n_rows - 1);
@@ -176,6 +176,7 @@ __global__ __launch_bounds__(64) void scalar_gate_scan_kernel(SgArgs p) {
 }
 
 // Any D and V: a thread a column, the column's state in the request's slot.
+template <typename T>
 __global__ void scalar_gate_any_kernel(SgArgs p, int D) {
   extern __shared__ float sh[];
   float *sk = sh, *sq = sh + D;
@@ -193,8 +194,8 @@ __global__ void scalar_gate_any_kernel(SgArgs p, int D) {
     const int64_t row = row0 + t;
     __syncthreads();
     for (int i = threadIdx.x; i < D; i += blockDim.x) {
-      sk[i] = sg_act(p.k[row * p.k_stride + qk_col + i], p.silu);
-      sq[i] = sg_act(p.q[row * p.q_stride + qk_col + i], p.silu) * p.q_scale;
+      sk[i] = sg_act(to_f32(((const T*)p.k)[row * p.k_stride + qk_col + i]), p.silu);
+      sq[i] = sg_act(to_f32(((const T*)p.q)[row * p.q_stride + qk_col + i]), p.silu) * p.q_scale;
     }
     __syncthreads();
     if (!live) continue;
@@ -208,7 +209,7 @@ __global__ void scalar_gate_any_kernel(SgArgs p, int D) {
     } else {
       a = p.decay[head];
     }
-    const float v = is_n ? 1.f : sg_act(p.v[row * p.v_stride + v_col + c], p.silu), bv = b * v;
+    const float v = is_n ? 1.f : sg_act(to_f32(((const T*)p.v)[row * p.v_stride + v_col + c]), p.silu), bv = b * v;
     float o = 0.f;
     for (int i = 0; i < D; ++i) {
       const float s = fmaf(a, st[i], bv * sk[i]);
@@ -273,14 +274,14 @@ __global__ __launch_bounds__(256) void scalar_gate_chunk_kernel(SgArgs p, const 
     for (int m = 0; m < QK_PER; ++m) {
       const int idx = tid + 256 * m, t = idx / D, d = idx - t * D;
       const int64_t row = row0 + min(t0 + t, n_rows - 1);
-      rk[m] = p.k[row * p.k_stride + qk_col + d];
-      rq[m] = p.q[row * p.q_stride + qk_col + d];
+      rk[m] = ((const float*)p.k)[row * p.k_stride + qk_col + d];
+      rq[m] = ((const float*)p.q)[row * p.q_stride + qk_col + d];
     }
 #pragma unroll
     for (int m = 0; m < V_PER; ++m) {
       const int idx = tid + 256 * m, t = idx / VS, j = idx - t * VS;
       const int64_t row = row0 + min(t0 + t, n_rows - 1);
-      rv[m] = p.v[row * p.v_stride + v_col + min(v0 + j, V - 1)];
+      rv[m] = ((const float*)p.v)[row * p.v_stride + v_col + min(v0 + j, V - 1)];
     }
     if (GATED) {
       const int64_t at = (int64_t)(row0 + min(t0 + lane, n_rows - 1)) * p.gate_stride + head;
@@ -511,16 +512,17 @@ int dli_exp_gates(const float* pre, int64_t stride, int i_off, int f_off, const 
 
 // keep, write: [rows][heads] or both nullptr (then decay [heads] and a write factor of one); floor and den
 // [rows][heads] come together, and with them the state has a column more a head. step [rows][heads] instead: factors from
-// softplus(step + step_bias) and -exp(step_rate), the result plus skip (may be nullptr) times v.
-int dli_scalar_gate_scan(const float* q, int64_t q_stride, const float* k, int64_t k_stride, const float* v, int64_t v_stride,
+// softplus(step + step_bias) and -exp(step_rate), the result plus skip (may be nullptr) times v; q, k and v may then be
+// bfloat16 (is_bf16).
+int dli_scalar_gate_scan(const void* q, int64_t q_stride, const void* k, int64_t k_stride, const void* v, int64_t v_stride,
                          const float* keep, const float* write, const float* log_keep, int64_t gate_stride, const float* decay,
                          const float* floor, float* den, float* state, int64_t state_stride, const int* q_start, const int* positions,
                          const int* state_slots, float* o, int64_t o_stride, int entries, int rows, int heads, int dim,
                          int vdim, float q_scale, int silu, int chunked, int qk_heads, const float* step, int64_t step_stride,
-                         const float* step_bias, const float* step_rate, const float* skip, hipStream_t stream) {
+                         const float* step_bias, const float* step_rate, const float* skip, int is_bf16, hipStream_t stream) {
   if (rows <= 0 || entries <= 0) return DLI_OK;
   if (qk_heads <= 0 || heads % qk_heads || (step != nullptr && (step_stride < heads || step_bias == nullptr || step_rate == nullptr ||
-      keep != nullptr || silu)) || (skip != nullptr && step == nullptr))
+      keep != nullptr || silu)) || (is_bf16 && step == nullptr) || (skip != nullptr && step == nullptr))
     return DLI_ERR_ARGUMENT;
   const int vx = vdim + (floor != nullptr ? 1 : 0);
   if (rows < entries || heads <= 0 || heads > 65535 || dim <= 0 || dim > 4096 || vdim <= 0 ||
@@ -540,7 +542,7 @@ int dli_scalar_gate_scan(const float* q, int64_t q_stride, const float* k, int64
   if (grid.z > 65535) return DLI_ERR_ARGUMENT;
   const bool gated = keep != nullptr;
   if (gated && floor == nullptr) return DLI_ERR_ARGUMENT;   // (gates without a normaliser: no model asks for them yet)
-  if (!single && !silu && dim % 16 == 0 && dim <= 64 && (!gated || log_keep != nullptr) && chunked) {
+  if (!is_bf16 && !single && !silu && dim % 16 == 0 && dim <= 64 && (!gated || log_keep != nullptr) && chunked) {
     // a step with portions: chunks of 64 tokens on the matrix cores
     const dim3 cgrid(entries, heads, (vdim + 15) / 16);
     if (cgrid.z > 65535) return DLI_ERR_ARGUMENT;
@@ -556,10 +558,11 @@ int dli_scalar_gate_scan(const float* q, int64_t q_stride, const float* k, int64
   }
 #define SG_LAUNCH(NK, TBV)                                                                                  \
   {                                                                                                         \
-    if (gated) scalar_gate_scan_kernel<NK, TBV, SG_EXP, false><<<grid, 64, 0, stream>>>(p);                \
-    else if (step != nullptr) scalar_gate_scan_kernel<NK, TBV, SG_STEP, false><<<grid, 64, 0, stream>>>(p); \
-    else if (silu) scalar_gate_scan_kernel<NK, TBV, SG_DECAY, true><<<grid, 64, 0, stream>>>(p);           \
-    else scalar_gate_scan_kernel<NK, TBV, SG_DECAY, false><<<grid, 64, 0, stream>>>(p);                    \
+    if (gated) scalar_gate_scan_kernel<NK, TBV, SG_EXP, false, float><<<grid, 64, 0, stream>>>(p);         \
+    else if (is_bf16) scalar_gate_scan_kernel<NK, TBV, SG_STEP, false, bf16_t><<<grid, 64, 0, stream>>>(p); \
+    else if (step != nullptr) scalar_gate_scan_kernel<NK, TBV, SG_STEP, false, float><<<grid, 64, 0, stream>>>(p); \
+    else if (silu) scalar_gate_scan_kernel<NK, TBV, SG_DECAY, true, float><<<grid, 64, 0, stream>>>(p);    \
+    else scalar_gate_scan_kernel<NK, TBV, SG_DECAY, false, float><<<grid, 64, 0, stream>>>(p);             \
   }
 #define SG_CASE(NK, TBM)                                                                     \
   case NK * 16:                                                                              \
@@ -570,8 +573,9 @@ int dli_scalar_gate_scan(const float* q, int64_t q_stride, const float* k, int64
     SG_CASE(12, 4) SG_CASE(16, 4)
     default: {
       const int threads = vx >= 256 ? 256 : (vx + 63) / 64 * 64;
-      scalar_gate_any_kernel<<<dim3(entries, heads, (vx + threads - 1) / threads), threads, 2 * dim * sizeof(float), stream>>>(
-          p, dim);
+      const dim3 any(entries, heads, (vx + threads - 1) / threads);
+      if (is_bf16) scalar_gate_any_kernel<bf16_t><<<any, threads, 2 * dim * sizeof(float), stream>>>(p, dim);
+      else scalar_gate_any_kernel<float><<<any, threads, 2 * dim * sizeof(float), stream>>>(p, dim);
     }
   }
 #undef SG_CASE

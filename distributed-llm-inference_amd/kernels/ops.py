@@ -167,7 +167,12 @@ _SIGNATURES = {
                       _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_ptr],
     "dli_scalar_gate_scan": [_c_ptr, _c_i64, _c_ptr, _c_i64, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr,
                              _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_int,
-                             _c_int, _c_float, _c_int, _c_int, _c_int, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr],
+                             _c_int, _c_float, _c_int, _c_int, _c_int, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr],
+    "dli_state_space_tile_rows": [],
+    "dli_state_space_tiles_supports": [_c_int, _c_int],
+    "dli_state_space_tiles": [_c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr,
+                              _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_int,
+                              _c_int, _c_ptr],
     "dli_group_norm": [_c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_int, _c_ptr],
     "dli_branch_norm_mean": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_int, _c_int, _c_float, _c_ptr],
     "dli_head_norm_gate": [_c_ptr, _c_i64, _c_ptr, _c_i64, _c_ptr, _c_float, _c_ptr, _c_i64, _c_int, _c_int, _c_int, _c_int,
@@ -2196,15 +2201,15 @@ def _state_rows(state: torch.Tensor, floats: int) -> None:
 
 
 def causal_conv(x: torch.Tensor, conv_w: torch.Tensor, bias: Optional[torch.Tensor], state: torch.Tensor, kept_offset: int,
-                q_start: torch.Tensor, positions: torch.Tensor, state_slots: torch.Tensor, out: torch.Tensor,
-                rounded: Optional[torch.Tensor] = None, act: str = "silu",
+                q_start: torch.Tensor, positions: torch.Tensor, state_slots: torch.Tensor,
+                out: Optional[torch.Tensor], rounded: Optional[torch.Tensor] = None, act: str = "silu",
                 in_bias: Optional[torch.Tensor] = None) -> None:
     """A short causal convolution over time per channel: ``out[t, c] = act(bias[c] + sum_j conv_w[c, taps-1-j] x[t-j, c])``
     with zeros before position 0. ``x`` float32 ``[n, >= channels]`` (rows contiguous; the channels from
     column 0), ``conv_w`` float32 ``[channels, taps]`` (the last column is the current token's). The inputs
     before an entry's first row come from ``state[slot, kept_offset:]`` (``[taps-1, channels]``, the newest
     last), which then receives the entry's last ``taps - 1`` inputs. ``out`` float32 ``[n, channels]``;
-    ``rounded``: the result once more (float32 or bfloat16), for the product that reads it next.
+    ``rounded``: the result once more (float32 or bfloat16), for the product that reads it next (``out`` may then be ``None``).
     ``act``: ``"silu"`` or ``"none"``. ``in_bias`` (float32 ``[channels]``): added to every input that exists (the kept inputs
     carry it, the zeros before position 0 do not)."""
     _f32_rows(x, "x")
@@ -2219,8 +2224,10 @@ def causal_conv(x: torch.Tensor, conv_w: torch.Tensor, bias: Optional[torch.Tens
     if in_bias is not None:
         _dense(in_bias, "in_bias", torch.float32, 1)
         _require(in_bias.shape[0] == channels, "in_bias must hold a value per channel")
-    _f32_rows(out, "out")
-    _require(out.shape == (n, channels), "out must be [n, channels]")
+    _require(out is not None or rounded is not None, "a result is wanted")
+    if out is not None:
+        _f32_rows(out, "out")
+        _require(out.shape == (n, channels), "out must be [n, channels]")
     r_stride, r_bf16 = 0, 0
     if rounded is not None:
         _rows(rounded, "rounded", rounded.dtype)
@@ -2231,7 +2238,7 @@ def causal_conv(x: torch.Tensor, conv_w: torch.Tensor, bias: Optional[torch.Tens
     entries = _step_arrays(q_start, positions, state_slots, n)
     _check(library().dli_causal_conv(
         _ptr(x), x.stride(0), _ptr(conv_w), _ptr(bias), _ptr(in_bias), _ptr(state), state.stride(0), int(kept_offset), _ptr(q_start),
-        _ptr(positions), _ptr(state_slots), _ptr(out), out.stride(0), _ptr(rounded), r_stride, r_bf16, entries, n,
+        _ptr(positions), _ptr(state_slots), _ptr(out), 0 if out is None else out.stride(0), _ptr(rounded), r_stride, r_bf16, entries, n,
         channels, taps, int(act == "silu"), _stream()), "causal_conv")
 
 
@@ -2439,11 +2446,14 @@ def scalar_gate_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: t
 
     ``qk_heads``: q and k hold that many heads, each shared by ``heads / qk_heads`` neighbours. ``step`` (float32 ``[n, heads]``,
     columns of a wider matrix will do) instead of factors: ``b = softplus(step + step_bias)``, ``a = exp(-exp(step_rate) b)``
-    (float32 ``[heads]`` each), and ``o`` gets ``skip * v`` on top (float32 ``[heads]``; ``None``: nothing)."""
+    (float32 ``[heads]`` each), and ``o`` gets ``skip * v`` on top (float32 ``[heads]``; ``None``: nothing); ``q``, ``k`` and ``v``
+    may then be bfloat16."""
+    is_bf16 = q.dtype == torch.bfloat16
+    _require(not is_bf16 or step is not None, "q, k and v are float32 but under a step size")
     qk_heads = heads if qk_heads is None else int(qk_heads)
     _require(qk_heads > 0 and heads % qk_heads == 0, "the heads do not group onto qk_heads")
     for name, t, width in (("q", q, qk_heads * dim), ("k", k, qk_heads * dim), ("v", v, heads * vdim), ("o", o, heads * vdim)):
-        _f32_rows(t, name)
+        _rows(t, name, torch.float32 if name == "o" else q.dtype)
         _require(t.shape[1] == width, f"{name} must hold {width} columns")
     n = q.shape[0]
     _require(k.shape[0] == n and v.shape[0] == n and o.shape[0] == n, "q, k, v and o differ in rows")
@@ -2472,8 +2482,58 @@ def scalar_gate_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: t
         _ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(v), v.stride(0), _ptr(keep), _ptr(write), _ptr(log_keep), heads,
         _ptr(decay), _ptr(floor), _ptr(den), _ptr(state), state.stride(0), _ptr(q_start), _ptr(positions), _ptr(state_slots),
         _ptr(o), o.stride(0), entries, n, heads, dim, vdim, float(q_scale), int(bool(silu)), int(bool(chunked)),
-        qk_heads, _ptr(step), 0 if step is None else step.stride(0), _ptr(step_bias), _ptr(step_rate), _ptr(skip), _stream()),
-        "scalar_gate_scan")
+        qk_heads, _ptr(step), 0 if step is None else step.stride(0), _ptr(step_bias), _ptr(step_rate), _ptr(skip),
+        int(is_bf16), _stream()), "scalar_gate_scan")
+
+
+def state_space_tile_rows() -> int:
+    return int(library().dli_state_space_tile_rows())
+
+
+def state_space_tiles_supports(state_size: int, value_dim: int) -> bool:
+    return bool(library().dli_state_space_tiles_supports(int(state_size), int(value_dim)))
+
+
+def state_space_tiles(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.Tensor, q_start: torch.Tensor,
+                      positions: torch.Tensor, state_slots: torch.Tensor, tiles: tuple, o: torch.Tensor, heads: int, dim: int,
+                      vdim: int, *, qk_heads: int, step: torch.Tensor, step_bias: torch.Tensor, step_rate: torch.Tensor,
+                      skip: Optional[torch.Tensor] = None) -> None:
+    """:func:`scalar_gate_scan` under a step size for the entries that ``tiles`` lists (``StepContext.q_tiles`` of
+    :func:`state_space_tile_rows` rows: all tiles of each entry), on the bfloat16 matrix cores and without a chain over the
+    tokens. ``q, k [n, qk_heads*dim]`` and ``v [n, heads*vdim]`` are bfloat16 columns of one matrix, sizes as
+    :func:`state_space_tiles_supports` takes them; steps, decays and the state are 32-bit. ``o``: rows of listed entries."""
+    n = q.shape[0]
+    _require(qk_heads > 0 and heads % qk_heads == 0 and state_space_tiles_supports(dim, vdim), "heads or sizes that the tiles do not take")
+    for name, t, width in (("q", q, qk_heads * dim), ("k", k, qk_heads * dim), ("v", v, heads * vdim)):
+        _rows(t, name, torch.bfloat16)
+        _require(t.shape == (n, width) and t.stride(0) == q.stride(0) and t.data_ptr() % 16 == 0,
+                 f"{name} must be [n, {width}], 16-byte aligned columns of the matrix that q and k lie in")
+    _f32_rows(o, "o")
+    _f32_rows(step, "step")
+    _require(q.stride(0) % 8 == 0 and o.shape == (n, heads * vdim) and o.stride(0) % 4 == 0 and o.data_ptr() % 16 == 0
+             and step.shape == (n, heads), "o must be [n, heads*vdim], step [n, heads], rows aligned")
+    for name, t in (("step_bias", step_bias), ("step_rate", step_rate), ("skip", skip)):
+        if t is not None:
+            _dense(t, name, torch.float32, 1)
+            _require(t.shape[0] == heads, f"{name} must hold a value per head")
+    _state_rows(state, heads * vdim * dim)
+    _require(state.stride(0) % 4 == 0 and state.data_ptr() % 16 == 0, "a slot of the state must begin on 16 bytes")
+    _step_arrays(q_start, positions, state_slots, n)
+    tile_entry, tile_q0 = tiles
+    _dense(tile_entry, "tile_entry", torch.int32, 1)
+    _dense(tile_q0, "tile_q0", torch.int32, 1)
+    _require(tile_entry.shape == tile_q0.shape, "tile lists differ in length")
+    count, size = tile_entry.shape[0], heads * vdim * dim
+    if count == 0:
+        return
+    ends = torch.empty(count, size, device=q.device, dtype=torch.float32)
+    total = torch.empty(count, heads, device=q.device, dtype=torch.float32)
+    planes = torch.empty(2, count, size, device=q.device, dtype=torch.bfloat16)
+    _check(library().dli_state_space_tiles(
+        _ptr(q), _ptr(k), _ptr(v), q.stride(0), _ptr(step), step.stride(0), _ptr(step_bias), _ptr(step_rate), _ptr(skip), _ptr(state),
+        state.stride(0), _ptr(q_start), _ptr(positions), _ptr(state_slots), _ptr(tile_entry), _ptr(tile_q0), count, _ptr(ends),
+        _ptr(total), _ptr(planes[0]), _ptr(planes[1]), _ptr(o), o.stride(0), heads, qk_heads, dim, vdim, _stream()),
+        "state_space_tiles")
 
 
 def diff_head_norm(a: torch.Tensor, lam: float, after: float, eps: float, gate: Optional[torch.Tensor], out: torch.Tensor,

@@ -8,9 +8,11 @@ reads ``B`` and ``C`` of group ``head // (num_heads / groups)``: ``S <- exp(-exp
 value_dim``), ``y = S^T C + D x``. The heads side by side are multiplied by ``silu(z)``, each of ``norm_groups`` equal parts
 is divided by its root mean square, the row is multiplied by ``norm``; then the output product.
 
-The recurrence is the one of ``csrc/scalar_gate_scan.hip`` with ``q = C``, ``k = B``, ``v = x``. The request's state slot
-holds ``S`` and the convolution's last ``conv_taps - 1`` inputs, all 32-bit; everything between the projections and the
-output product is 32-bit."""
+The recurrence is the one of ``csrc/scalar_gate_scan.hip`` under a step size, with ``q = C``, ``k = B``, ``v = x``; the portions
+of a bfloat16 step take ``csrc/state_space.hip``, tiles of tokens on the matrix cores. The request's state slot holds ``S``
+and the convolution's last ``conv_taps - 1`` inputs, all 32-bit. Step sizes, decays, the recurrence, gate and norm are 32-bit; in
+a bfloat16 runtime what leaves the convolution (``x``, ``B`` and ``C``) is rounded to bfloat16 once, for single tokens and
+portions alike, where the sizes let the matrix cores take the portions."""
 
 from __future__ import annotations
 
@@ -56,7 +58,7 @@ class StateSpace(Mixer):
         self.norm_w, self.w_o = tensors["norm"].contiguous(), tensors["o"]
 
     def cache_spec(self) -> StateSpec:
-        return StateSpec((self.state_floats + (self.taps - 1) * self.channels,), torch.float32)
+        return StateSpec((-(-(self.state_floats + (self.taps - 1) * self.channels) // 4) * 4,), torch.float32)  # (slots begin on 16 bytes)
 
     def graph_capturable(self, page_size: int) -> bool:
         return True  # kernels on the context's device arrays only; padding rows write the spare slot
@@ -76,14 +78,24 @@ class StateSpace(Mixer):
         n, c, gn, dev = x.shape[0], self.inner, self.groups * self.state_size, self.rt.device
         if proj is None:
             proj = linear_f32(self.rt, as_operand(self.rt, x, ctx), self.w_in)          # z | x | B | C | dt
-        xbc = torch.empty(n, self.channels, device=dev, dtype=torch.float32)
+        tiled = self.rt.is_bf16 and ops.state_space_tiles_supports(self.state_size, self.value_dim)
+        xbc = torch.empty(n, self.channels, device=dev, dtype=torch.bfloat16 if tiled else torch.float32)
         ops.causal_conv(proj[:, c:], self.conv_w, self.conv_b, state, self.state_floats, ctx.q_start, ctx.positions,
-                        ctx.state_slots, xbc, act="silu")
+                        ctx.state_slots, None if tiled else xbc, rounded=xbc if tiled else None, act="silu")
         y = torch.empty(n, c, device=dev, dtype=torch.float32)
-        ops.scalar_gate_scan(xbc[:, c + gn:], xbc[:, c:c + gn], xbc[:, :c], state, ctx.q_start, ctx.positions, ctx.state_slots, y,
-                             self.num_heads, self.state_size, self.value_dim, qk_heads=self.groups,
-                             step=proj[:, c + self.channels:c + self.channels + self.num_heads], step_bias=self.dt_bias,
-                             step_rate=self.a_log, skip=self.d)
+        C, B, v = xbc[:, c + gn:], xbc[:, c:c + gn], xbc[:, :c]
+        step = proj[:, c + self.channels:c + self.channels + self.num_heads]
+        sizes = (self.num_heads, self.state_size, self.value_dim)
+        rule = dict(qk_heads=self.groups, step_bias=self.dt_bias, step_rate=self.a_log, skip=self.d)
+        nd = ctx.num_decode if tiled else n     # (single tokens come first; without tiles the scan takes every entry)
+        if nd == n or not tiled:
+            ops.scalar_gate_scan(C, B, v, state, ctx.q_start, ctx.positions, ctx.state_slots, y, *sizes, step=step, **rule)
+        else:
+            if nd:
+                ops.scalar_gate_scan(C[:nd], B[:nd], v[:nd], state, ctx.q_start[:nd + 1], ctx.positions[:nd], ctx.state_slots[:nd], y[:nd],
+                                     *sizes, step=step[:nd], **rule)
+            ops.state_space_tiles(C, B, v, state, ctx.q_start, ctx.positions, ctx.state_slots,
+                                  ctx.q_tiles(ops.state_space_tile_rows(), first_entry=nd), y, *sizes, step=step, **rule)
         out = self.rt.empty(n, c)
         ops.head_norm_gate(y, proj[:, :c], self.norm_w, self.norm_eps, out, self.norm_groups, c // self.norm_groups,
                            gate="silu_first")

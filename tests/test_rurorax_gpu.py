@@ -296,6 +296,75 @@ def test_state_space_over_long_portions(ops, H, G, N, V):
         assert (held - S).abs().max() < 2e-5 * max(1.0, S.abs().max())
 
 
+def scan_tiles(ops, rows, state, q_start, positions, slots, H, G, N, V, p, singles_scanned=False):
+    """The same with x, B and C rounded to bfloat16, in tiles on the matrix cores (``singles_scanned``: entries of one row,
+    which must come first, by the scan)."""
+    x1, b1, c1 = H * V, H * V + G * N, H * V + 2 * G * N
+    n = rows.shape[0]
+    xbc = torch.empty(n, c1, dtype=torch.bfloat16).cuda()
+    xbc.copy_(rows[:, :c1])
+    o = torch.full((n, H * V), 77.0).cuda()
+    starts = q_start.tolist()
+    lengths = [b - a for a, b in zip(starts, starts[1:])]
+    step, rule = rows[:, c1:c1 + H], dict(qk_heads=G, step_bias=p["bias"].cuda(), step_rate=p["a_log"].cuda(), skip=p["d"].cuda())
+    nd = next((i for i, m in enumerate(lengths) if m > 1), len(lengths)) if singles_scanned else 0
+    if nd:
+        ops.scalar_gate_scan(xbc[:nd, b1:], xbc[:nd, x1:b1], xbc[:nd, :x1], state, q_start[:nd + 1], positions[:nd], slots[:nd], o[:nd],
+                             H, N, V, step=step[:nd], **rule)
+    tile = ops.state_space_tile_rows()
+    ent = [e for e in range(nd, len(lengths)) for _ in range(0, lengths[e], tile)]
+    q0 = [q for e in range(nd, len(lengths)) for q in range(0, lengths[e], tile)]
+    if ent:
+        ops.state_space_tiles(xbc[:, b1:], xbc[:, x1:b1], xbc[:, :x1], state, q_start, positions, slots, (i32(ent), i32(q0)), o, H, N, V,
+                              step=step, **rule)
+    return o
+
+
+def rounded_inputs(x, H, G, N, V):
+    c1 = H * V + 2 * G * N
+    return torch.cat([x[:, :c1].to(torch.bfloat16).float(), x[:, c1:]], dim=1)
+
+
+@pytest.mark.parametrize("singles_scanned", [False, True])
+@pytest.mark.parametrize("H,G,N,V", [(2, 1, 32, 8), (4, 2, 32, 48), (8, 1, 64, 64), (4, 2, 128, 64), (2, 1, 96, 40), (3, 3, 128, 104), (2, 2, 64, 136)])
+def test_state_space_in_tiles_against_whole(ops, H, G, N, V, singles_scanned):
+    """Portions shorter and longer than a tile and a tile's block, on fresh and on earlier states, beside single tokens."""
+    g = torch.Generator().manual_seed(N + V)
+    p, width = scan_params(H, g), H * V + 2 * G * N + H
+    lengths = {"a": 1300, "b": 700, "c": 5, "d": 64}
+    reqs = {r: (i, torch.randn(n, width, generator=g)) for i, (r, n) in enumerate(lengths.items())}
+    floats = H * V * N
+    state = torch.full((4, floats + 4), -9.0).cuda()
+    plan = [[("b", 1), ("a", 131)], [("b", 1), ("a", 1029), ("c", 2)], [("c", 1), ("a", 63), ("b", 513)], [("a", 1), ("c", 2), ("b", 128)],
+            [("b", 57), ("a", 76), ("d", 64)]]
+    got = in_steps(reqs, plan, lambda rows, qs, pos, sl: scan_tiles(ops, rows, state, qs, pos, sl, H, G, N, V, p, singles_scanned))
+    for r, (slot, x) in reqs.items():
+        ref, S = plain_scan(rounded_inputs(x, H, G, N, V), H, G, N, V, p)
+        # (the results' second operands are sums of two bfloat16 numbers: 2^-17; the state itself is 32-bit)
+        assert (got[r].double() - ref).abs().max() < 5e-5 * max(1.0, ref.abs().max()), (r, (got[r].double() - ref).abs().max())
+        held = state[slot, :floats].cpu().double().view(H, V, N).transpose(1, 2)
+        assert (held - S).abs().max() < 1e-5 * max(1.0, S.abs().max()), (r, (held - S).abs().max())
+    assert (state[:, floats:] == -9.0).all()
+
+
+def test_tiles_forget_and_remember(ops):
+    """Pre-activations of -60 and +60 token by token, a head that hardly decays and one that forgets within a token: the
+    factors span what 32-bit holds, and a value written 700 tokens ago is found again."""
+    H, G, N, V, n = 2, 1, 32, 8, 900
+    g = torch.Generator().manual_seed(3)
+    p = {"bias": torch.zeros(H), "a_log": torch.tensor([-30.0, 3.0]), "d": torch.tensor([0.0, 0.5])}
+    rows = torch.randn(n, H * V + 2 * G * N + H, generator=g)
+    rows[:, -H:] = torch.where(torch.rand(n, H, generator=g) < 0.7, torch.tensor(-60.0), torch.tensor(60.0))
+    rows[200:, H * V:H * V + N] = 0.0                           # nothing is written from here on
+    ref, S = plain_scan(rounded_inputs(rows, H, G, N, V), H, G, N, V, p)
+    state = torch.full((1, H * V * N), 5.0).cuda()
+    got = in_steps({"a": (0, rows)}, [[("a", 500)], [("a", 1)], [("a", 399)]],
+                   lambda r, qs, pos, sl: scan_tiles(ops, r, state, qs, pos, sl, H, G, N, V, p, True))["a"]
+    assert ref[700:, :V].abs().max() > 10
+    assert (got.double() - ref).abs().max() < 5e-5 * ref.abs().max()
+    assert (state[0].cpu().double().view(H, V, N).transpose(1, 2) - S).abs().max() < 1e-5 * S.abs().max()
+
+
 @pytest.mark.parametrize("N", [16, 128, 20])
 def test_a_state_written_long_ago_is_still_there(ops, N):
     """A head that hardly decays: what the first token wrote answers a query 900 tokens later, over portions and single
