@@ -31,6 +31,8 @@ typedef __attribute__((address_space(3))) ss_bf4* ss_lds4;
 
 #define SS_TILE 256
 
+template <int I> struct SsInt { static constexpr int value = I; };
+
 struct SsArgs {
   const bf16_t* q; const bf16_t* k; const bf16_t* v; int64_t stride;   // [rows][stride], each at its first column
   const float* step; int64_t step_stride; const float* bias; const float* rate; const float* skip;
@@ -81,7 +83,7 @@ __global__ __launch_bounds__(256, 2) void state_space_tile_state_kernel(SsArgs p
   __shared__ __align__(16) bf16_t sk[64 * LK], sv[3][64 * LV];
   __shared__ float sw[SS_TILE];
   __shared__ double sh[4];
-  const int tid = threadIdx.x, lane = tid % 64, wave = tid / 64, col = lane & 15, grp = lane >> 4;
+  const int tid = threadIdx.x, lane = tid % 64, wave = __builtin_amdgcn_readfirstlane(tid / 64), col = lane & 15, grp = lane >> 4;
   const int tile = blockIdx.x, head = blockIdx.y, v0 = blockIdx.z * 64;
   const int entry = p.tile_entry[tile], q0 = p.tile_q0[tile];
   const int row0 = p.q_start[entry] + q0, n_rows = min(SS_TILE, p.q_start[entry + 1] - row0);
@@ -169,192 +171,214 @@ __global__ __launch_bounds__(256, 2) void state_space_tile_state_kernel(SsArgs p
   }
 }
 
-// Four neighbours of the state a thread, of the entry that a tile with tile_q0 0 begins.
+// Two neighbours of the state a thread, of the entry that a tile with tile_q0 0 begins. (The tile is the grid's slowest
+// coordinate: the workgroups of such tiles, which do all the work, then lie side by side and go round all XCDs.)
 __global__ __launch_bounds__(256) void state_space_carry_kernel(SsArgs p) {
-  constexpr int AHEAD = 8;
-  const int first = blockIdx.x, head = blockIdx.y, i = 4 * (blockIdx.z * 256 + threadIdx.x), size = p.V * p.N;
+  typedef float f2 __attribute__((ext_vector_type(2)));
+  typedef __bf16 b2 __attribute__((ext_vector_type(2)));
+  constexpr int AHEAD = 8;                                  // tiles asked for at once, the next ones before these are walked
+  const int first = blockIdx.z, head = blockIdx.y, i = 2 * (blockIdx.x * 256 + threadIdx.x), size = p.V * p.N;
   if (p.tile_q0[first] != 0 || i >= size) return;
   const int entry = p.tile_entry[first];
   const int row0 = p.q_start[entry], tiles = (p.q_start[entry + 1] - row0 + SS_TILE - 1) / SS_TILE;
   float* st = p.state + (int64_t)p.state_slots[entry] * p.state_stride + (int64_t)head * size + i;
   const int64_t hop = (int64_t)p.heads * size;
   const int64_t at = ((int64_t)first * p.heads + head) * size + i;
-  ss_f4 S = *reinterpret_cast<const ss_f4*>(st);
-  if (p.positions[row0] == 0) S = ss_f4{0.f, 0.f, 0.f, 0.f};
-  ss_f4 e[AHEAD];
-  float a[AHEAD];
-  auto fetch = [&](int j, int t) {
-    t = min(t, tiles - 1);
-    e[j] = *reinterpret_cast<const ss_f4*>(p.ends + at + t * hop);
-    a[j] = p.total[(int64_t)(first + t) * p.heads + head];
-  };
+  f2 S = *reinterpret_cast<const f2*>(st);
+  if (p.positions[row0] == 0) S = f2{0.f, 0.f};
+  f2 e[2][AHEAD];
+  float a[2][AHEAD];
+  auto fetch = [&](int w, int t0) {
 #pragma unroll
-  for (int j = 0; j < AHEAD; ++j) fetch(j, j);
-  for (int t0 = 0; t0 < tiles; t0 += AHEAD) {
-#pragma unroll
-    for (int j = 0; j < AHEAD; ++j) {
-      if (t0 + j >= tiles) break;
-      ss_bf4 hi, lo;
-#pragma unroll
-      for (int c = 0; c < 4; ++c) {
-        hi[c] = (bf16_t)S[c];
-        lo[c] = (bf16_t)(S[c] - (float)hi[c]);
-        S[c] = fmaf(a[j], S[c], e[j][c]);
-      }
-      *reinterpret_cast<ss_bf4*>(p.in_hi + at + (t0 + j) * hop) = hi;
-      *reinterpret_cast<ss_bf4*>(p.in_lo + at + (t0 + j) * hop) = lo;
-      fetch(j, t0 + AHEAD + j);
+    for (int j = 0; j < AHEAD; ++j) {                       // (tiles past the last repeat it)
+      const int t = min(t0 + j, tiles - 1);
+      e[w][j] = *reinterpret_cast<const f2*>(p.ends + at + t * hop);
+      a[w][j] = p.total[(int64_t)(first + t) * p.heads + head];
     }
+  };
+  auto walk = [&](int w, int t0) {
+#pragma unroll
+    for (int j = 0; j < AHEAD; ++j)
+      if (t0 + j < tiles) {
+        b2 hi, lo;
+#pragma unroll
+        for (int c = 0; c < 2; ++c) {
+          hi[c] = (bf16_t)S[c];
+          lo[c] = (bf16_t)(S[c] - (float)hi[c]);
+          S[c] = fmaf(a[w][j], S[c], e[w][j][c]);
+        }
+        *reinterpret_cast<b2*>(p.in_hi + at + (t0 + j) * hop) = hi;
+        *reinterpret_cast<b2*>(p.in_lo + at + (t0 + j) * hop) = lo;
+      }
+  };
+  fetch(0, 0);
+  for (int t0 = 0; t0 < tiles; t0 += 2 * AHEAD) {
+    if (t0 + AHEAD < tiles) fetch(1, t0 + AHEAD);
+    walk(0, t0);
+    if (t0 + AHEAD >= tiles) break;
+    if (t0 + 2 * AHEAD < tiles) fetch(0, t0 + 2 * AHEAD);
+    walk(1, t0 + AHEAD);
   }
-  *reinterpret_cast<ss_f4*>(st) = S;
+  *reinterpret_cast<f2*>(st) = S;
 }
 
-// A workgroup a (tile, head, 64 values). Wave w takes the tokens 64 b + 16 w .. + 15 for b = 0 .. 3, so that all waves see as
-// many earlier tokens; k and v of 64 tokens at a time pass through LDS.
+// A workgroup a (tile, head, 64 values, half of the tile's runs of 16 tokens). Of the sixteen runs wave w takes j = 2 w + half
+// and 15 - j, so that all waves see as many earlier tokens. What is multiplied passes through LDS 64 rows at a time, the
+// next in flight meanwhile: first the two halves of the state at the tile's beginning (64 values' rows of N), then k and v of
+// 64 tokens after the other.
 template <int NT>
 __global__ __launch_bounds__(256, 2) void state_space_tile_result_kernel(SsArgs p) {
   constexpr int N = 32 * NT, LK = N + 8, LV = 64 + 8, KP = NT;
   __shared__ __align__(16) bf16_t sk[64 * LK], sv[64 * LV];
   __shared__ __align__(16) float s_hi[SS_TILE], s_lo[SS_TILE], s_dt[SS_TILE];
   __shared__ double sh[4];
-  const int tid = threadIdx.x, lane = tid % 64, wave = tid / 64, col = lane & 15, grp = lane >> 4;
-  const int tile = blockIdx.x, head = blockIdx.y, v0 = blockIdx.z * 64;
+  const int tid = threadIdx.x, lane = tid % 64, wave = __builtin_amdgcn_readfirstlane(tid / 64), col = lane & 15, grp = lane >> 4;
+  const int tile = blockIdx.x, head = blockIdx.y, v0 = (blockIdx.z >> 1) * 64;
   const int entry = p.tile_entry[tile], q0 = p.tile_q0[tile];
   const int start = p.q_start[entry], row0 = start + q0, n_rows = min(SS_TILE, p.q_start[entry + 1] - row0);
   if (n_rows <= 0) return;
+  const int half = 2 * wave + (blockIdx.z & 1);
+  const int run[2] = {16 * half, 16 * (15 - half)};         // the first token of each of this wave's runs
+  const int blocks = (n_rows + 63) / 64;
   const int group = head / (p.heads / p.qk_heads);
   const bf16_t* qq = p.q + (int64_t)group * N;
   const bf16_t* kk = p.k + (int64_t)group * N;
   const bf16_t* vv = p.v + (int64_t)head * p.V + v0;
   const int vlast = min(64, p.V - v0) - 8;
+  const int64_t in_at = ((int64_t)tile * p.heads + head) * p.V * N;
+  const bool carried = q0 != 0 || p.positions[start] != 0;  // (else the state at the tile's beginning is zero)
   ss_bf8 rk[KP], rv[2];
-  auto fetch = [&](int c0) {                                // rows past the last: the last again, with a step of zero
+  auto fetch = [&](int stage) {                             // (rows past the last: the last again; such tokens have a step of zero)
+    const bf16_t* base = stage == -2 ? p.in_hi + in_at : stage == -1 ? p.in_lo + in_at : kk + (int64_t)row0 * p.stride;
+    const int64_t hop = stage < 0 ? N : p.stride;
+    const int r0 = stage < 0 ? v0 : 64 * stage, last = stage < 0 ? p.V - 1 : n_rows - 1;
 #pragma unroll
     for (int m = 0; m < KP; ++m) {
       const int idx = tid + 256 * m, t = idx / (4 * NT), c = idx % (4 * NT);
-      rk[m] = *reinterpret_cast<const ss_bf8*>(kk + (int64_t)(row0 + min(c0 + t, n_rows - 1)) * p.stride + 8 * c);
+      rk[m] = *reinterpret_cast<const ss_bf8*>(base + min(r0 + t, last) * hop + 8 * c);
     }
+    if (stage >= 0)
 #pragma unroll
-    for (int m = 0; m < 2; ++m) {
-      const int idx = tid + 256 * m, t = idx / 8, c = idx % 8;
-      rv[m] = *reinterpret_cast<const ss_bf8*>(vv + (int64_t)(row0 + min(c0 + t, n_rows - 1)) * p.stride + min(8 * c, vlast));
-    }
+      for (int m = 0; m < 2; ++m) {
+        const int idx = tid + 256 * m, t = idx / 8, c = idx % 8;
+        rv[m] = *reinterpret_cast<const ss_bf8*>(vv + (int64_t)(row0 + min(64 * stage + t, n_rows - 1)) * p.stride + min(8 * c, vlast));
+      }
   };
-  fetch(0);
-  ss_bf8 qb[4][NT];
+  const int first = carried ? -2 : 0;
+  fetch(first);
+  ss_bf8 qb[2][NT];
 #pragma unroll
-  for (int b = 0; b < 4; ++b) {
-    const bf16_t* qr = qq + (int64_t)(row0 + min(64 * b + 16 * wave + col, n_rows - 1)) * p.stride + 8 * grp;
+  for (int b = 0; b < 2; ++b) {
+    const bf16_t* qr = qq + (int64_t)(row0 + min(run[b] + col, n_rows - 1)) * p.stride + 8 * grp;
 #pragma unroll
     for (int d = 0; d < NT; ++d) qb[b][d] = *reinterpret_cast<const ss_bf8*>(qr + 32 * d);
   }
   {
     float dt;
-    double run, all;
-    ss_steps(p, row0, n_rows, head, sh, &dt, &run, &all);
-    s_hi[tid] = (float)run;
-    s_lo[tid] = (float)(run - (double)(float)run);
+    double sum, all;
+    ss_steps(p, row0, n_rows, head, sh, &dt, &sum, &all);
+    s_hi[tid] = (float)sum;
+    s_lo[tid] = (float)(sum - (double)(float)sum);
     s_dt[tid] = dt;
   }
-  ss_f4 acc[4][4];
+  ss_f4 acc[2][4];
 #pragma unroll
-  for (int b = 0; b < 4; ++b)
+  for (int b = 0; b < 2; ++b)
 #pragma unroll
     for (int v = 0; v < 4; ++v) acc[b][v] = ss_f4{0.f, 0.f, 0.f, 0.f};
-  if (q0 != 0 || p.positions[start] != 0) {                 // (else the state at the tile's beginning is zero)
-    const int64_t at = ((int64_t)tile * p.heads + head) * p.V * N;
-#pragma unroll
-    for (int v = 0; v < 4; ++v) {
-      const int64_t row = at + (int64_t)min(v0 + 16 * v + col, p.V - 1) * N + 8 * grp;
-#pragma unroll
-      for (int d = 0; d < NT; ++d) {
-        const ss_bf8 hi = *reinterpret_cast<const ss_bf8*>(p.in_hi + row + 32 * d);
-        const ss_bf8 lo = *reinterpret_cast<const ss_bf8*>(p.in_lo + row + 32 * d);
-#pragma unroll
-        for (int b = 0; b < 4; ++b) {
-          acc[b][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(hi, qb[b][d], acc[b][v], 0, 0, 0);
-          acc[b][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lo, qb[b][d], acc[b][v], 0, 0, 0);
-        }
-      }
-    }
-  }
-  __syncthreads();                                          // the steps are in LDS
-  float t_hi[4], t_lo[4];
-#pragma unroll
-  for (int b = 0; b < 4; ++b) {
-    const int t = 64 * b + 16 * wave + col;
-    t_hi[b] = s_hi[t];
-    t_lo[b] = s_lo[t];
-    const float f = __builtin_amdgcn_exp2f(t_hi[b] + t_lo[b]);
-#pragma unroll
-    for (int v = 0; v < 4; ++v) acc[b][v] *= f;
-  }
-  const int blocks = (n_rows + 63) / 64;
-  for (int kb = 0; kb < blocks; ++kb) {
-    __syncthreads();                                        // the block before has been read
+  float t_hi[2], t_lo[2];
+  for (int stage = first; stage < blocks; ++stage) {
+    __syncthreads();                                        // the stage before has been read
 #pragma unroll
     for (int m = 0; m < KP; ++m) {
       const int idx = tid + 256 * m, t = idx / (4 * NT), c = idx % (4 * NT);
       *reinterpret_cast<ss_bf8*>(&sk[t * LK + 8 * c]) = rk[m];
     }
+    if (stage >= 0)
 #pragma unroll
-    for (int m = 0; m < 2; ++m) {
-      const int idx = tid + 256 * m, t = idx / 8, c = idx % 8;
-      *reinterpret_cast<ss_bf8*>(&sv[t * LV + 8 * c]) = rv[m];
-    }
+      for (int m = 0; m < 2; ++m) {
+        const int idx = tid + 256 * m, t = idx / 8, c = idx % 8;
+        *reinterpret_cast<ss_bf8*>(&sv[t * LV + 8 * c]) = rv[m];
+      }
     __syncthreads();
-    if (kb + 1 < blocks) fetch(64 * (kb + 1));
-#pragma unroll 1
-    for (int k = 0; k < 2; ++k) {                           // 32 tokens at a time
-      ss_f4 s[4][2];
+    if (stage + 1 < blocks) fetch(stage + 1);
+    if (stage < 0) {
 #pragma unroll
-      for (int b = 0; b < 4; ++b) s[b][0] = s[b][1] = ss_f4{0.f, 0.f, 0.f, 0.f};
+      for (int v = 0; v < 4; ++v)
+#pragma unroll
+        for (int d = 0; d < NT; ++d) {
+          const ss_bf8 f = *reinterpret_cast<const ss_bf8*>(&sk[(16 * v + col) * LK + 32 * d + 8 * grp]);
+#pragma unroll
+          for (int b = 0; b < 2; ++b) acc[b][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f, qb[b][d], acc[b][v], 0, 0, 0);
+        }
+      if (stage == -1)
+#pragma unroll
+        for (int b = 0; b < 2; ++b) {
+          const float f = __builtin_amdgcn_exp2f(s_hi[run[b] + col] + s_lo[run[b] + col]);
+#pragma unroll
+          for (int v = 0; v < 4; ++v) acc[b][v] *= f;
+        }
+      continue;
+    }
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+      t_hi[b] = s_hi[run[b] + col];
+      t_lo[b] = s_lo[run[b] + col];
+    }
+    // 32 tokens from j0 on against the wave's runs from FROM on
+    auto against = [&](auto from, int k) {
+      constexpr int FROM = decltype(from)::value;
+      const int j0 = 64 * stage + 32 * k;
+      ss_f4 s[2][2];
+#pragma unroll
+      for (int b = FROM; b < 2; ++b) s[b][0] = s[b][1] = ss_f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int u = 0; u < 2; ++u)
 #pragma unroll
         for (int d = 0; d < NT; ++d) {
           const ss_bf8 kf = *reinterpret_cast<const ss_bf8*>(&sk[(32 * k + 16 * u + col) * LK + 32 * d + 8 * grp]);
 #pragma unroll
-          for (int b = 0; b < 4; ++b)
-            if (b >= kb) s[b][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qb[b][d], s[b][u], 0, 0, 0);
+          for (int b = FROM; b < 2; ++b) s[b][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qb[b][d], s[b][u], 0, 0, 0);
         }
-      // s[b][u][i]: token 64 kb + 32 k + 16 u + 4 grp + i against this lane's token of b
-      ss_bf8 ph[4], pl[4];
+      // s[b][u][i]: token j0 + 16 u + 4 grp + i against this lane's token of run b
+      ss_bf8 ph[2], pl[2];
 #pragma unroll
       for (int u = 0; u < 2; ++u) {
-        const int at = 64 * kb + 32 * k + 16 * u + 4 * grp;
+        const int at = j0 + 16 * u + 4 * grp;
         const ss_f4 hi = *reinterpret_cast<const ss_f4*>(&s_hi[at]), lo = *reinterpret_cast<const ss_f4*>(&s_lo[at]);
         const ss_f4 dt = *reinterpret_cast<const ss_f4*>(&s_dt[at]);
 #pragma unroll
-        for (int b = 0; b < 4; ++b)
-          if (b >= kb) {
+        for (int b = FROM; b < 2; ++b)
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-              float x = (t_hi[b] - hi[i]) + (t_lo[b] - lo[i]);
-              if (b == kb) x = at + i <= 64 * b + 16 * wave + col ? x : -INFINITY;
-              const float w = s[b][u][i] * (__builtin_amdgcn_exp2f(x) * dt[i]);
-              const bf16_t h = (bf16_t)w;
-              ph[b][4 * u + i] = h;
-              pl[b][4 * u + i] = (bf16_t)(w - (float)h);
-            }
+          for (int i = 0; i < 4; ++i) {
+            const float x = (t_hi[b] - hi[i]) + (t_lo[b] - lo[i]);
+            const float w = s[b][u][i] * (__builtin_amdgcn_exp2f(at + i <= run[b] + col ? x : -INFINITY) * dt[i]);
+            const bf16_t h = (bf16_t)w;
+            ph[b][4 * u + i] = h;
+            pl[b][4 * u + i] = (bf16_t)(w - (float)h);
           }
       }
 #pragma unroll
       for (int v = 0; v < 4; ++v) {
         const ss_bf8 vf = ss_column(&sv[(32 * k + 4 * grp + col / 4) * LV + 16 * v + 4 * (col % 4)], LV);
 #pragma unroll
-        for (int b = 0; b < 4; ++b)
-          if (b >= kb) {
-            acc[b][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph[b], acc[b][v], 0, 0, 0);
-            acc[b][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl[b], acc[b][v], 0, 0, 0);
-          }
+        for (int b = FROM; b < 2; ++b) {
+          acc[b][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph[b], acc[b][v], 0, 0, 0);
+          acc[b][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl[b], acc[b][v], 0, 0, 0);
+        }
       }
+    };
+#pragma unroll 1
+    for (int k = 0; k < 2; ++k) {
+      const int j0 = 64 * stage + 32 * k;                   // (the second run lies behind the first)
+      if (j0 <= run[0] + 15) against(SsInt<0>{}, k);
+      else if (j0 <= run[1] + 15 && run[1] < n_rows) against(SsInt<1>{}, k);
     }
   }
   const float skip = p.skip != nullptr ? p.skip[head] : 0.f;
 #pragma unroll
-  for (int b = 0; b < 4; ++b) {
-    const int t = 64 * b + 16 * wave + col;
+  for (int b = 0; b < 2; ++b) {
+    const int t = run[b] + col;
     if (t >= n_rows) continue;
     const bf16_t* vr = vv + (int64_t)(row0 + t) * p.stride;
     float* out = p.o + (int64_t)(row0 + t) * p.o_stride + (int64_t)head * p.V + v0;
@@ -400,13 +424,13 @@ int dli_state_space_tiles(const void* q, const void* k, const void* v, int64_t s
   p.q_start = q_start; p.positions = positions; p.state_slots = state_slots; p.tile_entry = tile_entry; p.tile_q0 = tile_q0;
   p.ends = ends; p.total = total; p.in_hi = (bf16_t*)in_hi; p.in_lo = (bf16_t*)in_lo; p.o = o; p.o_stride = o_stride;
   p.heads = heads; p.qk_heads = qk_heads; p.V = value_dim; p.N = state_size;
-  const dim3 grid(tiles, heads, (value_dim + 63) / 64), carry(tiles, heads, (unsigned)((size / 4 + 255) / 256));
-  if (grid.z > 65535 || carry.z > 65535) return DLI_ERR_ARGUMENT;
+  const dim3 grid(tiles, heads, (value_dim + 63) / 64), result(tiles, heads, 2 * grid.z), carry((unsigned)((size / 2 + 255) / 256), heads, tiles);
+  if (result.z > 65535 || carry.z > 65535) return DLI_ERR_ARGUMENT;
 #define SS_CASE(NT)                                                                  \
   case NT:                                                                           \
     state_space_tile_state_kernel<NT><<<grid, 256, 0, stream>>>(p);                  \
     state_space_carry_kernel<<<carry, 256, 0, stream>>>(p);                          \
-    state_space_tile_result_kernel<NT><<<grid, 256, 0, stream>>>(p);                 \
+    state_space_tile_result_kernel<NT><<<result, 256, 0, stream>>>(p);                 \
     break;
   switch (state_size / 32) { SS_CASE(1) SS_CASE(2) SS_CASE(3) SS_CASE(4) }
 #undef SS_CASE

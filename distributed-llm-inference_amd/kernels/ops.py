@@ -110,6 +110,11 @@ _SIGNATURES = {
     "dli_attention_scored_mfma": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr,
                                   _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _c_ptr,
                                   _c_ptr, _c_ptr, _c_i64, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr],
+    "dli_attention_grouped_supports": [_c_int, _c_int, _c_int],
+    "dli_attention_grouped_tile_tokens": [_c_int, _c_int],
+    "dli_attention_grouped": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int,
+                              _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _c_int, _c_ptr,
+                              _c_ptr, _c_i64, _c_int, _c_ptr],
     "dli_attention_keyvalue_supports": [_c_int, _c_int],
     "dli_attention_keyvalue_tile_tokens": [_c_int, _c_int],
     "dli_attention_keyvalue_splits": [_c_int, _c_int, _c_int, _c_int],
@@ -1754,6 +1759,58 @@ def attention_scored_mfma(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch
         kv_heads, head_dim, value_dim, page_size, float(scale), int(window), int(chunk), int(bool(sink)), _ptr(r1),
         _ptr(r2), _ptr(gate), gate_stride, int(keep_first), v_heads, _ptr(out if out32 else None), _ptr(sinks), _stream()),
         "attention_scored_mfma")
+
+
+def attention_grouped_supports(head_dim: int, value_dim: int, page_size: int, dtype: torch.dtype) -> bool:
+    return dtype == torch.bfloat16 and bool(library().dli_attention_grouped_supports(int(head_dim), int(value_dim), int(page_size)))
+
+
+def attention_grouped_tile_tokens(q_heads: int, kv_heads: int) -> int:
+    return int(library().dli_attention_grouped_tile_tokens(int(q_heads), int(kv_heads)))
+
+
+def attention_grouped(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, out: torch.Tensor,
+                      q_start: torch.Tensor, kv_len: torch.Tensor, block_tables: torch.Tensor,
+                      tile_entry: torch.Tensor, tile_q0: torch.Tensor, q_heads: int, scale: float, *,
+                      window: int = 0, chunk: int = 0, sink: bool = False, gate: Optional[torch.Tensor] = None,
+                      keep_first: int = 0, sinks: Optional[torch.Tensor] = None) -> None:
+    """:func:`attention_scored` without a penalty on the distance, for the portions of a bfloat16 step, keys and values
+    passing through LDS once for all query heads of a kv head: tiles of :func:`attention_grouped_tile_tokens` tokens, sizes
+    that :func:`attention_grouped_supports` takes."""
+    _dense(k_pages, "k_pages", torch.bfloat16, 4)
+    _dense(v_pages, "v_pages", torch.bfloat16, 4)
+    _rows(q, "q", torch.bfloat16)
+    out32 = out.dtype == torch.float32
+    _rows(out, "out", torch.float32 if out32 else torch.bfloat16)
+    pages, kv_heads, page_size, head_dim = k_pages.shape
+    v_heads, value_dim = v_pages.shape[1], v_pages.shape[2]
+    _require(v_pages.shape == (pages, v_heads, value_dim, page_size) and v_heads > 0 and kv_heads % v_heads == 0,
+             "v_pages must be [pages, value heads, value_dim, page_size], the value heads a divisor of the kv heads")
+    _require(attention_grouped_supports(head_dim, value_dim, page_size, k_pages.dtype), "the grouped kernel does not take these sizes")
+    _require(q_heads % kv_heads == 0 and q.shape[1] == q_heads * head_dim and out.shape == (q.shape[0], q_heads * value_dim),
+             "q must be [tokens, q_heads*head_dim] and out [tokens, q_heads*value_dim], the query heads a multiple of the kv heads")
+    _require(q.stride(0) % 8 == 0 and out.stride(0) % 4 == 0 and q.data_ptr() % 16 == 0 and out.data_ptr() % 16 == 0
+             and k_pages.data_ptr() % 16 == 0 and v_pages.data_ptr() % 16 == 0, "q, out and the pages must be aligned for 16 bytes, row by row")
+    _require(keep_first >= 0, "keep_first must not be negative")
+    for name, t in (("q_start", q_start), ("kv_len", kv_len), ("tile_entry", tile_entry), ("tile_q0", tile_q0)):
+        _dense(t, name, torch.int32, 1)
+    _dense(block_tables, "block_tables", torch.int32, 2)
+    entries = kv_len.shape[0]
+    _require(q_start.shape[0] == entries + 1 and block_tables.shape[0] >= entries and tile_entry.shape == tile_q0.shape,
+             "q_start/kv_len/block_tables or the tile lists disagree")
+    if sinks is not None:
+        _dense(sinks, "sinks", torch.float32, 1)
+        _require(sinks.shape[0] == q_heads, "sinks must hold one value per query head")
+    gate_stride = 0
+    if gate is not None:
+        _f32_rows(gate, "gate")
+        _require(gate.shape == out.shape, "gate differs from out in shape")
+        gate_stride = gate.stride(0)
+    _check(library().dli_attention_grouped(
+        _ptr(q), q.stride(0), _ptr(k_pages), _ptr(v_pages), _ptr(out), out.stride(0), _ptr(q_start), _ptr(kv_len), _ptr(block_tables),
+        block_tables.stride(0), _ptr(tile_entry), _ptr(tile_q0), tile_entry.shape[0], q_heads, kv_heads, v_heads, head_dim, value_dim,
+        page_size, float(scale), int(window), int(chunk), int(keep_first), int(bool(sink)), _ptr(sinks), _ptr(gate), gate_stride,
+        int(out32), _stream()), "attention_grouped")
 
 
 def attention_keyvalue_supports(head_dim: int, value_dim: int, dtype: torch.dtype) -> bool:

@@ -62,8 +62,8 @@ def paged_scored_attention(rt: Runtime, ctx: Any, cache: Any, q: torch.Tensor, o
                            **changes: Any) -> None:
     """The attention of a step's rows over a paged cache, for any mixer that has written its keys and
     values there: steps of single tokens go to the kernel that reads the context's device arrays alone,
-    the portions of other steps to the matrix cores where they take the sizes (single tokens, which come
-    first, to their kernel), else to the vector-unit tile kernel. ``changes``: ``window``, ``chunk``, ``sink``,
+    the portions of other steps to the matrix cores where they take the sizes (with a penalty on the distance to a kernel of
+    their own; single tokens, which come first, to theirs), else to the vector-unit tile kernel. ``changes``: ``window``, ``chunk``, ``sink``,
     ``r1``, ``r2``, ``sinks`` as :func:`dli_amd.kernels.ops.attention_scored` takes them. A cache without value pages: the
     values are the keys' first ``value_dim`` components."""
     grp = ctx.groups[cache.group]
@@ -83,11 +83,17 @@ def paged_scored_attention(rt: Runtime, ctx: Any, cache: Any, q: torch.Tensor, o
         # every entry is one row: nothing is derived from the step's lengths on the host
         ops.attention_scored(q, cache.k_pages, cache.v_pages, out, ctx.q_start, ctx.kv_len, grp.block_tables,
                              None, None, num_heads, scale, gate=gate, **changes)
-    elif cache.v_pages is not None and ops.attention_scored_mfma_supports(head_dim, value_dim, ctx.page_size, rt.dtype):
+    elif cache.v_pages is not None and (_grouped_takes(rt, ctx, head_dim, value_dim, changes)
+                                        or ops.attention_scored_mfma_supports(head_dim, value_dim, ctx.page_size, rt.dtype)):
         if nd:
             ops.attention_scored(q[:nd], cache.k_pages, cache.v_pages, out[:nd], ctx.q_start[:nd + 1], ctx.kv_len[:nd],
                                  grp.block_tables[:nd], None, None, num_heads, scale,
                                  gate=None if gate is None else gate[:nd], **changes)
+        if _grouped_takes(rt, ctx, head_dim, value_dim, changes):
+            tiles = ctx.q_tiles(ops.attention_grouped_tile_tokens(num_heads, cache.k_pages.shape[1]), first_entry=nd)
+            ops.attention_grouped(q, cache.k_pages, cache.v_pages, out, ctx.q_start, ctx.kv_len, grp.block_tables, tiles[0], tiles[1],
+                                  num_heads, scale, gate=gate, **{n: v for n, v in changes.items() if n not in ("r1", "r2")})
+            return
         tiles = ctx.q_tiles(ops.SCORED_MFMA_TILE_ROWS, first_entry=nd)
         ops.attention_scored_mfma(q, cache.k_pages, cache.v_pages, out, ctx.q_start, ctx.kv_len, grp.block_tables,
                                   tiles[0], tiles[1], num_heads, scale, gate=gate, **changes)
@@ -95,6 +101,12 @@ def paged_scored_attention(rt: Runtime, ctx: Any, cache: Any, q: torch.Tensor, o
         tiles = ctx.q_tiles(ops.attention_generic_tile_rows(max(head_dim, value_dim)))
         ops.attention_scored(q, cache.k_pages, cache.v_pages, out, ctx.q_start, ctx.kv_len, grp.block_tables,
                              tiles[0], tiles[1], num_heads, scale, gate=gate, **changes)
+
+
+def _grouped_takes(rt: Runtime, ctx: Any, head_dim: int, value_dim: int, changes: Mapping[str, Any]) -> bool:
+    """Whether the matrix-core kernel that passes keys and values through LDS computes this attention: its sizes, no penalty
+    on the distance."""
+    return changes.get("r1") is None and ops.attention_grouped_supports(head_dim, value_dim, ctx.page_size, rt.dtype)
 
 
 def _keyvalue_takes(rt: Runtime, head_dim: int, value_dim: int, out: torch.Tensor, changes: Mapping[str, Any]) -> bool:

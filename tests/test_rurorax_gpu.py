@@ -460,12 +460,80 @@ def test_planted_keys_at_the_edges_of_chunks(ops, dtype, qh, kh, d, dv, size, ps
             out = torch.empty(m, qh * dv, dtype=dtype).cuda()
             ops.attention_scored_mfma(qd[rows], kp, vp, out, i32([0, m]), i32([n]), table, ent, q0, qh, scale, chunk=size)
             check(out, rows, ("matrix cores", first))
+        if dtype == torch.bfloat16 and ops.attention_grouped_supports(d, dv, ps, dtype):
+            tokens = ops.attention_grouped_tile_tokens(qh, kh)
+            ent, q0 = i32([0] * len(range(0, m, tokens))), i32(range(0, m, tokens))
+            out = torch.empty(m, qh * dv, dtype=dtype).cuda()
+            ops.attention_grouped(qd[rows], kp, vp, out, i32([0, m]), i32([n]), table, ent, q0, qh, scale, chunk=size)
+            check(out, rows, ("grouped", first))
     for t in range(100, n, 3):
         rows = [t, min(t + 1, n - 1), min(t + 2, n - 1)]
         out = torch.empty(3, qh * dv, dtype=dtype).cuda()
         ops.attention_scored(qd[rows], kp, vp, out, i32([0, 1, 2, 3]), i32([r + 1 for r in rows]), table.repeat(3, 1).contiguous(),
                              None, None, qh, scale, chunk=size)
         check(out, rows, ("single", t))
+
+
+def plain_masked(q, k, v, first, scale, low, keep, sink, v_heads):
+    """Softmax over ``low(i) <= j <= i`` and ``j < keep``, ``exp(sink[h])`` more in the denominator; key head ``g`` reads value head
+    ``g % v_heads``."""
+    n, H, _ = q.shape
+    G = k.shape[1]
+    out = torch.zeros(n, H, v.shape[2], dtype=F)
+    for t in range(n):
+        i = first + t
+        seen = [j for j in range(i + 1) if j >= low(i) or j < keep]
+        for h in range(H):
+            g = h // (H // G)
+            w = torch.exp(k[seen, g] @ q[t, h] * scale)
+            out[t, h] = (w @ v[seen, g % v_heads]) / (w.sum() + (math.exp(sink[h]) if sink is not None else 0.0))
+    return out
+
+
+@pytest.mark.parametrize("out32", [False, True])
+@pytest.mark.parametrize("qh,kh,vh,d,dv,window,chunk,keep,sink,gated,ps", [
+    (4, 2, 2, 64, 64, 70, 0, 0, True, False, 16), (8, 4, 2, 40, 128, 33, 0, 70, False, False, 8), (6, 2, 1, 128, 20, 64, 90, 5, True, True, 16),
+    (3, 3, 3, 8, 4, 0, 0, 0, False, True, 8), (66, 1, 1, 16, 48, 0, 50, 0, True, False, 16), (5, 1, 1, 104, 112, 1, 0, 1, False, False, 32),
+    (4, 4, 2, 24, 100, 100, 64, 3, True, True, 8), (2, 1, 1, 96, 96, 200, 0, 130, False, False, 16)])
+def test_grouped_attention_with_every_change(ops, qh, kh, vh, d, dv, window, chunk, keep, sink, gated, ps, out32):
+    """Windows, kept first positions, chunks, sinks, gates, shared value heads, in two entries on one list of tiles (one a
+    portion on top of earlier keys), against the plain softmax; a negative scale once."""
+    g = torch.Generator().manual_seed(qh * 7 + d)
+    lens, news = [190, 75], [97, 75]
+    scale = (-1 if kh == 3 else 1) * d ** -0.5
+    need = [-(-n // ps) for n in lens]
+    order = torch.randperm(sum(need) + 2, generator=g).tolist()
+    orders = [order[:need[0]], order[need[0]:need[0] + need[1]]]
+    kp, vp = torch.zeros(len(order), kh, ps, d, dtype=torch.bfloat16).cuda(), torch.zeros(len(order), vh, dv, ps, dtype=torch.bfloat16).cuda()
+    sinks = torch.randn(qh, generator=g) if sink else None
+    qs, refs = [], []
+    low = lambda i: max(i - window + 1 if window else 0, i // chunk * chunk if chunk else 0)
+    for n, m, o in zip(lens, news, orders):
+        q, k, v = (torch.randn(n, h, s, generator=g).to(torch.bfloat16) for h, s in ((qh, d), (kh, d), (vh, dv)))
+        for t in range(n):
+            kp[o[t // ps], :, t % ps] = k[t].cuda()
+            vp[o[t // ps], :, :, t % ps] = v[t].cuda()
+        qs.append(q[n - m:])
+        ref = torch.zeros(m, qh, dv, dtype=F)
+        for t in range(m):                                     # (kept positions count within the query's own chunk alone)
+            i = n - m + t
+            start = i // chunk * chunk if chunk else 0
+            ref[t] = plain_masked(q[i:i + 1].double(), k[start:].double(), v[start:].double(), i - start, scale, lambda x: low(x + start) - start,
+                                  max(0, keep - start) if window else 0, sinks, vh)[0]
+        refs.append(ref)
+    q = torch.cat(qs).reshape(sum(news), qh * d).cuda()
+    gate = torch.randn(sum(news), qh * dv, generator=g) if gated else None
+    ref = torch.cat(refs).reshape(sum(news), qh * dv)
+    if gated:
+        ref = ref * P.sigmoid(gate.double())
+    table = i32([p for o in orders for p in (o + [0] * max(need))[:max(need)]]).view(2, max(need))
+    tokens = ops.attention_grouped_tile_tokens(qh, kh)
+    ent = [e for e, m in enumerate(news) for _ in range(0, m, tokens)]
+    q0 = [x for m in news for x in range(0, m, tokens)]
+    out = torch.empty(sum(news), qh * dv, dtype=torch.float32 if out32 else torch.bfloat16).cuda()
+    ops.attention_grouped(q, kp, vp, out, i32([0, news[0], sum(news)]), i32(lens), table, i32(ent), i32(q0), qh, scale, window=window,
+                          chunk=chunk, keep_first=keep, sinks=sinks.cuda() if sink else None, gate=gate.cuda() if gated else None)
+    assert (out.cpu().double() - ref).abs().max() < 2e-2 * ref.abs().max()
 
 
 # ------------------------------------------------------------------------------ whole models
