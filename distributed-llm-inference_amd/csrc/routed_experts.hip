@@ -469,6 +469,104 @@ __global__ __launch_bounds__(256) void expert_down_mfma_kernel(ExpertArgs p, con
   }
 }
 
+// The same two products for many rows an expert (bfloat16, sizes that are multiples of 64 and 128 as the host checks): tiles of
+// EXL_BM sorted rows, a workgroup of four waves takes 128 rows of weights (the up product: 64 of each half), both
+// operands through LDS 64 k at a time, the next 64 in flight in registers meanwhile. A wave takes half of the
+// tile's rows and half of the weights' rows, sixteen 16 x 16 blocks. Rows in LDS are padded by 16 bytes. Every output sums its k in
+// ascending steps of 32, as in the kernels above. The workgroups of one XCD take neighbouring tiles with all their
+// features, so that an expert's weights are read into one L2 (or two).
+#define EXL_BM 128
+#define EXL_BK 64
+#define EXL_LD (EXL_BK + 8)
+template <bool UP>
+__global__ __launch_bounds__(256, 2) void expert_tiled_kernel(ExpertArgs p, const bf16_t* __restrict__ x, int64_t x_stride,
+                                                              const bf16_t* __restrict__ w0, const bf16_t* __restrict__ w1,
+                                                              bf16_t* __restrict__ y, float* __restrict__ z, int blocks_n,
+                                                              float limit, float alpha, float up_shift) {
+  __shared__ __align__(16) bf16_t xs[2][EXL_BM * EXL_LD], ws[2][128 * EXL_LD];
+  const int count = p.tile_count[0], per = (count + 7) / 8, local = blockIdx.x / 8;
+  const int tile = (blockIdx.x % 8) * per + local / blocks_n, block = local % blocks_n;
+  if (local / blocks_n >= per || tile >= count) return;
+  const int e = p.tile_expert[tile], r0 = p.tile_row0[tile], rend = min(p.offsets[e + 1], r0 + EXL_BM);
+  const int tid = threadIdx.x, lane = tid % 64, wave = __builtin_amdgcn_readfirstlane(tid / 64), c = lane % 16, g = lane / 16;
+  const int wm = wave & 1, wn = wave >> 1;
+  const int K = UP ? p.width : p.ff;
+  // this thread's 16-byte pieces: piece tid % 8 of the rows tid / 8 + 32 m
+  const bf16_t *xr[4], *wr[4];
+#pragma unroll
+  for (int m = 0; m < 4; ++m) {
+    const int row = tid / 8 + 32 * m, r = min(r0 + row, rend - 1);              // (a row past the end repeats the last)
+    xr[m] = x + (int64_t)(UP ? p.order[r] / p.top : r) * x_stride + 8 * (tid % 8);
+    if (UP) wr[m] = (row < 64 ? w0 : w1) + ((int64_t)e * p.ff + 64 * block + row % 64) * K + 8 * (tid % 8);
+    else wr[m] = w0 + ((int64_t)e * p.width + 128 * block + row) * K + 8 * (tid % 8);
+  }
+  exm_bf16x8 rx[4], rw[4];
+  auto fetch = [&](int k) {
+#pragma unroll
+    for (int m = 0; m < 4; ++m) { rx[m] = exm_load(xr[m] + k); rw[m] = exm_load(wr[m] + k); }
+  };
+  auto put = [&](int buf) {
+#pragma unroll
+    for (int m = 0; m < 4; ++m) {
+      const int at = (tid / 8 + 32 * m) * EXL_LD + 8 * (tid % 8);
+      *reinterpret_cast<exm_bf16x8*>(&xs[buf][at]) = rx[m];
+      *reinterpret_cast<exm_bf16x8*>(&ws[buf][at]) = rw[m];
+    }
+  };
+  exm_float4 acc[4][4];                                                          // [weights' block][rows' block]
+#pragma unroll
+  for (int n = 0; n < 4; ++n)
+#pragma unroll
+    for (int m = 0; m < 4; ++m) acc[n][m] = exm_float4{0.f, 0.f, 0.f, 0.f};
+  // the weights' blocks: gate 32 wn and 32 wn + 16, then the same of up; or 64 wn on
+  int wrow[4];
+#pragma unroll
+  for (int n = 0; n < 4; ++n) wrow[n] = UP ? 64 * (n / 2) + 32 * wn + 16 * (n % 2) : 64 * wn + 16 * n;
+  fetch(0);
+  put(0);
+  __syncthreads();
+  int buf = 0;
+  for (int k = 0; k < K; k += EXL_BK, buf ^= 1) {
+    const bool more = k + EXL_BK < K;
+    if (more) fetch(k + EXL_BK);
+#pragma unroll
+    for (int s = 0; s < 2; ++s) {
+      exm_bf16x8 a[4], b[4];
+#pragma unroll
+      for (int n = 0; n < 4; ++n) a[n] = exm_load(&ws[buf][(wrow[n] + c) * EXL_LD + 32 * s + 8 * g]);
+#pragma unroll
+      for (int m = 0; m < 4; ++m) b[m] = exm_load(&xs[buf][(64 * wm + 16 * m + c) * EXL_LD + 32 * s + 8 * g]);
+#pragma unroll
+      for (int n = 0; n < 4; ++n)
+#pragma unroll
+        for (int m = 0; m < 4; ++m) acc[n][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[n], b[m], acc[n][m], 0, 0, 0);
+    }
+    if (more) put(buf ^ 1);
+    __syncthreads();
+  }
+  typedef __bf16 bf4 __attribute__((ext_vector_type(4)));
+#pragma unroll
+  for (int m = 0; m < 4; ++m) {
+    const int r = r0 + 64 * wm + 16 * m + c;
+    if (r >= rend) continue;
+    if (UP) {
+      const float iw = p.in_weight != nullptr ? p.in_weight[p.order[r]] : 1.f;
+#pragma unroll
+      for (int n = 0; n < 2; ++n) {
+        bf4 o;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[i] = (bf16_t)clamped_glu(iw * acc[n][m][i], iw * acc[n + 2][m][i], limit, alpha, up_shift);
+        *reinterpret_cast<bf4*>(y + (int64_t)r * p.ff + 64 * block + 32 * wn + 16 * n + 4 * g) = o;
+      }
+    } else {
+      const int64_t slot = p.order[r];
+#pragma unroll
+      for (int n = 0; n < 4; ++n)
+        *reinterpret_cast<exm_float4*>(z + slot * p.width + 128 * block + wrow[n] + 4 * g) = acc[n][m];
+    }
+  }
+}
+
 // (weights nullptr: ones)
 // out[token] = sum_j weights[token][j] * (ids[token][j] < experts ? z[token * top + j] : h[token])
 //            + sigmoid(shared_gate[token]) * shared[token]       (the shared expert, if there is one)
@@ -543,7 +641,13 @@ int dli_router_choose(const float* logits, int64_t stride, const float* bias, co
 
 // Whether the matrix-core kernels take these sizes, and the rows of a tile of the kernels that will run.
 static bool expert_mfma(int width, int ff, int is_bf16) { return is_bf16 && width % 32 == 0 && ff % 32 == 0; }
-int dli_expert_tile_rows(int width, int ff, int is_bf16) { return expert_mfma(width, ff, is_bf16) ? EXM_BM : EX_BM; }
+// Many rows an expert, and sizes that tile: the kernels that pass both operands through LDS.
+static bool expert_tiled(int64_t slots, int experts, int width, int ff, int is_bf16) {
+  return is_bf16 && width % 128 == 0 && ff % 64 == 0 && slots >= 48 * (int64_t)experts;
+}
+int dli_expert_tile_rows(int64_t slots, int experts, int width, int ff, int is_bf16) {
+  return expert_tiled(slots, experts, width, ff, is_bf16) ? EXL_BM : expert_mfma(width, ff, is_bf16) ? EXM_BM : EX_BM;
+}
 
 // The experts' part of a mixture for `rows` tokens: sort, up product with activation, down product.
 // ids [rows][top]; scratch: offsets [experts + 1], order [rows * top], tile_expert and tile_row0 [max_tiles],
@@ -563,11 +667,21 @@ int dli_expert_products(const int* ids, const void* h, int64_t h_stride, const v
                ((uintptr_t)w_down % 16) || ((uintptr_t)y % 16)))
     return DLI_ERR_ARGUMENT;
   expert_sort_kernel<<<1, 1024, 2 * experts * sizeof(int), stream>>>(ids, (int)slots, experts, offsets, order, tile_expert,
-                                                                     tile_row0, tile_count, max_tiles, mfma ? EXM_BM : EX_BM);
+                                                                     tile_row0, tile_count, max_tiles,
+                                                                     dli_expert_tile_rows(slots, experts, width, ff, is_bf16));
   if (dli_launch_status() != DLI_OK) return DLI_ERR_LAUNCH;
   ExpertArgs p;
   p.tile_expert = tile_expert; p.tile_row0 = tile_row0; p.tile_count = tile_count; p.offsets = offsets; p.order = order;
   p.top = top; p.width = width; p.ff = ff; p.in_weight = in_weight;
+  if (expert_tiled(slots, experts, width, ff, is_bf16)) {
+    const unsigned tiles8 = 8 * ((max_tiles + 7) / 8);
+    if ((int64_t)tiles8 * (ff / 64 + width / 128) > 0x7fffffff || ((uintptr_t)z % 16)) return DLI_ERR_ARGUMENT;
+    expert_tiled_kernel<true><<<tiles8 * (ff / 64), 256, 0, stream>>>(p, (const bf16_t*)h, h_stride, (const bf16_t*)w_gate,
+                                                                      (const bf16_t*)w_up, (bf16_t*)y, nullptr, ff / 64, limit, alpha, up_shift);
+    expert_tiled_kernel<false><<<tiles8 * (width / 128), 256, 0, stream>>>(p, (const bf16_t*)y, ff, (const bf16_t*)w_down, nullptr,
+                                                                           nullptr, z, width / 128, 0.f, 0.f, 0.f);
+    return dli_launch_status();
+  }
   const int bn = mfma ? EXM_BN : EX_BN;
   const dim3 up_grid(max_tiles, (ff + bn - 1) / bn), down_grid(max_tiles, (width + bn - 1) / bn);
   if (mfma) {

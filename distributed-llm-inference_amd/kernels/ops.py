@@ -191,7 +191,7 @@ _SIGNATURES = {
     "dli_clamped_glu": [_c_ptr, _c_i64, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_int, _c_ptr],
     "dli_router_choose": [_c_ptr, _c_i64, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int,
                           _c_ptr, _c_ptr, _c_ptr],
-    "dli_expert_tile_rows": [_c_int, _c_int, _c_int],
+    "dli_expert_tile_rows": [_c_i64, _c_int, _c_int, _c_int, _c_int],
     "dli_expert_products": [_c_ptr, _c_ptr, _c_i64, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int,
                             _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_int,
                             _c_ptr],
@@ -2194,7 +2194,7 @@ def expert_products(ids: torch.Tensor, h: torch.Tensor, w_gate: torch.Tensor, w_
         _dense(in_weights, "in_weights", torch.float32, 2)
         _require(in_weights.shape == (n, top), "in_weights must be [n, top]")
     slots = n * top
-    tile_rows = int(library().dli_expert_tile_rows(width, ff, _is_bf16(h.dtype)))
+    tile_rows = int(library().dli_expert_tile_rows(slots, experts, width, ff, _is_bf16(h.dtype)))
     max_tiles = max(1, min(slots, slots // tile_rows + experts))
     ints = torch.empty(experts + 1 + slots + 2 * max_tiles + 1, device=h.device, dtype=torch.int32)
     offsets, order = ints[:experts + 1], ints[experts + 1:experts + 1 + slots]

@@ -189,7 +189,8 @@ def test_gelu_gate_with_biases(ops, rows, width, ff, dtype):
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("n,experts,top,width,ff", [(1, 4, 1, 64, 32), (9, 5, 2, 40, 12), (70, 12, 3, 64, 96), (33, 3, 3, 96, 64), (200, 70, 1, 32, 32)])
+@pytest.mark.parametrize("n,experts,top,width,ff", [(1, 4, 1, 64, 32), (9, 5, 2, 40, 12), (70, 12, 3, 64, 96), (33, 3, 3, 96, 64), (200, 70, 1, 32, 32),
+                                                      (300, 4, 2, 256, 128), (513, 5, 3, 128, 64), (260, 5, 1, 384, 192)])
 def test_sigmoid_scores_scale_what_the_experts_read(ops, dtype, n, experts, top, width, ff):
     """Scores as they are, largest first, on the experts' inputs: with weights below one half of the result that
     a weight on the output would give differs, since the activation bends."""
