@@ -327,84 +327,89 @@ __global__ __launch_bounds__(256) void expert_down_kernel(ExpertArgs p, const T*
   }
 }
 
-// The same two products on the matrix cores (bfloat16; width and ff multiples of 32): tiles of EXM_BM
-// sorted rows, a workgroup of four waves takes 128 features, each wave 32 of them (two blocks of 16) for
-// all rows of the tile. v_mfma_f32_16x16x32_bf16 with the weights as the first operand: lane l supplies
-// feature l % 16 of a block and row l % 16 of each block of 16 rows, and the eight k values
-// 8 (l / 16) .. + 7 of a step of 32, read straight from memory (16 bytes a lane and operand; the rows of
-// a tile are re-read by the four waves from the cache); the operands of the next step are asked for
-// before this step's products are issued. A lane's results are four neighbouring features of one row.
+// The same two products on the matrix cores (bfloat16; width and ff multiples of 32): tiles of 16 MB sorted rows, a
+// workgroup of four waves takes 64 NB features, each wave 16 NB of them for all rows of the tile.
+// v_mfma_f32_16x16x32_bf16 with the weights as the first operand: lane l supplies feature l % 16 of a block and row
+// l % 16 of each block of 16 rows, and the eight k values 8 (l / 16) .. + 7 of a step of 32, read straight from memory (16
+// bytes a lane and operand; the rows of a tile are re-read by the four waves from the cache); the operands of the next DEPTH
+// steps are on their way while a step's products are issued. A lane's results are four neighbouring features of one row.
 // Every output sums its k in ascending steps of 32 whatever its tile, so a row's result depends on
-// nothing beside the row.
+// nothing beside the row. Few rows an expert (MB 1) wait for the weights alone: one block of features a wave, many steps ahead.
 #define EXM_BM 64
-#define EXM_MB (EXM_BM / 16)
-#define EXM_BN 128
+#define EXM_FEW 16
 typedef __bf16 exm_bf16x8 __attribute__((ext_vector_type(8)));
 typedef float exm_float4 __attribute__((ext_vector_type(4)));
 
 __device__ __forceinline__ exm_bf16x8 exm_load(const bf16_t* p) { return *reinterpret_cast<const exm_bf16x8*>(p); }
 
+template <int MB, int NB, int DEPTH>
 __global__ __launch_bounds__(256) void expert_up_mfma_kernel(ExpertArgs p, const bf16_t* __restrict__ h, int64_t h_stride,
                                                              const bf16_t* __restrict__ w_gate,
                                                              const bf16_t* __restrict__ w_up, bf16_t* __restrict__ y,
                                                              float limit, float alpha, float up_shift) {
   const int tile = blockIdx.x;
   if (tile >= p.tile_count[0]) return;
-  const int e = p.tile_expert[tile], r0 = p.tile_row0[tile], rend = p.offsets[e + 1];
+  const int e = p.tile_expert[tile], r0 = p.tile_row0[tile], rend = min(p.offsets[e + 1], r0 + 16 * MB);
   const int lane = threadIdx.x % DLI_WAVE, wave = threadIdx.x / DLI_WAVE;
   const int c = lane % 16, kq = (lane / 16) * 8;
-  const int nw = blockIdx.y * EXM_BN + wave * 32;
-  const bf16_t *wg[2], *wu[2], *xr[EXM_MB];
+  const int nw = (blockIdx.y * 4 + wave) * 16 * NB;
+  const bf16_t *wg[NB], *wu[NB], *xr[MB];
 #pragma unroll
-  for (int nb = 0; nb < 2; ++nb) {
+  for (int nb = 0; nb < NB; ++nb) {
     const int n = min(nw + nb * 16 + c, p.ff - 1);                              // (a feature past the end repeats the last)
     wg[nb] = w_gate + ((int64_t)e * p.ff + n) * p.width + kq;
     wu[nb] = w_up + ((int64_t)e * p.ff + n) * p.width + kq;
   }
 #pragma unroll
-  for (int mb = 0; mb < EXM_MB; ++mb) {
+  for (int mb = 0; mb < MB; ++mb) {
     const int r = min(r0 + mb * 16 + c, rend - 1);                              // (a row past the end repeats the last)
     xr[mb] = h + (int64_t)(p.order[r] / p.top) * h_stride + kq;
   }
-  exm_float4 accg[2][EXM_MB], accu[2][EXM_MB];
+  exm_float4 accg[NB][MB], accu[NB][MB];
 #pragma unroll
-  for (int nb = 0; nb < 2; ++nb)
+  for (int nb = 0; nb < NB; ++nb)
 #pragma unroll
-    for (int mb = 0; mb < EXM_MB; ++mb) accg[nb][mb] = accu[nb][mb] = exm_float4{0.f, 0.f, 0.f, 0.f};
+    for (int mb = 0; mb < MB; ++mb) accg[nb][mb] = accu[nb][mb] = exm_float4{0.f, 0.f, 0.f, 0.f};
   const int blocks = (rend - r0 + 15) / 16;                                     // blocks of 16 rows that hold a row
-  exm_bf16x8 a[2], b[2], x[EXM_MB];
-  auto fetch = [&](int k) {
+  exm_bf16x8 a[DEPTH][NB], b[DEPTH][NB], x[DEPTH][MB];
+  auto fetch = [&](int j, int k) {
 #pragma unroll
-    for (int nb = 0; nb < 2; ++nb) { a[nb] = exm_load(wg[nb] + k); b[nb] = exm_load(wu[nb] + k); }
+    for (int nb = 0; nb < NB; ++nb) { a[j][nb] = exm_load(wg[nb] + k); b[j][nb] = exm_load(wu[nb] + k); }
 #pragma unroll
-    for (int mb = 0; mb < EXM_MB; ++mb) x[mb] = exm_load(xr[mb] + k);            // (unconditional: clamped rows are valid memory)
+    for (int mb = 0; mb < MB; ++mb) x[j][mb] = exm_load(xr[mb] + k);             // (unconditional: clamped rows are valid memory)
   };
-  fetch(0);
-  for (int k = 0; k < p.width; k += 32) {
-    exm_bf16x8 a0[2], b0[2], x0[EXM_MB];
 #pragma unroll
-    for (int nb = 0; nb < 2; ++nb) { a0[nb] = a[nb]; b0[nb] = b[nb]; }
+  for (int j = 0; j < DEPTH; ++j) fetch(j, min(32 * j, p.width - 32));
+  for (int k0 = 0; k0 < p.width; k0 += 32 * DEPTH) {
 #pragma unroll
-    for (int mb = 0; mb < EXM_MB; ++mb) x0[mb] = x[mb];
-    fetch(min(k + 32, p.width - 32));                                           // the last turn asks for its own step again
+    for (int j = 0; j < DEPTH; ++j) {
+      const int k = k0 + 32 * j;
+      exm_bf16x8 a0[NB], b0[NB], x0[MB];
 #pragma unroll
-    for (int mb = 0; mb < EXM_MB; ++mb) {
-      if (mb < blocks) {
+      for (int nb = 0; nb < NB; ++nb) { a0[nb] = a[j][nb]; b0[nb] = b[j][nb]; }
 #pragma unroll
-        for (int nb = 0; nb < 2; ++nb) {
-          accg[nb][mb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a0[nb], x0[mb], accg[nb][mb], 0, 0, 0);
-          accu[nb][mb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(b0[nb], x0[mb], accu[nb][mb], 0, 0, 0);
+      for (int mb = 0; mb < MB; ++mb) x0[mb] = x[j][mb];
+      if (DEPTH > 1 && k >= p.width) x0[0] = exm_bf16x8{};                       // (past the last step: a product of zero)
+      fetch(j, min(k + 32 * DEPTH, p.width - 32));                              // the last turn asks for its own step again
+#pragma unroll
+      for (int mb = 0; mb < MB; ++mb) {
+        if (MB == 1 || mb < blocks) {
+#pragma unroll
+          for (int nb = 0; nb < NB; ++nb) {
+            accg[nb][mb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a0[nb], x0[mb], accg[nb][mb], 0, 0, 0);
+            accu[nb][mb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(b0[nb], x0[mb], accu[nb][mb], 0, 0, 0);
+          }
         }
       }
     }
   }
 #pragma unroll
-  for (int mb = 0; mb < EXM_MB; ++mb) {
+  for (int mb = 0; mb < MB; ++mb) {
     const int r = r0 + mb * 16 + c;
     if (r >= rend) continue;
     const float iw = p.in_weight != nullptr ? p.in_weight[p.order[r]] : 1.f;
 #pragma unroll
-    for (int nb = 0; nb < 2; ++nb) {
+    for (int nb = 0; nb < NB; ++nb) {
       const int n0 = nw + nb * 16 + (lane / 16) * 4;
 #pragma unroll
       for (int i = 0; i < 4; ++i)
@@ -414,53 +419,60 @@ __global__ __launch_bounds__(256) void expert_up_mfma_kernel(ExpertArgs p, const
   }
 }
 
+template <int MB, int NB, int DEPTH>
 __global__ __launch_bounds__(256) void expert_down_mfma_kernel(ExpertArgs p, const bf16_t* __restrict__ y,
                                                                const bf16_t* __restrict__ w_down, float* __restrict__ z) {
   const int tile = blockIdx.x;
   if (tile >= p.tile_count[0]) return;
-  const int e = p.tile_expert[tile], r0 = p.tile_row0[tile], rend = p.offsets[e + 1];
+  const int e = p.tile_expert[tile], r0 = p.tile_row0[tile], rend = min(p.offsets[e + 1], r0 + 16 * MB);
   const int lane = threadIdx.x % DLI_WAVE, wave = threadIdx.x / DLI_WAVE;
   const int c = lane % 16, kq = (lane / 16) * 8;
-  const int nw = blockIdx.y * EXM_BN + wave * 32;
-  const bf16_t *wd[2], *yr[EXM_MB];
+  const int nw = (blockIdx.y * 4 + wave) * 16 * NB;
+  const bf16_t *wd[NB], *yr[MB];
 #pragma unroll
-  for (int nb = 0; nb < 2; ++nb) wd[nb] = w_down + ((int64_t)e * p.width + min(nw + nb * 16 + c, p.width - 1)) * p.ff + kq;
+  for (int nb = 0; nb < NB; ++nb) wd[nb] = w_down + ((int64_t)e * p.width + min(nw + nb * 16 + c, p.width - 1)) * p.ff + kq;
 #pragma unroll
-  for (int mb = 0; mb < EXM_MB; ++mb) yr[mb] = y + (int64_t)min(r0 + mb * 16 + c, rend - 1) * p.ff + kq;
-  exm_float4 acc[2][EXM_MB];
+  for (int mb = 0; mb < MB; ++mb) yr[mb] = y + (int64_t)min(r0 + mb * 16 + c, rend - 1) * p.ff + kq;
+  exm_float4 acc[NB][MB];
 #pragma unroll
-  for (int nb = 0; nb < 2; ++nb)
+  for (int nb = 0; nb < NB; ++nb)
 #pragma unroll
-    for (int mb = 0; mb < EXM_MB; ++mb) acc[nb][mb] = exm_float4{0.f, 0.f, 0.f, 0.f};
+    for (int mb = 0; mb < MB; ++mb) acc[nb][mb] = exm_float4{0.f, 0.f, 0.f, 0.f};
   const int blocks = (rend - r0 + 15) / 16;
-  exm_bf16x8 a[2], x[EXM_MB];
-  auto fetch = [&](int k) {
+  exm_bf16x8 a[DEPTH][NB], x[DEPTH][MB];
+  auto fetch = [&](int j, int k) {
 #pragma unroll
-    for (int nb = 0; nb < 2; ++nb) a[nb] = exm_load(wd[nb] + k);
+    for (int nb = 0; nb < NB; ++nb) a[j][nb] = exm_load(wd[nb] + k);
 #pragma unroll
-    for (int mb = 0; mb < EXM_MB; ++mb) x[mb] = exm_load(yr[mb] + k);
+    for (int mb = 0; mb < MB; ++mb) x[j][mb] = exm_load(yr[mb] + k);
   };
-  fetch(0);
-  for (int k = 0; k < p.ff; k += 32) {
-    exm_bf16x8 a0[2], x0[EXM_MB];
 #pragma unroll
-    for (int nb = 0; nb < 2; ++nb) a0[nb] = a[nb];
+  for (int j = 0; j < DEPTH; ++j) fetch(j, min(32 * j, p.ff - 32));
+  for (int k0 = 0; k0 < p.ff; k0 += 32 * DEPTH) {
 #pragma unroll
-    for (int mb = 0; mb < EXM_MB; ++mb) x0[mb] = x[mb];
-    fetch(min(k + 32, p.ff - 32));
+    for (int j = 0; j < DEPTH; ++j) {
+      const int k = k0 + 32 * j;
+      exm_bf16x8 a0[NB], x0[MB];
 #pragma unroll
-    for (int mb = 0; mb < EXM_MB; ++mb)
-      if (mb < blocks)
+      for (int nb = 0; nb < NB; ++nb) a0[nb] = a[j][nb];
 #pragma unroll
-        for (int nb = 0; nb < 2; ++nb) acc[nb][mb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a0[nb], x0[mb], acc[nb][mb], 0, 0, 0);
+      for (int mb = 0; mb < MB; ++mb) x0[mb] = x[j][mb];
+      if (DEPTH > 1 && k >= p.ff) x0[0] = exm_bf16x8{};
+      fetch(j, min(k + 32 * DEPTH, p.ff - 32));
+#pragma unroll
+      for (int mb = 0; mb < MB; ++mb)
+        if (MB == 1 || mb < blocks)
+#pragma unroll
+          for (int nb = 0; nb < NB; ++nb) acc[nb][mb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a0[nb], x0[mb], acc[nb][mb], 0, 0, 0);
+    }
   }
 #pragma unroll
-  for (int mb = 0; mb < EXM_MB; ++mb) {
+  for (int mb = 0; mb < MB; ++mb) {
     const int r = r0 + mb * 16 + c;
     if (r >= rend) continue;
     const int64_t slot = p.order[r];
 #pragma unroll
-    for (int nb = 0; nb < 2; ++nb) {
+    for (int nb = 0; nb < NB; ++nb) {
       const int n0 = nw + nb * 16 + (lane / 16) * 4;
 #pragma unroll
       for (int i = 0; i < 4; ++i)
@@ -645,8 +657,12 @@ static bool expert_mfma(int width, int ff, int is_bf16) { return is_bf16 && widt
 static bool expert_tiled(int64_t slots, int experts, int width, int ff, int is_bf16) {
   return is_bf16 && width % 128 == 0 && ff % 64 == 0 && slots >= 48 * (int64_t)experts;
 }
+// Few rows an expert: the kernels that wait for the weights alone.
+static bool expert_few(int64_t slots, int experts) { return slots <= 16 * (int64_t)experts; }
 int dli_expert_tile_rows(int64_t slots, int experts, int width, int ff, int is_bf16) {
-  return expert_tiled(slots, experts, width, ff, is_bf16) ? EXL_BM : expert_mfma(width, ff, is_bf16) ? EXM_BM : EX_BM;
+  if (expert_tiled(slots, experts, width, ff, is_bf16)) return EXL_BM;
+  if (!expert_mfma(width, ff, is_bf16)) return EX_BM;
+  return expert_few(slots, experts) ? EXM_FEW : EXM_BM;
 }
 
 // The experts' part of a mixture for `rows` tokens: sort, up product with activation, down product.
@@ -682,12 +698,16 @@ int dli_expert_products(const int* ids, const void* h, int64_t h_stride, const v
                                                                            nullptr, z, width / 128, 0.f, 0.f, 0.f);
     return dli_launch_status();
   }
-  const int bn = mfma ? EXM_BN : EX_BN;
+  const int bn = !mfma ? EX_BN : expert_few(slots, experts) ? 64 : 128;
   const dim3 up_grid(max_tiles, (ff + bn - 1) / bn), down_grid(max_tiles, (width + bn - 1) / bn);
-  if (mfma) {
-    expert_up_mfma_kernel<<<up_grid, 256, 0, stream>>>(p, (const bf16_t*)h, h_stride, (const bf16_t*)w_gate,
-                                                       (const bf16_t*)w_up, (bf16_t*)y, limit, alpha, up_shift);
-    expert_down_mfma_kernel<<<down_grid, 256, 0, stream>>>(p, (const bf16_t*)y, (const bf16_t*)w_down, z);
+#define EXM_LAUNCH(MB, NB, DU, DD)                                                                                                 \
+  expert_up_mfma_kernel<MB, NB, DU><<<up_grid, 256, 0, stream>>>(p, (const bf16_t*)h, h_stride, (const bf16_t*)w_gate,             \
+                                                                 (const bf16_t*)w_up, (bf16_t*)y, limit, alpha, up_shift);          \
+  expert_down_mfma_kernel<MB, NB, DD><<<down_grid, 256, 0, stream>>>(p, (const bf16_t*)y, (const bf16_t*)w_down, z)
+  if (mfma && expert_few(slots, experts)) {
+    EXM_LAUNCH(1, 1, 8, 8);
+  } else if (mfma) {
+    EXM_LAUNCH(4, 2, 1, 1);
   } else if (is_bf16) {
     expert_up_kernel<bf16_t><<<up_grid, 256, 0, stream>>>(p, (const bf16_t*)h, h_stride, (const bf16_t*)w_gate,
                                                           (const bf16_t*)w_up, (bf16_t*)y, limit, alpha, up_shift);
