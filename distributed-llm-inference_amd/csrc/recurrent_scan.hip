@@ -298,6 +298,51 @@ __global__ __launch_bounds__(256) void row_norm_gate_kernel(const float* __restr
   }
 }
 
+// The same for long heads of whole 16-byte pieces, at most 4096 values: every value is read once and stays in registers.
+template <typename T, int RULE>
+__global__ __launch_bounds__(256) void row_norm_gate_wide_kernel(const float* __restrict__ o, int64_t o_stride,
+                                                                 const float* __restrict__ g_pre, int64_t g_stride,
+                                                                 const float* __restrict__ norm_w, float eps, T* __restrict__ out,
+                                                                 int64_t out_stride, int dim, const float* __restrict__ den) {
+  __shared__ float scratch[16];
+  const int64_t row = blockIdx.x, at = (int64_t)blockIdx.y * dim;
+  const float dn = den != nullptr ? 1.f / den[row * gridDim.y + blockIdx.y] : 1.f;
+  float v[4][4], g[4][4], ss = 0.f;
+#pragma unroll
+  for (int t = 0; t < 4; ++t) {
+    const int c = (t * blockDim.x + threadIdx.x) * 4;
+    if (c >= dim) continue;
+    const float4 a = *reinterpret_cast<const float4*>(o + row * o_stride + at + c);
+    v[t][0] = a.x; v[t][1] = a.y; v[t][2] = a.z; v[t][3] = a.w;
+    if (RULE != GATE_NONE) {
+      const float4 b = *reinterpret_cast<const float4*>(g_pre + row * g_stride + at + c);
+      g[t][0] = b.x; g[t][1] = b.y; g[t][2] = b.z; g[t][3] = b.w;
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      if (RULE == GATE_FIRST) g[t][j] = silu<float>(g[t][j]);
+      const float f = RULE == GATE_FIRST ? v[t][j] * dn * g[t][j] : v[t][j] * dn;
+      ss += f * f;
+    }
+  }
+  const float r = dn / sqrtf(block_sum(ss, scratch) / (float)dim + eps);
+#pragma unroll
+  for (int t = 0; t < 4; ++t) {
+    const int c = (t * blockDim.x + threadIdx.x) * 4;
+    if (c >= dim) continue;
+    struct alignas(sizeof(T) * 4) Packed { T v[4]; } y;
+    const float4 w = *reinterpret_cast<const float4*>(norm_w + at + c);
+    const float ws[4] = {w.x, w.y, w.z, w.w};
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const float gate = RULE == GATE_NONE ? 1.f : RULE == GATE_FIRST ? g[t][j]
+                         : RULE == RULE_DELTA ? 1.f / (1.f + expf(-g[t][j])) : g[t][j] / (1.f + expf(-g[t][j]));
+      y.v[j] = from_f32<T>(v[t][j] * r * ws[j] * gate);
+    }
+    *reinterpret_cast<Packed*>(out + row * out_stride + at + c) = y;
+  }
+}
+
 template <int RULE>
 static int launch_scan(const ScanArgs& p, int entries, int rows, int dim, int out_is_bf16, hipStream_t stream) {
   // sixteen lanes a column (four columns a wave) where the head's size is a multiple of 16, else eight
@@ -373,10 +418,17 @@ extern "C" int dli_head_norm_gate(const float* o, int64_t o_stride, const float*
       (gate != GATE_NONE && (g_pre == nullptr || g_stride < width)))
     return DLI_ERR_ARGUMENT;
   const dim3 grid(rows, (heads + 3) / 4);
-  if (grid.y > 65535) return DLI_ERR_ARGUMENT;
+  if (heads > 65535) return DLI_ERR_ARGUMENT;
+  auto whole = [](const void* at, size_t bytes) { return (uintptr_t)at % bytes == 0; };
+  const bool wide = dim > 256 && dim <= 4096 && dim % 4 == 0 && (heads == 1 || gate == GATE_FIRST) && o_stride % 4 == 0 &&
+                    g_stride % 4 == 0 && out_stride % 4 == 0 && whole(o, 16) && whole(norm_w, 16) &&
+                    whole(out, out_is_bf16 ? 8 : 16) && (gate == GATE_NONE || whole(g_pre, 16));
+  const int wide_threads = dim >= 1024 ? 256 : (dim / 4 + 63) / 64 * 64;
 #define HNG(T, RULE)                                                                                                     \
   do {                                                                                                                   \
-    if (dim > 256 && (heads == 1 || gate == GATE_FIRST))                                                                 \
+    if (wide)                                                                                                            \
+      row_norm_gate_wide_kernel<T, RULE><<<dim3(rows, heads), wide_threads, 0, stream>>>(o, o_stride, g_pre, g_stride, norm_w, eps, (T*)out, out_stride, dim, den); \
+    else if (dim > 256 && (heads == 1 || gate == GATE_FIRST))                                                                 \
       row_norm_gate_kernel<T, RULE><<<dim3(rows, heads), 256, 0, stream>>>(o, o_stride, g_pre, g_stride, norm_w, eps, (T*)out, out_stride, dim, den); \
     else                                                                                                                 \
       head_norm_gate_kernel<T, RULE><<<grid, 256, 0, stream>>>(o, o_stride, g_pre, g_stride, norm_w, eps, (T*)out, out_stride, heads, dim, den); \

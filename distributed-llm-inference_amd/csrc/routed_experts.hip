@@ -604,6 +604,38 @@ __global__ void expert_combine_kernel(const int* __restrict__ ids, const float* 
   out[row * width + c] = sum;
 }
 
+// The same with four columns a thread: widths, strides and addresses of whole 16-byte pieces.
+template <typename T>
+__global__ __launch_bounds__(256) void expert_combine4_kernel(const int* __restrict__ ids, const float* __restrict__ weights,
+                                                              const float* __restrict__ z, const T* __restrict__ h, int64_t h_stride,
+                                                              const float* __restrict__ shared_gate, int64_t gate_stride,
+                                                              const float* __restrict__ shared, int64_t shared_stride,
+                                                              float* __restrict__ out, int top, int experts, int width) {
+  const int64_t row = blockIdx.x;
+  const int c = (blockIdx.y * blockDim.x + threadIdx.x) * 4;
+  if (c >= width) return;
+  float sum[4] = {0.f, 0.f, 0.f, 0.f};
+  for (int j = 0; j < top; ++j) {
+    const float wt = weights != nullptr ? weights[row * top + j] : 1.f;
+    float v[4];
+    if (ids[row * top + j] < experts) {
+      const float4 f = *reinterpret_cast<const float4*>(z + (row * top + j) * width + c);
+      v[0] = f.x; v[1] = f.y; v[2] = f.z; v[3] = f.w;
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[i] = to_f32(h[row * h_stride + c + i]);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) sum[i] = fmaf(wt, v[i], sum[i]);
+  }
+  if (shared != nullptr) {
+    const float g = shared_gate != nullptr ? 1.f / (1.f + expf(-shared_gate[row * gate_stride])) : 1.f;
+    const float4 f = *reinterpret_cast<const float4*>(shared + row * shared_stride + c);
+    sum[0] = fmaf(g, f.x, sum[0]); sum[1] = fmaf(g, f.y, sum[1]); sum[2] = fmaf(g, f.z, sum[2]); sum[3] = fmaf(g, f.w, sum[3]);
+  }
+  *reinterpret_cast<float4*>(out + row * width + c) = float4{sum[0], sum[1], sum[2], sum[3]};
+}
+
 // A router that is a table: the experts of a token are the row of `table` [vocabulary][top] at its token id,
 // each with the weight 1 / top. A thread a (token, choice).
 __global__ void table_choose_kernel(const int* __restrict__ table, const int* __restrict__ token_ids, int n, int top,
@@ -725,13 +757,16 @@ int dli_expert_combine(const int* ids, const float* weights, const float* z, con
                        int rows, int top, int experts, int width, int is_bf16, hipStream_t stream) {
   if (rows <= 0) return DLI_OK;
   if (top < 1 || width <= 0 || h_stride < width || (shared != nullptr && shared_stride < width)) return DLI_ERR_ARGUMENT;
-  const dim3 grid(rows, (width + 255) / 256);
-  if (is_bf16)
-    expert_combine_kernel<bf16_t><<<grid, 256, 0, stream>>>(ids, weights, z, (const bf16_t*)h, h_stride, shared_gate, gate_stride,
-                                                            shared, shared_stride, out, top, experts, width);
-  else
-    expert_combine_kernel<float><<<grid, 256, 0, stream>>>(ids, weights, z, (const float*)h, h_stride, shared_gate, gate_stride,
-                                                           shared, shared_stride, out, top, experts, width);
+  auto whole = [](const void* at) { return (uintptr_t)at % 16 == 0; };
+  // (with few rows the extra workgroups of one column a thread hide more of the wait)
+  const bool fours = rows >= 256 && width % 4 == 0 && whole(z) && whole(out) && (shared == nullptr || (whole(shared) && shared_stride % 4 == 0));
+  const int cols = fours ? 1024 : 256;
+  const dim3 grid(rows, (width + cols - 1) / cols);
+#define COMBINE(KERNEL, T) KERNEL<T><<<grid, 256, 0, stream>>>(ids, weights, z, (const T*)h, h_stride, shared_gate, gate_stride, \
+                                                               shared, shared_stride, out, top, experts, width)
+  if (is_bf16) { if (fours) COMBINE(expert_combine4_kernel, bf16_t); else COMBINE(expert_combine_kernel, bf16_t); }
+  else { if (fours) COMBINE(expert_combine4_kernel, float); else COMBINE(expert_combine_kernel, float); }
+#undef COMBINE
   return dli_launch_status();
 }
 

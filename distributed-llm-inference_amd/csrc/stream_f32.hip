@@ -345,8 +345,30 @@ __global__ void qk_unit_cache_kernel(const float* __restrict__ proj, int64_t str
 // NORM: q, over all its heads at once, is divided by its root mean square and multiplied by q_norm (a value a
 // column), and k alike by k_norm, after the bias and before the rotation.
 // The cos and sin of a row's angles are made once, in LDS (rows of more pairs: element by element).
+// E elements a thread and turn: 4 where every size and offset is a multiple of 4 (16-byte loads), else 1.
 #define ROTARY_LDS_PAIRS 512
-template <typename T, bool NORM>
+template <int E>
+struct RotaryElements { float v[E]; };
+template <int E>
+__device__ __forceinline__ RotaryElements<E> rotary_load(const float* p) {
+  RotaryElements<E> r;
+  if constexpr (E == 4) {
+    const float4 f = *reinterpret_cast<const float4*>(p);
+    r.v[0] = f.x; r.v[1] = f.y; r.v[2] = f.z; r.v[3] = f.w;
+  } else {
+    r.v[0] = p[0];
+  }
+  return r;
+}
+template <typename T, int E>
+__device__ __forceinline__ void rotary_store(T* p, const float* v) {
+  struct alignas(sizeof(T) * E) Packed { T v[E]; } o;
+#pragma unroll
+  for (int j = 0; j < E; ++j) o.v[j] = from_f32<T>(v[j]);
+  *reinterpret_cast<Packed*>(p) = o;
+}
+
+template <typename T, bool NORM, int E>
 __global__ __launch_bounds__(256) void rotary_cache_kernel(const float* __restrict__ proj, int64_t stride, int q_off, int k_off, int v_off,
                                     const float* __restrict__ bias,
                                     const int* __restrict__ positions, const float* __restrict__ inv_freq, int rot_dims,
@@ -371,9 +393,13 @@ __global__ __launch_bounds__(256) void rotary_cache_kernel(const float* __restri
   if (NORM) {
     auto rms = [&](int off, int size) {
       float ss = 0.f;
-      for (int i = threadIdx.x; i < size; i += blockDim.x) {
-        const float v = pr[off + i] + (bias != nullptr ? bias[off + i] : 0.f);
-        ss += v * v;
+      for (int i = threadIdx.x * E; i < size; i += blockDim.x * E) {
+        const RotaryElements<E> x = rotary_load<E>(pr + off + i);
+#pragma unroll
+        for (int j = 0; j < E; ++j) {
+          const float v = x.v[j] + (bias != nullptr ? bias[off + i + j] : 0.f);
+          ss += v * v;
+        }
       }
       return 1.f / sqrtf(block_sum(ss, scratch) / (float)size + eps);
     };
@@ -382,7 +408,7 @@ __global__ __launch_bounds__(256) void rotary_cache_kernel(const float* __restri
   }
   __syncthreads();
   // (a row of a step with few rows is shared by gridDim.y workgroups)
-  const int at0 = blockIdx.y * blockDim.x + threadIdx.x, stride0 = gridDim.y * blockDim.x;
+  const int at0 = (blockIdx.y * blockDim.x + threadIdx.x) * E, stride0 = gridDim.y * blockDim.x * E;
   for (int i = at0; i < (q_heads + kv_heads) * dim; i += stride0) {
     const int h = i / dim, c = i - h * dim;
     const bool is_q = h < q_heads;
@@ -391,28 +417,54 @@ __global__ __launch_bounds__(256) void rotary_cache_kernel(const float* __restri
     const float* bs = bias != nullptr ? bias + at : nullptr;
     const float r = is_q ? rq : rk;
     const float* nw = NORM ? (is_q ? q_norm + (int64_t)h * dim : k_norm + (int64_t)(h - q_heads) * dim) : nullptr;
-    float y = src[c] + (bs != nullptr ? bs[c] : 0.f);
-    if (NORM) y = y * r * nw[c];
+    auto read = [&](int from) {
+      RotaryElements<E> x = rotary_load<E>(src + from);
+      if (bs != nullptr) {
+#pragma unroll
+        for (int j = 0; j < E; ++j) x.v[j] += bs[from + j];
+      }
+      if (NORM) {
+#pragma unroll
+        for (int j = 0; j < E; ++j) x.v[j] = x.v[j] * r * nw[from + j];
+      }
+      return x;
+    };
+    RotaryElements<E> y = read(c);
     if (c < rot_dims) {
-      int pair, partner;
-      bool first;
-      if (interleaved) { pair = c >> 1; partner = c ^ 1; first = (c & 1) == 0; }
-      else { first = c < half; pair = first ? c : c - half; partner = first ? c + half : c - half; }
-      float cs, sn;
-      if (in_lds) { cs = cs_[pair]; sn = sn_[pair]; }
-      else rotary_cos_sin(p, inv_freq[pair], &cs, &sn);
-      float other = src[partner] + (bs != nullptr ? bs[partner] : 0.f);
-      if (NORM) other = other * r * nw[partner];
-      y = first ? y * cs - other * sn : y * cs + other * sn;
+      RotaryElements<E> other;
+      bool first = true;
+      if (!interleaved) { first = c < half; other = read(first ? c + half : c - half); }
+      else if (E == 1) { first = (c & 1) == 0; other = read(c ^ 1); }
+      else {
+#pragma unroll
+        for (int j = 0; j < E; ++j) other.v[j] = y.v[j ^ 1];
+      }
+#pragma unroll
+      for (int j = 0; j < E; ++j) {
+        const int pair = interleaved ? (c + j) >> 1 : first ? c + j : c + j - half;
+        float cs, sn;
+        if (in_lds) { cs = cs_[pair]; sn = sn_[pair]; }
+        else rotary_cos_sin(p, inv_freq[pair], &cs, &sn);
+        const bool lower = interleaved && E > 1 ? (j & 1) == 0 : first;
+        y.v[j] = lower ? y.v[j] * cs - other.v[j] * sn : y.v[j] * cs + other.v[j] * sn;
+      }
     }
-    if (is_q) q_out[(row * q_heads + h) * dim + c] = from_f32<T>(y * q_temp);
-    else if (slot >= 0) k_pages[((page * kv_heads + (h - q_heads)) * page_size + off) * dim + c] = from_f32<T>(y);
+    if (is_q) {
+#pragma unroll
+      for (int j = 0; j < E; ++j) y.v[j] *= q_temp;
+      rotary_store<T, E>(q_out + (row * q_heads + h) * dim + c, y.v);
+    } else if (slot >= 0) {
+      rotary_store<T, E>(k_pages + ((page * kv_heads + (h - q_heads)) * page_size + off) * dim + c, y.v);
+    }
   }
   if (slot >= 0)
     for (int i = at0; i < v_heads * vdim; i += stride0) {
       const int g = i / vdim, c = i - g * vdim;
-      v_pages[((page * v_heads + g) * vdim + c) * page_size + off] =
-          from_f32<T>(pr[v_off + i] + (bias != nullptr ? bias[v_off + i] : 0.f));
+      const RotaryElements<E> x = rotary_load<E>(pr + v_off + i);
+#pragma unroll
+      for (int j = 0; j < E; ++j)
+        v_pages[((page * v_heads + g) * vdim + c + j) * page_size + off] =
+            from_f32<T>(x.v[j] + (bias != nullptr ? bias[v_off + i + j] : 0.f));
     }
 }
 
@@ -752,16 +804,22 @@ int dli_rotary_cache(const float* proj, int64_t stride, int q_off, int k_off, in
       rot_dims > dim || rot_dims % 2 || (rot_dims > 0 && inv_freq == nullptr) || (q_norm != nullptr && kv_heads > 0 && k_norm == nullptr) ||
       (kv_heads > 0 && (k_pages == nullptr || slots == nullptr)) || (v_heads > 0 && (v_pages == nullptr || slots == nullptr)))
     return DLI_ERR_ARGUMENT;
-  const int64_t shares = ((int64_t)(q_heads + kv_heads) * dim + 511) / 512;
+  auto whole = [](const void* at, size_t bytes) { return (uintptr_t)at % bytes == 0; };
+  const bool fours = dim % 4 == 0 && vdim % 4 == 0 && rot_dims % (interleaved ? 4 : 8) == 0 && stride % 4 == 0 && q_off % 4 == 0 &&
+                     k_off % 4 == 0 && v_off % 4 == 0 && whole(proj, 16) && whole(q_out, is_bf16 ? 8 : 16) &&
+                     whole(k_pages, is_bf16 ? 8 : 16);
+  const int64_t shares = ((int64_t)(q_heads + kv_heads) * dim + (fours ? 1023 : 511)) / (fours ? 1024 : 512);
   const dim3 grid(rows, rows >= 128 ? 1 : (unsigned)(shares < 16 ? shares : 16));
-#define ROTARY_CACHE(T, NORM)                                                                                             \
-  rotary_cache_kernel<T, NORM><<<grid, 256, 0, stream>>>(proj, stride, q_off, k_off, v_off, bias, positions, inv_freq,    \
+#define ROTARY_CACHE_E(T, NORM, E)                                                                                        \
+  rotary_cache_kernel<T, NORM, E><<<grid, 256, 0, stream>>>(proj, stride, q_off, k_off, v_off, bias, positions, inv_freq,    \
                                                          rot_dims, interleaved, (T*)q_out, slots, (T*)k_pages, (T*)v_pages, \
                                                          q_heads, kv_heads, v_heads, dim, vdim, page_size, q_coef, q_every, \
                                                          q_norm, k_norm, eps)
+#define ROTARY_CACHE(T, NORM) do { if (fours) ROTARY_CACHE_E(T, NORM, 4); else ROTARY_CACHE_E(T, NORM, 1); } while (0)
   if (is_bf16) { if (q_norm != nullptr) ROTARY_CACHE(bf16_t, true); else ROTARY_CACHE(bf16_t, false); }
   else { if (q_norm != nullptr) ROTARY_CACHE(float, true); else ROTARY_CACHE(float, false); }
 #undef ROTARY_CACHE
+#undef ROTARY_CACHE_E
   return dli_launch_status();
 }
 
