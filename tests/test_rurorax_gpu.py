@@ -113,26 +113,29 @@ def test_the_norm_part_applies_itself(ops):
 
 
 @pytest.mark.parametrize("dtype,tol", [(torch.float32, 5e-6), (torch.bfloat16, 8e-3)])
-@pytest.mark.parametrize("parts,size", [(1, 40), (3, 24), (2, 96), (1, 300), (4, 520), (5, 1), (2, 2052)])
-def test_gate_before_the_norm_in_parts(ops, parts, size, dtype, tol):
+@pytest.mark.parametrize("at", [3, 4], ids=["unaligned", "aligned"])
+@pytest.mark.parametrize("parts,size", [(1, 40), (3, 24), (2, 96), (1, 300), (4, 520), (5, 1), (2, 2052), (1, 4096), (1, 4100)])
+def test_gate_before_the_norm_in_parts(ops, parts, size, at, dtype, tol):
     torch.manual_seed(parts * 7 + size)
     n, width = 6, parts * size
-    y, z, w = 2 * torch.randn(n, width), 2 * torch.randn(n, width + 3), 1 + 0.3 * torch.randn(width)
-    ref = P.gated_parts_norm(y.double(), z.double()[:, 3:], w.double(), parts, 1e-4)
+    y, z, w = 2 * torch.randn(n, width), 2 * torch.randn(n, width + 4), 1 + 0.3 * torch.randn(width)
+    ref = P.gated_parts_norm(y.double(), z.double()[:, at:at + width], w.double(), parts, 1e-4)
     out = torch.empty(n, width, dtype=dtype).cuda()
-    ops.head_norm_gate(y.cuda(), z.cuda()[:, 3:], w.cuda(), 1e-4, out, parts, size, gate="silu_first")
+    ops.head_norm_gate(y.cuda(), z.cuda()[:, at:at + width], w.cuda(), 1e-4, out, parts, size, gate="silu_first")
     assert (out.cpu().double() - ref).abs().max() < tol * ref.abs().max()
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("n", [9, 150])
-@pytest.mark.parametrize("qh,kh,d,dv,rot_dims", [(6, 2, 24, 10, 16), (3, 1, 5, 8, 2), (4, 4, 64, 80, 64), (8, 2, 40, 40, 0), (1, 1, 130, 3, 128)])
-def test_norms_over_whole_projections_before_the_rotation(ops, dtype, n, qh, kh, d, dv, rot_dims):
+@pytest.mark.parametrize("more", [3, 4], ids=["rows_unaligned", "rows_aligned"])
+@pytest.mark.parametrize("qh,kh,d,dv,rot_dims", [(6, 2, 24, 10, 16), (3, 1, 5, 8, 2), (4, 4, 64, 80, 64), (6, 3, 24, 16, 8), (8, 2, 40, 40, 0),
+                                                 (4, 2, 20, 12, 12), (1, 1, 130, 3, 128)])
+def test_norms_over_whole_projections_before_the_rotation(ops, dtype, n, more, qh, kh, d, dv, rot_dims):
     """q and k, heads of very different size, each by one root mean square over all heads; biases first, rotation last, v untouched."""
     g = torch.Generator().manual_seed(qh * 10 + d)
     cols, ps = (qh + kh) * d + kh * dv, 4
-    size = torch.cat([torch.linspace(0.1, 3.0, cols), torch.ones(3)])
-    proj, bias = torch.randn(n, cols + 3, generator=g) * size, torch.randn(cols + 3, generator=g)
+    size = torch.cat([torch.linspace(0.1, 3.0, cols), torch.ones(more)])
+    proj, bias = torch.randn(n, cols + more, generator=g) * size, torch.randn(cols + more, generator=g)
     qw, kw = 1 + 0.3 * torch.randn(qh * d, generator=g), 1 + 0.3 * torch.randn(kh * d, generator=g)
     rot = {"dims": rot_dims, "base": 100.0, "scaling": {"factor": 3.0}} if rot_dims else None
     pos = torch.tensor([0, 1, 2, 700, 701, 5, 9000, 3, 4] + list(range(9, n)))
